@@ -1,4 +1,4 @@
-"""In-tree build of the HIP extension ``eventgpt_amd/_C.so`` for gfx950.
+"""In-tree build of the HIP extensions ``eventgpt_amd/_C.so`` and ``_D.so`` for gfx950.
 
 Drives hipcc directly (no hipify, no JIT cache): every ``csrc/kernels/*.hip``
 is compiled to an object for ``--offload-arch=gfx950`` only, ``csrc/*.cpp`` are
@@ -7,7 +7,12 @@ into one shared library that registers its ops with ``TORCH_LIBRARY`` and is
 loaded with ``torch.ops.load_library``.  Objects are cached under ``build/`` by
 content hash, so rebuilding after a one-file edit takes seconds.
 
-    python -m eventgpt_amd.build          # build if stale
+``_C.so`` (ops ``evgpt::``) serves EventChat and its harness; ``_D.so`` (ops ``evlay::``) the layered
+decoders (``models/layered.py``).  The second one links its own kernels and the few it shares with the
+first, from the same objects, so a process that serves a layered decoder needs only that library.
+
+    python -m eventgpt_amd.build          # build both if stale
+    python -m eventgpt_amd.build --only layered
     python -m eventgpt_amd.build --force  # rebuild everything
 """
 from __future__ import annotations
@@ -26,6 +31,10 @@ PKG_DIR = os.path.dirname(os.path.abspath(__file__))
 CSRC = os.path.join(PKG_DIR, "csrc")
 BUILD_DIR = os.path.join(os.path.dirname(PKG_DIR), "build", "evgpt_C")
 SO_PATH = os.path.join(PKG_DIR, "_C.so")
+LAYERED_SO_PATH = os.path.join(PKG_DIR, "_D.so")
+# kernels of the layered decoders alone, and the ones they share with the rest
+LAYERED_KERNELS = ("attn_chunk", "conv1d", "gemm_f32", "linear_scan", "rowops")
+LAYERED_SHARED = ("attn_decode", "attn_prefill", "gemm", "sd")
 ARCH = "gfx950"
 
 # -packed-fp32-ops is disabled on purpose: some packed-fp32 forms have produced
@@ -82,16 +91,23 @@ def _compile(src: str, flags: List[str], verbose: bool) -> str:
 
 
 def sources():
-    hip = sorted(glob.glob(os.path.join(CSRC, "kernels", "*.hip")))
+    hip = [s for s in sorted(glob.glob(os.path.join(CSRC, "kernels", "*.hip")))
+           if os.path.basename(s)[:-4] not in LAYERED_KERNELS]
     cpp = sorted(glob.glob(os.path.join(CSRC, "*.cpp")))
     return hip, cpp
 
 
+def layered_sources():
+    hip = [os.path.join(CSRC, "kernels", n + ".hip") for n in sorted(LAYERED_KERNELS + LAYERED_SHARED)]
+    return hip, sorted(glob.glob(os.path.join(CSRC, "layered", "*.cpp")))
+
+
 def build(force: bool = False, verbose: bool = False, jobs: int = 8, extra: str = "",
-          out: str = SO_PATH) -> str:
+          out: str = SO_PATH, srcs=None) -> str:
     """``extra``: more hipcc flags for the kernels (``-DEVGPT_...=n`` tuning variants);
-    ``out``: where to link (a variant goes next to ``_C.so`` and is picked with ``EVGPT_SO``)."""
-    hip, cpp = sources()
+    ``out``: where to link (a variant goes next to ``_C.so`` and is picked with ``EVGPT_SO``);
+    ``srcs``: ``(hip, cpp)`` files, default those of ``_C.so``."""
+    hip, cpp = srcs or sources()
     inc, torch_lib = _torch_paths()
     inc_flags = [f"-I{p}" for p in inc] + [f"-I{CSRC}"]
     host_flags = ["-O2", "-std=c++17", "-fPIC",
@@ -108,7 +124,7 @@ def build(force: bool = False, verbose: bool = False, jobs: int = 8, extra: str 
     if (not force and os.path.exists(out) and os.path.exists(stamp_file)
             and open(stamp_file).read() == stamp):
         return out
-    cmd = [_hipcc(), "-shared", "-fPIC", f"--offload-arch={ARCH}", *objs, "-o", out,
+    cmd = [_hipcc(), "-shared", "-fPIC", "-Wl,-Bsymbolic", f"--offload-arch={ARCH}", *objs, "-o", out,
            f"-L{torch_lib}", "-ltorch", "-ltorch_cpu", "-lc10", "-ltorch_hip", "-lc10_hip",
            f"-Wl,-rpath,{torch_lib}"]
     if verbose:
@@ -120,6 +136,11 @@ def build(force: bool = False, verbose: bool = False, jobs: int = 8, extra: str 
     with open(stamp_file, "w") as f:
         f.write(stamp)
     return out
+
+
+def build_layered(verbose: bool = False, jobs: int = 8) -> str:
+    """``_D.so``: the kernels and ops of the layered decoders."""
+    return build(False, verbose, jobs, out=LAYERED_SO_PATH, srcs=layered_sources())
 
 
 def build_tools(verbose: bool = False) -> list:
@@ -152,8 +173,12 @@ def main():
     ap.add_argument("-j", "--jobs", type=int, default=8)
     ap.add_argument("--extra", default="", help="extra hipcc flags for the kernels (tuning variants)")
     ap.add_argument("--out", default=SO_PATH, help="output library (default eventgpt_amd/_C.so)")
+    ap.add_argument("--only", choices=["eventchat", "layered"], default=None, help="build one of the two libraries")
     a = ap.parse_args()
-    print(build(a.force, a.verbose, a.jobs, a.extra, a.out))
+    if a.only != "layered":
+        print(build(a.force, a.verbose, a.jobs, a.extra, a.out))
+    if a.only != "eventchat" and a.out == SO_PATH:
+        print(build_layered(a.verbose, a.jobs))
 
 
 if __name__ == "__main__":

@@ -1,0 +1,515 @@
+// Row kernels around the projections of a layered decoder: the residual stream x is fp32, every norm,
+// gate and rotation is fp32, and what a projection reads is written in the storage type T.
+//
+// One block per row.  A row of a projection (`SrcRows`) may still be split-K slabs, which are summed on
+// load.  Row widths are padded to multiples of 64 by zeros (weights are padded when they are packed), so
+// all accesses are aligned vectors; norms divide by the true width.
+#include "elem.h"
+#include "../layered_kernels.h"
+
+namespace evgpt {
+
+// eight consecutive values of a projection row
+__device__ __forceinline__ void src8(const SrcRows& s, long long row, int col, float (&o)[8]) {
+  if (!s.f32) {
+    load8(static_cast<const bf16_t*>(s.p) + row * s.ld + col, o);
+    return;
+  }
+  const float* p = static_cast<const float*>(s.p) + row * s.ld + col;
+  load8(p, o);
+  for (int k = 1; k < s.nslab; ++k) {
+    float t[8];
+    load8(p + k * s.slab, t);
+#pragma unroll
+    for (int i = 0; i < 8; ++i) o[i] += t[i];
+  }
+}
+__device__ __forceinline__ float src1(const SrcRows& s, long long row, int col) {
+  if (!s.f32) return bf16_to_f32(static_cast<const bf16_t*>(s.p)[row * s.ld + col]);
+  const float* p = static_cast<const float*>(s.p) + row * s.ld + col;
+  float v = p[0];
+  for (int k = 1; k < s.nslab; ++k) v += p[k * s.slab];
+  return v;
+}
+__device__ __forceinline__ float sumsq8(const float (&v)[8]) {
+  float s = 0.f;
+#pragma unroll
+  for (int i = 0; i < 8; ++i) s += v[i] * v[i];
+  return s;
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void embed_rows_kernel(const int* __restrict__ tok, const T* __restrict__ embed,
+                                                         float scale, float* __restrict__ x, int ld, int vocab) {
+  const long long row = blockIdx.x;
+  int t = tok[row];
+  if (t < 0 || t >= vocab) t = 0;
+  for (int c = threadIdx.x * 8; c < ld; c += 2048) {
+    float v[8];
+    load8(embed + static_cast<long long>(t) * ld + c, v);
+#pragma unroll
+    for (int i = 0; i < 8; ++i) v[i] *= scale;
+    store8(x + row * ld + c, v);
+  }
+}
+void launch_embed_rows(const int* tok, const void* embed, bool f32, float scale, float* x, int rows, int ld, int vocab,
+                       hipStream_t st) {
+  if (f32)
+    hipLaunchKernelGGL(embed_rows_kernel<float>, dim3(rows), dim3(256), 0, st, tok, static_cast<const float*>(embed),
+                       scale, x, ld, vocab);
+  else
+    hipLaunchKernelGGL(embed_rows_kernel<bf16_t>, dim3(rows), dim3(256), 0, st, tok,
+                       static_cast<const bf16_t*>(embed), scale, x, ld, vocab);
+}
+
+// The three residual kernels.  MODE 0: xn = norm(x).  MODE 1: x += a first.  MODE 2: x += (norm(a) wa +
+// norm(b) wb) / 2 first.  A thread keeps its first NC chunks of eight in registers between the passes.
+template <typename T, int MODE>
+__global__ __launch_bounds__(256) void residual_norm_kernel(float* __restrict__ x, const int* __restrict__ sel,
+                                                            SrcRows a, SrcRows b, const float* __restrict__ wa,
+                                                            const float* __restrict__ wb, const float* __restrict__ w,
+                                                            T* __restrict__ xn, int n, int ld, float eps) {
+  __shared__ float red[16];
+  const long long row = blockIdx.x, xrow = MODE == 0 && sel ? sel[row] : row;
+  const float inv_n = 1.f / static_cast<float>(n);
+  float* xr = x + xrow * ld;
+  float ra = 0.f, rb = 0.f;
+  if constexpr (MODE == 2) {
+    float sa = 0.f, sb = 0.f;
+    for (int c = threadIdx.x * 8; c < ld; c += 2048) {
+      float t[8];
+      src8(a, row, c, t);
+      sa += sumsq8(t);
+      src8(b, row, c, t);
+      sb += sumsq8(t);
+    }
+    ra = 0.5f * rsqrtf(block_sum(sa, red) * inv_n + eps);
+    rb = 0.5f * rsqrtf(block_sum(sb, red) * inv_n + eps);
+  }
+  constexpr int NC = 4;       // 8192 columns stay in registers
+  float keep[NC][8];
+  float ss = 0.f;
+  auto value = [&](int c, float (&v)[8]) {
+    load8(xr + c, v);
+    if constexpr (MODE == 1) {
+      float t[8];
+      src8(a, row, c, t);
+#pragma unroll
+      for (int i = 0; i < 8; ++i) v[i] += t[i];
+    }
+    if constexpr (MODE == 2) {
+      float t[8], u[8], p[8], q[8];
+      src8(a, row, c, t);
+      src8(b, row, c, u);
+      load8(wa + c, p);
+      load8(wb + c, q);
+#pragma unroll
+      for (int i = 0; i < 8; ++i) v[i] += t[i] * ra * p[i] + u[i] * rb * q[i];
+    }
+    if constexpr (MODE != 0) store8(xr + c, v);
+    ss += sumsq8(v);
+  };
+#pragma unroll
+  for (int k = 0; k < NC; ++k) {
+    const int c = (threadIdx.x + k * 256) * 8;
+    if (c < ld) value(c, keep[k]);
+  }
+  for (int c = (threadIdx.x + NC * 256) * 8; c < ld; c += 2048) {
+    float v[8];
+    value(c, v);
+  }
+  if (w == nullptr) return;
+  const float r = rsqrtf(block_sum(ss, red) * inv_n + eps);
+  T* o = xn + row * ld;
+  auto put = [&](int c, const float (&v)[8]) {
+    float g[8];
+    load8(w + c, g);
+#pragma unroll
+    for (int i = 0; i < 8; ++i) g[i] *= v[i] * r;
+    store8(o + c, g);
+  };
+#pragma unroll
+  for (int k = 0; k < NC; ++k) {
+    const int c = (threadIdx.x + k * 256) * 8;
+    if (c < ld) put(c, keep[k]);
+  }
+  for (int c = (threadIdx.x + NC * 256) * 8; c < ld; c += 2048) {   // each thread re-reads what it wrote
+    float v[8];
+    load8(xr + c, v);
+    put(c, v);
+  }
+}
+template <int MODE>
+static void launch_residual(float* x, const int* sel, const SrcRows& a, const SrcRows& b, const float* wa,
+                            const float* wb, const float* w, void* xn, bool f32, int rows, int n, int ld, float eps,
+                            hipStream_t st) {
+  if (f32)
+    hipLaunchKernelGGL((residual_norm_kernel<float, MODE>), dim3(rows), dim3(256), 0, st, x, sel, a, b, wa, wb, w,
+                       static_cast<float*>(xn), n, ld, eps);
+  else
+    hipLaunchKernelGGL((residual_norm_kernel<bf16_t, MODE>), dim3(rows), dim3(256), 0, st, x, sel, a, b, wa, wb, w,
+                       static_cast<bf16_t*>(xn), n, ld, eps);
+}
+void launch_norm_rows(const float* x, const int* sel, const float* w, void* xn, bool f32, int rows, int n, int ld,
+                      float eps, hipStream_t st) {
+  launch_residual<0>(const_cast<float*>(x), sel, SrcRows{}, SrcRows{}, nullptr, nullptr, w, xn, f32, rows, n, ld, eps, st);
+}
+void launch_add_norm_rows(float* x, const SrcRows& y, const float* w, void* xn, bool f32, int rows, int n, int ld,
+                          float eps, hipStream_t st) {
+  launch_residual<1>(x, nullptr, y, SrcRows{}, nullptr, nullptr, w, xn, f32, rows, n, ld, eps, st);
+}
+void launch_merge_norm_rows(float* x, const SrcRows& a, const SrcRows& b, const float* wa, const float* wb,
+                            const float* w, void* xn, bool f32, int rows, int n, int ld, float eps, hipStream_t st) {
+  launch_residual<2>(x, nullptr, a, b, wa, wb, w, xn, f32, rows, n, ld, eps, st);
+}
+
+template <typename T, int ACT>
+__global__ __launch_bounds__(256) void glu_rows_kernel(SrcRows src, T* __restrict__ h, long long total, int ip) {
+  const int per = ip >> 3;
+  for (long long i = blockIdx.x * 256ll + threadIdx.x; i < total; i += gridDim.x * 256ll) {
+    const long long row = i / per;
+    const int c = static_cast<int>(i % per) * 8;
+    float a[8], b[8];
+    src8(src, row, c, a);
+    src8(src, row, ip + c, b);
+#pragma unroll
+    for (int j = 0; j < 8; ++j) a[j] = (ACT == GLU_SILU ? a[j] * sigmoid_f(a[j]) : gelu_tanh_f(a[j])) * b[j];
+    store8(h + row * ip + c, a);
+  }
+}
+void launch_glu_rows(const SrcRows& src, void* h, bool f32, int rows, int ip, int act, hipStream_t st) {
+  const long long total = static_cast<long long>(rows) * (ip / 8);
+  const long long want = (total + 255) / 256;
+  const dim3 grid(static_cast<unsigned>(want < 4096 ? want : 4096)), block(256);
+  if (f32) {
+    if (act == GLU_SILU) hipLaunchKernelGGL((glu_rows_kernel<float, GLU_SILU>), grid, block, 0, st, src, static_cast<float*>(h), total, ip);
+    else hipLaunchKernelGGL((glu_rows_kernel<float, GLU_GELU_TANH>), grid, block, 0, st, src, static_cast<float*>(h), total, ip);
+  } else {
+    if (act == GLU_SILU) hipLaunchKernelGGL((glu_rows_kernel<bf16_t, GLU_SILU>), grid, block, 0, st, src, static_cast<bf16_t*>(h), total, ip);
+    else hipLaunchKernelGGL((glu_rows_kernel<bf16_t, GLU_GELU_TANH>), grid, block, 0, st, src, static_cast<bf16_t*>(h), total, ip);
+  }
+}
+
+// Group norm with a gate.  The row is staged in LDS (gated first when the gate comes before the norm), every
+// part's root mean square is taken over its run of true channels -- a wave per part -- and the row is written
+// with the part of each channel looked up.
+template <typename T, bool BEFORE>
+__global__ __launch_bounds__(256) void group_norm_kernel(const T* __restrict__ y, SrcRows gate, int gcol,
+                                                         const float* __restrict__ w, T* __restrict__ out, int heads,
+                                                         int v, int vp, int parts, int ld_out, float eps) {
+  extern __shared__ __attribute__((aligned(16))) float row_lds[];   // [heads * vp] values, then [parts]
+  const int slots = heads * vp, plen = heads * v / parts;
+  float* inv = row_lds + slots;
+  const long long row = blockIdx.x;
+  for (int c = threadIdx.x * 8; c < slots; c += 2048) {
+    float a[8];
+    load8(y + row * slots + c, a);
+    if constexpr (BEFORE) {
+      float g[8];
+      src8(gate, row, gcol + c, g);
+#pragma unroll
+      for (int i = 0; i < 8; ++i) a[i] *= g[i] * sigmoid_f(g[i]);
+    }
+    store8(row_lds + c, a);
+  }
+  __syncthreads();
+  const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
+  if (parts >= 4) {
+    for (int p = wid; p < parts; p += 4) {
+      float s = 0.f;
+      for (int i = lane; i < plen; i += 64) {
+        const int c = p * plen + i;
+        const float t = row_lds[(c / v) * vp + c % v];
+        s += t * t;
+      }
+      s = wave_sum(s);
+      if (lane == 0) inv[p] = rsqrtf(s / static_cast<float>(plen) + eps);
+    }
+  } else {
+    __shared__ float red[16];
+    for (int p = 0; p < parts; ++p) {
+      float s = 0.f;
+      for (int i = threadIdx.x; i < plen; i += 256) {
+        const int c = p * plen + i;
+        const float t = row_lds[(c / v) * vp + c % v];
+        s += t * t;
+      }
+      s = block_sum(s, red);
+      if (threadIdx.x == 0) inv[p] = rsqrtf(s / static_cast<float>(plen) + eps);
+    }
+  }
+  __syncthreads();
+  for (int c = threadIdx.x * 8; c < ld_out; c += 2048) {
+    float a[8] = {0, 0, 0, 0, 0, 0, 0, 0};
+    if (c < slots) {
+      float g[8];
+      load8(row_lds + c, a);
+      load8(w + c, g);
+      const int h = c / vp, c0 = h * v + c % vp;      // vp is a multiple of 8: eight slots of one head
+#pragma unroll
+      for (int i = 0; i < 8; ++i) {
+        const int part = min((c0 + i) / plen, parts - 1);   // padding slots have zero weight
+        a[i] *= inv[part] * g[i];
+      }
+      if constexpr (!BEFORE) {
+        float t[8];
+        src8(gate, row, gcol + c, t);
+#pragma unroll
+        for (int i = 0; i < 8; ++i) a[i] *= sigmoid_f(t[i]);
+      }
+    }
+    store8(out + row * ld_out + c, a);
+  }
+}
+void launch_group_norm_rows(const void* y, const SrcRows& gate, int gcol, bool gate_before, const float* w, void* out,
+                            bool f32, int rows, int heads, int v, int vp, int parts, int ld_out, float eps,
+                            hipStream_t st) {
+  const size_t lds = (static_cast<size_t>(heads) * vp + parts) * 4;
+  auto go = [&](auto* kern, auto* t) {
+    typedef std::remove_pointer_t<decltype(t)> T;
+    hipLaunchKernelGGL(kern, dim3(rows), dim3(256), lds, st, static_cast<const T*>(y), gate, gcol, w,
+                       static_cast<T*>(out), heads, v, vp, parts, ld_out, eps);
+  };
+  if (f32) {
+    if (gate_before) go(group_norm_kernel<float, true>, static_cast<float*>(nullptr));
+    else go(group_norm_kernel<float, false>, static_cast<float*>(nullptr));
+  } else {
+    if (gate_before) go(group_norm_kernel<bf16_t, true>, static_cast<bf16_t*>(nullptr));
+    else go(group_norm_kernel<bf16_t, false>, static_cast<bf16_t*>(nullptr));
+  }
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void convert_rows_kernel(SrcRows src, int col0, T* __restrict__ out, long long total,
+                                                           int cols, int ld_out) {
+  const int per = cols >> 3;
+  for (long long i = blockIdx.x * 256ll + threadIdx.x; i < total; i += gridDim.x * 256ll) {
+    const long long row = i / per;
+    const int c = static_cast<int>(i % per) * 8;
+    float a[8];
+    src8(src, row, col0 + c, a);
+    store8(out + row * ld_out + c, a);
+  }
+}
+void launch_convert_rows(const SrcRows& src, int col0, void* out, bool f32, int rows, int cols, int ld_out,
+                         hipStream_t st) {
+  const long long total = static_cast<long long>(rows) * (cols / 8);
+  const long long want = (total + 255) / 256;
+  const dim3 grid(static_cast<unsigned>(want < 4096 ? want : 4096));
+  if (f32) hipLaunchKernelGGL(convert_rows_kernel<float>, grid, dim3(256), 0, st, src, col0, static_cast<float*>(out), total, cols, ld_out);
+  else hipLaunchKernelGGL(convert_rows_kernel<bf16_t>, grid, dim3(256), 0, st, src, col0, static_cast<bf16_t*>(out), total, cols, ld_out);
+}
+
+// First index of the row's maximum (NaN never wins).
+__global__ __launch_bounds__(1024) void argmax_logits_kernel(const float* __restrict__ logits, long long ld,
+                                                             int* __restrict__ out, int vocab) {
+  __shared__ float sv[16];
+  __shared__ int si[16];
+  const float* r = logits + blockIdx.x * ld;
+  float bv = -INFINITY;
+  int bi = 0x7fffffff;
+  for (int i = threadIdx.x; i < vocab; i += 1024) {
+    const float v = r[i];
+    if (v > bv || (v == bv && i < bi)) { bv = v; bi = i; }
+  }
+#pragma unroll
+  for (int off = 32; off > 0; off >>= 1) {
+    const float ov = __shfl_xor(bv, off, 64);
+    const int oi = __shfl_xor(bi, off, 64);
+    if (ov > bv || (ov == bv && oi < bi)) { bv = ov; bi = oi; }
+  }
+  const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
+  if (lane == 0) { sv[wid] = bv; si[wid] = bi; }
+  __syncthreads();
+  if (threadIdx.x == 0) {
+    for (int w = 1; w < 16; ++w)
+      if (sv[w] > bv || (sv[w] == bv && si[w] < bi)) { bv = sv[w]; bi = si[w]; }
+    out[blockIdx.x] = bi == 0x7fffffff ? 0 : bi;
+  }
+}
+void launch_argmax_logits(const float* logits, long long ld, int* out, int rows, int vocab, hipStream_t st) {
+  hipLaunchKernelGGL(argmax_logits_kernel, dim3(rows), dim3(1024), 0, st, logits, ld, out, vocab);
+}
+
+// Commit of one token per sequence, as commit_token_kernel does it, staging the scaled embedding row as
+// the fp32 residual stream of the next step.
+template <typename T>
+__global__ __launch_bounds__(256) void commit_rows_kernel(const int* __restrict__ sampled, const T* __restrict__ embed,
+                                                          float scale, float* __restrict__ x,
+                                                          int* __restrict__ out_tokens, int max_out,
+                                                          int* __restrict__ step, int* __restrict__ pos,
+                                                          int* __restrict__ done, int* __restrict__ cur_token, int eos,
+                                                          int ld, int vocab, const int* __restrict__ active) {
+  const int b = blockIdx.x;
+  if (active && !active[b]) return;
+  int tok = sampled[b];
+  if (tok < 0 || tok >= vocab) tok = 0;
+  for (int c = threadIdx.x * 8; c < ld; c += 2048) {
+    float v[8];
+    load8(embed + static_cast<long long>(tok) * ld + c, v);
+#pragma unroll
+    for (int i = 0; i < 8; ++i) v[i] *= scale;
+    store8(x + static_cast<long long>(b) * ld + c, v);
+  }
+  if (threadIdx.x == 0) {
+    const int st = step[b];
+    if (st >= 0 && st < max_out) out_tokens[static_cast<long long>(b) * max_out + st] = tok;
+    cur_token[b] = tok;
+    if (tok == eos) done[b] = 1;
+    step[b] = st + 1;
+    pos[b] = pos[b] + 1;
+  }
+}
+void launch_commit_rows(const int* sampled, const void* embed, bool f32, float scale, float* x, int* out_tokens,
+                        int max_out, int* step, int* pos, int* done, int* cur_token, int eos, int B, int ld, int vocab,
+                        const int* active, hipStream_t st) {
+  if (f32)
+    hipLaunchKernelGGL(commit_rows_kernel<float>, dim3(B), dim3(256), 0, st, sampled, static_cast<const float*>(embed),
+                       scale, x, out_tokens, max_out, step, pos, done, cur_token, eos, ld, vocab, active);
+  else
+    hipLaunchKernelGGL(commit_rows_kernel<bf16_t>, dim3(B), dim3(256), 0, st, sampled,
+                       static_cast<const bf16_t*>(embed), scale, x, out_tokens, max_out, step, pos, done, cur_token,
+                       eos, ld, vocab, active);
+}
+
+// Attention inputs of one row.
+template <typename T>
+__global__ __launch_bounds__(256) void attn_prep_kernel(AttnPrepArgs a) {
+  __shared__ float red[16];
+  const long long row = blockIdx.x;
+  const int qn = a.Hq * a.D, kn = a.Hkv * a.D, half = a.rot >> 1;
+  float rq = 1.f, rk = 1.f;
+  if (a.qw) {
+    float s = 0.f;
+    for (int c = threadIdx.x * 8; c < qn; c += 2048) {
+      float t[8];
+      src8(a.src, row, a.q_col + c, t);
+      s += sumsq8(t);
+    }
+    rq = rsqrtf(block_sum(s, red) / static_cast<float>(a.nq) + a.eps);
+  }
+  if (a.kw) {
+    float s = 0.f;
+    for (int c = threadIdx.x * 8; c < kn; c += 2048) {
+      float t[8];
+      src8(a.src, row, a.k_col + c, t);
+      s += sumsq8(t);
+    }
+    rk = rsqrtf(block_sum(s, red) / static_cast<float>(a.nk) + a.eps);
+  }
+  const int p = a.row_pos[row];
+  const int pt = min(max(p, 0), a.max_pos - 1);
+  const float* cs = a.cos_tab + static_cast<long long>(pt) * half;
+  const float* sn = a.sin_tab + static_cast<long long>(pt) * half;
+  const long long slot = a.row_slot ? a.row_slot[row] : row;
+  const bool keep = a.row_keep == nullptr || a.row_keep[row] != 0;
+  const long long kv = a.row_kv ? a.row_kv[row] : -1;
+  const int cslot = p % a.cap;
+  // normalised and rotated element d of head h of a section
+  auto value = [&](int col, const float* w, float r, int h, int d) {
+    const int c = h * a.D + d;
+    float u = src1(a.src, row, col + c) * r;
+    if (w) u *= w[c];
+    if (d < a.rot) {
+      const int i = d < half ? d : d - half, c2 = d < half ? c + half : c - half;
+      float o = src1(a.src, row, col + c2) * r;
+      if (w) o *= w[c2];
+      u = d < half ? u * cs[i] - o * sn[i] : u * cs[i] + o * sn[i];
+    }
+    return u;
+  };
+  T* q = static_cast<T*>(a.q_out) + row * qn;
+  for (int c = threadIdx.x; c < qn; c += 256) q[c] = from_f32<T>(value(a.q_col, a.qw, rq, c / a.D, c % a.D));
+  for (int c = threadIdx.x; c < kn; c += 256) {
+    const int h = c / a.D, d = c % a.D;
+    const T kk = from_f32<T>(value(a.k_col, a.kw, rk, h, d));
+    const T vv = from_f32<T>(src1(a.src, row, a.v_col + c));
+    if (kv >= 0) {
+      static_cast<T*>(a.k_buf)[kv * kn + c] = kk;
+      static_cast<T*>(a.v_buf)[kv * kn + c] = vv;
+    }
+    if (keep) {
+      const long long o = ((slot * a.Hkv + h) * a.cap + cslot) * a.D + d;
+      static_cast<T*>(a.k_cache)[o] = kk;
+      static_cast<T*>(a.v_cache)[o] = vv;
+    }
+  }
+}
+void launch_attn_prep(const AttnPrepArgs& a, bool f32, int rows, hipStream_t st) {
+  if (f32) hipLaunchKernelGGL(attn_prep_kernel<float>, dim3(rows), dim3(256), 0, st, a);
+  else hipLaunchKernelGGL(attn_prep_kernel<bf16_t>, dim3(rows), dim3(256), 0, st, a);
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void chunk_keys_copy_kernel(const T* __restrict__ kc, const T* __restrict__ vc,
+                                                              T* __restrict__ kb, T* __restrict__ vb,
+                                                              const int* __restrict__ copies, int Hkv, int cap, int D) {
+  const int* c = copies + blockIdx.y * 4;
+  const long long slot = c[0];
+  const int first = c[1], dst = c[2], count = c[3];
+  for (int i = blockIdx.x; i < count; i += gridDim.x)
+    for (int e = threadIdx.x; e < Hkv * D; e += 256) {
+      const long long s = ((slot * Hkv + e / D) * cap + (first + i) % cap) * D + e % D;
+      const long long o = static_cast<long long>(dst + i) * Hkv * D + e;
+      kb[o] = kc[s];
+      vb[o] = vc[s];
+    }
+}
+void launch_chunk_keys_copy(const void* k_cache, const void* v_cache, void* k_buf, void* v_buf, const int* copies, int n,
+                            bool f32, int Hkv, int cap, int D, hipStream_t st) {
+  const dim3 grid(256, n);
+  if (f32)
+    hipLaunchKernelGGL(chunk_keys_copy_kernel<float>, grid, dim3(256), 0, st, static_cast<const float*>(k_cache),
+                       static_cast<const float*>(v_cache), static_cast<float*>(k_buf), static_cast<float*>(v_buf), copies,
+                       Hkv, cap, D);
+  else
+    hipLaunchKernelGGL(chunk_keys_copy_kernel<bf16_t>, grid, dim3(256), 0, st, static_cast<const bf16_t*>(k_cache),
+                       static_cast<const bf16_t*>(v_cache), static_cast<bf16_t*>(k_buf), static_cast<bf16_t*>(v_buf),
+                       copies, Hkv, cap, D);
+}
+
+// log gates of the matrix memory
+__global__ __launch_bounds__(256) void mlstm_gates_kernel(SrcRows src, int i_col, int f_col,
+                                                          const float* __restrict__ ib, const float* __restrict__ fb,
+                                                          float cap, float* __restrict__ li, float* __restrict__ lf,
+                                                          int total, int H) {
+  const int i = blockIdx.x * 256 + threadIdx.x;
+  if (i >= total) return;
+  const int row = i / H, h = i % H;
+  li[i] = cap * tanhf((src1(src, row, i_col + h) + ib[h]) / cap);
+  const float f = cap * tanhf((src1(src, row, f_col + h) + fb[h]) / cap);
+  lf[i] = -softplus_f(-f);
+}
+void launch_mlstm_gates(const SrcRows& src, int i_col, int f_col, const float* ib, const float* fb, float cap, float* li,
+                        float* lf, int rows, int H, hipStream_t st) {
+  const int total = rows * H;
+  hipLaunchKernelGGL(mlstm_gates_kernel, dim3((total + 255) / 256), dim3(256), 0, st, src, i_col, f_col, ib, fb, cap, li,
+                     lf, total, H);
+}
+
+__global__ __launch_bounds__(256) void ssd_gates_kernel(SrcRows src, int col, const float* __restrict__ dt_bias,
+                                                        const float* __restrict__ a_log, float* __restrict__ log_decay,
+                                                        float* __restrict__ dt, int total, int H) {
+  const int i = blockIdx.x * 256 + threadIdx.x;
+  if (i >= total) return;
+  const int row = i / H, h = i % H;
+  const float d = softplus_f(src1(src, row, col + h) + dt_bias[h]);
+  dt[i] = d;
+  log_decay[i] = -expf(a_log[h]) * d;
+}
+void launch_ssd_gates(const SrcRows& src, int col, const float* dt_bias, const float* a_log, float* log_decay, float* dt,
+                      int rows, int H, hipStream_t st) {
+  const int total = rows * H;
+  hipLaunchKernelGGL(ssd_gates_kernel, dim3((total + 255) / 256), dim3(256), 0, st, src, col, dt_bias, a_log, log_decay,
+                     dt, total, H);
+}
+
+__global__ void mod_pos_kernel(const int* pos, int* out, int B, int cap) {
+  const int i = blockIdx.x * 256 + threadIdx.x;
+  if (i < B) out[i] = pos[i] % cap;
+}
+void launch_mod_pos(const int* pos, int* out, int B, int cap, hipStream_t st) {
+  hipLaunchKernelGGL(mod_pos_kernel, dim3((B + 255) / 256), dim3(256), 0, st, pos, out, B, cap);
+}
+
+}  // namespace evgpt

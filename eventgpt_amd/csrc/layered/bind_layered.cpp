@@ -1,0 +1,472 @@
+// torch op registration for the layered decoders (namespace `evlay`), a library of its own (`_D.so`): a
+// deployment of such a model builds these kernels and the shared GEMM / attention / sampling ones, nothing else.
+// As in bind.cpp, operands are checked here so that no kernel is launched on shapes its indexing does not assume.
+#include <algorithm>
+#include <ATen/ATen.h>
+#include <c10/hip/HIPStream.h>
+#include <torch/library.h>
+
+#include "../evgpt_kernels.h"
+#include "../layered_kernels.h"
+
+namespace {
+
+using at::Tensor;
+using OptTensor = c10::optional<Tensor>;
+using evgpt::SrcRows;
+
+hipStream_t cur_stream() { return c10::hip::getCurrentHIPStream().stream(); }
+
+void check_t(const Tensor& t, const char* name) {       // storage type T: bf16 or fp32
+  TORCH_CHECK(t.is_cuda() && t.is_contiguous(), name, " must be a contiguous GPU tensor");
+  TORCH_CHECK(t.scalar_type() == at::kBFloat16 || t.scalar_type() == at::kFloat, name, " must be bfloat16 or float32");
+  TORCH_CHECK((reinterpret_cast<uintptr_t>(t.data_ptr()) & 15) == 0, name, " must be 16-byte aligned");
+}
+bool is_f32(const Tensor& t) { return t.scalar_type() == at::kFloat; }
+void check_f(const Tensor& t, const char* name) { check_t(t, name); TORCH_CHECK(is_f32(t), name, " must be float32"); }
+void check_i(const Tensor& t, const char* name) {
+  TORCH_CHECK(t.is_cuda() && t.is_contiguous() && t.scalar_type() == at::kInt, name, " must be a contiguous int32 GPU tensor");
+}
+const float* fptr(const OptTensor& t) { return t.has_value() && t->defined() ? t->data_ptr<float>() : nullptr; }
+const int* iptr(const OptTensor& t) { return t.has_value() && t->defined() ? t->data_ptr<int>() : nullptr; }
+const evgpt::bf16_t* bptr(const Tensor& t) { return reinterpret_cast<const evgpt::bf16_t*>(t.data_ptr()); }
+evgpt::bf16_t* bptr_mut(const Tensor& t) { return reinterpret_cast<evgpt::bf16_t*>(t.data_ptr()); }
+at::ScalarType t_of(bool f32) { return f32 ? at::kFloat : at::kBFloat16; }
+
+// rows of a projection: [M, ld] of either type (ld may be a row stride of a wider matrix), or fp32 slabs [S, M, ld]
+SrcRows src_of(const Tensor& t, const char* name, int64_t* rows, int64_t* cols) {
+  TORCH_CHECK(t.is_cuda() && (t.dim() == 2 || t.dim() == 3) && t.stride(-1) == 1, name, " must be [M, N] or [S, M, N]");
+  TORCH_CHECK(t.scalar_type() == at::kFloat || (t.scalar_type() == at::kBFloat16 && t.dim() == 2), name, ": bf16 or fp32");
+  const int64_t ld = t.stride(-2);
+  TORCH_CHECK((reinterpret_cast<uintptr_t>(t.data_ptr()) & 15) == 0 && (t.size(-2) == 1 || ld % 8 == 0) && t.size(-1) % 8 == 0,
+              name, ": rows must be aligned vectors of eight");
+  *rows = t.size(-2);
+  *cols = t.size(-1);
+  return SrcRows{t.data_ptr(), t.dim() == 3 ? t.stride(0) : 0, t.dim() == 3 ? (int)t.size(0) : 1, (int)ld, is_f32(t)};
+}
+
+// ---------------------------------------------------------------- projections
+Tensor linear(const Tensor& x, const Tensor& w, bool out_f32) {
+  check_t(x, "x"); check_t(w, "w");
+  TORCH_CHECK(x.dim() == 2 && w.dim() == 2 && x.scalar_type() == w.scalar_type(), "linear: x [M, K], w [N, K] of one type");
+  const int64_t M = x.size(0), K = x.size(1), N = w.size(0);
+  TORCH_CHECK(w.size(1) == K && K % 64 == 0 && K > 0 && N % 8 == 0, "linear: K % 64 == 0, N % 8 == 0");
+  TORCH_CHECK(M * K < (1ll << 30) && N * K < (1ll << 30) && M * N < (1ll << 31), "linear: operands are addressed with 32-bit offsets");
+  if (is_f32(x)) {
+    Tensor y = at::empty({M, N}, x.options());
+    if (M > 0)
+      evgpt::launch_gemm_f32(x.data_ptr<float>(), w.data_ptr<float>(), y.data_ptr<float>(), (int)M, (int)N, (int)K, (int)K,
+                             (int)K, (int)N, cur_stream());
+    return y;
+  }
+  Tensor y = at::empty({M, N}, x.options().dtype(t_of(out_f32)));
+  if (M == 0) return y;
+  const int sk = evgpt::gemm_splitk((int)M, (int)N, (int)K);
+  Tensor ws;
+  if (sk > 1) {
+    ws = at::empty({sk * M * N}, x.options().dtype(at::kFloat));
+  } else {
+    const int64_t tail = evgpt::gemm_tail_ws_floats((int)M, (int)N, (int)K);
+    if (tail > 0) ws = at::empty({tail}, x.options().dtype(at::kFloat));
+  }
+  evgpt::launch_gemm_bf16(bptr(x), bptr(w), out_f32 ? nullptr : bptr_mut(y), out_f32 ? y.data_ptr<float>() : nullptr, nullptr,
+                          nullptr, (int)M, (int)N, (int)K, (int)K, (int)K, (int)N, 0, nullptr, nullptr,
+                          ws.defined() ? ws.data_ptr<float>() : nullptr, sk, cur_stream());
+  return y;
+}
+
+// fp32 split-K slabs [S, M, N] for a consumer that sums them (fp32 operands: one slab)
+Tensor linear_slabs(const Tensor& x, const Tensor& w) {
+  if (is_f32(x)) return linear(x, w, true).unsqueeze(0);
+  check_t(x, "x"); check_t(w, "w");
+  TORCH_CHECK(x.dim() == 2 && w.dim() == 2 && !is_f32(w), "linear_slabs: x [M, K], w [N, K] of one type");
+  const int64_t M = x.size(0), K = x.size(1), N = w.size(0);
+  TORCH_CHECK(M >= 1 && w.size(1) == K && K % 64 == 0 && K > 0 && N % 8 == 0, "linear_slabs: K % 64 == 0, N % 8 == 0");
+  TORCH_CHECK(M * K < (1ll << 30) && N * K < (1ll << 30), "linear_slabs: operands are addressed with 32-bit offsets");
+  const int sk = evgpt::gemm_splitk_slabs((int)M, (int)N, (int)K);
+  Tensor ws = at::empty({sk, M, N}, x.options().dtype(at::kFloat));
+  const int used = evgpt::launch_gemm_partial(bptr(x), bptr(w), ws.data_ptr<float>(), (int)M, (int)N, (int)K, (int)K, (int)K,
+                                              cur_stream(), 0);
+  return used == sk ? ws : ws.narrow(0, 0, used);
+}
+
+// ---------------------------------------------------------------- rows
+Tensor embed_rows(const Tensor& tok, const Tensor& embed, double scale) {
+  check_i(tok, "tokens"); check_t(embed, "embed");
+  TORCH_CHECK(embed.dim() == 2 && embed.size(1) % 64 == 0, "embed: [V, padded width]");
+  const int64_t M = tok.numel(), ld = embed.size(1);
+  Tensor x = at::empty({M, ld}, embed.options().dtype(at::kFloat));
+  if (M > 0)
+    evgpt::launch_embed_rows(tok.data_ptr<int>(), embed.data_ptr(), is_f32(embed), (float)scale, x.data_ptr<float>(), (int)M,
+                             (int)ld, (int)embed.size(0), cur_stream());
+  return x;
+}
+
+void check_stream(const Tensor& x, int64_t n) {
+  check_f(x, "x");
+  TORCH_CHECK(x.dim() == 2 && x.size(1) % 64 == 0 && n >= 1 && n <= x.size(1), "x: [M, padded width]");
+}
+Tensor norm_rows(const Tensor& x, const OptTensor& sel, const Tensor& w, int64_t n, double eps, bool f32) {
+  check_stream(x, n); check_f(w, "w");
+  TORCH_CHECK(w.numel() == x.size(1), "norm_rows: weight size");
+  if (sel.has_value()) check_i(*sel, "sel");
+  const int64_t M = sel.has_value() ? sel->numel() : x.size(0);
+  Tensor xn = at::empty({M, x.size(1)}, x.options().dtype(t_of(f32)));
+  if (M > 0)
+    evgpt::launch_norm_rows(x.data_ptr<float>(), iptr(sel), w.data_ptr<float>(), xn.data_ptr(), f32, (int)M, (int)n,
+                            (int)x.size(1), (float)eps, cur_stream());
+  return xn;
+}
+SrcRows stream_src(const Tensor& y, const Tensor& x, const char* name) {
+  int64_t r, c;
+  const SrcRows s = src_of(y, name, &r, &c);
+  TORCH_CHECK(r == x.size(0) && c >= x.size(1), name, ": rows of the residual stream");
+  return s;
+}
+Tensor xn_of(const Tensor& x, const OptTensor& w, bool f32) {
+  if (!w.has_value()) return at::empty({0}, x.options().dtype(t_of(f32)));
+  check_f(*w, "w");
+  TORCH_CHECK(w->numel() == x.size(1), "norm weight size");
+  return at::empty({x.size(0), x.size(1)}, x.options().dtype(t_of(f32)));
+}
+Tensor add_norm_rows_(const Tensor& x, const Tensor& y, const OptTensor& w, int64_t n, double eps, bool f32) {
+  check_stream(x, n);
+  const SrcRows s = stream_src(y, x, "y");
+  Tensor xn = xn_of(x, w, f32);
+  evgpt::launch_add_norm_rows(x.data_ptr<float>(), s, fptr(w), xn.data_ptr(), f32, (int)x.size(0), (int)n, (int)x.size(1),
+                              (float)eps, cur_stream());
+  return xn;
+}
+Tensor merge_norm_rows_(const Tensor& x, const Tensor& a, const Tensor& b, const Tensor& wa, const Tensor& wb,
+                        const OptTensor& w, int64_t n, double eps, bool f32) {
+  check_stream(x, n); check_f(wa, "wa"); check_f(wb, "wb");
+  TORCH_CHECK(wa.numel() == x.size(1) && wb.numel() == x.size(1), "merge_norm_rows: branch weights");
+  const SrcRows sa = stream_src(a, x, "a"), sb = stream_src(b, x, "b");
+  Tensor xn = xn_of(x, w, f32);
+  evgpt::launch_merge_norm_rows(x.data_ptr<float>(), sa, sb, wa.data_ptr<float>(), wb.data_ptr<float>(), fptr(w),
+                                xn.data_ptr(), f32, (int)x.size(0), (int)n, (int)x.size(1), (float)eps, cur_stream());
+  return xn;
+}
+Tensor glu_rows(const Tensor& src, int64_t act, bool f32) {
+  int64_t M, N;
+  const SrcRows s = src_of(src, "src", &M, &N);
+  TORCH_CHECK(N % 16 == 0 && (act == evgpt::GLU_GELU_TANH || act == evgpt::GLU_SILU), "glu_rows: [M, 2 I], act 0 or 1");
+  Tensor h = at::empty({M, N / 2}, src.options().dtype(t_of(f32)));
+  evgpt::launch_glu_rows(s, h.data_ptr(), f32, (int)M, (int)(N / 2), (int)act, cur_stream());
+  return h;
+}
+Tensor group_norm_rows(const Tensor& y, const Tensor& gate, int64_t gcol, bool before, const Tensor& w, int64_t heads,
+                       int64_t v, int64_t vp, int64_t parts, int64_t ld_out, double eps) {
+  check_t(y, "y"); check_f(w, "w");
+  int64_t M, N;
+  const SrcRows s = src_of(gate, "gate", &M, &N);
+  TORCH_CHECK(y.numel() == M * heads * vp && w.numel() == heads * vp && vp % 8 == 0 && v >= 1 && v <= vp, "group_norm_rows: y [M, heads, vp]");
+  TORCH_CHECK(gcol >= 0 && gcol % 8 == 0 && gcol + heads * vp <= N, "group_norm_rows: gate columns");
+  TORCH_CHECK(parts >= 1 && heads * v % parts == 0 && ld_out % 8 == 0 && ld_out >= heads * vp, "group_norm_rows: parts, ld_out");
+  TORCH_CHECK((heads * vp + parts) * 4 <= 150 * 1024, "group_norm_rows: row too wide for LDS");
+  Tensor o = at::empty({M, ld_out}, y.options());
+  evgpt::launch_group_norm_rows(y.data_ptr(), s, (int)gcol, before, w.data_ptr<float>(), o.data_ptr(), is_f32(y), (int)M,
+                                (int)heads, (int)v, (int)vp, (int)parts, (int)ld_out, (float)eps, cur_stream());
+  return o;
+}
+Tensor convert_rows(const Tensor& src, int64_t col0, int64_t cols, bool f32) {
+  int64_t M, N;
+  const SrcRows s = src_of(src, "src", &M, &N);
+  TORCH_CHECK(col0 >= 0 && col0 % 8 == 0 && cols > 0 && cols % 8 == 0 && col0 + cols <= N, "convert_rows: columns");
+  Tensor o = at::empty({M, cols}, src.options().dtype(t_of(f32)));
+  evgpt::launch_convert_rows(s, (int)col0, o.data_ptr(), f32, (int)M, (int)cols, (int)cols, cur_stream());
+  return o;
+}
+void argmax_logits_(const Tensor& logits, const Tensor& out, int64_t vocab) {
+  TORCH_CHECK(logits.is_cuda() && logits.dim() == 2 && is_f32(logits) && logits.stride(1) == 1, "logits: fp32 [B, V]");
+  check_i(out, "out");
+  TORCH_CHECK(vocab >= 1 && vocab <= logits.size(1) && out.numel() >= logits.size(0), "argmax_logits: sizes");
+  evgpt::launch_argmax_logits(logits.data_ptr<float>(), logits.stride(0), out.data_ptr<int>(), (int)logits.size(0),
+                              (int)vocab, cur_stream());
+}
+void commit_rows_(const Tensor& sampled, const Tensor& embed, double scale, const Tensor& x, const Tensor& out_tokens,
+                  const Tensor& step, const Tensor& pos, const Tensor& done, const Tensor& cur, int64_t eos,
+                  const OptTensor& active) {
+  check_i(sampled, "sampled"); check_t(embed, "embed"); check_f(x, "x"); check_i(out_tokens, "out_tokens");
+  check_i(step, "step"); check_i(pos, "pos"); check_i(done, "done"); check_i(cur, "cur_token");
+  const int64_t B = x.size(0);
+  TORCH_CHECK(embed.dim() == 2 && embed.size(1) == x.size(1) && x.size(1) % 64 == 0, "commit_rows: embedding width");
+  TORCH_CHECK(sampled.numel() >= B && step.numel() >= B && pos.numel() >= B && done.numel() >= B && cur.numel() >= B &&
+              out_tokens.dim() == 2 && out_tokens.size(0) >= B, "commit_rows: per-sequence buffers");
+  if (active.has_value()) { check_i(*active, "active"); TORCH_CHECK(active->numel() >= B, "active"); }
+  evgpt::launch_commit_rows(sampled.data_ptr<int>(), embed.data_ptr(), is_f32(embed), (float)scale, x.data_ptr<float>(),
+                            out_tokens.data_ptr<int>(), (int)out_tokens.size(1), step.data_ptr<int>(), pos.data_ptr<int>(),
+                            done.data_ptr<int>(), cur.data_ptr<int>(), (int)eos, (int)B, (int)x.size(1),
+                            (int)embed.size(0), iptr(active), cur_stream());
+}
+void sample_top_p(const Tensor& logits, const Tensor& out, double temperature, double top_p, int64_t seed,
+                  const Tensor& step, int64_t top_k) {
+  check_f(logits, "logits"); check_i(out, "out"); check_i(step, "step");
+  TORCH_CHECK(logits.dim() == 2 && out.numel() >= logits.size(0) && step.numel() >= logits.size(0) && temperature > 0,
+              "sample_top_p: logits [B, V], temperature > 0");
+  evgpt::launch_sample_top_p(logits.data_ptr<float>(), out.data_ptr<int>(), (int)logits.size(0), (int)logits.size(1),
+                             (float)temperature, (int)top_k, (float)top_p, (unsigned long long)seed, step.data_ptr<int>(),
+                             cur_stream());
+}
+
+// ---------------------------------------------------------------- attention
+// returns q [M, Hq, D]; k_buf / v_buf and / or the chunk cache are written in place
+Tensor attn_prep_(const Tensor& src, int64_t q_col, int64_t k_col, int64_t v_col, const OptTensor& qw, const OptTensor& kw,
+                  int64_t Hq, int64_t Hkv, int64_t D, int64_t nq, int64_t nk, double eps, const Tensor& cos, const Tensor& sin,
+                  const OptTensor& row_slot, const Tensor& row_pos, const OptTensor& row_kv, const OptTensor& row_keep,
+                  const OptTensor& k_buf, const OptTensor& v_buf, const Tensor& k_cache, const Tensor& v_cache) {
+  int64_t M, N;
+  evgpt::AttnPrepArgs a{};
+  a.src = src_of(src, "src", &M, &N);
+  check_t(k_cache, "k_cache"); check_t(v_cache, "v_cache");
+  const bool f32 = is_f32(k_cache);
+  TORCH_CHECK(Hq >= 1 && Hkv >= 1 && Hq % Hkv == 0 && D % 64 == 0 && D >= 64, "attn_prep: heads");
+  TORCH_CHECK(q_col % 8 == 0 && k_col % 8 == 0 && v_col % 8 == 0 && q_col >= 0 && k_col >= 0 && v_col >= 0 &&
+              q_col + Hq * D <= N && k_col + Hkv * D <= N && v_col + Hkv * D <= N, "attn_prep: sections");
+  TORCH_CHECK(k_cache.dim() == 4 && k_cache.sizes() == v_cache.sizes() && k_cache.size(1) == Hkv && k_cache.size(3) == D &&
+              k_cache.size(2) >= 1 && is_f32(v_cache) == f32, "attn_prep: caches [slots, Hkv, cap, D]");
+  check_f(cos, "cos"); check_f(sin, "sin");
+  TORCH_CHECK(cos.dim() == 2 && cos.sizes() == sin.sizes() && cos.size(0) >= 1 && cos.size(1) * 2 <= D, "attn_prep: rotation tables");
+  check_i(row_pos, "row_pos");
+  TORCH_CHECK(row_pos.numel() >= M, "attn_prep: row_pos");
+  if (qw.has_value()) { check_f(*qw, "qw"); TORCH_CHECK(qw->numel() == Hq * D && nq >= 1); }
+  if (kw.has_value()) { check_f(*kw, "kw"); TORCH_CHECK(kw->numel() == Hkv * D && nk >= 1); }
+  if (row_slot.has_value()) { check_i(*row_slot, "row_slot"); TORCH_CHECK(row_slot->numel() == M); }
+  else TORCH_CHECK(M <= k_cache.size(0), "attn_prep: more rows than cache slots");
+  if (row_keep.has_value()) { check_i(*row_keep, "row_keep"); TORCH_CHECK(row_keep->numel() == M); }
+  if (row_kv.has_value()) {
+    check_i(*row_kv, "row_kv");
+    TORCH_CHECK(row_kv->numel() == M && k_buf.has_value() && v_buf.has_value(), "attn_prep: key buffer");
+    check_t(*k_buf, "k_buf"); check_t(*v_buf, "v_buf");
+    TORCH_CHECK(k_buf->numel() % (Hkv * D) == 0 && k_buf->numel() >= M * Hkv * D && v_buf->numel() == k_buf->numel() &&
+                is_f32(*k_buf) == f32 && is_f32(*v_buf) == f32, "attn_prep: key buffer size");
+    a.k_buf = k_buf->data_ptr();
+    a.v_buf = v_buf->data_ptr();
+  }
+  Tensor q = at::empty({M, Hq, D}, k_cache.options());
+  a.q_col = (int)q_col; a.k_col = (int)k_col; a.v_col = (int)v_col;
+  a.qw = fptr(qw); a.kw = fptr(kw);
+  a.Hq = (int)Hq; a.Hkv = (int)Hkv; a.D = (int)D; a.nq = (int)nq; a.nk = (int)nk; a.eps = (float)eps;
+  a.cos_tab = cos.data_ptr<float>(); a.sin_tab = sin.data_ptr<float>();
+  a.rot = (int)cos.size(1) * 2; a.max_pos = (int)cos.size(0);
+  a.row_slot = iptr(row_slot); a.row_pos = row_pos.data_ptr<int>(); a.row_kv = iptr(row_kv); a.row_keep = iptr(row_keep);
+  a.q_out = q.data_ptr(); a.k_cache = k_cache.data_ptr(); a.v_cache = v_cache.data_ptr(); a.cap = (int)k_cache.size(2);
+  if (M > 0) evgpt::launch_attn_prep(a, f32, (int)M, cur_stream());
+  return q;
+}
+void chunk_keys_copy_(const Tensor& k_cache, const Tensor& v_cache, const Tensor& k_buf, const Tensor& v_buf, const Tensor& copies) {
+  check_t(k_cache, "k_cache"); check_t(v_cache, "v_cache"); check_t(k_buf, "k_buf"); check_t(v_buf, "v_buf"); check_i(copies, "copies");
+  TORCH_CHECK(k_cache.dim() == 4 && k_cache.sizes() == v_cache.sizes() && copies.dim() == 2 && copies.size(1) == 4 &&
+              copies.size(0) < 65536, "chunk_keys_copy: copies [n, 4]");
+  TORCH_CHECK(is_f32(k_cache) == is_f32(k_buf) && is_f32(v_cache) == is_f32(v_buf) && is_f32(k_buf) == is_f32(v_buf), "chunk_keys_copy: types");
+  if (copies.size(0) > 0)
+    evgpt::launch_chunk_keys_copy(k_cache.data_ptr(), v_cache.data_ptr(), k_buf.data_ptr(), v_buf.data_ptr(),
+                                  copies.data_ptr<int>(), (int)copies.size(0), is_f32(k_cache), (int)k_cache.size(1),
+                                  (int)k_cache.size(2), (int)k_cache.size(3), cur_stream());
+}
+void check_qkv(const Tensor& q, const Tensor& k, const Tensor& v) {
+  check_t(q, "q"); check_t(k, "k"); check_t(v, "v");
+  TORCH_CHECK(q.dim() == 3 && k.dim() == 3 && k.sizes() == v.sizes() && q.size(2) == k.size(2) && q.size(1) % k.size(1) == 0 &&
+              q.scalar_type() == k.scalar_type() && q.scalar_type() == v.scalar_type(), "attention: q [M, Hq, D], k / v [R, Hkv, D]");
+  TORCH_CHECK(q.size(2) % 64 == 0 && q.size(2) <= 512, "attention: head size a multiple of 64 up to 512");
+}
+Tensor attn_chunk(const Tensor& q, const Tensor& k, const Tensor& v, const Tensor& items, double scale) {
+  check_qkv(q, k, v); check_i(items, "items");
+  TORCH_CHECK(items.dim() == 2 && items.size(1) == 4, "attn_chunk: items [n, 4]");
+  Tensor o = at::empty_like(q);
+  if (items.size(0) > 0)
+    evgpt::launch_attn_chunk(q.data_ptr(), k.data_ptr(), v.data_ptr(), o.data_ptr(), items.data_ptr<int>(), (int)items.size(0),
+                             is_f32(q), (int)q.size(1), (int)k.size(1), (int)q.size(2), (float)scale, cur_stream());
+  return o;
+}
+// `n` equal runs of `rows` query rows starting at q0, each with its keys `stride` key rows after the one before, the
+// run's first query at position `off` of its chunk, on the flash kernel (bf16, head size 64 or 128)
+void attn_runs_(const Tensor& q, const Tensor& k, const Tensor& v, const Tensor& o, int64_t q0, int64_t rows, int64_t kv0,
+                int64_t off, int64_t n, double scale) {
+  check_qkv(q, k, v); check_t(o, "o");
+  const int64_t Hq = q.size(1), Hkv = k.size(1), D = q.size(2);
+  TORCH_CHECK(!is_f32(q) && (D == 64 || D == 128) && o.sizes() == q.sizes() && !is_f32(o), "attn_runs: bf16, head size 64 or 128");
+  TORCH_CHECK(rows >= 1 && n >= 1 && q0 >= 0 && kv0 >= 0 && off >= 0 && (n == 1 || off == 0) && q0 + n * rows <= q.size(0) &&
+              kv0 + off + n * rows <= k.size(0), "attn_runs: rows");
+  const long long st[12] = {rows * Hq * D, Hq * D, D, rows * Hkv * D, Hkv * D, D, rows * Hkv * D, Hkv * D, D, rows * Hq * D, Hq * D, D};
+  evgpt::launch_attn_prefill(bptr(q) + q0 * Hq * D, bptr(k) + kv0 * Hkv * D, bptr(v) + kv0 * Hkv * D, bptr_mut(o) + q0 * Hq * D,
+                             st, nullptr, (int)n, (int)rows, (int)(off + rows), (int)Hq, (int)Hkv, (int)D, 1, (int)off, 0,
+                             (float)scale, cur_stream());
+}
+// split-KV decode attention of the other models on the chunk cache (bf16, head size 64 or 128); part_o / part_ml: scratch
+Tensor attn_chunk_decode(const Tensor& q, const Tensor& k_cache, const Tensor& v_cache, const Tensor& pos, double scale,
+                         int64_t nsplit) {
+  check_t(q, "q"); check_t(k_cache, "k_cache"); check_t(v_cache, "v_cache"); check_i(pos, "pos");
+  TORCH_CHECK(q.dim() == 3 && k_cache.dim() == 4 && k_cache.sizes() == v_cache.sizes(), "attn_chunk_decode: shapes");
+  const int64_t B = q.size(0), Hq = q.size(1), D = q.size(2), Hkv = k_cache.size(1), cap = k_cache.size(2);
+  TORCH_CHECK(k_cache.size(0) >= B && k_cache.size(3) == D && Hq % Hkv == 0 && pos.numel() >= B && D % 64 == 0 && D <= 512 &&
+              q.scalar_type() == k_cache.scalar_type() && q.scalar_type() == v_cache.scalar_type(), "attn_chunk_decode: shapes");
+  Tensor o = at::empty_like(q);
+  if (!is_f32(q) && (D == 64 || D == 128)) {
+    nsplit = std::min<int64_t>(std::max<int64_t>(nsplit, 1), 16);
+    Tensor at_pos = at::empty({B}, pos.options());
+    evgpt::launch_mod_pos(pos.data_ptr<int>(), at_pos.data_ptr<int>(), (int)B, (int)cap, cur_stream());
+    auto f = q.options().dtype(at::kFloat);
+    Tensor po = at::empty({nsplit > 1 ? B * Hq * nsplit * D : 1}, f), pm = at::empty({nsplit > 1 ? B * Hq * nsplit * 2 : 1}, f);
+    evgpt::launch_attn_decode(bptr(q), bptr(k_cache), bptr(v_cache), bptr_mut(o), po.data_ptr<float>(), pm.data_ptr<float>(),
+                              at_pos.data_ptr<int>(), (int)B, (int)Hq, (int)Hkv, (int)D, (int)cap, (int)nsplit, (float)scale,
+                              cur_stream());
+    return o;
+  }
+  evgpt::launch_attn_chunk_decode(q.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(), o.data_ptr(), pos.data_ptr<int>(),
+                                  is_f32(q), (int)B, (int)Hq, (int)Hkv, (int)D, (int)cap, (float)scale, cur_stream());
+  return o;
+}
+
+// ---------------------------------------------------------------- recurrences
+// q / k / v: 2-D views (rows, columns from the head section's start) of T matrices
+evgpt::ScanArgs scan_args(const Tensor& q, const Tensor& k, const Tensor& v, int64_t H, int64_t per_group, int64_t N, int64_t V,
+                          double qscale, const Tensor& log_decay, const OptTensor& log_in, const OptTensor& scale_in,
+                          const OptTensor& skip, const Tensor& S, const OptTensor& n, const OptTensor& m) {
+  const int64_t M = q.size(0);
+  auto view = [&](const Tensor& t, int64_t cols, const char* name) {
+    TORCH_CHECK(t.is_cuda() && t.dim() == 2 && t.stride(1) == 1 && t.size(0) == M && t.size(1) >= cols && t.scalar_type() == q.scalar_type() &&
+                (M <= 1 || t.stride(0) % 8 == 0) && (reinterpret_cast<uintptr_t>(t.data_ptr()) & 15) == 0, name, ": aligned rows of one type");
+  };
+  TORCH_CHECK(q.scalar_type() == at::kBFloat16 || q.scalar_type() == at::kFloat, "scan: bf16 or fp32");
+  TORCH_CHECK(H >= 1 && per_group >= 1 && H % per_group == 0 && N >= 32 && N % 32 == 0 && (V == 32 || (V >= 64 && V % 64 == 0)), "scan: sizes");
+  view(q, H / per_group * N, "q"); view(k, H / per_group * N, "k"); view(v, H * V, "v");
+  check_f(log_decay, "log_decay");
+  TORCH_CHECK(log_decay.numel() == M * H, "scan: log_decay [M, H]");
+  TORCH_CHECK(log_in.has_value() != scale_in.has_value(), "scan: log_in or scale_in");
+  if (log_in.has_value()) {
+    check_f(*log_in, "log_in");
+    TORCH_CHECK(log_in->numel() == M * H && n.has_value() && m.has_value(), "scan: log_in [M, H], normaliser, maximum");
+    check_f(*n, "n"); check_f(*m, "m");
+    TORCH_CHECK(n->numel() == S.size(0) * H * N && m->numel() == S.size(0) * H, "scan: normaliser sizes");
+  } else {
+    check_f(*scale_in, "scale_in");
+    TORCH_CHECK(scale_in->numel() == M * H, "scan: scale_in [M, H]");
+  }
+  if (skip.has_value()) { check_f(*skip, "skip"); TORCH_CHECK(skip->numel() == H, "scan: skip [H]"); }
+  check_f(S, "S");
+  TORCH_CHECK(S.dim() == 4 && S.size(1) == H && S.size(2) == V && S.size(3) == N, "scan: S [slots, H, V, N]");
+  evgpt::ScanArgs a{};
+  a.q = q.data_ptr(); a.k = k.data_ptr(); a.v = v.data_ptr();
+  a.ldq = q.stride(0); a.ldk = k.stride(0); a.ldv = v.stride(0);
+  a.per_group = (int)per_group; a.H = (int)H; a.N = (int)N; a.V = (int)V; a.qscale = (float)qscale;
+  a.log_decay = log_decay.data_ptr<float>(); a.log_in = fptr(log_in); a.scale_in = fptr(scale_in); a.skip = fptr(skip);
+  a.S = S.data_ptr<float>();
+  a.n = const_cast<float*>(fptr(n)); a.m = const_cast<float*>(fptr(m));
+  return a;
+}
+Tensor scan_prefill_(const Tensor& q, const Tensor& k, const Tensor& v, int64_t H, int64_t per_group, int64_t N, int64_t V,
+                     double qscale, const Tensor& log_decay, const OptTensor& log_in, const OptTensor& scale_in, const OptTensor& skip,
+                     const Tensor& S, const OptTensor& n, const OptTensor& m, const Tensor& chunks, const Tensor& seqs) {
+  evgpt::ScanArgs a = scan_args(q, k, v, H, per_group, N, V, qscale, log_decay, log_in, scale_in, skip, S, n, m);
+  check_i(chunks, "chunks"); check_i(seqs, "seqs");
+  TORCH_CHECK(chunks.dim() == 2 && chunks.size(1) == 4 && seqs.dim() == 2 && seqs.size(1) == 4, "scan: tables [n, 4]");
+  const int64_t C = chunks.size(0);
+  TORCH_CHECK(C < 65536 && H < 65536 && seqs.size(0) < 65536, "scan: grid");
+  Tensor o = at::empty({q.size(0), H * V}, q.options());
+  if (C == 0) return o;
+  auto f = q.options().dtype(at::kFloat);
+  Tensor dS = at::empty({C, H, V, N}, f), dn = at::empty({C, H, N}, f), sc = at::empty({3, C, H}, f);
+  evgpt::ScanChunks c{chunks.data_ptr<int>(), seqs.data_ptr<int>(), (int)C, (int)seqs.size(0), dS.data_ptr<float>(),
+                      dn.data_ptr<float>(), sc.data_ptr<float>(), sc.data_ptr<float>() + C * H, sc.data_ptr<float>() + 2 * C * H};
+  a.out = o.data_ptr();
+  evgpt::launch_scan_prefill(a, c, is_f32(q), cur_stream());
+  return o;
+}
+Tensor scan_step_(const Tensor& q, const Tensor& k, const Tensor& v, int64_t H, int64_t per_group, int64_t N, int64_t V,
+                  double qscale, const Tensor& log_decay, const OptTensor& log_in, const OptTensor& scale_in, const OptTensor& skip,
+                  const Tensor& S, const OptTensor& n, const OptTensor& m, const Tensor& pos,
+                  const OptTensor& live) {
+  evgpt::ScanArgs a = scan_args(q, k, v, H, per_group, N, V, qscale, log_decay, log_in, scale_in, skip, S, n, m);
+  check_i(pos, "pos");
+  const int64_t B = q.size(0);
+  TORCH_CHECK(pos.numel() >= B && S.size(0) >= B && B < 65536, "scan_step: one row per slot");
+  if (live.has_value()) { check_i(*live, "live"); TORCH_CHECK(live->numel() >= B, "live"); }
+  Tensor o = at::empty({B, H * V}, q.options());
+  a.out = o.data_ptr();
+  if (B > 0) evgpt::launch_scan_step(a, pos.data_ptr<int>(), iptr(live), is_f32(q), (int)B, cur_stream());
+  return o;
+}
+std::tuple<Tensor, Tensor> mlstm_gates(const Tensor& src, int64_t i_col, int64_t f_col, const Tensor& ib, const Tensor& fb, double cap) {
+  int64_t M, N;
+  const SrcRows s = src_of(src, "src", &M, &N);
+  check_f(ib, "ib"); check_f(fb, "fb");
+  const int64_t H = ib.numel();
+  TORCH_CHECK(fb.numel() == H && i_col >= 0 && f_col >= 0 && i_col + H <= N && f_col + H <= N && cap > 0 && M * H < (1ll << 31), "mlstm_gates: columns");
+  Tensor li = at::empty({M, H}, ib.options()), lf = at::empty({M, H}, ib.options());
+  if (M > 0)
+    evgpt::launch_mlstm_gates(s, (int)i_col, (int)f_col, ib.data_ptr<float>(), fb.data_ptr<float>(), (float)cap,
+                              li.data_ptr<float>(), lf.data_ptr<float>(), (int)M, (int)H, cur_stream());
+  return {li, lf};
+}
+std::tuple<Tensor, Tensor> ssd_gates(const Tensor& src, int64_t col, const Tensor& dt_bias, const Tensor& a_log) {
+  int64_t M, N;
+  const SrcRows s = src_of(src, "src", &M, &N);
+  check_f(dt_bias, "dt_bias"); check_f(a_log, "a_log");
+  const int64_t H = dt_bias.numel();
+  TORCH_CHECK(a_log.numel() == H && col >= 0 && col + H <= N && M * H < (1ll << 31), "ssd_gates: columns");
+  Tensor ld = at::empty({M, H}, a_log.options()), dt = at::empty({M, H}, a_log.options());
+  if (M > 0)
+    evgpt::launch_ssd_gates(s, (int)col, dt_bias.data_ptr<float>(), a_log.data_ptr<float>(), ld.data_ptr<float>(),
+                            dt.data_ptr<float>(), (int)M, (int)H, cur_stream());
+  return {ld, dt};
+}
+Tensor conv_rows_(const Tensor& src, int64_t col0, const Tensor& w, const Tensor& bias, const Tensor& ring,
+                  const OptTensor& row_slot, const Tensor& row_pos, const OptTensor& row_first, bool update,
+                  const OptTensor& live) {
+  int64_t M, N;
+  const SrcRows s = src_of(src, "src", &M, &N);
+  check_f(w, "w"); check_f(bias, "bias"); check_t(ring, "ring"); check_i(row_pos, "row_pos");
+  TORCH_CHECK(w.dim() == 2 && bias.numel() == w.size(0) && ring.dim() == 3 && ring.size(1) == w.size(1) && ring.size(2) == w.size(0),
+              "conv_rows: w [C, taps], ring [slots, taps, C]");
+  const int64_t C = w.size(0);
+  TORCH_CHECK(col0 >= 0 && col0 + C <= N && row_pos.numel() >= M, "conv_rows: columns, rows");
+  if (row_slot.has_value()) { check_i(*row_slot, "row_slot"); TORCH_CHECK(row_slot->numel() == M); }
+  else TORCH_CHECK(M <= ring.size(0), "conv_rows: more rows than slots");
+  if (row_first.has_value()) { check_i(*row_first, "row_first"); TORCH_CHECK(row_first->numel() == M); }
+  if (live.has_value()) { check_i(*live, "live"); TORCH_CHECK(live->numel() >= M, "live"); }
+  TORCH_CHECK(!update || !row_first.has_value(), "conv_rows: the ring is updated in place by single-token rows only");
+  Tensor o = at::empty({M, C}, ring.options());
+  if (M > 0)
+    evgpt::launch_conv_rows(s, (int)col0, w.data_ptr<float>(), bias.data_ptr<float>(), ring.data_ptr(), o.data_ptr(),
+                            is_f32(ring), iptr(row_slot), row_pos.data_ptr<int>(), iptr(row_first), (int)M, (int)C,
+                            (int)w.size(1), update, iptr(live), cur_stream());
+  return o;
+}
+void conv_tail_(const Tensor& src, int64_t col0, const Tensor& ring, const Tensor& tails) {
+  int64_t M, N;
+  const SrcRows s = src_of(src, "src", &M, &N);
+  check_t(ring, "ring"); check_i(tails, "tails");
+  TORCH_CHECK(ring.dim() == 3 && tails.dim() == 2 && tails.size(1) == 4 && col0 >= 0 && col0 + ring.size(2) <= N, "conv_tail: shapes");
+  if (tails.size(0) > 0)
+    evgpt::launch_conv_tail(s, (int)col0, ring.data_ptr(), is_f32(ring), tails.data_ptr<int>(), (int)tails.size(0),
+                            (int)ring.size(2), (int)ring.size(1), cur_stream());
+}
+
+}  // namespace
+
+TORCH_LIBRARY(evlay, m) {
+  m.def("linear(Tensor x, Tensor w, bool out_f32) -> Tensor", &linear);
+  m.def("linear_slabs(Tensor x, Tensor w) -> Tensor", &linear_slabs);
+  m.def("embed_rows(Tensor tok, Tensor embed, float scale) -> Tensor", &embed_rows);
+  m.def("norm_rows(Tensor x, Tensor? sel, Tensor w, int n, float eps, bool f32) -> Tensor", &norm_rows);
+  m.def("add_norm_rows_(Tensor(a!) x, Tensor y, Tensor? w, int n, float eps, bool f32) -> Tensor", &add_norm_rows_);
+  m.def("merge_norm_rows_(Tensor(a!) x, Tensor a, Tensor b, Tensor wa, Tensor wb, Tensor? w, int n, float eps, bool f32) -> Tensor", &merge_norm_rows_);
+  m.def("glu_rows(Tensor src, int act, bool f32) -> Tensor", &glu_rows);
+  m.def("group_norm_rows(Tensor y, Tensor gate, int gcol, bool before, Tensor w, int heads, int v, int vp, int parts, int ld_out, float eps) -> Tensor", &group_norm_rows);
+  m.def("convert_rows(Tensor src, int col0, int cols, bool f32) -> Tensor", &convert_rows);
+  m.def("argmax_logits_(Tensor logits, Tensor(a!) out, int vocab) -> ()", &argmax_logits_);
+  m.def("commit_rows_(Tensor sampled, Tensor embed, float scale, Tensor(a!) x, Tensor(b!) out_tokens, Tensor(c!) step, Tensor(d!) pos, Tensor(e!) done, Tensor(f!) cur_token, int eos, Tensor? active) -> ()", &commit_rows_);
+  m.def("sample_top_p(Tensor logits, Tensor(a!) out, float temperature, float top_p, int seed, Tensor step, int top_k=0) -> ()", &sample_top_p);
+  m.def("attn_prep_(Tensor src, int q_col, int k_col, int v_col, Tensor? qw, Tensor? kw, int Hq, int Hkv, int D, int nq, int nk, float eps, Tensor cos, Tensor sin, Tensor? row_slot, Tensor row_pos, Tensor? row_kv, Tensor? row_keep, Tensor(a!)? k_buf, Tensor(b!)? v_buf, Tensor(c!) k_cache, Tensor(d!) v_cache) -> Tensor", &attn_prep_);
+  m.def("chunk_keys_copy_(Tensor k_cache, Tensor v_cache, Tensor(a!) k_buf, Tensor(b!) v_buf, Tensor copies) -> ()", &chunk_keys_copy_);
+  m.def("attn_chunk(Tensor q, Tensor k, Tensor v, Tensor items, float scale) -> Tensor", &attn_chunk);
+  m.def("attn_runs_(Tensor q, Tensor k, Tensor v, Tensor(a!) o, int q0, int rows, int kv0, int off, int n, float scale) -> ()", &attn_runs_);
+  m.def("attn_chunk_decode(Tensor q, Tensor k_cache, Tensor v_cache, Tensor pos, float scale, int nsplit) -> Tensor", &attn_chunk_decode);
+  m.def("scan_prefill_(Tensor q, Tensor k, Tensor v, int H, int per_group, int N, int V, float qscale, Tensor log_decay, Tensor? log_in, Tensor? scale_in, Tensor? skip, Tensor(a!) S, Tensor(b!)? n, Tensor(c!)? m, Tensor chunks, Tensor seqs) -> Tensor", &scan_prefill_);
+  m.def("scan_step_(Tensor q, Tensor k, Tensor v, int H, int per_group, int N, int V, float qscale, Tensor log_decay, Tensor? log_in, Tensor? scale_in, Tensor? skip, Tensor(a!) S, Tensor(b!)? n, Tensor(c!)? m, Tensor pos, Tensor? live) -> Tensor", &scan_step_);
+  m.def("mlstm_gates(Tensor src, int i_col, int f_col, Tensor ib, Tensor fb, float cap) -> (Tensor, Tensor)", &mlstm_gates);
+  m.def("ssd_gates(Tensor src, int col, Tensor dt_bias, Tensor a_log) -> (Tensor, Tensor)", &ssd_gates);
+  m.def("conv_rows_(Tensor src, int col0, Tensor w, Tensor bias, Tensor(a!) ring, Tensor? row_slot, Tensor row_pos, Tensor? row_first, bool update, Tensor? live) -> Tensor", &conv_rows_);
+  m.def("conv_tail_(Tensor src, int col0, Tensor(a!) ring, Tensor tails) -> ()", &conv_tail_);
+}

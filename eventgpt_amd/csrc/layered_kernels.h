@@ -1,0 +1,137 @@
+// Launchers of the layered decoders' kernels (mixers with recurrent state, chunk-masked attention, an
+// fp32 residual stream).  As in evgpt_kernels.h they take raw pointers and a stream, allocate nothing
+// and never synchronise.  `f32` selects the storage type of weights and activations: float or bf16.
+#pragma once
+#include <hip/hip_runtime.h>
+
+namespace evgpt {
+
+typedef unsigned short bf16_t;
+
+// Rows produced by a projection: nslab fp32 slabs to be summed, or one matrix of bf16 / fp32.
+struct SrcRows {
+  const void* p;
+  long long slab;   // elements between slabs
+  int nslab;
+  int ld;           // elements between rows
+  int f32;
+};
+
+// ---- gemm_f32.hip
+void launch_gemm_f32(const float* A, const float* W, float* C, int M, int N, int K, int lda, int ldw, int ldc,
+                     hipStream_t st);
+
+// ---- rowops.hip.  Row widths are padded to a multiple of 64 with zeros (ld); norms divide by the true width n.
+enum { GLU_GELU_TANH = 0, GLU_SILU = 1 };
+void launch_embed_rows(const int* tok, const void* embed, bool f32, float scale, float* x, int rows, int ld, int vocab,
+                       hipStream_t st);
+// xn[i] = RMS norm of x[sel ? sel[i] : i] * w
+void launch_norm_rows(const float* x, const int* sel, const float* w, void* xn, bool f32, int rows, int n, int ld,
+                      float eps, hipStream_t st);
+// x += y; xn = RMS norm of x * w (skipped when w is null)
+void launch_add_norm_rows(float* x, const SrcRows& y, const float* w, void* xn, bool f32, int rows, int n, int ld,
+                          float eps, hipStream_t st);
+// x += (rms(a) * wa + rms(b) * wb) / 2; xn = RMS norm of x * w (skipped when w is null)
+void launch_merge_norm_rows(float* x, const SrcRows& a, const SrcRows& b, const float* wa, const float* wb,
+                            const float* w, void* xn, bool f32, int rows, int n, int ld, float eps, hipStream_t st);
+// h[row][i] = act(src[row][i]) * src[row][ip + i], i < ip
+void launch_glu_rows(const SrcRows& src, void* h, bool f32, int rows, int ip, int act, hipStream_t st);
+// Group norm of channels stored as heads of vp slots (v of them used): `parts` equal runs of the heads * v true
+// channels, each by its own root mean square, times w (laid out like the channels), with a gate read from `gate` at column
+// gcol + channel slot: silu(gate) multiplied in before the norm, or sigmoid(gate) after it.
+void launch_group_norm_rows(const void* y, const SrcRows& gate, int gcol, bool gate_before, const float* w, void* out,
+                            bool f32, int rows, int heads, int v, int vp, int parts, int ld_out, float eps,
+                            hipStream_t st);
+// out[row][c] = T(src[row][col0 + c]), c < cols (cols % 8 == 0)
+void launch_convert_rows(const SrcRows& src, int col0, void* out, bool f32, int rows, int cols, int ld_out,
+                         hipStream_t st);
+void launch_argmax_logits(const float* logits, long long ld, int* out, int rows, int vocab, hipStream_t st);
+void launch_commit_rows(const int* sampled, const void* embed, bool f32, float scale, float* x, int* out_tokens,
+                        int max_out, int* step, int* pos, int* done, int* cur_token, int eos, int B, int ld, int vocab,
+                        const int* active, hipStream_t st);
+
+// Attention inputs from a projection: RMS norm of all q rows / all k rows at once (weights or null), rotary embedding
+// of the first `rot` dimensions, q -> q_out rows, k / v -> rows of a key buffer and / or a per-sequence
+// cache of `cap` slots that holds the positions of the current chunk (slot = position % cap).
+struct AttnPrepArgs {
+  SrcRows src;
+  int q_col, k_col, v_col;         // columns of the sections in src
+  const float* qw;                 // [Hq][D] (zero in the padding) or null: no norm
+  const float* kw;
+  int Hq, Hkv, D;                  // D: padded head size of q, k and v
+  int nq, nk;                      // true widths of the q and k projections (norm divisors)
+  float eps;
+  const float* cos_tab;            // [max_pos][rot / 2]
+  const float* sin_tab;
+  int rot, max_pos;
+  const int* row_slot;             // [rows] cache slot, or null: the row's index
+  const int* row_pos;              // [rows]
+  const int* row_kv;               // [rows] row of the key buffer, or null: none
+  const int* row_keep;             // [rows] nonzero: also into the cache; null: all rows
+  void* q_out;                     // [rows][Hq][D]
+  void* k_buf; void* v_buf;        // [kv rows][Hkv][D]
+  void* k_cache; void* v_cache;    // [slots][Hkv][cap][D]
+  int cap;
+};
+void launch_attn_prep(const AttnPrepArgs& a, bool f32, int rows, hipStream_t st);
+// cached keys of a chunk that a portion continues, into the key buffer: copies [n][4] of
+// {slot, first cache slot, key buffer row, count}
+void launch_chunk_keys_copy(const void* k_cache, const void* v_cache, void* k_buf, void* v_buf, const int* copies, int n,
+                            bool f32, int Hkv, int cap, int D, hipStream_t st);
+
+// ---- attn_chunk.hip (D a multiple of 64, up to 512; any number of query heads per key head)
+// items [n][4]: {first query row, query rows (<= 64), key buffer row of the chunk's first key, position of the
+// first query within the chunk}
+void launch_attn_chunk(const void* q, const void* k, const void* v, void* o, const int* items, int n_items, bool f32,
+                       int Hq, int Hkv, int D, float scale, hipStream_t st);
+// keys 0 .. pos % cap of every sequence's cache
+void launch_attn_chunk_decode(const void* q, const void* k_cache, const void* v_cache, void* o, const int* pos,
+                              bool f32, int B, int Hq, int Hkv, int D, int cap, float scale, hipStream_t st);
+void launch_mod_pos(const int* pos, int* out, int B, int cap, hipStream_t st);
+
+// ---- linear_scan.hip: S_t = exp(a_t) S_(t-1) + b_t v_t k_t^T per head, y_t = S_t q_t
+struct ScanArgs {
+  const void* q; const void* k; const void* v;   // [rows][..], T
+  long long ldq, ldk, ldv;
+  int per_group;                   // heads per q / k head
+  int H, N, V;                     // padded sizes: N % 32 == 0, V == 32 or V % 64 == 0
+  float qscale;
+  const float* log_decay;          // [rows][H]
+  const float* log_in;             // [rows][H]: b = exp(log_in), with running maximum and normaliser; or null
+  const float* scale_in;           // [rows][H]: b; or null
+  const float* skip;               // [H]: y += skip * v; or null
+  void* out;                       // [rows][H][V]
+  float* S;                        // [slots][H][V][N]
+  float* n;                        // [slots][H][N]
+  float* m;                        // [slots][H]
+};
+struct ScanChunks {
+  const int* chunks;               // [C][4]: first row, rows (<= 64), slot, last chunk of its sequence
+  const int* seqs;                 // [nseq][4]: first chunk, chunks, slot, starts at position 0
+  int C, nseq;
+  float* dS;                       // [C][H][V][N]
+  float* dn;                       // [C][H][N]
+  float* am; float* fl; float* m0; // [C][H]
+};
+constexpr int SCAN_CHUNK = 64;
+void launch_scan_prefill(const ScanArgs& a, const ScanChunks& c, bool f32, hipStream_t st);
+// one token of every sequence: row b is slot b; pos[b] == 0 starts from the zero state; rows whose live is 0 are
+// left alone (their output too)
+void launch_scan_step(const ScanArgs& a, const int* pos, const int* live, bool f32, int B, hipStream_t st);
+// log gates of the matrix memory: cap * tanh((x + b) / cap), and the log sigmoid of it for the forget gate
+void launch_mlstm_gates(const SrcRows& src, int i_col, int f_col, const float* ib, const float* fb, float cap, float* li,
+                        float* lf, int rows, int H, hipStream_t st);
+// dt = softplus(x + bias), log decay = -exp(a_log) * dt
+void launch_ssd_gates(const SrcRows& src, int col, const float* dt_bias, const float* a_log, float* log_decay, float* dt,
+                      int rows, int H, hipStream_t st);
+
+// ---- conv1d.hip: causal per-channel convolution + silu; the state is the last inputs in a ring of `taps`
+// slots (slot = position % taps).  update: a decode step, which also stores its input (of the rows whose live is set)
+void launch_conv_rows(const SrcRows& src, int col0, const float* w, const float* bias, void* ring, void* out, bool f32,
+                      const int* row_slot, const int* row_pos, const int* row_first, int rows, int C, int taps,
+                      bool update, const int* live, hipStream_t st);
+// last inputs of every sequence of a prefill into the ring; tails [nseq][4]: {first row, rows, slot, start position}
+void launch_conv_tail(const SrcRows& src, int col0, void* ring, bool f32, const int* tails, int nseq, int C, int taps,
+                      hipStream_t st);
+
+}  // namespace evgpt

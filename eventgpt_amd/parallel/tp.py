@@ -600,18 +600,6 @@ class TensorParallelEngine(GenerationEngine):
         raw.argmax_pair_select(self._pairs, self.tp_world, self.B, self.sampled)
         self._commit_sampled()
 
-    # ----------------------------------------------------------------- batching
-    @torch.no_grad()
-    def prefill_batch(self, embeds_list: Sequence[torch.Tensor]) -> None:
-        """Prefill sequence ``b`` with ``embeds_list[b]`` for every slot, then pick and
-        commit the first token of all of them in one step."""
-        if len(embeds_list) != self.B:
-            raise ValueError(f"need {self.B} prompts, got {len(embeds_list)}")
-        self.reset()
-        self._prefill_slots(list(range(self.B)), list(embeds_list))
-        self._logits_and_commit(greedy=True)
-        self._after_prefill()
-
     def _after_prefill(self) -> None:
         """The in-tree collectives of a prefill are checked once its work is done (one device sync per
         prompt, where the library collective would have synchronised the ranks anyway)."""
@@ -629,44 +617,3 @@ class TensorParallelEngine(GenerationEngine):
             out = super().prefill(embeds, batch, start, None, return_hidden)
         self._after_prefill()
         return out
-
-    # ------------------------------------------------------ slot-wise scheduling
-    def enable_slot_masks(self) -> None:
-        """Give the commit kernel a per-slot "may advance" mask (all ones).  Captured
-        graphs bake the pointer, so earlier captures are dropped."""
-        if self.active is None:
-            self.active = torch.ones(self.B, dtype=torch.int32, device=self.device)
-            self._graph_greedy.clear()
-            self._graph_logits = None
-
-    @torch.no_grad()
-    def admit(self, slots: Sequence[int], embeds_list: Sequence[torch.Tensor]) -> None:
-        """Start new sequences in ``slots`` while the other slots keep their state:
-        prefill each slot's cache, then pick and commit the first token of exactly those
-        slots (every other slot is masked out of the commit)."""
-        self.enable_slot_masks()
-        if len(slots) != len(embeds_list) or not slots:
-            raise ValueError("one prompt per admitted slot")
-        keep = self.active.clone()
-        self._prefill_slots(list(slots), list(embeds_list))
-        self.step[list(slots)] = 0
-        self.done[list(slots)] = 0
-        self.active.zero_()
-        self.active[list(slots)] = 1
-        self._logits_and_commit(greedy=True)
-        keep[list(slots)] = 1
-        self.active.copy_(keep)
-        self._after_prefill()
-
-    def park(self, slots: Sequence[int]) -> None:
-        """Stop advancing ``slots`` (finished or cancelled sequences)."""
-        self.enable_slot_masks()
-        if slots:
-            self.active[list(slots)] = 0
-            # a parked slot still rides through the batched kernels: with position 0 its
-            # attention reads one key instead of a finished sequence's whole cache
-            self.pos[list(slots)] = 0
-
-    def tokens(self, batch: int) -> torch.Tensor:
-        n = int(self.step[batch].item())
-        return self.out_tokens[batch, :n].to(torch.long)

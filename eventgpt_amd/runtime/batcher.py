@@ -1,7 +1,8 @@
 """Continuous batching over a multi-slot engine: requests join and leave a running
 decode batch one slot at a time.
 
-The engine (``parallel.tp.TensorParallelEngine`` with ``max_batch`` slots) keeps every
+The engine (``parallel.tp.TensorParallelEngine`` or ``runtime.layered_engine.LayeredEngine`` with
+``max_batch`` slots; a prompt is what its engine prefills, embedding rows or token ids) keeps every
 sequence's position, step counter, EOS flag and token ring in device memory and advances
 all slots with ONE captured decode graph per step.  The scheduler only edits the per-slot
 ``active`` mask that the commit kernel reads:
@@ -48,8 +49,8 @@ class Request:
 
 class ContinuousBatcher:
     def __init__(self, engine, eos_token_id: int = 2, poll_every: int = 8, max_admit_per_step: int = 8):
-        if not hasattr(engine, "admit"):
-            raise TypeError("ContinuousBatcher needs a multi-slot engine (TensorParallelEngine)")
+        if not hasattr(engine, "_prefill_slots"):
+            raise TypeError("ContinuousBatcher needs a multi-slot engine (TensorParallelEngine, LayeredEngine)")
         self.e = engine
         self.e.eos = int(eos_token_id)
         self.e.enable_slot_masks()

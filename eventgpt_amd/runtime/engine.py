@@ -100,7 +100,283 @@ def persistent_state(method):
     return wrapped
 
 
-class GenerationEngine:
+class DecodeEngine:
+    """What serving an autoregressive decoder needs besides its layers: per-sequence state in device memory
+    (position, step, EOS flag, token ring, logits), graph capture and replay of the decode step, greedy
+    and sampled generation, and slot-wise scheduling (admit / park).
+
+    A subclass provides ``_layers_step`` (all layers of one decode step, on the residual rows ``self.x``),
+    ``_logits_and_commit`` / ``_commit_sampled``, ``prefill`` and -- for several sequences --
+    ``_prefill_slots``; it sets ``raw`` (an op namespace with ``sample_top_p``), ``device``, ``B``, ``V``,
+    ``l_max``, ``max_out``, ``use_graph`` and ``poll_every`` before ``_init_decode_state``.
+    """
+
+    def _init_decode_state(self, x: torch.Tensor, eos_token_id: Optional[int]) -> None:
+        """``x``: the residual rows of the decode step, one per sequence."""
+        B = self.B
+        i32 = dict(dtype=torch.int32, device=self.device)
+        self.x = x
+        self.logits = torch.zeros(B, self.V, dtype=torch.float32, device=self.device)
+        self.out_tokens = torch.zeros(B, self.max_out, **i32)
+        self.step = torch.zeros(B, **i32)
+        self.pos = torch.zeros(B, **i32)
+        self.done = torch.zeros(B, **i32)
+        self.cur_token = torch.zeros(B, **i32)
+        self.sampled = torch.zeros(B, **i32)
+        # per-sequence "may advance" flags read by the commit kernel; None = all.  A batch
+        # scheduler allocates them (enable_slot_masks).
+        self.active = None
+        self.eos = int(eos_token_id if eos_token_id is not None else -1)
+        # captured graphs bake the EOS id (a launch argument), so they are keyed by it
+        self._graph_greedy = {}
+        self._graph_logits = None
+
+    # ------------------------------------------------------------------ state
+    def reset(self) -> None:
+        for t in (self.step, self.pos, self.done, self.cur_token):
+            t.zero_()
+        self._pos_hi = 0
+
+    # Host-side upper bound of the device position counters.  The kernels clamp a position that
+    # runs past the cache (nothing faults), but a clamped verify silently accepts or emits wrong
+    # tokens, so multi-row passes are refused on the host before they can overrun: the bound is
+    # advanced by the most a call can append and re-read exactly (one small copy) only when it
+    # says the cache might be full.
+    _pos_hi = 0
+
+    def cache_room(self, rows: int) -> bool:
+        """True if ``rows`` more positions fit the cache of every sequence."""
+        if self._pos_hi + rows > self.l_max:
+            self._pos_hi = int(self.pos.max().item())
+        return self._pos_hi + rows <= self.l_max
+
+    def _poll_hook(self) -> None:
+        """Called where the host has just waited for the device anyway (EOS polls); a
+        tensor-parallel engine checks its collectives' error words here."""
+
+    def _step_greedy(self) -> None:
+        self._layers_step()
+        self._logits_and_commit(greedy=True)
+
+    def _step_logits(self) -> None:
+        self._layers_step()
+        self._logits_and_commit(greedy=False)
+
+    def _capture(self, fn):
+        """Capture ``fn`` into a HIP graph.  Warm-up and capture advance the device
+        counters, so they are snapshotted and restored (also when the capture fails)."""
+        state = (self.step, self.pos, self.done, self.cur_token, self.x)
+        saved = [t.clone() for t in state]
+        try:
+            side = torch.cuda.Stream()
+            side.wait_stream(torch.cuda.current_stream())
+            with torch.cuda.stream(side):
+                fn()  # warm-up (first-launch module load) outside the capture
+            torch.cuda.current_stream().wait_stream(side)
+            torch.cuda.synchronize()
+            g = torch.cuda.CUDAGraph()
+            # thread-local capture mode: another host thread driving a second engine on
+            # its own stream must not invalidate this capture
+            with capture_tensor_mode(), no_gc_during_capture(), \
+                    torch.cuda.graph(g, capture_error_mode="thread_local"):
+                fn()
+        finally:
+            for t, s in zip(state, saved):
+                t.copy_(s)
+            torch.cuda.synchronize()
+        return g
+
+    def _capture_or_eager(self, fn):
+        """``_capture`` that degrades to eager stepping when the step cannot be captured
+        (e.g. a collective backend that does not record into graphs): warns once, turns
+        graphs off for this engine, records the reason in ``graph_fallback`` (benchmarks
+        report it, so an eager run cannot pass for a captured one) and returns None."""
+        try:
+            return self._capture(fn)
+        except RuntimeError as e:
+            import warnings
+            warnings.warn(f"decode step could not be captured into a HIP graph ({e}); running eagerly")
+            self.use_graph = False
+            self.graph_fallback = str(e)[:200]
+            return None
+
+    graph_fallback: Optional[str] = None
+
+    @property
+    def graph_captured(self) -> bool:
+        """True when decode steps replay a captured graph (not the eager fallback)."""
+        return bool(self.use_graph and (self._graph_greedy or self._graph_logits is not None))
+
+    def ensure_graphs(self, eos_token_id: Optional[int] = None, greedy: bool = True) -> None:
+        """Capture the decode graph for this EOS id now, if it is not captured yet.
+        Schedulers call this before they start timed or multi-threaded regions, so
+        that no capture (which synchronises the device) lands inside them."""
+        if eos_token_id is not None:
+            self.eos = int(eos_token_id)
+        if not self.use_graph:
+            return
+        if greedy:
+            if self.eos not in self._graph_greedy:
+                self._graph_greedy[self.eos] = self._capture(self._step_greedy)
+        elif self._graph_logits is None:
+            self._graph_logits = self._capture(self._step_logits)
+
+    def decode_step(self, greedy: bool = True) -> None:
+        """Advance every sequence by one token (graph replay when enabled)."""
+        self._pos_hi += 1
+        if not self.use_graph:
+            (self._step_greedy if greedy else self._step_logits)()
+            return
+        if greedy:
+            g = self._graph_greedy.get(self.eos)
+            if g is None:
+                g = self._capture_or_eager(self._step_greedy)
+                if g is None:
+                    return self._step_greedy()
+                self._graph_greedy[self.eos] = g
+            g.replay()
+        else:
+            if self._graph_logits is None:
+                self._graph_logits = self._capture_or_eager(self._step_logits)
+                if self._graph_logits is None:
+                    return self._step_logits()
+            self._graph_logits.replay()
+
+    # --------------------------------------------------------------- generate
+    def _sample_and_commit(self, temperature: float, top_p: float, generator, top_k: int = 0) -> None:
+        """Draw the next token on the device (top-k / top-p by bisection, keyed by
+        ``(seed, step)``) and commit it; no host round trip."""
+        seed = int(generator.initial_seed()) if generator is not None else 0
+        self.raw.sample_top_p(self.logits, self.sampled, float(temperature), float(top_p),
+                              seed & 0x7FFFFFFFFFFFFFFF, self.step, int(top_k))
+        self._commit_sampled()
+
+    @torch.no_grad()
+    def generate(self, embeds: torch.Tensor, max_new_tokens: int = 512, temperature: float = 0.0,
+                 top_p: float = 1.0, eos_token_id: Optional[int] = None,
+                 generator: Optional[torch.Generator] = None, top_k: int = 0) -> torch.Tensor:
+        """Greedy / sampled generation for one sequence; returns new token ids (long).
+        Sampling applies temperature, then ``top_k`` (0 = off), then ``top_p``.
+
+        Greedy decoding replays one captured graph per token and syncs with the
+        host only every ``poll_every`` tokens to read the EOS flag.  Sampling
+        replays the layers+logits graph, then draws the token on the device.
+        """
+        if eos_token_id is not None:
+            self.eos = int(eos_token_id)
+        if max_new_tokens > self.max_out:
+            raise ValueError(f"max_new_tokens {max_new_tokens} > engine ring {self.max_out}")
+        self.reset()
+        greedy = temperature <= 0
+        self.prefill(embeds, select="greedy" if greedy else "logits")
+        if not greedy:
+            self._sample_and_commit(temperature, top_p, generator, top_k)
+        budget = min(max_new_tokens, self.l_max - embeds.shape[0])
+        return self.generate_continue(budget, None, temperature, top_p, generator, top_k)
+
+    @torch.no_grad()
+    def score(self, embeds: torch.Tensor, tokens: torch.Tensor) -> torch.Tensor:
+        """Teacher-forced logits of sequence 0: row 0 predicts the token after the prompt, row
+        ``i`` the token after ``tokens[i-1]`` -- ``[len(tokens)+1, V]`` fp32.  The given tokens
+        are committed instead of the model's own choice (one decode step each), so two
+        implementations can be compared on logits along the SAME path rather than on how
+        long their greedy outputs happen to agree."""
+        eos, self.eos = self.eos, -1
+        self.reset()
+        self.prefill(embeds, select="logits")
+        rows = [self.logits[0].float().clone()]
+        for t in tokens.tolist():
+            self.sampled[0] = int(t)
+            self._commit_sampled()
+            self.decode_step(greedy=False)
+            rows.append(self.logits[0].float().clone())
+        self.eos = eos
+        return torch.stack(rows)
+
+    @torch.no_grad()
+    def generate_continue(self, max_new_tokens: int, eos_token_id: Optional[int] = None,
+                          temperature: float = 0.0, top_p: float = 1.0,
+                          generator: Optional[torch.Generator] = None, top_k: int = 0) -> torch.Tensor:
+        """Keep decoding sequence 0 until ``max_new_tokens`` tokens have been emitted in
+        total (counting those already committed) or EOS; returns all emitted tokens."""
+        if eos_token_id is not None:
+            self.eos = int(eos_token_id)
+        greedy = temperature <= 0
+        n = int(self.step[0].item())
+        budget = min(max_new_tokens, self.max_out)
+        while n < budget and not int(self.done[0].item()):
+            self._poll_hook()
+            chunk = min(self.poll_every, budget - n)
+            for _ in range(chunk):
+                self.decode_step(greedy)
+                if not greedy:
+                    self._sample_and_commit(temperature, top_p, generator, top_k)
+            n += chunk
+        toks = self.out_tokens[0, :n].to(torch.long)
+        if self.eos >= 0:
+            hit = (toks == self.eos).nonzero()
+            if hit.numel():
+                toks = toks[: int(hit[0]) + 1]
+        return toks
+
+    # ----------------------------------------------------------------- batching
+    @torch.no_grad()
+    def prefill_batch(self, embeds_list: Sequence[torch.Tensor]) -> None:
+        """Prefill sequence ``b`` with ``embeds_list[b]`` for every slot, then pick and
+        commit the first token of all of them in one step."""
+        if len(embeds_list) != self.B:
+            raise ValueError(f"need {self.B} prompts, got {len(embeds_list)}")
+        self.reset()
+        self._prefill_slots(list(range(self.B)), list(embeds_list))
+        self._logits_and_commit(greedy=True)
+        self._after_prefill()
+
+    def _after_prefill(self) -> None:
+        """Called when a prefill has been issued; a tensor-parallel engine checks its collectives here."""
+
+    # ------------------------------------------------------ slot-wise scheduling
+    def enable_slot_masks(self) -> None:
+        """Give the commit kernel a per-slot "may advance" mask (all ones).  Captured
+        graphs bake the pointer, so earlier captures are dropped."""
+        if self.active is None:
+            self.active = torch.ones(self.B, dtype=torch.int32, device=self.device)
+            self._graph_greedy.clear()
+            self._graph_logits = None
+
+    @torch.no_grad()
+    def admit(self, slots: Sequence[int], embeds_list: Sequence[torch.Tensor]) -> None:
+        """Start new sequences in ``slots`` while the other slots keep their state:
+        prefill each slot's cache, then pick and commit the first token of exactly those
+        slots (every other slot is masked out of the commit)."""
+        self.enable_slot_masks()
+        if len(slots) != len(embeds_list) or not slots:
+            raise ValueError("one prompt per admitted slot")
+        keep = self.active.clone()
+        self._prefill_slots(list(slots), list(embeds_list))
+        self.step[list(slots)] = 0
+        self.done[list(slots)] = 0
+        self.active.zero_()
+        self.active[list(slots)] = 1
+        self._logits_and_commit(greedy=True)
+        keep[list(slots)] = 1
+        self.active.copy_(keep)
+        self._after_prefill()
+
+    def park(self, slots: Sequence[int]) -> None:
+        """Stop advancing ``slots`` (finished or cancelled sequences)."""
+        self.enable_slot_masks()
+        if slots:
+            self.active[list(slots)] = 0
+            # a parked slot still rides through the batched kernels: with position 0 its
+            # attention reads one key instead of a finished sequence's whole cache
+            self.pos[list(slots)] = 0
+
+    def tokens(self, batch: int) -> torch.Tensor:
+        n = int(self.step[batch].item())
+        return self.out_tokens[batch, :n].to(torch.long)
+
+
+class GenerationEngine(DecodeEngine):
     @persistent_state
     def __init__(self, model, max_len: int = 2560, max_batch: int = 1, nsplit: Optional[int] = None,
                  use_graph: bool = True, max_new_tokens: int = 1024, poll_every: int = 16,
@@ -155,7 +431,7 @@ class GenerationEngine:
         bf = dict(dtype=torch.bfloat16, device=dev)
         i32 = dict(dtype=torch.int32, device=dev)
         f32 = dict(dtype=torch.float32, device=dev)
-        self.x = torch.zeros(B, self.H, **bf)           # residual stream of the decode step
+        self._init_decode_state(torch.zeros(B, self.H, **bf), cfg.eos_token_id)
         self.q = torch.zeros(B, self.Hq * self.D, **bf)
         self.attn = torch.zeros(B, self.Hq * self.D, **bf)
         self.h = torch.zeros(B, self.I, **bf)
@@ -164,23 +440,9 @@ class GenerationEngine:
         self.n_part = int(self.raw.logits_partials(self.V))
         self.part_val = torch.zeros(B * self.n_part, **f32)
         self.part_idx = torch.zeros(B * self.n_part, **i32)
-        self.logits = torch.zeros(B, self.V, **f32)
-        self.out_tokens = torch.zeros(B, self.max_out, **i32)
-        self.step = torch.zeros(B, **i32)
-        self.pos = torch.zeros(B, **i32)
-        self.done = torch.zeros(B, **i32)
-        self.cur_token = torch.zeros(B, **i32)
-        self.sampled = torch.zeros(B, **i32)
         self.sd_result = torch.zeros(8, **i32)  # [n_accepted, next_token, n_emitted, step, done, pos, -, -]
         self.sd_limit = None     # device int32 [1]: freeze verify rounds once this many tokens are out
         self.sd_stats = None     # device int32 [4]: drafted, accepted, rounds (device-resident SD loops)
-        # per-sequence "may advance" flags read by the commit kernel; None = all.  A batch
-        # scheduler allocates them (TensorParallelEngine.enable_slot_masks).
-        self.active = None
-        self.eos = int(cfg.eos_token_id if cfg.eos_token_id is not None else -1)
-        # captured graphs bake the EOS id (a launch argument), so they are keyed by it
-        self._graph_greedy = {}
-        self._graph_logits = None
         self._verify_graphs = {}
 
     # ---------------------------------------------------------------- weights
@@ -260,25 +522,6 @@ class GenerationEngine:
         if self.w4:
             return sum(q.nbytes for l in self.layers for q in l.q4.values())
         return sum(getattr(l, n).numel() * 2 for l in self.layers for n in self._W4_NAMES)
-
-    # ------------------------------------------------------------------ state
-    def reset(self) -> None:
-        for t in (self.step, self.pos, self.done, self.cur_token):
-            t.zero_()
-        self._pos_hi = 0
-
-    # Host-side upper bound of the device position counters.  The kernels clamp a position that
-    # runs past the cache (nothing faults), but a clamped verify silently accepts or emits wrong
-    # tokens, so multi-row passes are refused on the host before they can overrun: the bound is
-    # advanced by the most a call can append and re-read exactly (one small copy) only when it
-    # says the cache might be full.
-    _pos_hi = 0
-
-    def cache_room(self, rows: int) -> bool:
-        """True if ``rows`` more positions fit the cache of every sequence."""
-        if self._pos_hi + rows > self.l_max:
-            self._pos_hi = int(self.pos.max().item())
-        return self._pos_hi + rows <= self.l_max
 
     @property
     def kv_bytes_per_token(self) -> int:
@@ -593,172 +836,3 @@ class GenerationEngine:
         self.raw.commit_token(self.part_val, self.part_idx, self.n_part, self.sampled, self.embed,
                               self.x, self.out_tokens, self.step, self.pos, self.done,
                               self.cur_token, self.eos, self.active)
-
-    def _poll_hook(self) -> None:
-        """Called where the host has just waited for the device anyway (EOS polls); a
-        tensor-parallel engine checks its collectives' error words here."""
-
-    def _step_greedy(self) -> None:
-        self._layers_step()
-        self._logits_and_commit(greedy=True)
-
-    def _step_logits(self) -> None:
-        self._layers_step()
-        self._logits_and_commit(greedy=False)
-
-    def _capture(self, fn):
-        """Capture ``fn`` into a HIP graph.  Warm-up and capture advance the device
-        counters, so they are snapshotted and restored (also when the capture fails)."""
-        state = (self.step, self.pos, self.done, self.cur_token, self.x)
-        saved = [t.clone() for t in state]
-        try:
-            side = torch.cuda.Stream()
-            side.wait_stream(torch.cuda.current_stream())
-            with torch.cuda.stream(side):
-                fn()  # warm-up (first-launch module load) outside the capture
-            torch.cuda.current_stream().wait_stream(side)
-            torch.cuda.synchronize()
-            g = torch.cuda.CUDAGraph()
-            # thread-local capture mode: another host thread driving a second engine on
-            # its own stream must not invalidate this capture
-            with capture_tensor_mode(), no_gc_during_capture(), \
-                    torch.cuda.graph(g, capture_error_mode="thread_local"):
-                fn()
-        finally:
-            for t, s in zip(state, saved):
-                t.copy_(s)
-            torch.cuda.synchronize()
-        return g
-
-    def _capture_or_eager(self, fn):
-        """``_capture`` that degrades to eager stepping when the step cannot be captured
-        (e.g. a collective backend that does not record into graphs): warns once, turns
-        graphs off for this engine, records the reason in ``graph_fallback`` (benchmarks
-        report it, so an eager run cannot pass for a captured one) and returns None."""
-        try:
-            return self._capture(fn)
-        except RuntimeError as e:
-            import warnings
-            warnings.warn(f"decode step could not be captured into a HIP graph ({e}); running eagerly")
-            self.use_graph = False
-            self.graph_fallback = str(e)[:200]
-            return None
-
-    graph_fallback: Optional[str] = None
-
-    @property
-    def graph_captured(self) -> bool:
-        """True when decode steps replay a captured graph (not the eager fallback)."""
-        return bool(self.use_graph and (self._graph_greedy or self._graph_logits is not None))
-
-    def ensure_graphs(self, eos_token_id: Optional[int] = None, greedy: bool = True) -> None:
-        """Capture the decode graph for this EOS id now, if it is not captured yet.
-        Schedulers call this before they start timed or multi-threaded regions, so
-        that no capture (which synchronises the device) lands inside them."""
-        if eos_token_id is not None:
-            self.eos = int(eos_token_id)
-        if not self.use_graph:
-            return
-        if greedy:
-            if self.eos not in self._graph_greedy:
-                self._graph_greedy[self.eos] = self._capture(self._step_greedy)
-        elif self._graph_logits is None:
-            self._graph_logits = self._capture(self._step_logits)
-
-    def decode_step(self, greedy: bool = True) -> None:
-        """Advance every sequence by one token (graph replay when enabled)."""
-        self._pos_hi += 1
-        if not self.use_graph:
-            (self._step_greedy if greedy else self._step_logits)()
-            return
-        if greedy:
-            g = self._graph_greedy.get(self.eos)
-            if g is None:
-                g = self._capture_or_eager(self._step_greedy)
-                if g is None:
-                    return self._step_greedy()
-                self._graph_greedy[self.eos] = g
-            g.replay()
-        else:
-            if self._graph_logits is None:
-                self._graph_logits = self._capture_or_eager(self._step_logits)
-                if self._graph_logits is None:
-                    return self._step_logits()
-            self._graph_logits.replay()
-
-    # --------------------------------------------------------------- generate
-    def _sample_and_commit(self, temperature: float, top_p: float, generator, top_k: int = 0) -> None:
-        """Draw the next token on the device (top-k / top-p by bisection, keyed by
-        ``(seed, step)``) and commit it; no host round trip."""
-        seed = int(generator.initial_seed()) if generator is not None else 0
-        self.raw.sample_top_p(self.logits, self.sampled, float(temperature), float(top_p),
-                              seed & 0x7FFFFFFFFFFFFFFF, self.step, int(top_k))
-        self._commit_sampled()
-
-    @torch.no_grad()
-    def generate(self, embeds: torch.Tensor, max_new_tokens: int = 512, temperature: float = 0.0,
-                 top_p: float = 1.0, eos_token_id: Optional[int] = None,
-                 generator: Optional[torch.Generator] = None, top_k: int = 0) -> torch.Tensor:
-        """Greedy / sampled generation for one sequence; returns new token ids (long).
-        Sampling applies temperature, then ``top_k`` (0 = off), then ``top_p``.
-
-        Greedy decoding replays one captured graph per token and syncs with the
-        host only every ``poll_every`` tokens to read the EOS flag.  Sampling
-        replays the layers+logits graph, then draws the token on the device.
-        """
-        if eos_token_id is not None:
-            self.eos = int(eos_token_id)
-        if max_new_tokens > self.max_out:
-            raise ValueError(f"max_new_tokens {max_new_tokens} > engine ring {self.max_out}")
-        self.reset()
-        greedy = temperature <= 0
-        self.prefill(embeds, select="greedy" if greedy else "logits")
-        if not greedy:
-            self._sample_and_commit(temperature, top_p, generator, top_k)
-        budget = min(max_new_tokens, self.l_max - embeds.shape[0])
-        return self.generate_continue(budget, None, temperature, top_p, generator, top_k)
-
-    @torch.no_grad()
-    def score(self, embeds: torch.Tensor, tokens: torch.Tensor) -> torch.Tensor:
-        """Teacher-forced logits of sequence 0: row 0 predicts the token after the prompt, row
-        ``i`` the token after ``tokens[i-1]`` -- ``[len(tokens)+1, V]`` fp32.  The given tokens
-        are committed instead of the model's own choice (one decode step each), so two
-        implementations can be compared on logits along the SAME path rather than on how
-        long their greedy outputs happen to agree."""
-        eos, self.eos = self.eos, -1
-        self.reset()
-        self.prefill(embeds, select="logits")
-        rows = [self.logits[0].float().clone()]
-        for t in tokens.tolist():
-            self.sampled[0] = int(t)
-            self._commit_sampled()
-            self.decode_step(greedy=False)
-            rows.append(self.logits[0].float().clone())
-        self.eos = eos
-        return torch.stack(rows)
-
-    @torch.no_grad()
-    def generate_continue(self, max_new_tokens: int, eos_token_id: Optional[int] = None,
-                          temperature: float = 0.0, top_p: float = 1.0,
-                          generator: Optional[torch.Generator] = None, top_k: int = 0) -> torch.Tensor:
-        """Keep decoding sequence 0 until ``max_new_tokens`` tokens have been emitted in
-        total (counting those already committed) or EOS; returns all emitted tokens."""
-        if eos_token_id is not None:
-            self.eos = int(eos_token_id)
-        greedy = temperature <= 0
-        n = int(self.step[0].item())
-        budget = min(max_new_tokens, self.max_out)
-        while n < budget and not int(self.done[0].item()):
-            self._poll_hook()
-            chunk = min(self.poll_every, budget - n)
-            for _ in range(chunk):
-                self.decode_step(greedy)
-                if not greedy:
-                    self._sample_and_commit(temperature, top_p, generator, top_k)
-            n += chunk
-        toks = self.out_tokens[0, :n].to(torch.long)
-        if self.eos >= 0:
-            hit = (toks == self.eos).nonzero()
-            if hit.numel():
-                toks = toks[: int(hit[0]) + 1]
-        return toks

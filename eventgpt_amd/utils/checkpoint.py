@@ -49,12 +49,12 @@ def iter_checkpoint_tensors(path: str) -> Iterator[Tuple[str, torch.Tensor]]:
 
 
 def load_into(model: torch.nn.Module, path: str, strict: bool = True,
-              ignore_suffixes: Tuple[str, ...] = ("position_ids", "rotary_emb.inv_freq")
-              ) -> Tuple[List[str], List[str]]:
+              ignore_suffixes: Tuple[str, ...] = ("position_ids", "rotary_emb.inv_freq"),
+              grown_vocab: bool = True) -> Tuple[List[str], List[str]]:
     """Copy checkpoint tensors into ``model`` in place (dtype/device of the model).
 
     Returns ``(missing, unexpected)``.  Rows are copied into a *prefix* of a
-    larger parameter when the only mismatch is a grown vocabulary.
+    larger parameter when the only mismatch is a grown vocabulary (not with ``grown_vocab=False``).
     """
     target = dict(model.state_dict(keep_vars=True))
     seen = set()
@@ -69,7 +69,7 @@ def load_into(model: torch.nn.Module, path: str, strict: bool = True,
                 continue
             if t.shape == v.shape:
                 t.copy_(v)
-            elif t.ndim == v.ndim and t.shape[1:] == v.shape[1:] and t.shape[0] > v.shape[0]:
+            elif grown_vocab and t.ndim == v.ndim and t.shape[1:] == v.shape[1:] and t.shape[0] > v.shape[0]:
                 t[: v.shape[0]].copy_(v)
             else:
                 raise ValueError(f"{k}: checkpoint {tuple(v.shape)} vs model {tuple(t.shape)}")
