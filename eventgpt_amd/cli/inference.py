@@ -8,6 +8,10 @@ file into 5 frames, generate, print the decoded answer.
 Extras for environments without a checkpoint: ``--random_init {7b,stub125m,tiny}``
 builds a random-initialised model instead of reading ``--model_path``, and
 ``--device/--dtype`` override placement (CPU fp32 is the plumbing configuration).
+
+The model class is the one the checkpoint's ``config.json`` names (``models/registry.py``).  A text
+decoder takes ``--query`` as it is, or ``--token_ids`` where no tokenizer fits its vocabulary, and no
+event file.
 """
 from __future__ import annotations
 
@@ -24,13 +28,14 @@ from ..data.conversation import prepare_event_prompt
 from ..data.events import event_frames, load_event_npy
 from ..data.tokenizer import ByteTokenizer, load_tokenizer, tokenizer_event_token
 from ..models import EventChatConfig, EventChatModel
+from ..models.registry import read_config
 
 
 def build_parser() -> argparse.ArgumentParser:
     p = argparse.ArgumentParser(description="EventGPT inference")
     p.add_argument("--model_path", type=str, default=None)
     p.add_argument("--model_base", type=str, default=None)
-    p.add_argument("--query", type=str, required=True)
+    p.add_argument("--query", type=str, default=None)
     p.add_argument("--conv_mode", type=str, default="eventgpt_v1")
     p.add_argument("--sep", type=str, default=",")
     p.add_argument("--context_len", type=int, default=2048)
@@ -42,8 +47,10 @@ def build_parser() -> argparse.ArgumentParser:
     p.add_argument("--num_beams", type=int, default=1)
     p.add_argument("--max_new_tokens", type=int, default=512)
     p.add_argument("--spatial_temporal_encoder", type=bool, default=True)
-    p.add_argument("--event_frame", type=str, required=True)
+    p.add_argument("--event_frame", type=str, default=None)
     # extensions
+    p.add_argument("--token_ids", type=str, default=None,
+                   help="text decoders: prompt as comma-separated token ids (the answer is printed as ids too)")
     p.add_argument("--random_init", choices=["7b", "stub125m", "tiny"], default=None)
     from ..quant import add_quant_args
     add_quant_args(p)
@@ -70,10 +77,15 @@ def process_event_data(event_frame_path: str, event_processor, device, dtype=tor
     return size, tensors
 
 
-def load_model(args):
+def _placement(args):
     device = torch.device(args.device or ("cuda" if torch.cuda.is_available() else "cpu"))
     dtype = {"bfloat16": torch.bfloat16, "float32": torch.float32}[
         args.dtype or ("bfloat16" if device.type == "cuda" else "float32")]
+    return device, dtype
+
+
+def load_model(args):
+    device, dtype = _placement(args)
     if args.random_init:
         cfg = {"7b": EventChatConfig.eventgpt_7b, "stub125m": EventChatConfig.stub_125m,
                "tiny": EventChatConfig.tiny}[args.random_init]()
@@ -89,8 +101,40 @@ def load_model(args):
     return model, tokenizer, device, dtype
 
 
+def run_text(args) -> str:
+    """Generation with a text decoder: prompt ids in, text (or ids) out."""
+    device, dtype = _placement(args)
+    if args.use_4bit:
+        raise SystemExit("--use_4bit: 4-bit weights are implemented for the EventChat decoders")
+    if args.num_beams != 1:
+        raise SystemExit("--num_beams: beam search is implemented for the EventChat decoders")
+    entry, cfg = read_config(args.model_path)
+    tokenizer = None
+    if args.token_ids is not None:
+        ids = [int(t) for t in args.token_ids.split(",") if t.strip()]
+    else:
+        if args.query is None:
+            raise SystemExit("--query or --token_ids is required")
+        tokenizer = load_tokenizer(args.model_path, cfg.vocab_size)
+        ids = list(tokenizer(args.query).input_ids)
+    if not ids or min(ids) < 0 or max(ids) >= cfg.vocab_size:
+        raise SystemExit(f"prompt token ids must lie in 0..{cfg.vocab_size - 1}")
+    model = entry.model.from_pretrained(args.model_path, torch_dtype=dtype, config=cfg, device=device)
+    gen = torch.Generator(device=device).manual_seed(args.seed)
+    out = model.generate(torch.tensor(ids), do_sample=args.temperature > 0, temperature=args.temperature,
+                         top_p=args.top_p, top_k=args.top_k, max_new_tokens=args.max_new_tokens, generator=gen)
+    text = tokenizer.batch_decode(out, skip_special_tokens=True)[0].strip() if tokenizer is not None \
+        else ",".join(str(t) for t in out[0].tolist())
+    print(text)
+    return text
+
+
 def run(argv: Optional[Sequence[str]] = None) -> str:
     args = build_parser().parse_args(argv)
+    if args.model_path and not args.random_init and read_config(args.model_path)[0].modality == "text":
+        return run_text(args)
+    if args.query is None or args.event_frame is None:
+        raise SystemExit("--query and --event_frame are required")
     model, tokenizer, device, dtype = load_model(args)
     if args.use_4bit and device.type != "cuda":
         raise SystemExit("--use_4bit selects the GPU engine's weight format; on the CPU use "

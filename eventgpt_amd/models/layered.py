@@ -268,6 +268,8 @@ class LayeredDecoder:
                 z = z - 2
             elif name.endswith(".f.b"):
                 z = z + 3
+            elif name.endswith(".i.b"):
+                z = z - 3
             elif t.dim() == 2:
                 z = z / t.shape[1] ** 0.5
             t.copy_(z)
