@@ -100,6 +100,12 @@ def parse_args(argv=None):
                     help="tensor-parallel collective (default: EVGPT_TP_ALLREDUCE or rccl)")
     ap.add_argument("--weight-format", choices=["bf16", "nf4", "fp4"], default="bf16",
                     help="nf4/fp4: the reference's 4-bit rows (bitsandbytes load_in_4bit); not the headline config")
+    ap.add_argument("--layered", default=None, metavar="SIZES",
+                    help="instead of the headline: prefill and decode of a layered decoder (Nusitar) beside a LLaMA decoder "
+                         "of equal size, one JSON line per pass (1b, 7b or both with a comma); one GPU")
+    ap.add_argument("--layered-only", choices=["both", "nusitar", "llama"], default="both", help="measure one of the two models")
+    ap.add_argument("--layered-pass", default=None, metavar="PASS",
+                    help="one pass only, e.g. prefill:1x4096 or decode:8 (for profiling)")
     ap.add_argument("--rehearsal", action="store_true",
                     help="run the multi-rank flow on ONE GPU: every rank drives cuda:0 and the group is gloo "
                          "(host-copied collectives, no graphs); exercises the code path, measures nothing useful")
@@ -230,6 +236,20 @@ def run_oneshot_child(args, dist, rank: int, world: int, local_rank: int, dev):
 
 
 # --------------------------------------------------------------------- bench
+def layered_main(args) -> None:
+    from eventgpt_amd.benchmarks import layered_bench
+    kw = {}
+    if args.layered_pass:
+        kind, _, what = args.layered_pass.partition(":")
+        kw = dict(prompts=(), packs=(), streams=())
+        if kind == "decode":
+            kw["streams"] = (int(what),)
+        else:
+            b, n = (int(v) for v in what.split("x"))
+            kw.update({"prompts": (n,)} if b == 1 else {"packs": ((b, n),)})
+    layered_bench.run(sizes=tuple(args.layered.split(",")), only=args.layered_only, emit=lambda s: print(s, flush=True), **kw)
+
+
 def build_model(args, dev):
     import torch
     from eventgpt_amd.models import ClipVisionConfig, EventChatConfig, EventChatModel
@@ -331,6 +351,8 @@ def main(argv=None):
         raise SystemExit(launch_ranks(args.gpus, sys.argv[1:] if argv is None else argv))
     if args.probe:
         return probe_main(args)
+    if args.layered:
+        return layered_main(args)
 
     import torch
     world = int(os.environ.get("WORLD_SIZE", "1"))
