@@ -22,6 +22,7 @@ import concurrent.futures as cf
 import glob
 import hashlib
 import os
+import re
 import shutil
 import subprocess
 import sys
@@ -63,13 +64,23 @@ def _torch_paths():
     return inc, lib
 
 
+def _local_includes(path: str, seen=None) -> List[str]:
+    """The headers a source includes with quotes, recursively."""
+    seen = [] if seen is None else seen
+    with open(path) as f:
+        for name in re.findall(r'^\s*#\s*include\s*"([^"]+)"', f.read(), re.M):
+            hdr = os.path.normpath(os.path.join(os.path.dirname(path), name))
+            if os.path.exists(hdr) and hdr not in seen:
+                seen.append(hdr)
+                _local_includes(hdr, seen)
+    return seen
+
+
 def _digest(path: str, extra: str) -> str:
     h = hashlib.sha256()
     h.update(extra.encode())
-    with open(path, "rb") as f:
-        h.update(f.read())
-    for hdr in sorted(glob.glob(os.path.join(CSRC, "**", "*.h"), recursive=True)):
-        with open(hdr, "rb") as f:
+    for name in [path] + sorted(_local_includes(path)):
+        with open(name, "rb") as f:
             h.update(f.read())
     return h.hexdigest()[:16]
 

@@ -101,7 +101,7 @@ void launch_gemm_bf16(const bf16_t* A, const bf16_t* W, bf16_t* C, float* Cf, co
                       float* amax_val, int* amax_idx, float* splitk_ws, int splitk,
                       hipStream_t st);
 void launch_gemm_glu(const bf16_t* A, const bf16_t* W, bf16_t* H, int M, int I, int K, int lda, int ldw, int ldc,
-                     hipStream_t st);
+                     hipStream_t st, int glu_act = 0);   // 0: silu, 1: gelu (tanh form)
 bool launch_gemm_qkv_rope(const bf16_t* A, const bf16_t* W, int M, int K, bf16_t* q_out, bf16_t* k_cache,
                           bf16_t* v_cache, const float* cos_tab, const float* sin_tab, const int* pos0, int Hq,
                           int Hkv, int l_max, hipStream_t st);

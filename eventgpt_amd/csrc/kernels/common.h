@@ -120,6 +120,12 @@ __device__ __forceinline__ float gelu_f(float x) {
 __device__ __forceinline__ float quick_gelu_f(float x) { return x / (1.f + __expf(-1.702f * x)); }
 
 enum Act : int { ACT_NONE = 0, ACT_GELU = 1, ACT_QUICK_GELU = 2, ACT_SILU = 3, ACT_RELU = 4 };
+// gate of a gated linear unit: x sigmoid(x), or the tanh form of gelu as x sigmoid(2 sqrt(2 / pi) (x + 0.044715 x^3))
+enum GluAct : int { GLU_ACT_SILU = 0, GLU_ACT_GELU_TANH = 1 };
+__device__ __forceinline__ float glu_gate(float x, int act) {
+  const float z = act == GLU_ACT_GELU_TANH ? x * (1.5957691216057308f + 0.07135481627159854f * x * x) : x;
+  return x / (1.f + __expf(-z));
+}
 
 __device__ __forceinline__ float apply_act(float x, int act) {
   switch (act) {

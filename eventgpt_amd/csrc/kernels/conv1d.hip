@@ -46,9 +46,85 @@ __global__ __launch_bounds__(256) void conv_rows_kernel(SrcRows src, int col0, c
   out[row * C + c] = from_f32<T>(acc * sigmoid_f(acc));
   if (update && (live == nullptr || live[row])) ring[(slot * taps + p % taps) * C + c] = cur;
 }
+// The same over the rows of a pack whose projection is stored in T: a thread walks CR rows of eight channels with
+// the last inputs in registers; only a sequence's first taps - 1 rows of a pass look into the ring.
+constexpr int CR = 16;
+template <typename T, int TAPS>
+__global__ __launch_bounds__(256) void conv_pack_kernel(const T* __restrict__ src, long long ld, const float* __restrict__ w,
+                                                        const float* __restrict__ bias, const T* __restrict__ ring,
+                                                        T* __restrict__ out, const int* __restrict__ row_slot,
+                                                        const int* __restrict__ row_pos,
+                                                        const int* __restrict__ row_first, int rows, int C) {
+  const int c = (blockIdx.x * 256 + threadIdx.x) * 8;
+  if (c >= C) return;
+  const int r0 = blockIdx.y * CR, r1 = min(r0 + CR, rows);
+  float wv[TAPS][8], b[8], win[TAPS][8];            // win[d]: input d rows back
+#pragma unroll
+  for (int i = 0; i < 8; ++i)
+#pragma unroll
+    for (int j = 0; j < TAPS; ++j) wv[j][i] = w[static_cast<long long>(c + i) * TAPS + j];
+  load8(bias + c, b);
+#pragma unroll
+  for (int d = 1; d < TAPS; ++d) load8(src + static_cast<long long>(max(r0 - d, 0)) * ld + c, win[d - 1]);
+  for (int row = r0; row < r1; ++row) {
+#pragma unroll
+    for (int d = TAPS - 1; d > 0; --d)
+#pragma unroll
+      for (int i = 0; i < 8; ++i) win[d][i] = win[d - 1][i];
+    load8(src + static_cast<long long>(row) * ld + c, win[0]);
+    const int back = row - row_first[row];
+    float acc[8];
+#pragma unroll
+    for (int i = 0; i < 8; ++i) acc[i] = b[i];
+    if (back >= TAPS - 1) {
+#pragma unroll
+      for (int d = TAPS - 1; d >= 0; --d)
+#pragma unroll
+        for (int i = 0; i < 8; ++i) acc[i] += wv[TAPS - 1 - d][i] * win[d][i];
+    } else {
+      const int p = row_pos[row];
+      const long long slot = row_slot[row];
+#pragma unroll
+      for (int d = TAPS - 1; d >= 0; --d) {
+        if (p - d < 0) continue;
+        float x[8];
+        if (d <= back) {
+#pragma unroll
+          for (int i = 0; i < 8; ++i) x[i] = win[d][i];
+        } else {
+          load8(ring + (slot * TAPS + (p - d) % TAPS) * C + c, x);
+        }
+#pragma unroll
+        for (int i = 0; i < 8; ++i) acc[i] += wv[TAPS - 1 - d][i] * x[i];
+      }
+    }
+#pragma unroll
+    for (int i = 0; i < 8; ++i) acc[i] *= sigmoid_f(acc[i]);
+    store8(out + static_cast<long long>(row) * C + c, acc);
+  }
+}
+template <typename T>
+static bool launch_pack(const SrcRows& src, int col0, const float* w, const float* bias, const void* ring, void* out,
+                        const int* row_slot, const int* row_pos, const int* row_first, int rows, int C, int taps, hipStream_t st) {
+  const dim3 grid((C / 8 + 255) / 256, (rows + CR - 1) / CR);
+  if (C % 8 || col0 % 8 || src.nslab != 1 || grid.y > 65535 || taps < 2 || taps > 4) return false;
+  const T* p = static_cast<const T*>(src.p) + col0;
+#define EVGPT_CONV(TAPS) hipLaunchKernelGGL((conv_pack_kernel<T, TAPS>), grid, dim3(256), 0, st, p, src.ld, w, bias, \
+                                            static_cast<const T*>(ring), static_cast<T*>(out), row_slot, row_pos, row_first, rows, C)
+  if (taps == 2) EVGPT_CONV(2);
+  else if (taps == 3) EVGPT_CONV(3);
+  else EVGPT_CONV(4);
+#undef EVGPT_CONV
+  return true;
+}
+
 void launch_conv_rows(const SrcRows& src, int col0, const float* w, const float* bias, void* ring, void* out, bool f32,
                       const int* row_slot, const int* row_pos, const int* row_first, int rows, int C, int taps,
                       bool update, const int* live, hipStream_t st) {
+  if (!update && row_slot && row_first && (src.f32 != 0) == f32) {
+    if (f32 ? launch_pack<float>(src, col0, w, bias, ring, out, row_slot, row_pos, row_first, rows, C, taps, st)
+            : launch_pack<bf16_t>(src, col0, w, bias, ring, out, row_slot, row_pos, row_first, rows, C, taps, st)) return;
+  }
   const dim3 grid(rows, (C + 255) / 256);
   if (f32)
     hipLaunchKernelGGL(conv_rows_kernel<float>, grid, dim3(256), 0, st, src, col0, w, bias, static_cast<float*>(ring),

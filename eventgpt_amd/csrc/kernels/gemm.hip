@@ -81,6 +81,7 @@ struct GemmParams {
   // up region, so a lane holds both factors of its output columns and the intermediate [M, 2I]
   // tensor is never written.
   int glu_half;
+  int glu_act;         // GluAct of that mode
   // K-contiguous operands only: the columns a row really has when that is not a multiple of 64
   // (0: K itself).  K is then the contraction rounded up to 64, and the last K-tile's chunks past
   // k_cols -- which in memory are the start of the next row -- are staged as zeros.
@@ -189,7 +190,7 @@ __device__ __forceinline__ void gemm_epilogue(const GemmParams& p, f32x4_t (&acc
           float v[4];
 #pragma unroll
           for (int r = 0; r < 4; ++r)
-            v[r] = silu_f(bf16_to_f32(f32_to_bf16(acc[i][j][r]))) * bf16_to_f32(f32_to_bf16(acc[i][j + TN / 2][r]));
+            v[r] = glu_gate(bf16_to_f32(f32_to_bf16(acc[i][j][r])), p.glu_act) * bf16_to_f32(f32_to_bf16(acc[i][j + TN / 2][r]));
           const size_t o = static_cast<size_t>(m) * p.ldc + n;
           if (n + 3 < p.N && (p.ldc & 3) == 0) {
             u32x2_t w = {pack_bf16x2(v[0], v[1]), pack_bf16x2(v[2], v[3])};
@@ -274,8 +275,12 @@ __device__ __forceinline__ void gemm_epilogue(const GemmParams& p, f32x4_t (&acc
           if (n + r < p.N) v[r] = bf16_to_f32(f32_to_bf16(v[r])) + bf16_to_f32(p.res[o + r]);
       }
       if (p.Cf) {
+        if (full) {
+          *reinterpret_cast<f32x4_t*>(p.Cf + o) = f32x4_t{v[0], v[1], v[2], v[3]};
+        } else {
 #pragma unroll
-        for (int r = 0; r < 4; ++r) if (n + r < p.N) p.Cf[o + r] = v[r];
+          for (int r = 0; r < 4; ++r) if (n + r < p.N) p.Cf[o + r] = v[r];
+        }
       }
       if (p.C) {
         if (full) {
@@ -1364,13 +1369,14 @@ int gemm_splitk_t(int M, int N, int K) {
   return s < 1 ? 1 : (s > 4 ? 4 : s);
 }
 
-// H[M, I] = silu(A · Wgate^T) * (A · Wup^T) with W = [gate rows | up rows] ([2I, K]): the gate/up
+// H[M, I] = act(A · Wgate^T) * (A · Wup^T), act = silu or (glu_act) gelu, with W = [gate rows | up rows] ([2I, K]): the gate/up
 // projection of a SwiGLU MLP with the activation applied in the epilogue (GemmParams::glu_half).
 void launch_gemm_glu(const bf16_t* A, const bf16_t* W, bf16_t* H, int M, int I, int K, int lda, int ldw, int ldc,
-                     hipStream_t st) {
+                     hipStream_t st, int glu_act) {
   GemmParams p{A, W, H, nullptr, nullptr, nullptr, M, I, K, lda, ldw, ldc, ACT_NONE, nullptr, nullptr, 1, K,
                nullptr, 0, K, K};
   p.glu_half = I;
+  p.glu_act = glu_act;
   auto tiles = [&](int bm, int bn) { return static_cast<long long>((M + bm - 1) / bm) * ((2 * I + bn - 1) / bn); };
   if (g_forced_cfg < 0 && use_256(M, 2 * I, K) && g_tail_splitk && I % 128 == 0) {
     // a handful of 256 x 128 output tiles past the last full round (2115 rows x 11008: 774 = 3 x 256 + 6)

@@ -9,7 +9,7 @@
 //      chunk's slot of dS ends up holding the state at the chunk's START;
 //   3. scan_chunk_out: y_t = exp(F_t) S_start q_t + sum_{s <= t} exp(F_t - F_s) b_s (q_t . k_s) v_s.
 // The products run on MFMA.  Whatever belongs to the recurrence -- states, decays, weighted scores --
-// stays fp32: decay sums are accumulated in double (differences of long sums are taken), and fp32 MFMA
+// stays fp32: decay sums and maxima are kept in double (differences of long sums are taken), and fp32 MFMA
 // operands go in as two bf16 parts (`WideFrag`).
 //
 // With a running maximum (log_in given; b = exp(log_in)) the stored state is S exp(-m), with
@@ -37,13 +37,18 @@ __device__ __forceinline__ double wave_scan_add(double v) {
   }
   return v;
 }
-__device__ __forceinline__ float wave_scan_max(float v) {
+__device__ __forceinline__ double wave_scan_max(double v) {
   const int lane = threadIdx.x & 63;
 #pragma unroll
   for (int d = 1; d < 64; d <<= 1) {
-    const float o = __shfl_up(v, d, 64);
-    if (lane >= d) v = fmaxf(v, o);
+    const double o = __shfl_up(v, d, 64);
+    if (lane >= d) v = fmax(v, o);
   }
+  return v;
+}
+__device__ __forceinline__ double wave_max_f64(double v) {
+#pragma unroll
+  for (int off = 32; off > 0; off >>= 1) v = fmax(v, __shfl_xor(v, off, 64));
   return v;
 }
 
@@ -72,43 +77,40 @@ __device__ __forceinline__ void load_transposed(const T* __restrict__ p, long lo
   }
 }
 
+// Block: 64 value rows of one head and chunk, all of N in runs of 64.
 template <typename T, bool STAB>
 __global__ __launch_bounds__(256) void scan_chunk_state_kernel(ScanArgs a, ScanChunks c) {
   __shared__ __attribute__((aligned(16))) T kt[64 * TS];
   __shared__ __attribute__((aligned(16))) T vt[64 * TS];
   __shared__ __attribute__((aligned(16))) float wgt[SL];
-  const int nt = (a.N + 63) >> 6;
-  const int n0 = (blockIdx.x % nt) * 64, v0 = (blockIdx.x / nt) * 64;
-  const int h = blockIdx.y, ci = blockIdx.z;
+  const int v0 = blockIdx.x * 64, h = blockIdx.y, ci = blockIdx.z;
   const int row0 = c.chunks[ci * 4], len = min(c.chunks[ci * 4 + 1], SL);
   const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6, fr = lane & 15, g = lane >> 4;
-  const int nn = min(64, a.N - n0), nv = min(64, a.V - v0);
-  load_transposed(static_cast<const T*>(a.k), a.ldk, row0, len, (h / a.per_group) * a.N + n0, nn, kt);
+  const int nv = min(64, a.V - v0), k_col = (h / a.per_group) * a.N;
   load_transposed(static_cast<const T*>(a.v), a.ldv, row0, len, h * a.V + v0, nv, vt);
+  load_transposed(static_cast<const T*>(a.k), a.ldk, row0, len, k_col, min(64, a.N), kt);
   if (wid == 0) {
     const bool in = lane < len;
     const long long gi = static_cast<long long>(row0 + lane) * a.H + h;
     const double F = wave_scan_add(in ? static_cast<double>(a.log_decay[gi]) : 0.0);
     const double FL = __shfl(F, 63, 64);
-    float e = static_cast<float>(FL - F), top = 0.f, b = 1.f;
+    double e = FL - F, top = 0.0;
+    float b = 1.f;
     if constexpr (STAB) {
       e = in ? e + a.log_in[gi] : -INFINITY;
-      top = wave_max(e);
+      top = wave_max_f64(e);
     } else {
       b = in ? a.scale_in[gi] : 0.f;
     }
-    wgt[lane] = in ? expf(e - top) * b : 0.f;
+    wgt[lane] = in ? expf(static_cast<float>(e - top)) * b : 0.f;
     if (blockIdx.x == 0 && lane == 0) {
       const long long o = static_cast<long long>(ci) * a.H + h;
       c.am[o] = top;
-      c.fl[o] = static_cast<float>(FL);
+      c.fl[o] = FL;
     }
   }
   __syncthreads();
-  // D[v][n]: a wave owns 16 value rows
-  f32x4_t acc[4];
-#pragma unroll
-  for (int i = 0; i < 4; ++i) acc[i] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+  WideFrag<T> vf[SL / 32];          // a wave owns 16 value rows, weighted
 #pragma unroll
   for (int ks = 0; ks < SL / 32; ++ks) {
     float x[8], w[8];
@@ -116,23 +118,35 @@ __global__ __launch_bounds__(256) void scan_chunk_state_kernel(ScanArgs a, ScanC
     load8(wgt + ks * 32 + g * 8, w);
 #pragma unroll
     for (int j = 0; j < 8; ++j) x[j] *= w[j];
-    const WideFrag<T> vf = wide_frag<T>(x);
-#pragma unroll
-    for (int i = 0; i < 4; ++i) acc[i] = mma(vf, load_frag(kt + (i * 16 + fr) * TS + ks * 32 + g * 8), acc[i]);
+    vf[ks] = wide_frag<T>(x);
   }
-  float* dS = c.dS + (static_cast<long long>(ci) * a.H + h) * a.V * a.N;
-#pragma unroll
-  for (int i = 0; i < 4; ++i)
-#pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      const int v = wid * 16 + g * 4 + r, n = i * 16 + fr;
-      if (v < nv && n < nn) dS[static_cast<long long>(v0 + v) * a.N + n0 + n] = acc[i][r];
+  float* dS = c.dS + ((static_cast<long long>(ci) * a.H + h) * a.V + v0) * a.N;
+  for (int n0 = 0; n0 < a.N; n0 += 64) {
+    const int nn = min(64, a.N - n0);
+    if (n0 > 0) {
+      __syncthreads();
+      load_transposed(static_cast<const T*>(a.k), a.ldk, row0, len, k_col + n0, nn, kt);
+      __syncthreads();
     }
-  if constexpr (STAB) {
-    if (v0 == 0 && tid < nn) {
-      float s = 0.f;
-      for (int t = 0; t < SL; ++t) s += wgt[t] * to_f32(kt[tid * TS + t]);
-      c.dn[(static_cast<long long>(ci) * a.H + h) * a.N + n0 + tid] = s;
+    f32x4_t acc[4];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) acc[i] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int ks = 0; ks < SL / 32; ++ks)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) acc[i] = mma(load_frag(kt + (i * 16 + fr) * TS + ks * 32 + g * 8), vf[ks], acc[i]);
+    // D[n][v]: a lane holds four consecutive n of value row fr
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int v = wid * 16 + fr, n = i * 16 + g * 4;
+      if (v < nv && n < nn) *reinterpret_cast<f32x4_t*>(dS + static_cast<long long>(v) * a.N + n0 + n) = acc[i];
+    }
+    if constexpr (STAB) {
+      if (v0 == 0 && tid < nn) {
+        float s = 0.f;
+        for (int t = 0; t < SL; ++t) s += wgt[t] * to_f32(kt[tid * TS + t]);
+        c.dn[(static_cast<long long>(ci) * a.H + h) * a.N + n0 + tid] = s;
+      }
     }
   }
 }
@@ -169,16 +183,16 @@ __global__ __launch_bounds__(256) void scan_chunk_pass_kernel(ScanArgs a, ScanCh
         const f32x4_t d = nxt[k];
         if (k0 + k + PF < nc) nxt[k] = load4(dbase + (o + static_cast<long long>(PF) * a.H) * size + e);
         *reinterpret_cast<f32x4_t*>(dbase + o * size + e) = s;
-        const float fl = c.fl[o];
+        const double fl = c.fl[o];
         if constexpr (STAB) {
-          const float am = c.am[o];
+          const double am = c.am[o];
           if (lead) c.m0[o] = m;
-          const float m1 = fmaxf(fl + m, am);
-          const float x = expf(fl + m - m1), y = expf(am - m1);
+          const float m1 = static_cast<float>(fmax(fl + m, am));
+          const float x = expf(static_cast<float>(fl + m - m1)), y = expf(static_cast<float>(am - m1));
           s = s * x + d * y;
           m = m1;
         } else {
-          s = s * expf(fl) + d;
+          s = s * expf(static_cast<float>(fl)) + d;
         }
       }
     }
@@ -186,18 +200,24 @@ __global__ __launch_bounds__(256) void scan_chunk_pass_kernel(ScanArgs a, ScanCh
   }
 }
 
+// Block: 64 value columns of one head and chunk.  Scores are computed transposed, a wave per sixteen keys, and
+// meet in LDS; then a wave owns sixteen value rows for all tokens, so that the chunk's start state -- most of the
+// bytes this kernel reads -- is read once.
 template <typename T, bool STAB>
 __global__ __launch_bounds__(256) void scan_chunk_out_kernel(ScanArgs a, ScanChunks c) {
-  __shared__ __attribute__((aligned(16))) T vt[64 * TS];
+  constexpr int PS = SL + 4;                      // floats per row of the score tile
+  __shared__ __attribute__((aligned(16))) T vt[64 * TS];      // [value][key]
+  __shared__ __attribute__((aligned(16))) T qs[SL * TS];      // [token][64 of N]
+  __shared__ __attribute__((aligned(16))) float ps[SL * PS];  // [token][key] weighted scores
   __shared__ double F_s[SL];
-  __shared__ float in_s[SL], m_s[SL], b_s[SL];
+  __shared__ float in_s[SL], m_s[SL], b_s[SL], inv_s[SL];
   const int v0 = blockIdx.x * 64, h = blockIdx.y, ci = blockIdx.z;
   const int row0 = c.chunks[ci * 4], len = min(c.chunks[ci * 4 + 1], SL);
   const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6, fr = lane & 15, g = lane >> 4;
   const int nv = min(64, a.V - v0), hk = h / a.per_group;
   const long long ho = static_cast<long long>(ci) * a.H + h;
-  load_transposed(static_cast<const T*>(a.v), a.ldv, row0, len, h * a.V + v0, nv, vt);
   const float m0 = STAB ? c.m0[ho] : 0.f;
+  load_transposed(static_cast<const T*>(a.v), a.ldv, row0, len, h * a.V + v0, nv, vt);
   if (wid == 0) {
     const bool in = lane < len;
     const long long gi = static_cast<long long>(row0 + lane) * a.H + h;
@@ -206,118 +226,124 @@ __global__ __launch_bounds__(256) void scan_chunk_out_kernel(ScanArgs a, ScanChu
     if constexpr (STAB) {
       const float li = in ? a.log_in[gi] : -INFINITY;
       in_s[lane] = li;
-      const float top = fmaxf(m0, wave_scan_max(static_cast<float>(static_cast<double>(li) - F)));
-      const float m = static_cast<float>(F + static_cast<double>(top));
-      m_s[lane] = m;
+      m_s[lane] = static_cast<float>(F + fmax(static_cast<double>(m0), wave_scan_max(static_cast<double>(li) - F)));
       if (blockIdx.x == 0 && lane == len - 1 && c.chunks[ci * 4 + 3])
-        a.m[static_cast<long long>(c.chunks[ci * 4 + 2]) * a.H + h] = fmaxf(c.fl[ho] + m0, c.am[ho]);
+        a.m[static_cast<long long>(c.chunks[ci * 4 + 2]) * a.H + h] = static_cast<float>(fmax(c.fl[ho] + m0, c.am[ho]));
     } else {
       b_s[lane] = in ? a.scale_in[gi] : 0.f;
     }
   }
-  __syncthreads();
-  if (wid * 16 >= len) return;
-  // lane: token t of this wave's sixteen
-  const int t = wid * 16 + fr, tc = min(t, len - 1);
-  const T* qp = static_cast<const T*>(a.q) + (row0 + tc) * a.ldq + static_cast<long long>(hk) * a.N;
-  const T* kp = static_cast<const T*>(a.k) + static_cast<long long>(hk) * a.N;
-  const float* S0 = c.dS + ho * a.V * a.N + static_cast<long long>(v0) * a.N;
+  const T* qp = static_cast<const T*>(a.q) + static_cast<long long>(hk) * a.N;
+  const T* kp = static_cast<const T*>(a.k) + (row0 + min(wid * 16 + fr, len - 1)) * a.ldk + static_cast<long long>(hk) * a.N;
+  const float* S0 = c.dS + (ho * a.V + v0 + wid * 16 + fr) * a.N;
   const float* nrm = STAB ? c.dn + ho * a.N : nullptr;
-  f32x4_t st[4], inter[4], y[4];
+  const bool rows_v = wid * 16 < nv;              // this wave has value rows
+  f32x4_t st[4], inter[4];
 #pragma unroll
-  for (int i = 0; i < 4; ++i) st[i] = inter[i] = y[i] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+  for (int i = 0; i < 4; ++i) st[i] = inter[i] = f32x4_t{0.f, 0.f, 0.f, 0.f};
   float nq = 0.f;
-  for (int n = g * 8; n < a.N; n += 32) {
-    const Frag<T> qf = load_frag(qp + n);
+  for (int n0 = 0; n0 < a.N; n0 += 64) {
+    const int nn = min(64, a.N - n0);
+    __syncthreads();
 #pragma unroll
-    for (int i = 0; i < 4; ++i)
-      if (i <= wid) {
-        const int s = min(i * 16 + fr, len - 1);
-        st[i] = mma(load_frag(kp + (row0 + s) * a.ldk + n), qf, st[i]);
+    for (int i = 0; i < 2; ++i) {
+      const int idx = tid + i * 256, t = idx >> 3, c8 = (idx & 7) * 8;
+      if (c8 < nn) {
+        const T* p = qp + (row0 + min(t, len - 1)) * a.ldq + n0 + c8;
+        T* d = qs + t * TS + c8;
+        *reinterpret_cast<u32x4_t*>(d) = load16(p);
+        if constexpr (sizeof(T) == 4) *reinterpret_cast<u32x4_t*>(d + 4) = load16(p + 4);
       }
+    }
+    __syncthreads();
+    for (int n = 0; n < nn; n += 32) {
+      Frag<T> qf[4];
 #pragma unroll
-    for (int i = 0; i < 4; ++i)
-      if (i * 16 < nv) {
+      for (int j = 0; j < 4; ++j) qf[j] = load_frag(qs + (j * 16 + fr) * TS + n + g * 8);
+      const Frag<T> kf = load_frag(kp + n0 + n + g * 8);
+#pragma unroll
+      for (int j = 0; j < 4; ++j)
+        if (j >= wid) st[j] = mma(kf, qf[j], st[j]);
+      if (rows_v) {
         float x[8];
-        load8(S0 + static_cast<long long>(i * 16 + fr) * a.N + n, x);
-        inter[i] = mma(wide_frag<T>(x), qf, inter[i]);
-      }
-    if constexpr (STAB) {
-      float x[8], q8[8];
-      load8(nrm + n, x);
-      load8(qp + n, q8);
+        load8(S0 + n0 + n + g * 8, x);
+        const WideFrag<T> sf = wide_frag<T>(x);
 #pragma unroll
-      for (int j = 0; j < 8; ++j) nq += x[j] * q8[j];
+        for (int j = 0; j < 4; ++j) inter[j] = mma(sf, qf[j], inter[j]);
+      }
+    }
+    if constexpr (STAB) {
+      const int t = tid >> 2, part = (tid & 3) * 16;
+      for (int n = part; n < min(part + 16, nn); ++n) nq += nrm[n0 + n] * to_f32(qs[t * TS + n]);
     }
   }
-  // weighted scores of this lane's token; the accumulator layout is the operand layout of the next product
-  // with contraction slot (g, j) <-> key 32 b + 4 g + j (j < 4) or 32 b + 16 + 4 g + j - 4
-  const double Ft = F_s[tc];
-  const float mt = STAB ? m_s[tc] : 0.f;
-  float den = 0.f;
+  // weighted scores of keys 16 wid + 4 g + r and token 16 j + fr
 #pragma unroll
-  for (int i = 0; i < 4; ++i)
+  for (int j = 0; j < 4; ++j) {
+    const int t = j * 16 + fr;
+    const double Ft = F_s[t];
+    const float mt = STAB ? m_s[t] : 0.f;
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
-      const int s = i * 16 + g * 4 + r;
+      const int s = wid * 16 + g * 4 + r;
       float w = 0.f;
-      if (s <= t && s < len) {
-        w = static_cast<float>(Ft - F_s[s]);
-        if constexpr (STAB) w = expf(w + in_s[s] - mt);
-        else w = expf(w) * b_s[s];
+      if (s <= t && t < len) {
+        if constexpr (STAB) w = expf(static_cast<float>(Ft - F_s[s] + static_cast<double>(in_s[s] - mt)));
+        else w = expf(static_cast<float>(Ft - F_s[s])) * b_s[s];
       }
-      st[i][r] *= w * a.qscale;
-      den += st[i][r];
+      st[j][r] *= w * a.qscale;
     }
-#pragma unroll
-  for (int kb = 0; kb < 2; ++kb) {
-    if (kb * 2 > wid) break;
-    float x[8];
-#pragma unroll
-    for (int j = 0; j < 4; ++j) { x[j] = st[kb * 2][j]; x[4 + j] = st[kb * 2 + 1][j]; }
-    const WideFrag<T> pf = wide_frag<T>(x);
-#pragma unroll
-    for (int i = 0; i < 4; ++i)
-      if (i * 16 < nv) {
-        const T* vr = vt + (i * 16 + fr) * TS + kb * 32 + g * 4;
-        Frag<T> vf;
-        if constexpr (sizeof(T) == 2) {
-          const u32x2_t lo = *reinterpret_cast<const u32x2_t*>(vr), hi = *reinterpret_cast<const u32x2_t*>(vr + 16);
-          vf.v = __builtin_bit_cast(bf16x8_t, u32x4_t{lo[0], lo[1], hi[0], hi[1]});
-        } else {
-#pragma unroll
-          for (int j = 0; j < 4; ++j) { vf.v[j] = vr[j]; vf.v[4 + j] = vr[16 + j]; }
-        }
-        y[i] = mma(vf, pf, y[i]);
-      }
+    *reinterpret_cast<f32x4_t*>(ps + t * PS + wid * 16 + g * 4) = st[j];
   }
-  const float carry = expf(static_cast<float>(Ft + static_cast<double>(m0)) - mt) * a.qscale;
-  float inv = 1.f;
+  __syncthreads();
   if constexpr (STAB) {
-    den += __shfl_xor(den, 16, 64);
-    den += __shfl_xor(den, 32, 64);
-    nq += __shfl_xor(nq, 16, 64);
-    nq += __shfl_xor(nq, 32, 64);
-    inv = 1.f / (fmaxf(fabsf(nq * carry + den), expf(-mt)) + 1e-6f);
-  }
-  if (t >= len) return;
-  const float skip = a.skip ? a.skip[h] : 0.f;
-  T* o = static_cast<T*>(a.out) + (static_cast<long long>(row0 + t) * a.H + h) * a.V + v0;
-  const T* vrow = static_cast<const T*>(a.v) + (row0 + t) * a.ldv + static_cast<long long>(h) * a.V + v0;
+    const int t = tid >> 2, part = (tid & 3) * 16;
+    float den = 0.f;
 #pragma unroll
-  for (int i = 0; i < 4; ++i)
-    if (i * 16 < nv) {
-      const int v = i * 16 + g * 4;
-      f32x4_t r = (inter[i] * carry + y[i]) * inv;
-      if (a.skip) r += load4(vrow + v) * skip;
-      store4(o + v, r[0], r[1], r[2], r[3]);
+    for (int i = 0; i < 16; i += 4) {
+      const f32x4_t x = *reinterpret_cast<const f32x4_t*>(ps + t * PS + part + i);
+      den += x[0] + x[1] + x[2] + x[3];
     }
+    const float carry = expf(static_cast<float>(F_s[t] + static_cast<double>(m0 - m_s[t]))) * a.qscale;
+    den += nq * carry;
+    den += __shfl_xor(den, 1, 64);
+    den += __shfl_xor(den, 2, 64);
+    if ((tid & 3) == 0) inv_s[t] = 1.f / (fmaxf(fabsf(den), expf(-m_s[t])) + 1e-6f);
+    __syncthreads();
+  }
+  if (!rows_v) return;
+  Frag<T> vf[SL / 32];
+#pragma unroll
+  for (int kb = 0; kb < SL / 32; ++kb) vf[kb] = load_frag(vt + (wid * 16 + fr) * TS + kb * 32 + g * 8);
+  const float skip = a.skip ? a.skip[h] : 0.f;
+#pragma unroll
+  for (int j = 0; j < 4; ++j) {
+    const int t = j * 16 + fr;
+    f32x4_t y = f32x4_t{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int kb = 0; kb < SL / 32; ++kb)
+      if (kb * 2 <= j) {
+        float x[8];
+        load8(ps + t * PS + kb * 32 + g * 8, x);
+        y = mma(vf[kb], wide_frag<T>(x), y);
+      }
+    if (t >= len) continue;
+    const float carry = expf(static_cast<float>(F_s[t] + static_cast<double>(m0 - (STAB ? m_s[t] : 0.f)))) * a.qscale;
+    y += inter[j] * carry;
+    if constexpr (STAB) y *= inv_s[t];
+    const int v = wid * 16 + g * 4;
+    if (a.skip) {
+#pragma unroll
+      for (int r = 0; r < 4; ++r) y[r] += skip * to_f32(vt[(v + r) * TS + t]);
+    }
+    store4(static_cast<T*>(a.out) + (static_cast<long long>(row0 + t) * a.H + h) * a.V + v0 + v, y[0], y[1], y[2], y[3]);
+  }
 }
 
 void launch_scan_prefill(const ScanArgs& a, const ScanChunks& c, bool f32, hipStream_t st) {
-  const int nt = (a.N + 63) / 64, vt = (a.V + 63) / 64;
+  const int vt = (a.V + 63) / 64;
   const bool stab = a.log_in != nullptr;
-  const dim3 g1(nt * vt, a.H, c.C), g3(vt, a.H, c.C);
+  const dim3 g1(vt, a.H, c.C), g3(vt, a.H, c.C);
   const long long quads = static_cast<long long>(a.V) * a.N / 4;
   const dim3 g2(static_cast<unsigned>((quads + 255) / 256) + (stab ? 1 : 0), a.H, c.nseq);
   if (f32) {

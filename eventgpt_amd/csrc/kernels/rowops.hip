@@ -214,7 +214,18 @@ __global__ __launch_bounds__(256) void group_norm_kernel(const T* __restrict__ y
   }
   __syncthreads();
   const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
-  if (parts >= 4) {
+  if (v == vp && (plen & 7) == 0 && parts >= 4) {      // no padding between heads: a part is a run of the row
+    for (int p = wid; p < parts; p += 4) {
+      float s = 0.f;
+      for (int i = lane * 8; i < plen; i += 512) {
+        float t[8];
+        load8(row_lds + p * plen + i, t);
+        s += sumsq8(t);
+      }
+      s = wave_sum(s);
+      if (lane == 0) inv[p] = rsqrtf(s / static_cast<float>(plen) + eps);
+    }
+  } else if (parts >= 4) {
     for (int p = wid; p < parts; p += 4) {
       float s = 0.f;
       for (int i = lane; i < plen; i += 64) {
@@ -246,9 +257,11 @@ __global__ __launch_bounds__(256) void group_norm_kernel(const T* __restrict__ y
       load8(row_lds + c, a);
       load8(w + c, g);
       const int h = c / vp, c0 = h * v + c % vp;      // vp is a multiple of 8: eight slots of one head
+      const int part0 = min(c0 / plen, parts - 1), next = (part0 + 1) * plen;
 #pragma unroll
       for (int i = 0; i < 8; ++i) {
-        const int part = min((c0 + i) / plen, parts - 1);   // padding slots have zero weight
+        // (padding slots have zero weight)
+        const int part = c0 + i < next ? part0 : min((c0 + i) / plen, parts - 1);
         a[i] *= inv[part] * g[i];
       }
       if constexpr (!BEFORE) {
@@ -419,6 +432,53 @@ __global__ __launch_bounds__(256) void attn_prep_kernel(AttnPrepArgs a) {
     return u;
   };
   T* q = static_cast<T*>(a.q_out) + row * qn;
+  if ((half & 7) == 0) {
+    // eight elements of a head at a time, with the eight they are paired with
+    auto value8 = [&](int col, const float* w, float r, int c, float (&u)[8]) {
+      const int d = c % a.D;
+      src8(a.src, row, col + c, u);
+      float g[8];
+      if (w) {
+        load8(w + c, g);
+#pragma unroll
+        for (int i = 0; i < 8; ++i) u[i] *= r * g[i];
+      }
+      if (d >= a.rot) return;
+      const bool lo = d < half;
+      const int c2 = lo ? c + half : c - half, i0 = lo ? d : d - half;
+      float o[8], cc[8], ss[8];
+      src8(a.src, row, col + c2, o);
+      if (w) {
+        load8(w + c2, g);
+#pragma unroll
+        for (int i = 0; i < 8; ++i) o[i] *= r * g[i];
+      }
+      load8(cs + i0, cc);
+      load8(sn + i0, ss);
+#pragma unroll
+      for (int i = 0; i < 8; ++i) u[i] = lo ? u[i] * cc[i] - o[i] * ss[i] : u[i] * cc[i] + o[i] * ss[i];
+    };
+    for (int c = threadIdx.x * 8; c < qn; c += 2048) {
+      float u[8];
+      value8(a.q_col, a.qw, rq, c, u);
+      store8(q + c, u);
+    }
+    for (int c = threadIdx.x * 8; c < kn; c += 2048) {
+      float u[8], v[8];
+      value8(a.k_col, a.kw, rk, c, u);
+      src8(a.src, row, a.v_col + c, v);
+      if (kv >= 0) {
+        store8(static_cast<T*>(a.k_buf) + kv * kn + c, u);
+        store8(static_cast<T*>(a.v_buf) + kv * kn + c, v);
+      }
+      if (keep) {
+        const long long o = ((slot * a.Hkv + c / a.D) * a.cap + cslot) * a.D + c % a.D;
+        store8(static_cast<T*>(a.k_cache) + o, u);
+        store8(static_cast<T*>(a.v_cache) + o, v);
+      }
+    }
+    return;
+  }
   for (int c = threadIdx.x; c < qn; c += 256) q[c] = from_f32<T>(value(a.q_col, a.qw, rq, c / a.D, c % a.D));
   for (int c = threadIdx.x; c < kn; c += 256) {
     const int h = c / a.D, d = c % a.D;

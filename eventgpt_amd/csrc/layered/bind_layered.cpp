@@ -90,6 +90,28 @@ Tensor linear_slabs(const Tensor& x, const Tensor& w) {
   return used == sk ? ws : ws.narrow(0, 0, used);
 }
 
+// act(x Wgate^T) * (x Wup^T), w_gate_up [2 I, K]; bf16: the activation in the GEMM's epilogue
+Tensor linear_glu(const Tensor& x, const Tensor& w, int64_t act) {
+  TORCH_CHECK(act == evgpt::GLU_GELU_TANH || act == evgpt::GLU_SILU, "linear_glu: act 0 or 1");
+  TORCH_CHECK(w.dim() == 2 && w.size(0) % 64 == 0, "linear_glu: w_gate_up [2 I, K], I % 32 == 0");
+  const int64_t I = w.size(0) / 2;
+  if (is_f32(x) || x.size(0) <= 32) {
+    const Tensor y = is_f32(x) ? linear(x, w, true) : linear_slabs(x, w);
+    Tensor h = at::empty({x.size(0), I}, x.options());
+    const SrcRows s{y.data_ptr(), y.dim() == 3 ? y.stride(0) : 0, y.dim() == 3 ? (int)y.size(0) : 1, (int)(2 * I), 1};
+    evgpt::launch_glu_rows(s, h.data_ptr(), is_f32(x), (int)x.size(0), (int)I, (int)act, cur_stream());
+    return h;
+  }
+  check_t(x, "x"); check_t(w, "w");
+  const int64_t M = x.size(0), K = x.size(1);
+  TORCH_CHECK(x.dim() == 2 && !is_f32(w) && w.size(1) == K && K % 64 == 0 && K > 0, "linear_glu: x [M, K], K % 64 == 0");
+  TORCH_CHECK(2 * I * K * 2 < (1ll << 31) && M * K * 2 < (1ll << 31), "linear_glu: operands over 2 GiB");
+  Tensor h = at::empty({M, I}, x.options());
+  evgpt::launch_gemm_glu(bptr(x), bptr(w), bptr_mut(h), (int)M, (int)I, (int)K, (int)K, (int)K, (int)I, cur_stream(),
+                         act == evgpt::GLU_SILU ? 0 : 1);
+  return h;
+}
+
 // ---------------------------------------------------------------- rows
 Tensor embed_rows(const Tensor& tok, const Tensor& embed, double scale) {
   check_i(tok, "tokens"); check_t(embed, "embed");
@@ -366,9 +388,10 @@ Tensor scan_prefill_(const Tensor& q, const Tensor& k, const Tensor& v, int64_t 
   Tensor o = at::empty({q.size(0), H * V}, q.options());
   if (C == 0) return o;
   auto f = q.options().dtype(at::kFloat);
-  Tensor dS = at::empty({C, H, V, N}, f), dn = at::empty({C, H, N}, f), sc = at::empty({3, C, H}, f);
+  Tensor dS = at::empty({C, H, V, N}, f), dn = at::empty({C, H, N}, f), m0 = at::empty({C, H}, f);
+  Tensor sc = at::empty({2, C, H}, f.dtype(at::kDouble));
   evgpt::ScanChunks c{chunks.data_ptr<int>(), seqs.data_ptr<int>(), (int)C, (int)seqs.size(0), dS.data_ptr<float>(),
-                      dn.data_ptr<float>(), sc.data_ptr<float>(), sc.data_ptr<float>() + C * H, sc.data_ptr<float>() + 2 * C * H};
+                      dn.data_ptr<float>(), sc.data_ptr<double>(), sc.data_ptr<double>() + C * H, m0.data_ptr<float>()};
   a.out = o.data_ptr();
   evgpt::launch_scan_prefill(a, c, is_f32(q), cur_stream());
   return o;
@@ -448,6 +471,7 @@ void conv_tail_(const Tensor& src, int64_t col0, const Tensor& ring, const Tenso
 TORCH_LIBRARY(evlay, m) {
   m.def("linear(Tensor x, Tensor w, bool out_f32) -> Tensor", &linear);
   m.def("linear_slabs(Tensor x, Tensor w) -> Tensor", &linear_slabs);
+  m.def("linear_glu(Tensor x, Tensor w_gate_up, int act) -> Tensor", &linear_glu);
   m.def("embed_rows(Tensor tok, Tensor embed, float scale) -> Tensor", &embed_rows);
   m.def("norm_rows(Tensor x, Tensor? sel, Tensor w, int n, float eps, bool f32) -> Tensor", &norm_rows);
   m.def("add_norm_rows_(Tensor(a!) x, Tensor y, Tensor? w, int n, float eps, bool f32) -> Tensor", &add_norm_rows_);

@@ -111,7 +111,8 @@ struct ScanChunks {
   int C, nseq;
   float* dS;                       // [C][H][V][N]
   float* dn;                       // [C][H][N]
-  float* am; float* fl; float* m0; // [C][H]
+  double* am; double* fl;          // [C][H]
+  float* m0;                       // [C][H]
 };
 constexpr int SCAN_CHUNK = 64;
 void launch_scan_prefill(const ScanArgs& a, const ScanChunks& c, bool f32, hipStream_t st);

@@ -341,8 +341,7 @@ class DenseMLP(Mixer):
 
     def residual(self, rows: RowBatch, x: torch.Tensor, xn: torch.Tensor, norm: Optional[torch.Tensor]) -> torch.Tensor:
         raw = self.raw
-        h = raw.glu_rows(raw.linear_slabs(xn, self.w_gate_up) if rows.decode else raw.linear(xn, self.w_gate_up, False),
-                         self.act, self.f32)
+        h = raw.linear_glu(xn, self.w_gate_up, self.act)
         return raw.add_norm_rows_(x, self._out(rows, self.w_down, h), norm, self.width, self.eps, self.f32)
 
 

@@ -304,7 +304,9 @@ def test_matrix_memory_extreme_gates(raw, dev, dtype):
     o = raw.scan_prefill_(q.view(T, -1), k.view(T, -1), v.view(T, -1), H, 1, Nn, V, 1.0, lf.to(dev), li.to(dev), None, None, *st,
                           rb.chunks, rb.scan_seqs)
     err = (o.cpu().double().view(T, H, V) - want).pow(2).mean(-1).sqrt() / want.pow(2).mean(-1).sqrt().clamp_min(1e-3)
-    assert float(err.max()) < (1e-4 if dtype == torch.float32 else 3e-2)
+    # (a token whose query is nearly orthogonal to the one stored key is ill-conditioned: 2e-4 in a plain 32-bit scan)
+    assert float(err.max()) < (1e-3 if dtype == torch.float32 else 3e-2)
+    assert float(err.median()) < (1e-6 if dtype == torch.float32 else 5e-3)
 
 
 def prep(raw, dev, dtype, src, cfg, D, rb, cache, eps=1e-3, qw=None, kw=None, k_buf=None, v_buf=None, row_kv=None, keep=None):
