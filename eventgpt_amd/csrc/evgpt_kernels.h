@@ -276,7 +276,7 @@ void launch_argmax_pair_select(const unsigned* pairs, int W, int B, int* token, 
 // ---- attn_decode.hip
 void launch_attn_decode(const bf16_t* q, const bf16_t* k_cache, const bf16_t* v_cache,
                         bf16_t* out, float* part_o, float* part_ml, const int* pos, int B, int Hq,
-                        int Hkv, int D, int l_max, int nsplit, float scale, hipStream_t st);
+                        int Hkv, int D, int l_max, int nsplit, float scale, hipStream_t st, int ring = 0);
 
 // ---- attn_prefill.hip
 void launch_attn_prefill(const bf16_t* q, const bf16_t* k, const bf16_t* v, bf16_t* o,

@@ -21,14 +21,15 @@ template <int D, bool FINAL = false>
 __global__ __launch_bounds__(AD_WAVES * 64) void attn_decode_split_kernel(
     const bf16_t* __restrict__ q, const bf16_t* __restrict__ k_cache,
     const bf16_t* __restrict__ v_cache, float* __restrict__ part_o, float* __restrict__ part_ml,
-    const int* __restrict__ pos, int Hq, int Hkv, int l_max, float scale, bf16_t* __restrict__ out) {
+    const int* __restrict__ pos, int Hq, int Hkv, int l_max, float scale, bf16_t* __restrict__ out, int ring) {
   constexpr int LPK = D / 8;       // lanes per key row
   constexpr int KPW = 64 / LPK;    // keys per wave-instruction
   const int h = blockIdx.x, split = blockIdx.y, b = blockIdx.z, nsplit = gridDim.y;
   const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6;
   const int sub = lane / LPK, dl = lane % LPK;
   // the current token's K/V were appended by the QKV kernel; never read past the cache
-  const int len = min(max(pos[b] + 1, 1), l_max);
+  // (ring: the cache holds the last pos % l_max + 1 positions only, from slot 0 on)
+  const int len = ring ? max(pos[b], 0) % l_max + 1 : min(max(pos[b] + 1, 1), l_max);
   const int hk = h / (Hq / Hkv);
 
   // this split's key range, in units of KPW-key groups
@@ -157,25 +158,26 @@ __global__ __launch_bounds__(D) void attn_decode_combine_kernel(const float* __r
 
 void launch_attn_decode(const bf16_t* q, const bf16_t* k_cache, const bf16_t* v_cache,
                         bf16_t* out, float* part_o, float* part_ml, const int* pos, int B, int Hq,
-                        int Hkv, int D, int l_max, int nsplit, float scale, hipStream_t st) {
+                        int Hkv, int D, int l_max, int nsplit, float scale, hipStream_t st,
+                        int ring) {
   dim3 grid(Hq, nsplit, B), block(AD_WAVES * 64);
   if (nsplit == 1) {   // many streams: no partial results, no second launch
     if (D == 128)
       hipLaunchKernelGGL((attn_decode_split_kernel<128, true>), grid, block, 0, st, q, k_cache, v_cache,
-                         part_o, part_ml, pos, Hq, Hkv, l_max, scale, out);
+                         part_o, part_ml, pos, Hq, Hkv, l_max, scale, out, ring);
     else
       hipLaunchKernelGGL((attn_decode_split_kernel<64, true>), grid, block, 0, st, q, k_cache, v_cache,
-                         part_o, part_ml, pos, Hq, Hkv, l_max, scale, out);
+                         part_o, part_ml, pos, Hq, Hkv, l_max, scale, out, ring);
     return;
   }
   if (D == 128) {
     hipLaunchKernelGGL((attn_decode_split_kernel<128, false>), grid, block, 0, st, q, k_cache, v_cache,
-                       part_o, part_ml, pos, Hq, Hkv, l_max, scale, out);
+                       part_o, part_ml, pos, Hq, Hkv, l_max, scale, out, ring);
     hipLaunchKernelGGL(attn_decode_combine_kernel<128>, dim3(Hq, B), dim3(128), 0, st, part_o,
                        part_ml, out, Hq, nsplit);
   } else {
     hipLaunchKernelGGL((attn_decode_split_kernel<64, false>), grid, block, 0, st, q, k_cache, v_cache,
-                       part_o, part_ml, pos, Hq, Hkv, l_max, scale, out);
+                       part_o, part_ml, pos, Hq, Hkv, l_max, scale, out, ring);
     hipLaunchKernelGGL(attn_decode_combine_kernel<64>, dim3(Hq, B), dim3(64), 0, st, part_o,
                        part_ml, out, Hq, nsplit);
   }

@@ -17,8 +17,8 @@
 // output: y_t = S_t q_t / (max(|n_t . q_t|, exp(-m_t)) + 1e-6).  m is a max-plus scan, so it chunks too:
 // m_t = F_t + max(m_start, max_{s <= t}(log_in_s - F_s)).
 //
-// Decode (scan_step) streams the state once: sixteen lanes per state row, read, decayed, updated, dotted
-// with q and written back in one pass.
+// n and m are stored twice, indexed by the parity of the position they are read at, so that a decode step
+// (decode_step.hip) can write the next ones while other blocks still read the old ones.
 #include "elem.h"
 #include "../layered_kernels.h"
 
@@ -157,18 +157,21 @@ __global__ __launch_bounds__(256) void scan_chunk_pass_kernel(ScanArgs a, ScanCh
   const int* sq = c.seqs + blockIdx.z * 4;
   const int c0 = sq[0], nc = sq[1];
   const long long slot = sq[2];
-  const bool fresh = sq[3] != 0;
+  const bool fresh = (sq[3] & 1) != 0;
+  const long long nm_in = (static_cast<long long>(sq[3] >> 1 & 1) * a.slots + slot) * a.H;    // [2][slots][H]
+  const long long nm_out = (static_cast<long long>(sq[3] >> 2 & 1) * a.slots + slot) * a.H;
   const int h = blockIdx.y;
   const long long per = static_cast<long long>(a.V) * a.N;
   const bool norm = STAB && blockIdx.x == gridDim.x - 1;
   const long long size = norm ? a.N : per;
   const long long e0 = norm ? threadIdx.x * 4ll : (static_cast<long long>(blockIdx.x) * 256 + threadIdx.x) * 4;
-  const float m_in = STAB && !fresh ? a.m[slot * a.H + h] : 0.f;
-  float* state = norm ? a.n + (slot * a.H + h) * a.N : a.S + (slot * a.H + h) * per;
+  const float m_in = STAB && !fresh ? a.m[nm_in + h] : 0.f;
+  const float* from = norm ? a.n + (nm_in + h) * a.N : a.S + (slot * a.H + h) * per;
+  float* to = norm ? a.n + (nm_out + h) * a.N : a.S + (slot * a.H + h) * per;
   float* dbase = norm ? c.dn : c.dS;
   const bool lead = blockIdx.x == 0 && threadIdx.x == 0;
   for (long long e = e0; e < size; e += norm ? 1024 : size) {
-    f32x4_t s = fresh ? f32x4_t{0.f, 0.f, 0.f, 0.f} : load4(state + e);
+    f32x4_t s = fresh ? f32x4_t{0.f, 0.f, 0.f, 0.f} : load4(from + e);
     float m = m_in;
     constexpr int PF = 4;            // chunk slots in flight
     f32x4_t nxt[PF];
@@ -196,7 +199,7 @@ __global__ __launch_bounds__(256) void scan_chunk_pass_kernel(ScanArgs a, ScanCh
         }
       }
     }
-    *reinterpret_cast<f32x4_t*>(state + e) = s;
+    *reinterpret_cast<f32x4_t*>(to + e) = s;
   }
 }
 
@@ -227,8 +230,9 @@ __global__ __launch_bounds__(256) void scan_chunk_out_kernel(ScanArgs a, ScanChu
       const float li = in ? a.log_in[gi] : -INFINITY;
       in_s[lane] = li;
       m_s[lane] = static_cast<float>(F + fmax(static_cast<double>(m0), wave_scan_max(static_cast<double>(li) - F)));
-      if (blockIdx.x == 0 && lane == len - 1 && c.chunks[ci * 4 + 3])
-        a.m[static_cast<long long>(c.chunks[ci * 4 + 2]) * a.H + h] = static_cast<float>(fmax(c.fl[ho] + m0, c.am[ho]));
+      const int last = c.chunks[ci * 4 + 3];
+      if (blockIdx.x == 0 && lane == len - 1 && (last & 1))
+        a.m[(static_cast<long long>(last >> 1 & 1) * a.slots + c.chunks[ci * 4 + 2]) * a.H + h] = static_cast<float>(fmax(c.fl[ho] + m0, c.am[ho]));
     } else {
       b_s[lane] = in ? a.scale_in[gi] : 0.f;
     }
@@ -361,98 +365,6 @@ void launch_scan_prefill(const ScanArgs& a, const ScanChunks& c, bool f32, hipSt
   } else {
     if (stab) hipLaunchKernelGGL((scan_chunk_out_kernel<bf16_t, true>), g3, dim3(256), 0, st, a, c);
     else hipLaunchKernelGGL((scan_chunk_out_kernel<bf16_t, false>), g3, dim3(256), 0, st, a, c);
-  }
-}
-
-// One token.  Block: sixteen state rows of one head; sixteen lanes per row.  Every block of a head computes
-// the new maximum and the normaliser's dot product itself; the normaliser and the maximum are stored by a
-// second launch, when all of them have read the old ones.
-template <typename T, bool STAB>
-__global__ __launch_bounds__(256) void scan_step_kernel(ScanArgs a, const int* __restrict__ pos,
-                                                        const int* __restrict__ live) {
-  const int h = blockIdx.y, b = blockIdx.z, v0 = blockIdx.x * 16;
-  if (live && !live[b]) return;       // a parked sequence keeps its state
-  const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6, l16 = lane & 15, rg = lane >> 4;
-  const bool fresh = pos[b] <= 0;
-  const int hk = h / a.per_group;
-  const T* q = static_cast<const T*>(a.q) + b * a.ldq + static_cast<long long>(hk) * a.N;
-  const T* k = static_cast<const T*>(a.k) + b * a.ldk + static_cast<long long>(hk) * a.N;
-  const int gi = b * a.H + h;
-  float decay, add, inv = 1.f;
-  const int v = v0 + wid * 4 + rg;
-  float* Sr = a.S + (static_cast<long long>(gi) * a.V + v) * a.N;
-  if constexpr (STAB) {
-    const float m = fresh ? 0.f : a.m[gi];
-    const float lf = a.log_decay[gi], li = a.log_in[gi];
-    const float m1 = fmaxf(lf + m, li);
-    decay = expf(lf + m - m1);
-    add = expf(li - m1);
-    float dot = 0.f;
-    const float* n = a.n + static_cast<long long>(gi) * a.N;
-    for (int e = l16 * 4; e < a.N; e += 64) {
-      const f32x4_t kk = load4(k + e), qq = load4(q + e);
-      const f32x4_t nn = fresh ? kk * add : load4(n + e) * decay + kk * add;
-#pragma unroll
-      for (int i = 0; i < 4; ++i) dot += nn[i] * qq[i];
-    }
-    dot = group_sum<16>(dot) * a.qscale;
-    inv = 1.f / (fmaxf(fabsf(dot), expf(-m1)) + 1e-6f);
-  } else {
-    decay = expf(a.log_decay[gi]);
-    add = a.scale_in[gi];
-  }
-  const float vv = to_f32(static_cast<const T*>(a.v)[b * a.ldv + static_cast<long long>(h) * a.V + v]);
-  const float av = add * vv;
-  float y = 0.f;
-  for (int e = l16 * 4; e < a.N; e += 64) {
-    const f32x4_t kk = load4(k + e), qq = load4(q + e);
-    f32x4_t s = kk * av;
-    if (!fresh) s += load4(Sr + e) * decay;
-    *reinterpret_cast<f32x4_t*>(Sr + e) = s;
-#pragma unroll
-    for (int i = 0; i < 4; ++i) y += s[i] * qq[i];
-  }
-  y = group_sum<16>(y) * a.qscale * inv;
-  if (a.skip) y += a.skip[h] * vv;
-  if (l16 == 0) static_cast<T*>(a.out)[(static_cast<long long>(b) * a.H + h) * a.V + v] = from_f32<T>(y);
-}
-
-// normaliser and maximum of the step, after every block of scan_step has read the old ones
-template <typename T>
-__global__ __launch_bounds__(256) void scan_step_norm_kernel(ScanArgs a, const int* __restrict__ pos,
-                                                             const int* __restrict__ live) {
-  const int h = blockIdx.x, b = blockIdx.y;
-  if (live && !live[b]) return;
-  const bool fresh = pos[b] <= 0;
-  const int gi = b * a.H + h;
-  const T* k = static_cast<const T*>(a.k) + b * a.ldk + static_cast<long long>(h / a.per_group) * a.N;
-  const float m = fresh ? 0.f : a.m[gi];
-  const float lf = a.log_decay[gi], li = a.log_in[gi];
-  const float m1 = fmaxf(lf + m, li);
-  const float decay = expf(lf + m - m1), add = expf(li - m1);
-  float* n = a.n + static_cast<long long>(gi) * a.N;
-  for (int e = threadIdx.x * 4; e < a.N; e += 1024) {
-    f32x4_t nn = load4(k + e) * add;
-    if (!fresh) nn += load4(n + e) * decay;
-    *reinterpret_cast<f32x4_t*>(n + e) = nn;
-  }
-  __syncthreads();
-  if (threadIdx.x == 0) a.m[gi] = m1;
-}
-
-void launch_scan_step(const ScanArgs& a, const int* pos, const int* live, bool f32, int B, hipStream_t st) {
-  const dim3 grid(a.V / 16, a.H, B);
-  const bool stab = a.log_in != nullptr;
-  if (f32) {
-    if (stab) {
-      hipLaunchKernelGGL((scan_step_kernel<float, true>), grid, dim3(256), 0, st, a, pos, live);
-      hipLaunchKernelGGL(scan_step_norm_kernel<float>, dim3(a.H, B), dim3(256), 0, st, a, pos, live);
-    } else hipLaunchKernelGGL((scan_step_kernel<float, false>), grid, dim3(256), 0, st, a, pos, live);
-  } else {
-    if (stab) {
-      hipLaunchKernelGGL((scan_step_kernel<bf16_t, true>), grid, dim3(256), 0, st, a, pos, live);
-      hipLaunchKernelGGL(scan_step_norm_kernel<bf16_t>, dim3(a.H, B), dim3(256), 0, st, a, pos, live);
-    } else hipLaunchKernelGGL((scan_step_kernel<bf16_t, false>), grid, dim3(256), 0, st, a, pos, live);
   }
 }
 

@@ -4,39 +4,9 @@
 // One block per row.  A row of a projection (`SrcRows`) may still be split-K slabs, which are summed on
 // load.  Row widths are padded to multiples of 64 by zeros (weights are padded when they are packed), so
 // all accesses are aligned vectors; norms divide by the true width.
-#include "elem.h"
-#include "../layered_kernels.h"
+#include "src_rows.h"
 
 namespace evgpt {
-
-// eight consecutive values of a projection row
-__device__ __forceinline__ void src8(const SrcRows& s, long long row, int col, float (&o)[8]) {
-  if (!s.f32) {
-    load8(static_cast<const bf16_t*>(s.p) + row * s.ld + col, o);
-    return;
-  }
-  const float* p = static_cast<const float*>(s.p) + row * s.ld + col;
-  load8(p, o);
-  for (int k = 1; k < s.nslab; ++k) {
-    float t[8];
-    load8(p + k * s.slab, t);
-#pragma unroll
-    for (int i = 0; i < 8; ++i) o[i] += t[i];
-  }
-}
-__device__ __forceinline__ float src1(const SrcRows& s, long long row, int col) {
-  if (!s.f32) return bf16_to_f32(static_cast<const bf16_t*>(s.p)[row * s.ld + col]);
-  const float* p = static_cast<const float*>(s.p) + row * s.ld + col;
-  float v = p[0];
-  for (int k = 1; k < s.nslab; ++k) v += p[k * s.slab];
-  return v;
-}
-__device__ __forceinline__ float sumsq8(const float (&v)[8]) {
-  float s = 0.f;
-#pragma unroll
-  for (int i = 0; i < 8; ++i) s += v[i] * v[i];
-  return s;
-}
 
 template <typename T>
 __global__ __launch_bounds__(256) void embed_rows_kernel(const int* __restrict__ tok, const T* __restrict__ embed,
@@ -193,8 +163,8 @@ void launch_glu_rows(const SrcRows& src, void* h, bool f32, int rows, int ip, in
 // Group norm with a gate.  The row is staged in LDS (gated first when the gate comes before the norm), every
 // part's root mean square is taken over its run of true channels -- a wave per part -- and the row is written
 // with the part of each channel looked up.
-template <typename T, bool BEFORE>
-__global__ __launch_bounds__(256) void group_norm_kernel(const T* __restrict__ y, SrcRows gate, int gcol,
+template <typename T, int GATE>
+__global__ __launch_bounds__(256) void group_norm_kernel(SrcRows y, SrcRows gate, int gcol,
                                                          const float* __restrict__ w, T* __restrict__ out, int heads,
                                                          int v, int vp, int parts, int ld_out, float eps) {
   extern __shared__ __attribute__((aligned(16))) float row_lds[];   // [heads * vp] values, then [parts]
@@ -203,8 +173,8 @@ __global__ __launch_bounds__(256) void group_norm_kernel(const T* __restrict__ y
   const long long row = blockIdx.x;
   for (int c = threadIdx.x * 8; c < slots; c += 2048) {
     float a[8];
-    load8(y + row * slots + c, a);
-    if constexpr (BEFORE) {
+    src8(y, row, c, a);
+    if constexpr (GATE == GATE_SILU_BEFORE) {
       float g[8];
       src8(gate, row, gcol + c, g);
 #pragma unroll
@@ -264,7 +234,7 @@ __global__ __launch_bounds__(256) void group_norm_kernel(const T* __restrict__ y
         const int part = c0 + i < next ? part0 : min((c0 + i) / plen, parts - 1);
         a[i] *= inv[part] * g[i];
       }
-      if constexpr (!BEFORE) {
+      if constexpr (GATE == GATE_SIGMOID_AFTER) {
         float t[8];
         src8(gate, row, gcol + c, t);
 #pragma unroll
@@ -274,43 +244,28 @@ __global__ __launch_bounds__(256) void group_norm_kernel(const T* __restrict__ y
     store8(out + row * ld_out + c, a);
   }
 }
-void launch_group_norm_rows(const void* y, const SrcRows& gate, int gcol, bool gate_before, const float* w, void* out,
-                            bool f32, int rows, int heads, int v, int vp, int parts, int ld_out, float eps,
-                            hipStream_t st) {
-  const size_t lds = (static_cast<size_t>(heads) * vp + parts) * 4;
-  auto go = [&](auto* kern, auto* t) {
-    typedef std::remove_pointer_t<decltype(t)> T;
-    hipLaunchKernelGGL(kern, dim3(rows), dim3(256), lds, st, static_cast<const T*>(y), gate, gcol, w,
-                       static_cast<T*>(out), heads, v, vp, parts, ld_out, eps);
-  };
-  if (f32) {
-    if (gate_before) go(group_norm_kernel<float, true>, static_cast<float*>(nullptr));
-    else go(group_norm_kernel<float, false>, static_cast<float*>(nullptr));
-  } else {
-    if (gate_before) go(group_norm_kernel<bf16_t, true>, static_cast<bf16_t*>(nullptr));
-    else go(group_norm_kernel<bf16_t, false>, static_cast<bf16_t*>(nullptr));
-  }
-}
-
 template <typename T>
-__global__ __launch_bounds__(256) void convert_rows_kernel(SrcRows src, int col0, T* __restrict__ out, long long total,
-                                                           int cols, int ld_out) {
-  const int per = cols >> 3;
-  for (long long i = blockIdx.x * 256ll + threadIdx.x; i < total; i += gridDim.x * 256ll) {
-    const long long row = i / per;
-    const int c = static_cast<int>(i % per) * 8;
-    float a[8];
-    src8(src, row, col0 + c, a);
-    store8(out + row * ld_out + c, a);
-  }
+static void launch_group_norm(const SrcRows& y, const SrcRows& gate, int gcol, int mode, const float* w, void* out, int rows,
+                              int heads, int v, int vp, int parts, int ld_out, float eps, hipStream_t st) {
+  const size_t lds = (static_cast<size_t>(heads) * vp + parts) * 4;
+  const dim3 grid(rows), block(256);
+  T* o = static_cast<T*>(out);
+  if (lds > 64 * 1024)
+    hipFuncSetAttribute(mode == GATE_SILU_BEFORE ? reinterpret_cast<const void*>(&group_norm_kernel<T, GATE_SILU_BEFORE>)
+                        : mode == GATE_SIGMOID_AFTER ? reinterpret_cast<const void*>(&group_norm_kernel<T, GATE_SIGMOID_AFTER>)
+                                                     : reinterpret_cast<const void*>(&group_norm_kernel<T, GATE_NONE>),
+                        hipFuncAttributeMaxDynamicSharedMemorySize, static_cast<int>(lds));
+  if (mode == GATE_SILU_BEFORE)
+    hipLaunchKernelGGL((group_norm_kernel<T, GATE_SILU_BEFORE>), grid, block, lds, st, y, gate, gcol, w, o, heads, v, vp, parts, ld_out, eps);
+  else if (mode == GATE_SIGMOID_AFTER)
+    hipLaunchKernelGGL((group_norm_kernel<T, GATE_SIGMOID_AFTER>), grid, block, lds, st, y, gate, gcol, w, o, heads, v, vp, parts, ld_out, eps);
+  else
+    hipLaunchKernelGGL((group_norm_kernel<T, GATE_NONE>), grid, block, lds, st, y, gate, gcol, w, o, heads, v, vp, parts, ld_out, eps);
 }
-void launch_convert_rows(const SrcRows& src, int col0, void* out, bool f32, int rows, int cols, int ld_out,
-                         hipStream_t st) {
-  const long long total = static_cast<long long>(rows) * (cols / 8);
-  const long long want = (total + 255) / 256;
-  const dim3 grid(static_cast<unsigned>(want < 4096 ? want : 4096));
-  if (f32) hipLaunchKernelGGL(convert_rows_kernel<float>, grid, dim3(256), 0, st, src, col0, static_cast<float*>(out), total, cols, ld_out);
-  else hipLaunchKernelGGL(convert_rows_kernel<bf16_t>, grid, dim3(256), 0, st, src, col0, static_cast<bf16_t*>(out), total, cols, ld_out);
+void launch_group_norm_rows(const SrcRows& y, const SrcRows& gate, int gcol, int mode, const float* w, void* out, bool f32,
+                            int rows, int heads, int v, int vp, int parts, int ld_out, float eps, hipStream_t st) {
+  if (f32) launch_group_norm<float>(y, gate, gcol, mode, w, out, rows, heads, v, vp, parts, ld_out, eps, st);
+  else launch_group_norm<bf16_t>(y, gate, gcol, mode, w, out, rows, heads, v, vp, parts, ld_out, eps, st);
 }
 
 // First index of the row's maximum (NaN never wins).
@@ -562,14 +517,6 @@ void launch_ssd_gates(const SrcRows& src, int col, const float* dt_bias, const f
   const int total = rows * H;
   hipLaunchKernelGGL(ssd_gates_kernel, dim3((total + 255) / 256), dim3(256), 0, st, src, col, dt_bias, a_log, log_decay,
                      dt, total, H);
-}
-
-__global__ void mod_pos_kernel(const int* pos, int* out, int B, int cap) {
-  const int i = blockIdx.x * 256 + threadIdx.x;
-  if (i < B) out[i] = pos[i] % cap;
-}
-void launch_mod_pos(const int* pos, int* out, int B, int cap, hipStream_t st) {
-  hipLaunchKernelGGL(mod_pos_kernel, dim3((B + 255) / 256), dim3(256), 0, st, pos, out, B, cap);
 }
 
 }  // namespace evgpt

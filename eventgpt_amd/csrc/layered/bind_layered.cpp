@@ -177,26 +177,25 @@ Tensor glu_rows(const Tensor& src, int64_t act, bool f32) {
   evgpt::launch_glu_rows(s, h.data_ptr(), f32, (int)M, (int)(N / 2), (int)act, cur_stream());
   return h;
 }
-Tensor group_norm_rows(const Tensor& y, const Tensor& gate, int64_t gcol, bool before, const Tensor& w, int64_t heads,
-                       int64_t v, int64_t vp, int64_t parts, int64_t ld_out, double eps) {
-  check_t(y, "y"); check_f(w, "w");
-  int64_t M, N;
-  const SrcRows s = src_of(gate, "gate", &M, &N);
-  TORCH_CHECK(y.numel() == M * heads * vp && w.numel() == heads * vp && vp % 8 == 0 && v >= 1 && v <= vp, "group_norm_rows: y [M, heads, vp]");
-  TORCH_CHECK(gcol >= 0 && gcol % 8 == 0 && gcol + heads * vp <= N, "group_norm_rows: gate columns");
+// y: [M, heads * vp] rows of either type; gate_mode 0 none, 1 silu before the norm, 2 sigmoid after it
+Tensor group_norm_rows(const Tensor& y, const OptTensor& gate, int64_t gcol, int64_t gate_mode, const Tensor& w, int64_t heads,
+                       int64_t v, int64_t vp, int64_t parts, int64_t ld_out, double eps, bool f32) {
+  check_f(w, "w");
+  int64_t M, N, gm, gn;
+  const SrcRows ys = src_of(y, "y", &M, &N);
+  TORCH_CHECK(N == heads * vp && w.numel() == heads * vp && vp % 8 == 0 && v >= 1 && v <= vp, "group_norm_rows: y [M, heads * vp]");
+  SrcRows gs{};
+  TORCH_CHECK(gate_mode >= 0 && gate_mode <= 2 && (gate_mode == 0 || gate.has_value()), "group_norm_rows: gate");
+  if (gate_mode) {
+    gs = src_of(*gate, "gate", &gm, &gn);
+    TORCH_CHECK(gm == M && gcol >= 0 && gcol % 8 == 0 && gcol + heads * vp <= gn, "group_norm_rows: gate columns");
+  }
   TORCH_CHECK(parts >= 1 && heads * v % parts == 0 && ld_out % 8 == 0 && ld_out >= heads * vp, "group_norm_rows: parts, ld_out");
   TORCH_CHECK((heads * vp + parts) * 4 <= 150 * 1024, "group_norm_rows: row too wide for LDS");
-  Tensor o = at::empty({M, ld_out}, y.options());
-  evgpt::launch_group_norm_rows(y.data_ptr(), s, (int)gcol, before, w.data_ptr<float>(), o.data_ptr(), is_f32(y), (int)M,
-                                (int)heads, (int)v, (int)vp, (int)parts, (int)ld_out, (float)eps, cur_stream());
-  return o;
-}
-Tensor convert_rows(const Tensor& src, int64_t col0, int64_t cols, bool f32) {
-  int64_t M, N;
-  const SrcRows s = src_of(src, "src", &M, &N);
-  TORCH_CHECK(col0 >= 0 && col0 % 8 == 0 && cols > 0 && cols % 8 == 0 && col0 + cols <= N, "convert_rows: columns");
-  Tensor o = at::empty({M, cols}, src.options().dtype(t_of(f32)));
-  evgpt::launch_convert_rows(s, (int)col0, o.data_ptr(), f32, (int)M, (int)cols, (int)cols, cur_stream());
+  Tensor o = at::empty({M, ld_out}, w.options().dtype(t_of(f32)));
+  if (M > 0)
+    evgpt::launch_group_norm_rows(ys, gs, (int)gcol, (int)gate_mode, w.data_ptr<float>(), o.data_ptr(), f32, (int)M, (int)heads,
+                                  (int)v, (int)vp, (int)parts, (int)ld_out, (float)eps, cur_stream());
   return o;
 }
 void argmax_logits_(const Tensor& logits, const Tensor& out, int64_t vocab) {
@@ -232,27 +231,45 @@ void sample_top_p(const Tensor& logits, const Tensor& out, double temperature, d
 }
 
 // ---------------------------------------------------------------- attention
+// the heads of an attention layer: columns of its sections in a projection, norms, rotation tables, chunk cache
+evgpt::AttnPrepArgs prep_args(const SrcRows& src, int64_t M, int64_t N, int64_t q_col, int64_t k_col, int64_t v_col,
+                              const OptTensor& qw, const OptTensor& kw, int64_t Hq, int64_t Hkv, int64_t D, int64_t nq, int64_t nk,
+                              double eps, const Tensor& cos, const Tensor& sin, const Tensor& row_pos, const Tensor& k_cache,
+                              const Tensor& v_cache) {
+  evgpt::AttnPrepArgs a{};
+  a.src = src;
+  check_t(k_cache, "k_cache"); check_t(v_cache, "v_cache");
+  TORCH_CHECK(Hq >= 1 && Hkv >= 1 && Hq % Hkv == 0 && D % 64 == 0 && D >= 64, "attention: heads");
+  TORCH_CHECK(q_col % 8 == 0 && k_col % 8 == 0 && v_col % 8 == 0 && q_col >= 0 && k_col >= 0 && v_col >= 0 &&
+              q_col + Hq * D <= N && k_col + Hkv * D <= N && v_col + Hkv * D <= N, "attention: sections");
+  TORCH_CHECK(k_cache.dim() == 4 && k_cache.sizes() == v_cache.sizes() && k_cache.size(1) == Hkv && k_cache.size(3) == D &&
+              k_cache.size(2) >= 1 && v_cache.scalar_type() == k_cache.scalar_type(), "attention: caches [slots, Hkv, cap, D]");
+  check_f(cos, "cos"); check_f(sin, "sin");
+  TORCH_CHECK(cos.dim() == 2 && cos.sizes() == sin.sizes() && cos.size(0) >= 1 && cos.size(1) * 2 <= D, "attention: rotation tables");
+  check_i(row_pos, "row_pos");
+  TORCH_CHECK(row_pos.numel() >= M, "attention: row_pos");
+  if (qw.has_value()) { check_f(*qw, "qw"); TORCH_CHECK(qw->numel() == Hq * D && nq >= 1); }
+  if (kw.has_value()) { check_f(*kw, "kw"); TORCH_CHECK(kw->numel() == Hkv * D && nk >= 1); }
+  a.q_col = (int)q_col; a.k_col = (int)k_col; a.v_col = (int)v_col;
+  a.qw = fptr(qw); a.kw = fptr(kw);
+  a.Hq = (int)Hq; a.Hkv = (int)Hkv; a.D = (int)D; a.nq = (int)nq; a.nk = (int)nk; a.eps = (float)eps;
+  a.cos_tab = cos.data_ptr<float>(); a.sin_tab = sin.data_ptr<float>();
+  a.rot = (int)cos.size(1) * 2; a.max_pos = (int)cos.size(0);
+  a.row_pos = row_pos.data_ptr<int>();
+  a.k_cache = k_cache.data_ptr(); a.v_cache = v_cache.data_ptr(); a.cap = (int)k_cache.size(2);
+  return a;
+}
+
 // returns q [M, Hq, D]; k_buf / v_buf and / or the chunk cache are written in place
 Tensor attn_prep_(const Tensor& src, int64_t q_col, int64_t k_col, int64_t v_col, const OptTensor& qw, const OptTensor& kw,
                   int64_t Hq, int64_t Hkv, int64_t D, int64_t nq, int64_t nk, double eps, const Tensor& cos, const Tensor& sin,
                   const OptTensor& row_slot, const Tensor& row_pos, const OptTensor& row_kv, const OptTensor& row_keep,
                   const OptTensor& k_buf, const OptTensor& v_buf, const Tensor& k_cache, const Tensor& v_cache) {
   int64_t M, N;
-  evgpt::AttnPrepArgs a{};
-  a.src = src_of(src, "src", &M, &N);
-  check_t(k_cache, "k_cache"); check_t(v_cache, "v_cache");
+  const SrcRows rows = src_of(src, "src", &M, &N);
+  evgpt::AttnPrepArgs a = prep_args(rows, M, N, q_col, k_col, v_col, qw, kw, Hq, Hkv, D, nq, nk, eps, cos, sin, row_pos,
+                                    k_cache, v_cache);
   const bool f32 = is_f32(k_cache);
-  TORCH_CHECK(Hq >= 1 && Hkv >= 1 && Hq % Hkv == 0 && D % 64 == 0 && D >= 64, "attn_prep: heads");
-  TORCH_CHECK(q_col % 8 == 0 && k_col % 8 == 0 && v_col % 8 == 0 && q_col >= 0 && k_col >= 0 && v_col >= 0 &&
-              q_col + Hq * D <= N && k_col + Hkv * D <= N && v_col + Hkv * D <= N, "attn_prep: sections");
-  TORCH_CHECK(k_cache.dim() == 4 && k_cache.sizes() == v_cache.sizes() && k_cache.size(1) == Hkv && k_cache.size(3) == D &&
-              k_cache.size(2) >= 1 && is_f32(v_cache) == f32, "attn_prep: caches [slots, Hkv, cap, D]");
-  check_f(cos, "cos"); check_f(sin, "sin");
-  TORCH_CHECK(cos.dim() == 2 && cos.sizes() == sin.sizes() && cos.size(0) >= 1 && cos.size(1) * 2 <= D, "attn_prep: rotation tables");
-  check_i(row_pos, "row_pos");
-  TORCH_CHECK(row_pos.numel() >= M, "attn_prep: row_pos");
-  if (qw.has_value()) { check_f(*qw, "qw"); TORCH_CHECK(qw->numel() == Hq * D && nq >= 1); }
-  if (kw.has_value()) { check_f(*kw, "kw"); TORCH_CHECK(kw->numel() == Hkv * D && nk >= 1); }
   if (row_slot.has_value()) { check_i(*row_slot, "row_slot"); TORCH_CHECK(row_slot->numel() == M); }
   else TORCH_CHECK(M <= k_cache.size(0), "attn_prep: more rows than cache slots");
   if (row_keep.has_value()) { check_i(*row_keep, "row_keep"); TORCH_CHECK(row_keep->numel() == M); }
@@ -266,13 +283,8 @@ Tensor attn_prep_(const Tensor& src, int64_t q_col, int64_t k_col, int64_t v_col
     a.v_buf = v_buf->data_ptr();
   }
   Tensor q = at::empty({M, Hq, D}, k_cache.options());
-  a.q_col = (int)q_col; a.k_col = (int)k_col; a.v_col = (int)v_col;
-  a.qw = fptr(qw); a.kw = fptr(kw);
-  a.Hq = (int)Hq; a.Hkv = (int)Hkv; a.D = (int)D; a.nq = (int)nq; a.nk = (int)nk; a.eps = (float)eps;
-  a.cos_tab = cos.data_ptr<float>(); a.sin_tab = sin.data_ptr<float>();
-  a.rot = (int)cos.size(1) * 2; a.max_pos = (int)cos.size(0);
-  a.row_slot = iptr(row_slot); a.row_pos = row_pos.data_ptr<int>(); a.row_kv = iptr(row_kv); a.row_keep = iptr(row_keep);
-  a.q_out = q.data_ptr(); a.k_cache = k_cache.data_ptr(); a.v_cache = v_cache.data_ptr(); a.cap = (int)k_cache.size(2);
+  a.row_slot = iptr(row_slot); a.row_kv = iptr(row_kv); a.row_keep = iptr(row_keep);
+  a.q_out = q.data_ptr();
   if (M > 0) evgpt::launch_attn_prep(a, f32, (int)M, cur_stream());
   return q;
 }
@@ -326,13 +338,11 @@ Tensor attn_chunk_decode(const Tensor& q, const Tensor& k_cache, const Tensor& v
   Tensor o = at::empty_like(q);
   if (!is_f32(q) && (D == 64 || D == 128)) {
     nsplit = std::min<int64_t>(std::max<int64_t>(nsplit, 1), 16);
-    Tensor at_pos = at::empty({B}, pos.options());
-    evgpt::launch_mod_pos(pos.data_ptr<int>(), at_pos.data_ptr<int>(), (int)B, (int)cap, cur_stream());
     auto f = q.options().dtype(at::kFloat);
     Tensor po = at::empty({nsplit > 1 ? B * Hq * nsplit * D : 1}, f), pm = at::empty({nsplit > 1 ? B * Hq * nsplit * 2 : 1}, f);
     evgpt::launch_attn_decode(bptr(q), bptr(k_cache), bptr(v_cache), bptr_mut(o), po.data_ptr<float>(), pm.data_ptr<float>(),
-                              at_pos.data_ptr<int>(), (int)B, (int)Hq, (int)Hkv, (int)D, (int)cap, (int)nsplit, (float)scale,
-                              cur_stream());
+                              pos.data_ptr<int>(), (int)B, (int)Hq, (int)Hkv, (int)D, (int)cap, (int)nsplit, (float)scale,
+                              cur_stream(), 1);
     return o;
   }
   evgpt::launch_attn_chunk_decode(q.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(), o.data_ptr(), pos.data_ptr<int>(),
@@ -360,7 +370,7 @@ evgpt::ScanArgs scan_args(const Tensor& q, const Tensor& k, const Tensor& v, int
     check_f(*log_in, "log_in");
     TORCH_CHECK(log_in->numel() == M * H && n.has_value() && m.has_value(), "scan: log_in [M, H], normaliser, maximum");
     check_f(*n, "n"); check_f(*m, "m");
-    TORCH_CHECK(n->numel() == S.size(0) * H * N && m->numel() == S.size(0) * H, "scan: normaliser sizes");
+    TORCH_CHECK(n->numel() == 2 * S.size(0) * H * N && m->numel() == 2 * S.size(0) * H, "scan: normaliser, maximum [2, slots, ..]");
   } else {
     check_f(*scale_in, "scale_in");
     TORCH_CHECK(scale_in->numel() == M * H, "scan: scale_in [M, H]");
@@ -375,6 +385,7 @@ evgpt::ScanArgs scan_args(const Tensor& q, const Tensor& k, const Tensor& v, int
   a.log_decay = log_decay.data_ptr<float>(); a.log_in = fptr(log_in); a.scale_in = fptr(scale_in); a.skip = fptr(skip);
   a.S = S.data_ptr<float>();
   a.n = const_cast<float*>(fptr(n)); a.m = const_cast<float*>(fptr(m));
+  a.slots = (int)S.size(0);
   return a;
 }
 Tensor scan_prefill_(const Tensor& q, const Tensor& k, const Tensor& v, int64_t H, int64_t per_group, int64_t N, int64_t V,
@@ -396,20 +407,188 @@ Tensor scan_prefill_(const Tensor& q, const Tensor& k, const Tensor& v, int64_t 
   evgpt::launch_scan_prefill(a, c, is_f32(q), cur_stream());
   return o;
 }
-Tensor scan_step_(const Tensor& q, const Tensor& k, const Tensor& v, int64_t H, int64_t per_group, int64_t N, int64_t V,
-                  double qscale, const Tensor& log_decay, const OptTensor& log_in, const OptTensor& scale_in, const OptTensor& skip,
-                  const Tensor& S, const OptTensor& n, const OptTensor& m, const Tensor& pos,
-                  const OptTensor& live) {
-  evgpt::ScanArgs a = scan_args(q, k, v, H, per_group, N, V, qscale, log_decay, log_in, scale_in, skip, S, n, m);
-  check_i(pos, "pos");
-  const int64_t B = q.size(0);
-  TORCH_CHECK(pos.numel() >= B && S.size(0) >= B && B < 65536, "scan_step: one row per slot");
+// ---------------------------------------------------------------- decode steps
+// One token per sequence from the projection rows `src`: the attention heads (norm, rotation, cache append; q is
+// returned) and the matrix memory (its output is returned, fp32).  Rows whose `live` is 0 change no state.
+std::tuple<Tensor, Tensor> parallel_step_(const Tensor& src, at::IntArrayRef attn, const OptTensor& qw, const OptTensor& kw,
+                                          double eps, const Tensor& cos, const Tensor& sin, const Tensor& k_cache, const Tensor& v_cache,
+                                          at::IntArrayRef mem, const Tensor& ib, const Tensor& fb, double cap, double qscale,
+                                          const Tensor& S, const Tensor& n, const Tensor& m, const Tensor& pos, const OptTensor& live) {
+  int64_t B, N;
+  const SrcRows rows = src_of(src, "src", &B, &N);
+  TORCH_CHECK(attn.size() == 8 && mem.size() == 8, "parallel_step: attn {q, k, v columns, Hq, Hkv, D, true q, true k widths}, "
+              "mem {q, k, v, i, f columns, H, N, V}");
+  evgpt::StepHeads sh{};
+  sh.a = prep_args(rows, B, N, attn[0], attn[1], attn[2], qw, kw, attn[3], attn[4], attn[5], attn[6], attn[7], eps, cos, sin, pos,
+                   k_cache, v_cache);
+  sh.on = 1;
+  const bool f32 = is_f32(k_cache);
+  const int64_t H = mem[5], Nq = mem[6], V = mem[7];
+  check_f(ib, "ib"); check_f(fb, "fb"); check_f(S, "S"); check_f(n, "n"); check_f(m, "m");
+  TORCH_CHECK(H >= 1 && Nq >= 32 && Nq % 32 == 0 && Nq <= 4096 && (V == 32 || (V >= 64 && V % 64 == 0)) && cap > 0, "parallel_step: memory sizes");
+  for (int i = 0; i < 3; ++i)
+    TORCH_CHECK(mem[i] >= 0 && mem[i] + H * (i == 2 ? V : Nq) <= N, "parallel_step: memory sections");
+  TORCH_CHECK(mem[3] >= 0 && mem[4] >= 0 && mem[3] + H <= N && mem[4] + H <= N && ib.numel() == H && fb.numel() == H, "parallel_step: gates");
+  TORCH_CHECK(S.dim() == 4 && S.size(0) >= B && S.size(1) == H && S.size(2) == V && S.size(3) == Nq &&
+              n.numel() == 2 * S.size(0) * H * Nq && m.numel() == 2 * S.size(0) * H && k_cache.size(0) >= B, "parallel_step: states");
   if (live.has_value()) { check_i(*live, "live"); TORCH_CHECK(live->numel() >= B, "live"); }
-  Tensor o = at::empty({B, H * V}, q.options());
-  a.out = o.data_ptr();
-  if (B > 0) evgpt::launch_scan_step(a, pos.data_ptr<int>(), iptr(live), is_f32(q), (int)B, cur_stream());
+  TORCH_CHECK(B < 65536, "parallel_step: rows");
+  Tensor q = at::empty({B, attn[3], attn[5]}, k_cache.options()), o = at::empty({B, H * V}, S.options());
+  sh.a.q_out = q.data_ptr();
+  evgpt::StepMemory sm{rows, (int)mem[0], (int)mem[1], (int)mem[2], (int)mem[3], (int)mem[4], ib.data_ptr<float>(), fb.data_ptr<float>(),
+                       (float)cap, (float)qscale, (int)H, (int)Nq, (int)V, S.data_ptr<float>(), n.data_ptr<float>(),
+                       m.data_ptr<float>(), (int)S.size(0), o.data_ptr<float>()};
+  if (B > 0) evgpt::launch_parallel_step(sh, sm, pos.data_ptr<int>(), iptr(live), f32, (int)B, cur_stream());
+  return {q, o};
+}
+// the state-space recurrence with its convolution and silu(z) gate: [B, H * V] fp32
+Tensor ssd_step_(const Tensor& src, at::IntArrayRef dims, const Tensor& conv_w, const Tensor& conv_b, const Tensor& ring,
+                 const Tensor& dt_bias, const Tensor& a_log, const Tensor& skip, const Tensor& S, const Tensor& pos, const OptTensor& live) {
+  int64_t B, N;
+  const SrcRows rows = src_of(src, "src", &B, &N);
+  TORCH_CHECK(dims.size() == 7, "ssd_step: {z, x, dt columns, H, G, N, V}");
+  const int64_t H = dims[3], G = dims[4], Ns = dims[5], V = dims[6], C = H * V + 2 * G * Ns;
+  check_f(conv_w, "conv_w"); check_f(conv_b, "conv_b"); check_t(ring, "ring"); check_f(dt_bias, "dt_bias"); check_f(a_log, "a_log");
+  check_f(skip, "skip"); check_f(S, "S"); check_i(pos, "pos");
+  TORCH_CHECK(H >= 1 && G >= 1 && H % G == 0 && Ns >= 32 && Ns % 32 == 0 && Ns <= 4096 && (V == 32 || (V >= 64 && V % 64 == 0)), "ssd_step: sizes");
+  TORCH_CHECK(dims[0] >= 0 && dims[1] >= 0 && dims[2] >= 0 && dims[0] + H * V <= N && dims[1] + C <= N && dims[2] + H <= N, "ssd_step: sections");
+  TORCH_CHECK(conv_w.dim() == 2 && conv_w.size(0) == C && conv_b.numel() == C && ring.dim() == 3 && ring.size(0) >= B &&
+              ring.size(1) == conv_w.size(1) && ring.size(2) == C, "ssd_step: convolution");
+  TORCH_CHECK(dt_bias.numel() == H && a_log.numel() == H && skip.numel() == H, "ssd_step: per-head constants");
+  TORCH_CHECK(S.dim() == 4 && S.size(0) >= B && S.size(1) == H && S.size(2) == V && S.size(3) == Ns && pos.numel() >= B && B < 65536, "ssd_step: state");
+  if (live.has_value()) { check_i(*live, "live"); TORCH_CHECK(live->numel() >= B, "live"); }
+  Tensor o = at::empty({B, H * V}, S.options());
+  evgpt::StepSsd a{rows, (int)dims[0], (int)dims[1], (int)dims[2], conv_w.data_ptr<float>(), conv_b.data_ptr<float>(), ring.data_ptr(),
+                   (int)conv_w.size(1), dt_bias.data_ptr<float>(), a_log.data_ptr<float>(), skip.data_ptr<float>(), (int)H, (int)G,
+                   (int)Ns, (int)V, S.data_ptr<float>(), o.data_ptr<float>()};
+  if (B > 0) evgpt::launch_ssd_step(a, pos.data_ptr<int>(), iptr(live), is_f32(ring), (int)B, cur_stream());
   return o;
 }
+
+// ---------------------------------------------------------------- up to four rows, weights streamed
+constexpr int64_t GEMV_LDS = 64 * 1024;
+void check_gemv_w(const Tensor& w, int64_t B, int64_t K, const char* name) {
+  check_t(w, name);
+  TORCH_CHECK(w.dim() == 2 && w.size(1) == K && K % 64 == 0 && K > 0 && w.size(0) % 8 == 0, name, ": [N, K], K % 64 == 0, N % 8 == 0");
+  TORCH_CHECK(B >= 1 && B <= evgpt::GEMV_ROWS_MAX, "row_gemv: one to four rows");
+}
+evgpt::GemvInput stream_input(const Tensor& x, const Tensor& w, int64_t n, double eps, const OptTensor& a, const OptTensor& b,
+                              const OptTensor& wa, const OptTensor& wb, const OptTensor& x_out) {
+  check_stream(x, n); check_f(w, "norm");
+  const int64_t K = x.size(1);
+  TORCH_CHECK(w.numel() == K, "row_gemv: norm weight size");
+  evgpt::GemvInput in{};
+  in.kind = evgpt::GV_NORM;
+  in.x = x.data_ptr(); in.w = w.data_ptr<float>(); in.n = (int)n; in.eps = (float)eps;
+  if (a.has_value()) {
+    TORCH_CHECK(b.has_value() && wa.has_value() && wb.has_value() && x_out.has_value(), "row_gemv: branches");
+    check_f(*a, "a"); check_f(*b, "b"); check_f(*wa, "wa"); check_f(*wb, "wb"); check_f(*x_out, "x_out");
+    TORCH_CHECK(a->numel() == x.numel() && b->numel() == x.numel() && wa->numel() == K && wb->numel() == K &&
+                x_out->numel() == x.numel() && x_out->data_ptr() != x.data_ptr(), "row_gemv: branch sizes");
+    in.kind = evgpt::GV_MERGE;
+    in.a = a->data_ptr<float>(); in.b = b->data_ptr<float>(); in.wa = wa->data_ptr<float>(); in.wb = wb->data_ptr<float>();
+    in.x_out = x_out->data_ptr<float>();
+  }
+  return in;
+}
+void run_gemv(const evgpt::GemvCall& c, bool f32, int64_t B) {
+  TORCH_CHECK((int64_t)evgpt::row_gemv_lds(c, f32, (int)B) <= GEMV_LDS, "row_gemv: input rows do not fit LDS");
+  evgpt::launch_row_gemv(c, f32, (int)B, cur_stream());
+}
+// W · norm(x): fp32 [B, N], or with act >= 0 act(gate) * up of [gate | up] rows in the storage type.  With branches a, b: x +
+// (rms(a) wa + rms(b) wb) / 2 takes x's place and is stored to x_out.
+Tensor gemv_norm(const Tensor& x, const Tensor& norm, int64_t n, double eps, const Tensor& w, int64_t act, const OptTensor& a,
+                 const OptTensor& b, const OptTensor& wa, const OptTensor& wb, const OptTensor& x_out) {
+  evgpt::GemvCall c{};
+  c.count = 1;
+  c.p[0].in = stream_input(x, norm, n, eps, a, b, wa, wb, x_out);
+  const int64_t B = x.size(0), N = w.size(0);
+  check_gemv_w(w, B, x.size(1), "w");
+  c.p[0].W = w.data_ptr(); c.p[0].N = (int)N; c.p[0].K = (int)x.size(1);
+  Tensor y;
+  if (act >= 0) {
+    TORCH_CHECK(act == evgpt::GLU_GELU_TANH || act == evgpt::GLU_SILU, "gemv_norm: act 0 or 1");
+    y = at::empty({B, N / 2}, w.options());
+    c.epilogue = evgpt::GV_GLU; c.h = y.data_ptr(); c.act = (int)act;
+  } else {
+    y = at::empty({B, N}, x.options());
+    c.epilogue = evgpt::GV_STORE; c.p[0].y = y.data_ptr<float>(); c.p[0].ldy = (int)N;
+  }
+  run_gemv(c, is_f32(w), B);
+  return y;
+}
+// x += W · h for rows h of the storage type
+void gemv_add_(const Tensor& x, const Tensor& w, const Tensor& h) {
+  check_stream(x, 1); check_t(h, "h");
+  const int64_t B = x.size(0);
+  TORCH_CHECK(h.dim() == 2 && h.size(0) == B && h.scalar_type() == w.scalar_type() && w.size(0) == x.size(1), "gemv_add: h [B, K], w [width, K]");
+  check_gemv_w(w, B, h.size(1), "w");
+  evgpt::GemvCall c{};
+  c.count = 1;
+  c.epilogue = evgpt::GV_ADD;
+  c.p[0].W = w.data_ptr(); c.p[0].N = (int)w.size(0); c.p[0].K = (int)w.size(1);
+  c.p[0].in.kind = evgpt::GV_PLAIN; c.p[0].in.x = h.data_ptr();
+  c.p[0].y = x.data_ptr<float>(); c.p[0].ldy = (int)x.size(1);
+  run_gemv(c, is_f32(w), B);
+}
+evgpt::GemvInput group_input(const Tensor& y, int64_t B, const OptTensor& gate, int64_t gcol, const Tensor& norm, int64_t heads,
+                             int64_t v, int64_t vp, int64_t parts, double eps) {
+  check_f(y, "y"); check_f(norm, "norm");
+  TORCH_CHECK(y.numel() == B * heads * vp && norm.numel() == heads * vp && vp % 8 == 0 && v >= 1 && v <= vp && parts >= 1 &&
+              heads * v % parts == 0, "row_gemv: group norm sizes");
+  evgpt::GemvInput in{};
+  in.kind = evgpt::GV_GROUP;
+  in.y = y.data_ptr<float>(); in.w = norm.data_ptr<float>(); in.eps = (float)eps;
+  in.heads = (int)heads; in.v = (int)v; in.vp = (int)vp; in.parts = (int)parts;
+  if (gate.has_value()) {
+    int64_t gm, gn;
+    in.gate = src_of(*gate, "gate", &gm, &gn);
+    TORCH_CHECK(gm == B && gcol >= 0 && gcol % 8 == 0 && gcol + heads * vp <= gn, "row_gemv: gate columns");
+    in.gcol = (int)gcol;
+    in.gate_mode = evgpt::GATE_SIGMOID_AFTER;
+  }
+  return in;
+}
+// x += W · groupnorm(y)
+void gemv_group_add_(const Tensor& x, const Tensor& w, const Tensor& y, const Tensor& norm, int64_t heads, int64_t v, int64_t vp,
+                     int64_t parts, double eps) {
+  check_stream(x, 1);
+  const int64_t B = x.size(0), K = w.size(1);
+  TORCH_CHECK(w.size(0) == x.size(1) && K >= heads * vp, "gemv_group_add: w [width, K]");
+  check_gemv_w(w, B, K, "w");
+  evgpt::GemvCall c{};
+  c.count = 1;
+  c.epilogue = evgpt::GV_ADD;
+  c.p[0].W = w.data_ptr(); c.p[0].N = (int)w.size(0); c.p[0].K = (int)K;
+  c.p[0].in = group_input(y, B, c10::nullopt, 0, norm, heads, v, vp, parts, eps);
+  c.p[0].y = x.data_ptr<float>(); c.p[0].ldy = (int)x.size(1);
+  run_gemv(c, is_f32(w), B);
+}
+// {Wa · h, Wb · (groupnorm(y) sigmoid(gate))} in one launch: the output projections of an attention branch and a gated
+// recurrent branch, fp32 [2, B, width]
+Tensor gemv_branches(const Tensor& wa, const Tensor& h, const Tensor& wb, const Tensor& y, const Tensor& gate, int64_t gcol,
+                     const Tensor& norm, int64_t heads, int64_t v, int64_t vp, double eps) {
+  check_t(h, "h");
+  TORCH_CHECK(h.dim() == 2 && h.scalar_type() == wa.scalar_type() && wa.scalar_type() == wb.scalar_type() && wa.size(0) == wb.size(0) &&
+              wb.size(1) >= heads * vp, "gemv_branches: h [B, Ka], weights [width, K]");
+  const int64_t B = h.size(0), N = wa.size(0);
+  check_gemv_w(wa, B, h.size(1), "wa"); check_gemv_w(wb, B, wb.size(1), "wb");
+  Tensor o = at::empty({2, B, N}, y.options());
+  evgpt::GemvCall c{};
+  c.count = 2;
+  c.epilogue = evgpt::GV_STORE;
+  c.p[0].W = wa.data_ptr(); c.p[0].N = (int)N; c.p[0].K = (int)wa.size(1);
+  c.p[0].in.kind = evgpt::GV_PLAIN; c.p[0].in.x = h.data_ptr();
+  c.p[0].y = o.data_ptr<float>(); c.p[0].ldy = (int)N;
+  c.p[1].W = wb.data_ptr(); c.p[1].N = (int)N; c.p[1].K = (int)wb.size(1);
+  c.p[1].in = group_input(y, B, gate, gcol, norm, heads, v, vp, heads, eps);
+  c.p[1].y = o.data_ptr<float>() + B * N; c.p[1].ldy = (int)N;
+  run_gemv(c, is_f32(wa), B);
+  return o;
+}
+int64_t gemv_rows_max() { return evgpt::GEMV_ROWS_MAX; }
+int64_t gemv_lds_bytes() { return GEMV_LDS; }
+
 std::tuple<Tensor, Tensor> mlstm_gates(const Tensor& src, int64_t i_col, int64_t f_col, const Tensor& ib, const Tensor& fb, double cap) {
   int64_t M, N;
   const SrcRows s = src_of(src, "src", &M, &N);
@@ -435,25 +614,20 @@ std::tuple<Tensor, Tensor> ssd_gates(const Tensor& src, int64_t col, const Tenso
   return {ld, dt};
 }
 Tensor conv_rows_(const Tensor& src, int64_t col0, const Tensor& w, const Tensor& bias, const Tensor& ring,
-                  const OptTensor& row_slot, const Tensor& row_pos, const OptTensor& row_first, bool update,
-                  const OptTensor& live) {
+                  const Tensor& row_slot, const Tensor& row_pos, const Tensor& row_first) {
   int64_t M, N;
   const SrcRows s = src_of(src, "src", &M, &N);
-  check_f(w, "w"); check_f(bias, "bias"); check_t(ring, "ring"); check_i(row_pos, "row_pos");
+  check_f(w, "w"); check_f(bias, "bias"); check_t(ring, "ring"); check_i(row_pos, "row_pos"); check_i(row_slot, "row_slot");
+  check_i(row_first, "row_first");
   TORCH_CHECK(w.dim() == 2 && bias.numel() == w.size(0) && ring.dim() == 3 && ring.size(1) == w.size(1) && ring.size(2) == w.size(0),
               "conv_rows: w [C, taps], ring [slots, taps, C]");
   const int64_t C = w.size(0);
-  TORCH_CHECK(col0 >= 0 && col0 + C <= N && row_pos.numel() >= M, "conv_rows: columns, rows");
-  if (row_slot.has_value()) { check_i(*row_slot, "row_slot"); TORCH_CHECK(row_slot->numel() == M); }
-  else TORCH_CHECK(M <= ring.size(0), "conv_rows: more rows than slots");
-  if (row_first.has_value()) { check_i(*row_first, "row_first"); TORCH_CHECK(row_first->numel() == M); }
-  if (live.has_value()) { check_i(*live, "live"); TORCH_CHECK(live->numel() >= M, "live"); }
-  TORCH_CHECK(!update || !row_first.has_value(), "conv_rows: the ring is updated in place by single-token rows only");
+  TORCH_CHECK(col0 >= 0 && col0 + C <= N && row_pos.numel() == M && row_slot.numel() == M && row_first.numel() == M, "conv_rows: columns, rows");
   Tensor o = at::empty({M, C}, ring.options());
   if (M > 0)
     evgpt::launch_conv_rows(s, (int)col0, w.data_ptr<float>(), bias.data_ptr<float>(), ring.data_ptr(), o.data_ptr(),
-                            is_f32(ring), iptr(row_slot), row_pos.data_ptr<int>(), iptr(row_first), (int)M, (int)C,
-                            (int)w.size(1), update, iptr(live), cur_stream());
+                            is_f32(ring), row_slot.data_ptr<int>(), row_pos.data_ptr<int>(), row_first.data_ptr<int>(), (int)M,
+                            (int)C, (int)w.size(1), cur_stream());
   return o;
 }
 void conv_tail_(const Tensor& src, int64_t col0, const Tensor& ring, const Tensor& tails) {
@@ -477,8 +651,7 @@ TORCH_LIBRARY(evlay, m) {
   m.def("add_norm_rows_(Tensor(a!) x, Tensor y, Tensor? w, int n, float eps, bool f32) -> Tensor", &add_norm_rows_);
   m.def("merge_norm_rows_(Tensor(a!) x, Tensor a, Tensor b, Tensor wa, Tensor wb, Tensor? w, int n, float eps, bool f32) -> Tensor", &merge_norm_rows_);
   m.def("glu_rows(Tensor src, int act, bool f32) -> Tensor", &glu_rows);
-  m.def("group_norm_rows(Tensor y, Tensor gate, int gcol, bool before, Tensor w, int heads, int v, int vp, int parts, int ld_out, float eps) -> Tensor", &group_norm_rows);
-  m.def("convert_rows(Tensor src, int col0, int cols, bool f32) -> Tensor", &convert_rows);
+  m.def("group_norm_rows(Tensor y, Tensor? gate, int gcol, int gate_mode, Tensor w, int heads, int v, int vp, int parts, int ld_out, float eps, bool f32) -> Tensor", &group_norm_rows);
   m.def("argmax_logits_(Tensor logits, Tensor(a!) out, int vocab) -> ()", &argmax_logits_);
   m.def("commit_rows_(Tensor sampled, Tensor embed, float scale, Tensor(a!) x, Tensor(b!) out_tokens, Tensor(c!) step, Tensor(d!) pos, Tensor(e!) done, Tensor(f!) cur_token, int eos, Tensor? active) -> ()", &commit_rows_);
   m.def("sample_top_p(Tensor logits, Tensor(a!) out, float temperature, float top_p, int seed, Tensor step, int top_k=0) -> ()", &sample_top_p);
@@ -488,9 +661,16 @@ TORCH_LIBRARY(evlay, m) {
   m.def("attn_runs_(Tensor q, Tensor k, Tensor v, Tensor(a!) o, int q0, int rows, int kv0, int off, int n, float scale) -> ()", &attn_runs_);
   m.def("attn_chunk_decode(Tensor q, Tensor k_cache, Tensor v_cache, Tensor pos, float scale, int nsplit) -> Tensor", &attn_chunk_decode);
   m.def("scan_prefill_(Tensor q, Tensor k, Tensor v, int H, int per_group, int N, int V, float qscale, Tensor log_decay, Tensor? log_in, Tensor? scale_in, Tensor? skip, Tensor(a!) S, Tensor(b!)? n, Tensor(c!)? m, Tensor chunks, Tensor seqs) -> Tensor", &scan_prefill_);
-  m.def("scan_step_(Tensor q, Tensor k, Tensor v, int H, int per_group, int N, int V, float qscale, Tensor log_decay, Tensor? log_in, Tensor? scale_in, Tensor? skip, Tensor(a!) S, Tensor(b!)? n, Tensor(c!)? m, Tensor pos, Tensor? live) -> Tensor", &scan_step_);
+  m.def("parallel_step_(Tensor src, int[] attn, Tensor? qw, Tensor? kw, float eps, Tensor cos, Tensor sin, Tensor(a!) k_cache, Tensor(b!) v_cache, int[] mem, Tensor ib, Tensor fb, float cap, float qscale, Tensor(c!) S, Tensor(d!) n, Tensor(e!) m, Tensor pos, Tensor? live) -> (Tensor, Tensor)", &parallel_step_);
+  m.def("ssd_step_(Tensor src, int[] dims, Tensor conv_w, Tensor conv_b, Tensor(a!) ring, Tensor dt_bias, Tensor a_log, Tensor skip, Tensor(b!) S, Tensor pos, Tensor? live) -> Tensor", &ssd_step_);
+  m.def("gemv_norm(Tensor x, Tensor norm, int n, float eps, Tensor w, int act, Tensor? a, Tensor? b, Tensor? wa, Tensor? wb, Tensor(a!)? x_out) -> Tensor", &gemv_norm);
+  m.def("gemv_add_(Tensor(a!) x, Tensor w, Tensor h) -> ()", &gemv_add_);
+  m.def("gemv_group_add_(Tensor(a!) x, Tensor w, Tensor y, Tensor norm, int heads, int v, int vp, int parts, float eps) -> ()", &gemv_group_add_);
+  m.def("gemv_branches(Tensor wa, Tensor h, Tensor wb, Tensor y, Tensor gate, int gcol, Tensor norm, int heads, int v, int vp, float eps) -> Tensor", &gemv_branches);
+  m.def("gemv_rows_max() -> int", &gemv_rows_max);
+  m.def("gemv_lds_bytes() -> int", &gemv_lds_bytes);
   m.def("mlstm_gates(Tensor src, int i_col, int f_col, Tensor ib, Tensor fb, float cap) -> (Tensor, Tensor)", &mlstm_gates);
   m.def("ssd_gates(Tensor src, int col, Tensor dt_bias, Tensor a_log) -> (Tensor, Tensor)", &ssd_gates);
-  m.def("conv_rows_(Tensor src, int col0, Tensor w, Tensor bias, Tensor(a!) ring, Tensor? row_slot, Tensor row_pos, Tensor? row_first, bool update, Tensor? live) -> Tensor", &conv_rows_);
+  m.def("conv_rows_(Tensor src, int col0, Tensor w, Tensor bias, Tensor ring, Tensor row_slot, Tensor row_pos, Tensor row_first) -> Tensor", &conv_rows_);
   m.def("conv_tail_(Tensor src, int col0, Tensor(a!) ring, Tensor tails) -> ()", &conv_tail_);
 }

@@ -39,12 +39,9 @@ void launch_glu_rows(const SrcRows& src, void* h, bool f32, int rows, int ip, in
 // Group norm of channels stored as heads of vp slots (v of them used): `parts` equal runs of the heads * v true
 // channels, each by its own root mean square, times w (laid out like the channels), with a gate read from `gate` at column
 // gcol + channel slot: silu(gate) multiplied in before the norm, or sigmoid(gate) after it.
-void launch_group_norm_rows(const void* y, const SrcRows& gate, int gcol, bool gate_before, const float* w, void* out,
-                            bool f32, int rows, int heads, int v, int vp, int parts, int ld_out, float eps,
-                            hipStream_t st);
-// out[row][c] = T(src[row][col0 + c]), c < cols (cols % 8 == 0)
-void launch_convert_rows(const SrcRows& src, int col0, void* out, bool f32, int rows, int cols, int ld_out,
-                         hipStream_t st);
+enum { GATE_NONE = 0, GATE_SILU_BEFORE = 1, GATE_SIGMOID_AFTER = 2 };
+void launch_group_norm_rows(const SrcRows& y, const SrcRows& gate, int gcol, int mode, const float* w, void* out, bool f32,
+                            int rows, int heads, int v, int vp, int parts, int ld_out, float eps, hipStream_t st);
 void launch_argmax_logits(const float* logits, long long ld, int* out, int rows, int vocab, hipStream_t st);
 void launch_commit_rows(const int* sampled, const void* embed, bool f32, float scale, float* x, int* out_tokens,
                         int max_out, int* step, int* pos, int* done, int* cur_token, int eos, int B, int ld, int vocab,
@@ -87,7 +84,6 @@ void launch_attn_chunk(const void* q, const void* k, const void* v, void* o, con
 // keys 0 .. pos % cap of every sequence's cache
 void launch_attn_chunk_decode(const void* q, const void* k_cache, const void* v_cache, void* o, const int* pos,
                               bool f32, int B, int Hq, int Hkv, int D, int cap, float scale, hipStream_t st);
-void launch_mod_pos(const int* pos, int* out, int B, int cap, hipStream_t st);
 
 // ---- linear_scan.hip: S_t = exp(a_t) S_(t-1) + b_t v_t k_t^T per head, y_t = S_t q_t
 struct ScanArgs {
@@ -102,12 +98,15 @@ struct ScanArgs {
   const float* skip;               // [H]: y += skip * v; or null
   void* out;                       // [rows][H][V]
   float* S;                        // [slots][H][V][N]
-  float* n;                        // [slots][H][N]
-  float* m;                        // [slots][H]
+  float* n;                        // [2][slots][H][N], indexed by the parity of the next position
+  float* m;                        // [2][slots][H]
+  int slots;
 };
 struct ScanChunks {
-  const int* chunks;               // [C][4]: first row, rows (<= 64), slot, last chunk of its sequence
-  const int* seqs;                 // [nseq][4]: first chunk, chunks, slot, starts at position 0
+  // [C][4]: first row, rows (<= 64), slot, flags (bit 0: the sequence's last chunk, bit 1: parity of the next position)
+  const int* chunks;
+  // [nseq][4]: first chunk, chunks, slot, flags (bit 0: from position 0, bits 1 and 2: parities of start and end)
+  const int* seqs;
   int C, nseq;
   float* dS;                       // [C][H][V][N]
   float* dn;                       // [C][H][N]
@@ -116,9 +115,6 @@ struct ScanChunks {
 };
 constexpr int SCAN_CHUNK = 64;
 void launch_scan_prefill(const ScanArgs& a, const ScanChunks& c, bool f32, hipStream_t st);
-// one token of every sequence: row b is slot b; pos[b] == 0 starts from the zero state; rows whose live is 0 are
-// left alone (their output too)
-void launch_scan_step(const ScanArgs& a, const int* pos, const int* live, bool f32, int B, hipStream_t st);
 // log gates of the matrix memory: cap * tanh((x + b) / cap), and the log sigmoid of it for the forget gate
 void launch_mlstm_gates(const SrcRows& src, int i_col, int f_col, const float* ib, const float* fb, float cap, float* li,
                         float* lf, int rows, int H, hipStream_t st);
@@ -126,11 +122,75 @@ void launch_mlstm_gates(const SrcRows& src, int i_col, int f_col, const float* i
 void launch_ssd_gates(const SrcRows& src, int col, const float* dt_bias, const float* a_log, float* log_decay, float* dt,
                       int rows, int H, hipStream_t st);
 
+// ---- decode_step.hip: one token per sequence (row b is slot b), straight from the projection's rows
+struct StepHeads {                 // attention half: heads of AttnPrepArgs, one block each
+  AttnPrepArgs a;
+  int on;
+};
+struct StepMemory {                // matrix memory half
+  SrcRows src;
+  int q_col, k_col, v_col, i_col, f_col;
+  const float* ib; const float* fb;
+  float cap, qscale;
+  int H, N, V;                     // padded sizes
+  float* S; float* n; float* m;    // as in ScanArgs
+  int slots;
+  float* out;                      // [B][H][V]
+};
+void launch_parallel_step(const StepHeads& h, const StepMemory& m, const int* pos, const int* live, bool f32, int B,
+                          hipStream_t st);
+struct StepSsd {
+  SrcRows src;
+  int z_col, x_col, dt_col;        // x, B and C are consecutive
+  const float* conv_w; const float* conv_b;     // [C][taps], [C]
+  void* ring;                      // [slots][taps][C], T
+  int taps;
+  const float* dt_bias; const float* a_log; const float* skip;
+  int H, G, N, V;
+  float* S;                        // [slots][H][V][N]
+  float* out;                      // [B][H][V]: y silu(z)
+};
+void launch_ssd_step(const StepSsd& a, const int* pos, const int* live, bool f32, int B, hipStream_t st);
+
+// ---- row_gemv.hip: up to four rows, weights streamed once, the input prepared and the output finished in the launch
+enum { GV_PLAIN = 0, GV_NORM = 1, GV_MERGE = 2, GV_GROUP = 3 };
+enum { GV_STORE = 0, GV_ADD = 1, GV_GLU = 2 };
+struct GemvInput {
+  int kind;
+  const void* x;                   // PLAIN: [B][K] of T; NORM, MERGE: the fp32 stream [B][K]
+  const float* a; const float* b;  // MERGE: branch outputs [B][K], x + (rms(a) wa + rms(b) wb) / 2
+  const float* wa; const float* wb;
+  float* x_out;                    // MERGE: the merged stream [B][K]
+  const float* w;                  // NORM, MERGE, GROUP: norm weights [K]
+  int n;                           // true width
+  float eps;
+  const float* y;                  // GROUP: [B][heads * vp] fp32
+  SrcRows gate;
+  int gcol, gate_mode;
+  int heads, v, vp, parts;
+};
+struct GemvProblem {
+  const void* W;                   // [N][K]
+  int N, K;
+  GemvInput in;
+  float* y; int ldy;               // STORE: [B][ldy] fp32; ADD: the stream, accumulated
+};
+struct GemvCall {
+  GemvProblem p[2];
+  int count;                       // problems in this launch (same epilogue)
+  int epilogue;
+  void* h;                         // GLU: [B][N / 2] of T (W is [gate rows | up rows])
+  int act;
+};
+constexpr int GEMV_ROWS_MAX = 4;
+size_t row_gemv_lds(const GemvCall& c, bool f32, int B);     // bytes of LDS the call needs
+void launch_row_gemv(const GemvCall& c, bool f32, int B, hipStream_t st);
+
 // ---- conv1d.hip: causal per-channel convolution + silu; the state is the last inputs in a ring of `taps`
-// slots (slot = position % taps).  update: a decode step, which also stores its input (of the rows whose live is set)
+// slots (slot = position % taps)
 void launch_conv_rows(const SrcRows& src, int col0, const float* w, const float* bias, void* ring, void* out, bool f32,
                       const int* row_slot, const int* row_pos, const int* row_first, int rows, int C, int taps,
-                      bool update, const int* live, hipStream_t st);
+                      hipStream_t st);
 // last inputs of every sequence of a prefill into the ring; tails [nseq][4]: {first row, rows, slot, start position}
 void launch_conv_tail(const SrcRows& src, int col0, void* ring, bool f32, const int* tails, int nseq, int C, int taps,
                       hipStream_t st);

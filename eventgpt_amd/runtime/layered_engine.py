@@ -20,7 +20,7 @@ from typing import Dict, List, Optional, Sequence, Tuple
 import torch
 
 from .engine import DecodeEngine, GenerationEngine, persistent_state
-from .mixers import MIXERS, DenseMLP, RowBatch, Sequence_, pad, pad_to
+from .mixers import MIXERS, DenseMLP, RowBatch, Sequence_, Stream, pad, pad_to
 
 
 class _Stage:
@@ -50,6 +50,11 @@ class LayeredEngine(DecodeEngine):
         self.f32 = self.dtype == torch.float32
         self.width, self.wp, self.eps = cfg.hidden_size, pad(cfg.hidden_size, 64), cfg.norm_eps
         self.V = cfg.vocab_size
+        # decode steps of up to this many sequences run on the weight-streaming kernels, more on the few-row GEMM
+        self.gemv_rows = int(self.raw.gemv_rows_max())
+        self.gemv_lds = int(self.raw.gemv_lds_bytes())
+        if self.wp * (4 if self.f32 else 2) * min(self.B, self.gemv_rows) > self.gemv_lds:
+            self.gemv_rows = 0
         self._rot: Dict[Tuple[float, int], Tuple[torch.Tensor, torch.Tensor]] = {}
         t = model.tensors
 
@@ -81,35 +86,37 @@ class LayeredEngine(DecodeEngine):
         return self._rot[key]
 
     # ------------------------------------------------------------------ layers
-    def _run_stages(self, rows: RowBatch, x: torch.Tensor, final: bool, collect: Optional[list] = None):
-        """All layers over the residual rows ``x`` (updated in place); the final norm's output if ``final``."""
-        xn = self.raw.norm_rows(x, None, self.stages[0].norm, self.width, self.eps, self.f32)
+    def _run_stages(self, rows: RowBatch, x: torch.Tensor, collect: Optional[list] = None) -> Stream:
+        """All layers over the residual rows ``x`` (updated in place, or replaced in the stream that is returned)."""
+        stream = Stream(self, x, rows.decode)
         for i, st in enumerate(self.stages):
-            nxt = self.stages[i + 1].norm if i + 1 < len(self.stages) else (self.final_norm if final else None)
-            xn = st.block.residual(rows, x, xn, nxt)
+            st.block.forward(rows, stream, st.norm)
             if collect is not None and i + 1 in self.layer_ends:
-                collect.append(x[:, :self.width].clone())
-        return xn
+                collect.append(stream.settle()[:, :self.width].clone())
+        return stream
 
     def _logits(self, xn: torch.Tensor) -> torch.Tensor:
         return self.raw.linear(xn, self.head, True)[:, :self.V]
 
     def _layers_step(self) -> None:
         rows = RowBatch(self.device, True, pos=self.pos, live=self.active)
-        self._xn = self._run_stages(rows, self.x, True)
+        self._stream = self._run_stages(rows, self.x)
 
     def _logits_and_commit(self, greedy: bool, want_logits: bool = False) -> None:
-        xn, self._xn = self._xn, None
-        if xn is None:                       # after a prefill: ``x`` holds the last rows' residual stream
-            xn = self.raw.norm_rows(self.x, None, self.final_norm, self.width, self.eps, self.f32)
-        logits = self._logits(xn)
+        stream, self._stream = self._stream, None
+        if stream is None:                   # after a prefill: ``x`` holds the last rows' residual stream
+            stream = Stream(self, self.x, True)
+        if stream.few:
+            logits = stream.gemv(self.final_norm, self.head)[:, :self.V]
+        else:
+            logits = self._logits(stream.normed(self.final_norm))
         if not greedy or want_logits:
             self.logits.copy_(logits)
         if greedy:
             self.raw.argmax_logits_(logits, self.sampled, self.V)
             self._commit_sampled()
 
-    _xn: Optional[torch.Tensor] = None
+    _stream: Optional[Stream] = None
 
     def _commit_sampled(self) -> None:
         self.raw.commit_rows_(self.sampled, self.embed, self.cfg.embedding_scale, self.x, self.out_tokens, self.step,
@@ -142,8 +149,8 @@ class LayeredEngine(DecodeEngine):
             n += int(t.numel())
         flat = torch.cat([t.reshape(-1).to("cpu", torch.int32) if not t.is_cuda else t.reshape(-1).to(torch.int32) for t in ids])
         x = self.raw.embed_rows(flat.to(self.device).contiguous(), self.embed, self.cfg.embedding_scale)
-        self._run_stages(RowBatch(self.device, False, seqs=seqs), x, False, collect)
-        return x, [s.row0 for s in seqs]
+        stream = self._run_stages(RowBatch(self.device, False, seqs=seqs), x, collect)
+        return stream.settle(), [s.row0 for s in seqs]
 
     def _packs(self, slots, ids, starts):
         """Cut portions into passes of at most ``PACK_ROWS`` rows: ``[(slots, ids, starts, indices, offsets)]``."""

@@ -137,10 +137,19 @@ def test_chunk_tables_cover_every_query_once(size):
 def test_scan_tables():
     seqs = [Sequence_(3, 0, 130, 0), Sequence_(1, 130, 2, 50), Sequence_(0, 132, 64, 0)]
     rb = RowBatch("cpu", False, seqs=seqs)
-    assert rb.chunks.tolist() == [[0, 64, 3, 0], [64, 64, 3, 0], [128, 2, 3, 1], [130, 2, 1, 1], [132, 64, 0, 1]]
-    assert rb.scan_seqs.tolist() == [[0, 3, 3, 1], [3, 1, 1, 0], [4, 1, 0, 1]]
-    assert rb.tails.tolist() == [[0, 130, 3, 0], [130, 2, 1, 50], [132, 64, 0, 0]]
+    rb = RowBatch("cpu", False, seqs=seqs + [Sequence_(2, 196, 3, 7), Sequence_(4, 199, 1, 0)])
+    assert rb.tails.tolist() == [[0, 130, 3, 0], [130, 2, 1, 50], [132, 64, 0, 0], [196, 3, 2, 7], [199, 1, 4, 0]]
     assert rb.pos.tolist()[126:134] == [126, 127, 128, 129, 50, 51, 0, 1]
+    # flags: first chunk from the zero state / last chunk of the sequence, and the parities of start and end
+    L, at = mixers.SCAN_CHUNK, 0
+    for (c0, n, slot, flags), s in zip(rb.scan_seqs.tolist(), rb.seqs):
+        assert (c0, n, slot) == (at, -(-s.rows // L), s.slot)
+        assert flags == int(s.start == 0) + 2 * (s.start % 2) + 4 * ((s.start + s.rows) % 2)
+        for c in range(n):
+            assert rb.chunks.tolist()[at + c] == [s.row0 + c * L, min(L, s.rows - c * L), s.slot,
+                                                  int(c == n - 1) + 2 * ((s.start + s.rows) % 2)]
+        at += n
+    assert at == rb.chunks.shape[0]
 
 
 def test_oracle_chunk_mask_and_state():

@@ -110,7 +110,8 @@ def test_group_norm_with_gate(raw, dev, dtype, heads, v, vp, parts, before):
     gate[:, 8:] = rnd(rows, slots, seed=1).float()
     w[:, :v] = 1 + 0.2 * rnd(heads, v, seed=2).float()
     (yd, yr), (gd, gr) = typed(y, dtype, dev), typed(gate, dtype, dev)
-    o = raw.group_norm_rows(yd, gd, 8, before, w.to(dev), heads, v, vp, parts, slots + 64, eps)
+    o = raw.group_norm_rows(yd.view(rows, -1), gd, 8, 1 if before else 2, w.to(dev), heads, v, vp, parts, slots + 64, eps,
+                            dtype == torch.float32)
     real = yr[..., :v].reshape(rows, -1)
     g = gr[:, 8:].view(rows, heads, vp)[..., :v].reshape(rows, -1)
     wr = w[:, :v].reshape(-1).double()
@@ -118,6 +119,9 @@ def test_group_norm_with_gate(raw, dev, dtype, heads, v, vp, parts, before):
     got = o[:, :slots].view(rows, heads, vp)
     assert N.rel_err(got[..., :v].reshape(rows, -1), want) < (2e-6 if dtype == torch.float32 else 6e-3)
     assert float(got[..., v:].float().abs().sum()) == 0 and float(o[:, slots:].float().abs().sum()) == 0
+    plain = raw.group_norm_rows(y.view(rows, -1).to(dev), None, 0, 0, w.to(dev), heads, v, vp, parts, slots, eps, True)
+    assert N.rel_err(plain.view(rows, heads, vp)[..., :v].reshape(rows, -1),
+                     oracle.rms(y[..., :v].reshape(rows, -1).double(), eps, wr, parts)) < 2e-6
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
@@ -127,6 +131,13 @@ def test_glu(raw, dev, dtype):
     tol = 1e-6 if dtype == torch.float32 else 6e-3
     assert N.rel_err(raw.glu_rows(src, 0, dtype == torch.float32), oracle.gelu_tanh(a) * b) < tol
     assert N.rel_err(raw.glu_rows(src, 1, dtype == torch.float32), oracle.silu(a) * b) < tol
+    # projection and gate together: slabs + gate for few rows, the GEMM's epilogue for many
+    for m in (3, 40, 300):
+        x, xr = typed(rnd(m, 128, seed=3), dtype, dev)
+        w, wr = typed(rnd(2 * 192, 128, seed=4, scale=128 ** -0.5), dtype, dev)
+        g, u = (xr @ wr.T).chunk(2, -1)
+        for act, f in ((0, oracle.gelu_tanh), (1, oracle.silu)):
+            assert N.rel_err(raw.linear_glu(x, w, act), f(g) * u) < (3e-6 if dtype == torch.float32 else 8e-3)
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
@@ -156,7 +167,7 @@ def pack(lens, starts=None):
 @pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("taps", [1, 2, 4, 7])
 def test_convolution(raw, dev, dtype, taps):
-    """Whole sequences, portions (also shorter than the taps) and single steps give the same rows."""
+    """Whole sequences, portions (also shorter than the taps) and single tokens give the same rows."""
     C, lens = 72, [1, 9, 30]
     w, b = rnd(C, taps, seed=1).float(), rnd(C, seed=2).float()
     x = [typed(rnd(n, C, seed=5 + n), dtype, dev) for n in lens]
@@ -175,7 +186,7 @@ def test_convolution(raw, dev, dtype, taps):
                 seqs.append(Sequence_(i, row, n[i], at[i]))
                 row += n[i]
             rb = RowBatch(dev, False, seqs=seqs)
-            o = raw.conv_rows_(src, 0, wd, bd, ring, rb.slot, rb.pos, rb.first, False, None)
+            o = raw.conv_rows_(src, 0, wd, bd, ring, rb.slot, rb.pos, rb.first)
             raw.conv_tail_(src, 0, ring, rb.tails)
             for s in seqs:
                 got[s.slot].append(o[s.row0:s.row0 + s.rows])
@@ -185,16 +196,6 @@ def test_convolution(raw, dev, dtype, taps):
     for cuts in ([100], [2] * 15, [5] * 6, [1] * 30, [3, 1, 100]):
         for g, r in zip(run(cuts), want):
             assert N.rel_err(g, r) < tol
-    # decode steps: row b is slot b; a row that is not live leaves its ring alone
-    ring = torch.full((1, taps, C), 77.0, dtype=dtype, device=dev)
-    live, pos = torch.ones(1, dtype=torch.int32, device=dev), torch.zeros(1, dtype=torch.int32, device=dev)
-    for t in range(lens[2]):
-        pos.fill_(t)
-        live.zero_()
-        raw.conv_rows_(torch.full_like(x[2][0][:1], 55.0), 0, wd, bd, ring, None, pos, None, True, live)
-        live.fill_(1)
-        o = raw.conv_rows_(x[2][0][t:t + 1], 0, wd, bd, ring, None, pos, None, True, live)
-        assert N.rel_err(o, want[2][t:t + 1]) < 4 * tol
 
 
 def scan_case(kind, dtype, dev, lens, H, per_group, Nn, V, seed=0):
@@ -230,8 +231,8 @@ def scan_case(kind, dtype, dev, lens, H, per_group, Nn, V, seed=0):
 @pytest.mark.parametrize("kind,H,per_group,Nn,V", [("ssd", 4, 2, 32, 64), ("ssd", 3, 3, 96, 32), ("ssd", 2, 1, 128, 64),
                                                    ("mlstm", 2, 1, 32, 32), ("mlstm", 3, 1, 160, 128), ("mlstm", 1, 1, 64, 192)])
 def test_recurrence(raw, dev, dtype, kind, H, per_group, Nn, V):
-    """Unequal sequences in one pack, in portions (whole chunks, two tokens, across chunk borders) and step by step,
-    from states that hold an earlier owner's values."""
+    """Unequal sequences in one pack, in portions (whole chunks, two tokens, single ones, across chunk borders), from
+    states that hold an earlier owner's values."""
     lens = [1, 63, 64, 65, 200]
     q, k, v, gates, scale, want = scan_case(kind, dtype, dev, lens, H, per_group, Nn, V)
     offs = [sum(lens[:i]) for i in range(len(lens))]
@@ -242,11 +243,11 @@ def test_recurrence(raw, dev, dtype, kind, H, per_group, Nn, V):
     def state():
         f = dict(device=dev, dtype=torch.float32)
         S = torch.full((B, H, V, Nn), 7.0, **f)
-        return (S, None, None) if kind == "ssd" else (S, torch.full((B, H, Nn), 7.0, **f), torch.full((B, H), 7.0, **f))
+        return (S, None, None) if kind == "ssd" else (S, torch.full((2, B, H, Nn), 7.0, **f), torch.full((2, B, H), 7.0, **f))
 
     def rows(t, idx):
         return None if t is None else (t if t.dim() == 1 else t[idx].contiguous())
-    for cuts in ([1000], [64] * 4, [2] * 100, [37] * 6, [130, 3, 70]):
+    for cuts in ([1000], [64] * 4, [2] * 100, [1] * 200, [37] * 6, [130, 3, 70]):
         st, at, got = state(), [0] * B, [[] for _ in lens]
         for cut in cuts:
             seqs, idx, row = [], [], 0
@@ -267,23 +268,160 @@ def test_recurrence(raw, dev, dtype, kind, H, per_group, Nn, V):
                 at[s.slot] += s.rows
         for g, w in zip(got, want):
             assert N.rel_err(torch.cat(g), w.reshape(w.shape[0], -1)) < tol, cuts
-    # steps: a parked slot keeps its state
-    st = state()
-    pos = torch.zeros(B, dtype=torch.int32, device=dev)
-    outs = [[] for _ in lens]
-    for t in range(max(lens)):
-        live = torch.tensor([int(t < n) for n in lens], dtype=torch.int32, device=dev)
-        ix = torch.tensor([offs[i] + min(t, lens[i] - 1) for i in range(B)], device=dev)
-        pos.fill_(t)
-        before = st[0][0].clone()
-        o = raw.scan_step_(q[ix], k[ix], v[ix], H, per_group, Nn, V, scale, *(rows(g, ix) for g in gates), *st, pos, live)
-        if t > 0:
-            assert torch.equal(before, st[0][0])
-        for i in range(B):
-            if t < lens[i]:
-                outs[i].append(o[i])
-    for g, w in zip(outs, want):
-        assert N.rel_err(torch.stack(g), w.reshape(w.shape[0], -1)) < tol
+
+
+def step_rows(dtype, dev, cols):
+    """Projection rows of a decode step: values that T holds, as one fp32 matrix and as three slabs that sum to it."""
+    x = torch.cat(cols, -1)
+    pad = torch.zeros(x.shape[0], -x.shape[1] % 8)
+    x = torch.cat([x, pad], -1).to(dev)
+    a = torch.round(x * 0.5 * 256) / 256
+    return x, torch.stack([a, x - a, torch.zeros_like(x)])
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("H,G,Nn,V,v_used", [(4, 2, 32, 64, 64), (3, 1, 96, 32, 20), (2, 2, 128, 128, 128)])
+def test_ssd_decode_step(raw, dev, dtype, H, G, Nn, V, v_used):
+    """Convolution, gates, recurrence and output gate of single tokens; unequal sequences, a slot that is parked now and
+    then, stale state of an earlier owner, rows as a matrix and as slabs."""
+    taps, lens, T = 3, [9, 5], 9
+    inner, C = H * V, H * V + 2 * G * Nn
+    f = dict(dtype=torch.float32, device=dev)
+    z, xbc = typed(rnd(2, T, inner), dtype, "cpu")[0].float(), typed(rnd(2, T, C, seed=1), dtype, "cpu")[0].float()
+    dt = rnd(2, T, H, seed=2).float()
+    cw, cb = rnd(C, taps, seed=3).float(), rnd(C, seed=4).float()
+    bias, a_log, skip = (rnd(H, seed=5 + i).float() for i in range(3))
+    S, ring = torch.full((2, H, V, Nn), 9.0, **f), torch.full((2, taps, C), 9.0, dtype=dtype, device=dev)
+    want = []
+    for b in range(2):
+        c = oracle.silu(oracle.causal_conv(xbc[b].double(), cw.double(), cb.double()))
+        c = c.to(dtype).double()
+        x, bb, cc = c.split([inner, G * Nn, G * Nn], -1)
+        y = oracle.ssd_scan(x.reshape(T, H, V), bb.reshape(T, G, Nn), cc.reshape(T, G, Nn),
+                            oracle.softplus(dt[b].double() + bias.double()), a_log.double(), skip.double())
+        want.append(y.reshape(T, inner) * oracle.silu(z[b].double()))
+    dims = [0, inner, inner + C, H, G, Nn, V]
+    args = [t.to(dev) for t in (cw, cb)] + [ring] + [t.to(dev) for t in (bias, a_log, skip)]
+    for t in range(T):
+        live = torch.tensor([1, int(t < lens[1])], dtype=torch.int32, device=dev)
+        pos = torch.full((2,), t, dtype=torch.int32, device=dev)
+        rows = step_rows(dtype, dev, [z[:, t], xbc[:, t], dt[:, t]])
+        off = torch.zeros(2, dtype=torch.int32, device=dev)
+        before = S.clone(), ring.clone()
+        raw.ssd_step_(rows[0] + 1, dims, *args, S, pos, off)
+        assert torch.equal(before[0], S) and torch.equal(before[1], ring)
+        o = raw.ssd_step_(rows[t % 2], dims, *args, S, pos, live)
+        for b in range(2):
+            if t < lens[b]:
+                assert N.rel_err(o[b:b + 1], want[b][t:t + 1]) < (1e-5 if dtype == torch.float32 else 1e-2), (t, b)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("Hr,Nn,V", [(3, 32, 64), (1, 160, 32), (2, 64, 192)])
+def test_parallel_decode_step(raw, dev, dtype, Hr, Nn, V):
+    """Attention heads (norm, rotation, cache append) and matrix memory of single tokens from one set of rows."""
+    H, G, d, D, dims, cap, eps, T, lens, mcap = 6, 2, 20, 64, 12, 4, 1e-3, 11, [11, 6], 5.0
+    f = dict(dtype=torch.float32, device=dev)
+    att = torch.zeros(2, T, H + 2 * G, D)
+    att[..., :d] = rnd(2, T, H + 2 * G, d).float()
+    att = att.to(dtype).float()
+    q, k = (typed(rnd(2, T, Hr, Nn, seed=s, scale=Nn ** -0.25), dtype, "cpu")[0].float() for s in (1, 2))
+    v = typed(rnd(2, T, Hr, V, seed=3), dtype, "cpu")[0].float()
+    gi, gf = 3 * rnd(2, T, Hr, seed=4).float(), 2 + rnd(2, T, Hr, seed=5).float()
+    ib, fb = rnd(Hr, seed=6).float(), rnd(Hr, seed=7).float()
+    qw, kw = torch.zeros(H, D), torch.zeros(G, D)
+    qw[:, :d], kw[:, :d] = 1 + 0.2 * rnd(H, d, seed=8).float(), 1 + 0.2 * rnd(G, d, seed=9).float()
+    ang = torch.arange(64, dtype=torch.float64)[:, None] * 50.0 ** (-2.0 * torch.arange(dims // 2, dtype=torch.float64) / dims)
+    cos, sin = ang.cos().float().to(dev), ang.sin().float().to(dev)
+    kc, vc = (torch.full((2, G, cap, D), 9.0, dtype=dtype, device=dev) for _ in range(2))
+    S, n, m = torch.full((2, Hr, V, Nn), 7.0, **f), torch.full((2, 2, Hr, Nn), 7.0, **f), torch.full((2, 2, Hr), 7.0, **f)
+    want, wq, wk = [], [], []
+    for b in range(2):
+        li = mcap * torch.tanh((gi[b] + ib).double() / mcap)
+        lf = -oracle.softplus(-mcap * torch.tanh((gf[b] + fb).double() / mcap))
+        want.append(oracle.mlstm_scan(q[b].double() * 0.4, k[b].double(), v[b].double(), li, lf).reshape(T, -1))
+        real, pos = att[b, ..., :d].double(), torch.arange(T)
+        wq.append(oracle.rotate(oracle.rms(real[:, :H].reshape(T, -1), eps, qw[:, :d].reshape(-1).double()).view(T, H, d), pos, dims, 50.0))
+        wk.append(oracle.rotate(oracle.rms(real[:, H:H + G].reshape(T, -1), eps, kw[:, :d].reshape(-1).double()).view(T, G, d), pos, dims, 50.0))
+    c0 = (H + 2 * G) * D
+    a_dims = [0, H * D, (H + G) * D, H, G, D, H * d, G * d]
+    m_dims = [c0, c0 + Hr * Nn, c0 + 2 * Hr * Nn, c0 + 2 * Hr * Nn + Hr * V, c0 + 2 * Hr * Nn + Hr * V + Hr, Hr, Nn, V]
+    tol = 2e-5 if dtype == torch.float32 else 6e-3
+
+    def step(rows, pos, live):
+        return raw.parallel_step_(rows, a_dims, qw.to(dev).view(-1), kw.to(dev).view(-1), eps, cos, sin, kc, vc, m_dims,
+                                  ib.to(dev), fb.to(dev), mcap, 0.4, S, n, m, pos, live)
+    for t in range(T):
+        live = torch.tensor([1, int(t < lens[1])], dtype=torch.int32, device=dev)
+        pos = torch.full((2,), t, dtype=torch.int32, device=dev)
+        rows = step_rows(dtype, dev, [att[:, t].reshape(2, -1), q[:, t].reshape(2, -1), k[:, t].reshape(2, -1),
+                                      v[:, t].reshape(2, -1), gi[:, t], gf[:, t]])
+        before = [x.clone() for x in (kc, vc, S, n, m)]
+        step(rows[0] + 1, pos, torch.zeros(2, dtype=torch.int32, device=dev))
+        assert all(torch.equal(x, y) for x, y in zip(before, (kc, vc, S, n, m)))
+        qo, o = step(rows[t % 2], pos, live)
+        for b in range(2):
+            if t < lens[b]:
+                assert N.rel_err(o[b:b + 1], want[b][t:t + 1]) < 10 * tol, (t, b)
+                assert N.rel_err(qo[b, :, :d].reshape(1, -1), wq[b][t].reshape(1, -1)) < tol
+                assert N.rel_err(kc[b, :, t % cap, :d].reshape(1, -1), wk[b][t].reshape(1, -1)) < tol
+                assert torch.equal(vc[b, :, t % cap, :d].float().cpu(), att[b, t, H + G:, :d])
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("B", [1, 2, 3, 4])
+@pytest.mark.parametrize("width,ff,heads,v,vp", [(100, 192, 3, 20, 32), (640, 1344, 5, 64, 64), (2112, 4352, 8, 128, 128)])
+def test_few_row_products(raw, dev, dtype, B, width, ff, heads, v, vp):
+    """The weight-streaming products with their inputs and epilogues: norm, branch merge, gated unit, group norm with
+    and without a gate, addition to the stream, two problems in a launch."""
+    ld, eps, slots = -(-width // 64) * 64, 1e-3, heads * vp
+    kp = -(-slots // 64) * 64
+    if B * max(ld, kp, ff) * (4 if dtype == torch.float32 else 2) > 60000:
+        pytest.skip("input rows do not fit the launch's LDS; the engine takes the GEMM path")
+
+    def padded(t, n=ld):
+        out = torch.zeros(*t.shape[:-1], n, dtype=t.dtype)
+        out[..., :t.shape[-1]] = t
+        return out
+    x, a, b = (rnd(B, width, seed=s).float() for s in range(3))
+    w, wa, wb = (1 + 0.3 * rnd(width, seed=10 + s).float() for s in range(3))
+    X, A, Bb, W, WA, WB = (padded(t).to(dev) for t in (x, a, b, w, wa, wb))
+    x, a, b, w, wa, wb = (t.double() for t in (x, a, b, w, wa, wb))
+    tol = 3e-6 if dtype == torch.float32 else 8e-3
+    M, Mr = typed(padded(rnd(104, width, seed=5, scale=width ** -0.5)), dtype, dev)
+    normed = padded(oracle.rms(x, eps, w))
+    y = raw.gemv_norm(X, W, width, eps, M, -1, None, None, None, None, None)
+    assert y.dtype == torch.float32 and N.rel_err(y, normed @ Mr.T) < tol
+    out = torch.empty_like(X)
+    merged = x + 0.5 * (oracle.rms(a, eps, wa) + oracle.rms(b, eps, wb))
+    U, Ur = typed(padded(rnd(2 * ff, width, seed=6, scale=width ** -0.5)), dtype, dev)
+    g, u = (padded(oracle.rms(merged, eps, w)) @ Ur.T).chunk(2, -1)
+    h = raw.gemv_norm(X, W, width, eps, U, 0, A, Bb, WA, WB, out)
+    assert h.dtype == dtype and N.rel_err(out[:, :width], merged) < 1e-6 and N.rel_err(h, oracle.gelu_tanh(g) * u) < 2 * tol
+    h, hr = typed(rnd(B, ff, seed=7), dtype, dev)
+    Dn, Dr = typed(padded(rnd(ff, width, seed=8, scale=ff ** -0.5)).T.contiguous(), dtype, dev)
+    Y = X.clone()
+    raw.gemv_add_(Y, Dn, h)
+    assert N.rel_err(Y[:, :width], x + (hr @ Dr.T)[:, :width]) < 2e-6
+    o, nw = torch.zeros(B, heads, vp), torch.zeros(heads, vp)
+    o[..., :v], nw[:, :v] = rnd(B, heads, v, seed=9).float(), 1 + 0.3 * rnd(heads, v, seed=13).float()
+    G, Gr = typed(padded(rnd(heads * vp, width, seed=14, scale=slots ** -0.5)).T.contiguous(), dtype, dev)
+    if kp > slots:
+        z = torch.zeros(ld, kp - slots)
+        G, Gr = torch.cat([G, z.to(dev, dtype)], 1).contiguous(), torch.cat([Gr, z.double()], 1)
+    real, nr = o[..., :v].reshape(B, -1).double(), nw[:, :v].reshape(-1).double()
+    for parts in {1, heads, 4 if heads * v % 4 == 0 else 1}:
+        full = torch.zeros(B, heads, vp, dtype=torch.float64)
+        full[..., :v] = oracle.rms(real, eps, nr, parts).view(B, heads, v)
+        Y = X.clone()
+        raw.gemv_group_add_(Y, G, o.to(dev).view(B, -1), nw.to(dev).view(-1), heads, v, vp, parts, eps)
+        assert N.rel_err(Y[:, :width], x + (padded(full.view(B, -1), kp) @ Gr.T)[:, :width]) < tol
+    gate = rnd(B, 16 + slots, seed=15).float()
+    full = torch.zeros(B, heads, vp, dtype=torch.float64)
+    full[..., :v] = oracle.rms(real, eps, nr, heads).view(B, heads, v)
+    full = full.view(B, -1) * torch.sigmoid(gate[:, 16:].double())
+    two = raw.gemv_branches(Dn, h, G, o.to(dev).view(B, -1), gate.to(dev), 16, nw.to(dev).view(-1), heads, v, vp, eps)
+    assert N.rel_err(two[0, :, :width], (hr @ Dr.T)[:, :width]) < tol and N.rel_err(two[1, :, :width], (padded(full, kp) @ Gr.T)[:, :width]) < tol
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
@@ -299,7 +437,7 @@ def test_matrix_memory_extreme_gates(raw, dev, dtype):
     li[100:, 1] = 14.9
     want = oracle.mlstm_scan(qr, kr, vr, li.double(), lf.double())
     f = dict(device=dev, dtype=torch.float32)
-    st = (torch.zeros(1, H, V, Nn, **f), torch.zeros(1, H, Nn, **f), torch.zeros(1, H, **f))
+    st = (torch.zeros(1, H, V, Nn, **f), torch.zeros(2, 1, H, Nn, **f), torch.zeros(2, 1, H, **f))
     rb = RowBatch(dev, False, seqs=pack([T]))
     o = raw.scan_prefill_(q.view(T, -1), k.view(T, -1), v.view(T, -1), H, 1, Nn, V, 1.0, lf.to(dev), li.to(dev), None, None, *st,
                           rb.chunks, rb.scan_seqs)
