@@ -2,7 +2,7 @@
 // memory of xLSTM):
 //     S_t = exp(a_t) S_(t-1) + b_t v_t k_t^T,      y_t = S_t q_t          (S is [V][N], value-major)
 //
-// Prefill runs in chunks of 64 tokens, three launches, all chunks of all sequences at once where the
+// Prefill runs in chunks of 128 tokens (64 with fp32 storage), three launches, all chunks of all sequences at once where the
 // recurrence allows it.  With F_t = sum of a over the chunk up to t:
 //   1. scan_chunk_state: what a chunk adds to the state,  dS = sum_s exp(F_L - F_s) b_s v_s k_s^T;
 //   2. scan_chunk_pass: the walk over a sequence's chunks, elementwise:  S <- exp(F_L) S + dS; every
@@ -23,9 +23,6 @@
 #include "../layered_kernels.h"
 
 namespace evgpt {
-
-constexpr int SL = SCAN_CHUNK;
-constexpr int TS = SL + 8;      // elements per row of a transposed LDS tile
 
 // inclusive sum over the wave, in double
 __device__ __forceinline__ double wave_scan_add(double v) {
@@ -54,12 +51,12 @@ __device__ __forceinline__ double wave_max_f64(double v) {
 
 // rows [row0, row0 + len) x 64 columns from col (nc of them exist) of a T matrix, transposed into
 // lds[column][row] with rows past len as zeros
-template <typename T>
+template <typename T, int SL>
 __device__ __forceinline__ void load_transposed(const T* __restrict__ p, long long ld, long long row0, int len, int col,
                                                 int nc, T* lds) {
 #pragma unroll
-  for (int i = 0; i < 2; ++i) {
-    const int idx = threadIdx.x + i * 256, s = idx & 63, c8 = (idx >> 6) * 8;
+  for (int i = 0; i < SL / 32; ++i) {
+    const int idx = threadIdx.x + i * 256, s = idx % SL, c8 = (idx / SL) * 8;
     T t[8];
     if (s < len && c8 < nc) {
       const T* g = p + (row0 + s) * ld + col + c8;
@@ -73,13 +70,47 @@ __device__ __forceinline__ void load_transposed(const T* __restrict__ p, long lo
       for (int j = 0; j < 8; ++j) t[j] = T(0);
     }
 #pragma unroll
-    for (int j = 0; j < 8; ++j) lds[(c8 + j) * TS + s] = t[j];
+    for (int j = 0; j < 8; ++j) lds[(c8 + j) * (SL + 8) + s] = t[j];
+  }
+}
+
+// One wave: decay sums F of a chunk's tokens (lane l: tokens l NH .. l NH + NH - 1), and with STAB the running maxima
+// of log_in - F.
+template <int NH, bool STAB>
+__device__ __forceinline__ void chunk_gates(const ScanArgs& a, int row0, int len, int h, double (&F)[NH], float (&li)[NH],
+                                            double (&top)[NH]) {
+  const int lane = threadIdx.x & 63;
+  double sum = 0.0;
+#pragma unroll
+  for (int i = 0; i < NH; ++i) {
+    const int t = lane * NH + i;
+    const long long gi = static_cast<long long>(row0 + t) * a.H + h;
+    sum += t < len ? static_cast<double>(a.log_decay[gi]) : 0.0;
+    F[i] = sum;
+    if constexpr (STAB) li[i] = t < len ? a.log_in[gi] : -INFINITY;
+    else li[i] = t < len ? a.scale_in[gi] : 0.f;
+  }
+  const double before = wave_scan_add(sum) - sum;
+#pragma unroll
+  for (int i = 0; i < NH; ++i) F[i] += before;
+  if constexpr (STAB) {
+    double m = -INFINITY;
+#pragma unroll
+    for (int i = 0; i < NH; ++i) {
+      m = fmax(m, static_cast<double>(li[i]) - F[i]);
+      top[i] = m;
+    }
+    const double up = __shfl_up(wave_scan_max(m), 1, 64);
+    if (lane > 0)
+#pragma unroll
+      for (int i = 0; i < NH; ++i) top[i] = fmax(top[i], up);
   }
 }
 
 // Block: 64 value rows of one head and chunk, all of N in runs of 64.
-template <typename T, bool STAB>
+template <typename T, bool STAB, int SL>
 __global__ __launch_bounds__(256) void scan_chunk_state_kernel(ScanArgs a, ScanChunks c) {
+  constexpr int TS = SL + 8, NH = SL / 64;
   __shared__ __attribute__((aligned(16))) T kt[64 * TS];
   __shared__ __attribute__((aligned(16))) T vt[64 * TS];
   __shared__ __attribute__((aligned(16))) float wgt[SL];
@@ -87,22 +118,20 @@ __global__ __launch_bounds__(256) void scan_chunk_state_kernel(ScanArgs a, ScanC
   const int row0 = c.chunks[ci * 4], len = min(c.chunks[ci * 4 + 1], SL);
   const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6, fr = lane & 15, g = lane >> 4;
   const int nv = min(64, a.V - v0), k_col = (h / a.per_group) * a.N;
-  load_transposed(static_cast<const T*>(a.v), a.ldv, row0, len, h * a.V + v0, nv, vt);
-  load_transposed(static_cast<const T*>(a.k), a.ldk, row0, len, k_col, min(64, a.N), kt);
+  load_transposed<T, SL>(static_cast<const T*>(a.v), a.ldv, row0, len, h * a.V + v0, nv, vt);
+  load_transposed<T, SL>(static_cast<const T*>(a.k), a.ldk, row0, len, k_col, min(64, a.N), kt);
   if (wid == 0) {
-    const bool in = lane < len;
-    const long long gi = static_cast<long long>(row0 + lane) * a.H + h;
-    const double F = wave_scan_add(in ? static_cast<double>(a.log_decay[gi]) : 0.0);
-    const double FL = __shfl(F, 63, 64);
-    double e = FL - F, top = 0.0;
-    float b = 1.f;
-    if constexpr (STAB) {
-      e = in ? e + a.log_in[gi] : -INFINITY;
-      top = wave_max_f64(e);
-    } else {
-      b = in ? a.scale_in[gi] : 0.f;
+    double F[NH], m[NH];
+    float li[NH];
+    chunk_gates<NH, STAB>(a, row0, len, h, F, li, m);
+    const double FL = __shfl(F[NH - 1], 63, 64);
+    double top = 0.0;
+    if constexpr (STAB) top = FL + __shfl(m[NH - 1], 63, 64);     // the largest FL - F + log_in
+#pragma unroll
+    for (int i = 0; i < NH; ++i) {
+      const float e = static_cast<float>(FL - F[i] + (STAB ? static_cast<double>(li[i]) - top : 0.0));
+      wgt[lane * NH + i] = lane * NH + i < len ? expf(e) * (STAB ? 1.f : li[i]) : 0.f;
     }
-    wgt[lane] = in ? expf(static_cast<float>(e - top)) * b : 0.f;
     if (blockIdx.x == 0 && lane == 0) {
       const long long o = static_cast<long long>(ci) * a.H + h;
       c.am[o] = top;
@@ -125,7 +154,7 @@ __global__ __launch_bounds__(256) void scan_chunk_state_kernel(ScanArgs a, ScanC
     const int nn = min(64, a.N - n0);
     if (n0 > 0) {
       __syncthreads();
-      load_transposed(static_cast<const T*>(a.k), a.ldk, row0, len, k_col + n0, nn, kt);
+      load_transposed<T, SL>(static_cast<const T*>(a.k), a.ldk, row0, len, k_col + n0, nn, kt);
       __syncthreads();
     }
     f32x4_t acc[4];
@@ -203,168 +232,194 @@ __global__ __launch_bounds__(256) void scan_chunk_pass_kernel(ScanArgs a, ScanCh
   }
 }
 
-// Block: 64 value columns of one head and chunk.  Scores are computed transposed, a wave per sixteen keys, and
-// meet in LDS; then a wave owns sixteen value rows for all tokens, so that the chunk's start state -- most of the
-// bytes this kernel reads -- is read once.
-template <typename T, bool STAB>
+// Block: 64 value columns of one head and chunk.  Scores are computed transposed, a wave per sixteen keys of every
+// 64, and meet in LDS (in the query tile's place); then a wave owns sixteen value rows for all tokens, so that the
+// chunk's start state -- most of the bytes this kernel reads -- is read once.
+template <typename T, bool STAB, int SL>
 __global__ __launch_bounds__(256) void scan_chunk_out_kernel(ScanArgs a, ScanChunks c) {
-  constexpr int PS = SL + 4;                      // floats per row of the score tile
-  __shared__ __attribute__((aligned(16))) T vt[64 * TS];      // [value][key]
-  __shared__ __attribute__((aligned(16))) T qs[SL * TS];      // [token][64 of N]
-  __shared__ __attribute__((aligned(16))) float ps[SL * PS];  // [token][key] weighted scores
+  constexpr int TS = SL + 8, NH = SL / 64, PS = SL + 4, QS = 64 + 8;
+  constexpr int Q_BYTES = SL * QS * sizeof(T), P_BYTES = 64 * PS * 4;
+  __shared__ __attribute__((aligned(16))) T vt[64 * TS];              // [value][key]
+  __shared__ __attribute__((aligned(16))) unsigned char qp_lds[Q_BYTES > P_BYTES ? Q_BYTES : P_BYTES];
+  T* qs = reinterpret_cast<T*>(qp_lds);                               // [token][64 of N]
+  float* ps = reinterpret_cast<float*>(qp_lds);                       // [token of a half][key] weighted scores
   __shared__ double F_s[SL];
-  __shared__ float in_s[SL], m_s[SL], b_s[SL], inv_s[SL];
+  __shared__ float in_s[SL], m_s[SL], inv_s[64];
   const int v0 = blockIdx.x * 64, h = blockIdx.y, ci = blockIdx.z;
   const int row0 = c.chunks[ci * 4], len = min(c.chunks[ci * 4 + 1], SL);
   const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6, fr = lane & 15, g = lane >> 4;
   const int nv = min(64, a.V - v0), hk = h / a.per_group;
   const long long ho = static_cast<long long>(ci) * a.H + h;
   const float m0 = STAB ? c.m0[ho] : 0.f;
-  load_transposed(static_cast<const T*>(a.v), a.ldv, row0, len, h * a.V + v0, nv, vt);
+  load_transposed<T, SL>(static_cast<const T*>(a.v), a.ldv, row0, len, h * a.V + v0, nv, vt);
   if (wid == 0) {
-    const bool in = lane < len;
-    const long long gi = static_cast<long long>(row0 + lane) * a.H + h;
-    const double F = wave_scan_add(in ? static_cast<double>(a.log_decay[gi]) : 0.0);
-    F_s[lane] = F;
+    double F[NH], top[NH];
+    float li[NH];
+    chunk_gates<NH, STAB>(a, row0, len, h, F, li, top);
+#pragma unroll
+    for (int i = 0; i < NH; ++i) {
+      const int t = lane * NH + i;
+      F_s[t] = F[i];
+      in_s[t] = li[i];
+      m_s[t] = STAB ? static_cast<float>(F[i] + fmax(static_cast<double>(m0), top[i])) : 0.f;
+    }
     if constexpr (STAB) {
-      const float li = in ? a.log_in[gi] : -INFINITY;
-      in_s[lane] = li;
-      m_s[lane] = static_cast<float>(F + fmax(static_cast<double>(m0), wave_scan_max(static_cast<double>(li) - F)));
       const int last = c.chunks[ci * 4 + 3];
-      if (blockIdx.x == 0 && lane == len - 1 && (last & 1))
-        a.m[(static_cast<long long>(last >> 1 & 1) * a.slots + c.chunks[ci * 4 + 2]) * a.H + h] = static_cast<float>(fmax(c.fl[ho] + m0, c.am[ho]));
-    } else {
-      b_s[lane] = in ? a.scale_in[gi] : 0.f;
+      if (blockIdx.x == 0 && lane == 0 && (last & 1))
+        a.m[(static_cast<long long>(last >> 1 & 1) * a.slots + c.chunks[ci * 4 + 2]) * a.H + h] =
+            static_cast<float>(fmax(c.fl[ho] + m0, c.am[ho]));
     }
   }
   const T* qp = static_cast<const T*>(a.q) + static_cast<long long>(hk) * a.N;
-  const T* kp = static_cast<const T*>(a.k) + (row0 + min(wid * 16 + fr, len - 1)) * a.ldk + static_cast<long long>(hk) * a.N;
+  const T* kp[NH];
+#pragma unroll
+  for (int k = 0; k < NH; ++k)
+    kp[k] = static_cast<const T*>(a.k) + (row0 + min(k * 64 + wid * 16 + fr, len - 1)) * a.ldk + static_cast<long long>(hk) * a.N;
   const float* S0 = c.dS + (ho * a.V + v0 + wid * 16 + fr) * a.N;
   const float* nrm = STAB ? c.dn + ho * a.N : nullptr;
   const bool rows_v = wid * 16 < nv;              // this wave has value rows
-  f32x4_t st[4], inter[4];
+  f32x4_t st[NH][NH][4], inter[NH][4];            // [key half][token half][token tile]
+  float nq[NH];
 #pragma unroll
-  for (int i = 0; i < 4; ++i) st[i] = inter[i] = f32x4_t{0.f, 0.f, 0.f, 0.f};
-  float nq = 0.f;
+  for (int k = 0; k < NH; ++k) {
+    nq[k] = 0.f;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      inter[k][i] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int j = 0; j < NH; ++j) st[k][j][i] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+    }
+  }
   for (int n0 = 0; n0 < a.N; n0 += 64) {
     const int nn = min(64, a.N - n0);
     __syncthreads();
 #pragma unroll
-    for (int i = 0; i < 2; ++i) {
+    for (int i = 0; i < 2 * NH; ++i) {
       const int idx = tid + i * 256, t = idx >> 3, c8 = (idx & 7) * 8;
       if (c8 < nn) {
         const T* p = qp + (row0 + min(t, len - 1)) * a.ldq + n0 + c8;
-        T* d = qs + t * TS + c8;
+        T* d = qs + t * QS + c8;
         *reinterpret_cast<u32x4_t*>(d) = load16(p);
         if constexpr (sizeof(T) == 4) *reinterpret_cast<u32x4_t*>(d + 4) = load16(p + 4);
       }
     }
     __syncthreads();
     for (int n = 0; n < nn; n += 32) {
-      Frag<T> qf[4];
+      Frag<T> kf[NH];
 #pragma unroll
-      for (int j = 0; j < 4; ++j) qf[j] = load_frag(qs + (j * 16 + fr) * TS + n + g * 8);
-      const Frag<T> kf = load_frag(kp + n0 + n + g * 8);
+      for (int k = 0; k < NH; ++k) kf[k] = load_frag(kp[k] + n0 + n + g * 8);
+      float x[8];
+      if (rows_v) load8(S0 + n0 + n + g * 8, x);
+      else
 #pragma unroll
-      for (int j = 0; j < 4; ++j)
-        if (j >= wid) st[j] = mma(kf, qf[j], st[j]);
-      if (rows_v) {
-        float x[8];
-        load8(S0 + n0 + n + g * 8, x);
-        const WideFrag<T> sf = wide_frag<T>(x);
+        for (int j = 0; j < 8; ++j) x[j] = 0.f;
+      const WideFrag<T> sf = wide_frag<T>(x);
 #pragma unroll
-        for (int j = 0; j < 4; ++j) inter[j] = mma(sf, qf[j], inter[j]);
-      }
+      for (int th = 0; th < NH; ++th)
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+          const Frag<T> qf = load_frag(qs + (th * 64 + j * 16 + fr) * QS + n + g * 8);
+#pragma unroll
+          for (int k = 0; k < NH; ++k)
+            if (k < th || (k == th && j >= wid)) st[k][th][j] = mma(kf[k], qf, st[k][th][j]);
+          inter[th][j] = mma(sf, qf, inter[th][j]);
+        }
     }
     if constexpr (STAB) {
-      const int t = tid >> 2, part = (tid & 3) * 16;
-      for (int n = part; n < min(part + 16, nn); ++n) nq += nrm[n0 + n] * to_f32(qs[t * TS + n]);
+      const int part = (tid & 3) * 16;
+#pragma unroll
+      for (int th = 0; th < NH; ++th)
+        for (int n = part; n < min(part + 16, nn); ++n) nq[th] += nrm[n0 + n] * to_f32(qs[(th * 64 + (tid >> 2)) * QS + n]);
     }
   }
-  // weighted scores of keys 16 wid + 4 g + r and token 16 j + fr
-#pragma unroll
-  for (int j = 0; j < 4; ++j) {
-    const int t = j * 16 + fr;
-    const double Ft = F_s[t];
-    const float mt = STAB ? m_s[t] : 0.f;
-#pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      const int s = wid * 16 + g * 4 + r;
-      float w = 0.f;
-      if (s <= t && t < len) {
-        if constexpr (STAB) w = expf(static_cast<float>(Ft - F_s[s] + static_cast<double>(in_s[s] - mt)));
-        else w = expf(static_cast<float>(Ft - F_s[s])) * b_s[s];
-      }
-      st[j][r] *= w * a.qscale;
-    }
-    *reinterpret_cast<f32x4_t*>(ps + t * PS + wid * 16 + g * 4) = st[j];
-  }
-  __syncthreads();
-  if constexpr (STAB) {
-    const int t = tid >> 2, part = (tid & 3) * 16;
-    float den = 0.f;
-#pragma unroll
-    for (int i = 0; i < 16; i += 4) {
-      const f32x4_t x = *reinterpret_cast<const f32x4_t*>(ps + t * PS + part + i);
-      den += x[0] + x[1] + x[2] + x[3];
-    }
-    const float carry = expf(static_cast<float>(F_s[t] + static_cast<double>(m0 - m_s[t]))) * a.qscale;
-    den += nq * carry;
-    den += __shfl_xor(den, 1, 64);
-    den += __shfl_xor(den, 2, 64);
-    if ((tid & 3) == 0) inv_s[t] = 1.f / (fmaxf(fabsf(den), expf(-m_s[t])) + 1e-6f);
-    __syncthreads();
-  }
-  if (!rows_v) return;
   Frag<T> vf[SL / 32];
 #pragma unroll
   for (int kb = 0; kb < SL / 32; ++kb) vf[kb] = load_frag(vt + (wid * 16 + fr) * TS + kb * 32 + g * 8);
   const float skip = a.skip ? a.skip[h] : 0.f;
 #pragma unroll
-  for (int j = 0; j < 4; ++j) {
-    const int t = j * 16 + fr;
-    f32x4_t y = f32x4_t{0.f, 0.f, 0.f, 0.f};
+  for (int th = 0; th < NH; ++th) {
+    if (th * 64 >= len) break;                    // block-uniform
+    __syncthreads();                              // the query tile, or the scores of the half before, are no longer read
 #pragma unroll
-    for (int kb = 0; kb < SL / 32; ++kb)
-      if (kb * 2 <= j) {
-        float x[8];
-        load8(ps + t * PS + kb * 32 + g * 8, x);
-        y = mma(vf[kb], wide_frag<T>(x), y);
+    for (int k = 0; k <= th; ++k)
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        // weighted scores of keys 64 k + 16 wid + 4 g + r and token 64 th + 16 j + fr
+        const int t = th * 64 + j * 16 + fr;
+        const double Ft = F_s[t];
+        f32x4_t w = st[k][th][j];
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const int s = k * 64 + wid * 16 + g * 4 + r;
+          float e = 0.f;
+          if (s <= t && t < len) {
+            if constexpr (STAB) e = expf(static_cast<float>(Ft - F_s[s] + static_cast<double>(in_s[s] - m_s[t])));
+            else e = expf(static_cast<float>(Ft - F_s[s])) * in_s[s];
+          }
+          w[r] *= e * a.qscale;
+        }
+        *reinterpret_cast<f32x4_t*>(ps + (j * 16 + fr) * PS + k * 64 + wid * 16 + g * 4) = w;
       }
-    if (t >= len) continue;
-    const float carry = expf(static_cast<float>(F_s[t] + static_cast<double>(m0 - (STAB ? m_s[t] : 0.f)))) * a.qscale;
-    y += inter[j] * carry;
-    if constexpr (STAB) y *= inv_s[t];
-    const int v = wid * 16 + g * 4;
-    if (a.skip) {
+    __syncthreads();
+    if constexpr (STAB) {
+      const int tl = tid >> 2, t = th * 64 + tl;
+      float den = 0.f;
 #pragma unroll
-      for (int r = 0; r < 4; ++r) y[r] += skip * to_f32(vt[(v + r) * TS + t]);
+      for (int k = 0; k <= th; ++k)
+#pragma unroll
+        for (int i = 0; i < 16; i += 4) {
+          const f32x4_t x = *reinterpret_cast<const f32x4_t*>(ps + tl * PS + k * 64 + (tid & 3) * 16 + i);
+          den += x[0] + x[1] + x[2] + x[3];
+        }
+      den += nq[th] * expf(static_cast<float>(F_s[t] + static_cast<double>(m0 - m_s[t]))) * a.qscale;
+      den += __shfl_xor(den, 1, 64);
+      den += __shfl_xor(den, 2, 64);
+      if ((tid & 3) == 0) inv_s[tl] = 1.f / (fmaxf(fabsf(den), expf(-m_s[t])) + 1e-6f);
+      __syncthreads();
     }
-    store4(static_cast<T*>(a.out) + (static_cast<long long>(row0 + t) * a.H + h) * a.V + v0 + v, y[0], y[1], y[2], y[3]);
+    if (!rows_v) continue;
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      const int tl = j * 16 + fr, t = th * 64 + tl;
+      f32x4_t y = f32x4_t{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int kb = 0; kb < SL / 32; ++kb)
+        if (kb < 2 * th || (kb < 2 * th + 2 && (kb - 2 * th) * 2 <= j)) {
+          float x[8];
+          load8(ps + tl * PS + kb * 32 + g * 8, x);
+          y = mma(vf[kb], wide_frag<T>(x), y);
+        }
+      if (t >= len) continue;
+      y += inter[th][j] * (expf(static_cast<float>(F_s[t] + static_cast<double>(m0 - m_s[t]))) * a.qscale);
+      if constexpr (STAB) y *= inv_s[tl];
+      const int v = wid * 16 + g * 4;
+      if (a.skip) {
+#pragma unroll
+        for (int r = 0; r < 4; ++r) y[r] += skip * to_f32(vt[(v + r) * TS + t]);
+      }
+      store4(static_cast<T*>(a.out) + (static_cast<long long>(row0 + t) * a.H + h) * a.V + v0 + v, y[0], y[1], y[2], y[3]);
+    }
   }
 }
 
-void launch_scan_prefill(const ScanArgs& a, const ScanChunks& c, bool f32, hipStream_t st) {
-  const int vt = (a.V + 63) / 64;
-  const bool stab = a.log_in != nullptr;
-  const dim3 g1(vt, a.H, c.C), g3(vt, a.H, c.C);
+template <typename T, bool STAB>
+static void launch_scan(const ScanArgs& a, const ScanChunks& c, hipStream_t st) {
+  constexpr int SL = sizeof(T) == 2 ? SCAN_CHUNK_BF16 : SCAN_CHUNK_F32;
+  const dim3 g1((a.V + 63) / 64, a.H, c.C), block(256);
   const long long quads = static_cast<long long>(a.V) * a.N / 4;
-  const dim3 g2(static_cast<unsigned>((quads + 255) / 256) + (stab ? 1 : 0), a.H, c.nseq);
+  const dim3 g2(static_cast<unsigned>((quads + 255) / 256) + (STAB ? 1 : 0), a.H, c.nseq);
+  hipLaunchKernelGGL((scan_chunk_state_kernel<T, STAB, SL>), g1, block, 0, st, a, c);
+  hipLaunchKernelGGL(scan_chunk_pass_kernel<STAB>, g2, block, 0, st, a, c);
+  hipLaunchKernelGGL((scan_chunk_out_kernel<T, STAB, SL>), g1, block, 0, st, a, c);
+}
+void launch_scan_prefill(const ScanArgs& a, const ScanChunks& c, bool f32, hipStream_t st) {
+  const bool stab = a.log_in != nullptr;
   if (f32) {
-    if (stab) hipLaunchKernelGGL((scan_chunk_state_kernel<float, true>), g1, dim3(256), 0, st, a, c);
-    else hipLaunchKernelGGL((scan_chunk_state_kernel<float, false>), g1, dim3(256), 0, st, a, c);
+    if (stab) launch_scan<float, true>(a, c, st);
+    else launch_scan<float, false>(a, c, st);
   } else {
-    if (stab) hipLaunchKernelGGL((scan_chunk_state_kernel<bf16_t, true>), g1, dim3(256), 0, st, a, c);
-    else hipLaunchKernelGGL((scan_chunk_state_kernel<bf16_t, false>), g1, dim3(256), 0, st, a, c);
-  }
-  if (stab) hipLaunchKernelGGL(scan_chunk_pass_kernel<true>, g2, dim3(256), 0, st, a, c);
-  else hipLaunchKernelGGL(scan_chunk_pass_kernel<false>, g2, dim3(256), 0, st, a, c);
-  if (f32) {
-    if (stab) hipLaunchKernelGGL((scan_chunk_out_kernel<float, true>), g3, dim3(256), 0, st, a, c);
-    else hipLaunchKernelGGL((scan_chunk_out_kernel<float, false>), g3, dim3(256), 0, st, a, c);
-  } else {
-    if (stab) hipLaunchKernelGGL((scan_chunk_out_kernel<bf16_t, true>), g3, dim3(256), 0, st, a, c);
-    else hipLaunchKernelGGL((scan_chunk_out_kernel<bf16_t, false>), g3, dim3(256), 0, st, a, c);
+    if (stab) launch_scan<bf16_t, true>(a, c, st);
+    else launch_scan<bf16_t, false>(a, c, st);
   }
 }
 

@@ -237,6 +237,9 @@ __global__ __launch_bounds__(256) void row_gemv_kernel(GemvCall call, int blocks
   }
 }
 
+static int g_blocks = 0;
+void row_gemv_blocks(int n) { g_blocks = n > 0 ? n : 0; }
+
 static int blocks_of(const GemvProblem& p, int budget) {
   const int units = p.N / GV_R;
   return units < budget ? units : budget;
@@ -253,8 +256,12 @@ size_t row_gemv_lds(const GemvCall& c, bool f32, int B) {
 }
 template <typename T, int B>
 static void launch_b(const GemvCall& c, size_t lds, hipStream_t st) {
-  // four to eight blocks per CU: enough waves to stream, few enough that the inputs are not prepared too often
-  const int budget = 1280;
+  // two or three blocks per CU: enough waves to stream, few enough that the inputs are not prepared too often.  Width 4096,
+  // us at 256 / 512 / 768 / 1280 / 2048 blocks: one row, norm + 18560 rows 38.5 / 26.5 / 26.8 / 28.9 / 29.9, merge + gate/up
+  // 45.8 / 33.4 / 35.4 / 40.2 / 42.0, two output projections 19.8 / 18.3 / 15.9 / 18.0 / 21.3; four rows, norm + 18560 rows
+  // 58.9 / 38.8 / 34.6 / 41.6 / 47.4
+  const int kind = c.p[0].in.kind;
+  const int budget = g_blocks ? g_blocks : (B == 1 && c.count == 1 && (kind == GV_NORM || kind == GV_MERGE) ? 512 : 768);
   const int b0 = blocks_of(c.p[0], c.count == 2 ? budget / 2 : budget), b1 = c.count == 2 ? blocks_of(c.p[1], budget / 2) : 0;
   const dim3 grid(b0 + b1), block(256);
   const bool plain = c.count == 1 && c.p[0].in.kind == GV_PLAIN;

@@ -268,51 +268,54 @@ void launch_group_norm_rows(const SrcRows& y, const SrcRows& gate, int gcol, int
   else launch_group_norm<bf16_t>(y, gate, gcol, mode, w, out, rows, heads, v, vp, parts, ld_out, eps, st);
 }
 
-// First index of the row's maximum (NaN never wins).
-__global__ __launch_bounds__(1024) void argmax_logits_kernel(const float* __restrict__ logits, long long ld,
-                                                             int* __restrict__ out, int vocab) {
+// Commit of one token per sequence, as commit_token_kernel does it, staging the scaled embedding row as
+// the fp32 residual stream of the next step.  With logits: the first index of the row's maximum (NaN never
+// wins), eight candidates per thread and pass in flight.
+template <typename T>
+__global__ __launch_bounds__(1024) void commit_rows_kernel(const float* __restrict__ logits, long long ld_logits,
+                                                           int* __restrict__ sampled, const T* __restrict__ embed,
+                                                           float scale, float* __restrict__ x, int* __restrict__ out_tokens,
+                                                           int max_out, int* __restrict__ step, int* __restrict__ pos,
+                                                           int* __restrict__ done, int* __restrict__ cur_token, int eos,
+                                                           int ld, int vocab, const int* __restrict__ active) {
   __shared__ float sv[16];
   __shared__ int si[16];
-  const float* r = logits + blockIdx.x * ld;
-  float bv = -INFINITY;
-  int bi = 0x7fffffff;
-  for (int i = threadIdx.x; i < vocab; i += 1024) {
-    const float v = r[i];
-    if (v > bv || (v == bv && i < bi)) { bv = v; bi = i; }
-  }
-#pragma unroll
-  for (int off = 32; off > 0; off >>= 1) {
-    const float ov = __shfl_xor(bv, off, 64);
-    const int oi = __shfl_xor(bi, off, 64);
-    if (ov > bv || (ov == bv && oi < bi)) { bv = ov; bi = oi; }
-  }
-  const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
-  if (lane == 0) { sv[wid] = bv; si[wid] = bi; }
-  __syncthreads();
-  if (threadIdx.x == 0) {
-    for (int w = 1; w < 16; ++w)
-      if (sv[w] > bv || (sv[w] == bv && si[w] < bi)) { bv = sv[w]; bi = si[w]; }
-    out[blockIdx.x] = bi == 0x7fffffff ? 0 : bi;
-  }
-}
-void launch_argmax_logits(const float* logits, long long ld, int* out, int rows, int vocab, hipStream_t st) {
-  hipLaunchKernelGGL(argmax_logits_kernel, dim3(rows), dim3(1024), 0, st, logits, ld, out, vocab);
-}
-
-// Commit of one token per sequence, as commit_token_kernel does it, staging the scaled embedding row as
-// the fp32 residual stream of the next step.
-template <typename T>
-__global__ __launch_bounds__(256) void commit_rows_kernel(const int* __restrict__ sampled, const T* __restrict__ embed,
-                                                          float scale, float* __restrict__ x,
-                                                          int* __restrict__ out_tokens, int max_out,
-                                                          int* __restrict__ step, int* __restrict__ pos,
-                                                          int* __restrict__ done, int* __restrict__ cur_token, int eos,
-                                                          int ld, int vocab, const int* __restrict__ active) {
+  __shared__ int tok_s;
   const int b = blockIdx.x;
   if (active && !active[b]) return;
-  int tok = sampled[b];
+  if (logits) {
+    const float* r = logits + b * ld_logits;
+    float bv = -INFINITY;
+    int bi = 0x7fffffff;
+    constexpr int U = 8;
+    for (int i0 = threadIdx.x; i0 < vocab; i0 += 1024 * U) {
+      float v[U];
+#pragma unroll
+      for (int u = 0; u < U; ++u) v[u] = r[min(i0 + u * 1024, vocab - 1)];
+#pragma unroll
+      for (int u = 0; u < U; ++u)
+        if (i0 + u * 1024 < vocab && v[u] > bv) { bv = v[u]; bi = i0 + u * 1024; }    // a thread's indices ascend
+    }
+#pragma unroll
+    for (int off = 32; off > 0; off >>= 1) {
+      const float ov = __shfl_xor(bv, off, 64);
+      const int oi = __shfl_xor(bi, off, 64);
+      if (ov > bv || (ov == bv && oi < bi)) { bv = ov; bi = oi; }
+    }
+    const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
+    if (lane == 0) { sv[wid] = bv; si[wid] = bi; }
+    __syncthreads();
+    if (threadIdx.x == 0) {
+      for (int w = 1; w < 16; ++w)
+        if (sv[w] > bv || (sv[w] == bv && si[w] < bi)) { bv = sv[w]; bi = si[w]; }
+      tok_s = bi == 0x7fffffff ? 0 : bi;
+      sampled[b] = tok_s;
+    }
+    __syncthreads();
+  }
+  int tok = logits ? tok_s : sampled[b];
   if (tok < 0 || tok >= vocab) tok = 0;
-  for (int c = threadIdx.x * 8; c < ld; c += 2048) {
+  for (int c = threadIdx.x * 8; c < ld; c += blockDim.x * 8) {
     float v[8];
     load8(embed + static_cast<long long>(tok) * ld + c, v);
 #pragma unroll
@@ -328,43 +331,45 @@ __global__ __launch_bounds__(256) void commit_rows_kernel(const int* __restrict_
     pos[b] = pos[b] + 1;
   }
 }
-void launch_commit_rows(const int* sampled, const void* embed, bool f32, float scale, float* x, int* out_tokens,
-                        int max_out, int* step, int* pos, int* done, int* cur_token, int eos, int B, int ld, int vocab,
-                        const int* active, hipStream_t st) {
+void launch_commit_rows(const float* logits, long long ld_logits, int* sampled, const void* embed, bool f32, float scale,
+                        float* x, int* out_tokens, int max_out, int* step, int* pos, int* done, int* cur_token, int eos, int B,
+                        int ld, int vocab, const int* active, hipStream_t st) {
+  const dim3 grid(B), block(logits ? 1024 : 256);
   if (f32)
-    hipLaunchKernelGGL(commit_rows_kernel<float>, dim3(B), dim3(256), 0, st, sampled, static_cast<const float*>(embed),
-                       scale, x, out_tokens, max_out, step, pos, done, cur_token, eos, ld, vocab, active);
+    hipLaunchKernelGGL(commit_rows_kernel<float>, grid, block, 0, st, logits, ld_logits, sampled,
+                       static_cast<const float*>(embed), scale, x, out_tokens, max_out, step, pos, done, cur_token, eos, ld,
+                       vocab, active);
   else
-    hipLaunchKernelGGL(commit_rows_kernel<bf16_t>, dim3(B), dim3(256), 0, st, sampled,
-                       static_cast<const bf16_t*>(embed), scale, x, out_tokens, max_out, step, pos, done, cur_token,
-                       eos, ld, vocab, active);
+    hipLaunchKernelGGL(commit_rows_kernel<bf16_t>, grid, block, 0, st, logits, ld_logits, sampled,
+                       static_cast<const bf16_t*>(embed), scale, x, out_tokens, max_out, step, pos, done, cur_token, eos, ld,
+                       vocab, active);
 }
 
-// Attention inputs of one row.
-template <typename T>
+// Attention inputs of one row.  The q and k sections are read once, into LDS (STAGED; rows too wide for it are read
+// again instead), where an element finds the one it is rotated with.
+template <typename T, bool STAGED>
 __global__ __launch_bounds__(256) void attn_prep_kernel(AttnPrepArgs a) {
+  extern __shared__ __attribute__((aligned(16))) float row_lds[];     // q section, k section
   __shared__ float red[16];
   const long long row = blockIdx.x;
   const int qn = a.Hq * a.D, kn = a.Hkv * a.D, half = a.rot >> 1;
-  float rq = 1.f, rk = 1.f;
-  if (a.qw) {
-    float s = 0.f;
-    for (int c = threadIdx.x * 8; c < qn; c += 2048) {
-      float t[8];
-      src8(a.src, row, a.q_col + c, t);
-      s += sumsq8(t);
-    }
-    rq = rsqrtf(block_sum(s, red) / static_cast<float>(a.nq) + a.eps);
+  float sq = 0.f, sk = 0.f;
+  for (int c = threadIdx.x * 8; c < qn; c += 2048) {
+    float t[8];
+    src8(a.src, row, a.q_col + c, t);
+    sq += sumsq8(t);
+    if constexpr (STAGED) store8(row_lds + c, t);
   }
-  if (a.kw) {
-    float s = 0.f;
-    for (int c = threadIdx.x * 8; c < kn; c += 2048) {
-      float t[8];
-      src8(a.src, row, a.k_col + c, t);
-      s += sumsq8(t);
-    }
-    rk = rsqrtf(block_sum(s, red) / static_cast<float>(a.nk) + a.eps);
+  for (int c = threadIdx.x * 8; c < kn; c += 2048) {
+    float t[8];
+    src8(a.src, row, a.k_col + c, t);
+    sk += sumsq8(t);
+    if constexpr (STAGED) store8(row_lds + qn + c, t);
   }
+  // (the sums' barriers also publish the staged row)
+  const float rq = a.qw ? rsqrtf(block_sum(sq, red) / static_cast<float>(a.nq) + a.eps) : 1.f;
+  const float rk = a.kw ? rsqrtf(block_sum(sk, red) / static_cast<float>(a.nk) + a.eps) : 1.f;
+  __syncthreads();
   const int p = a.row_pos[row];
   const int pt = min(max(p, 0), a.max_pos - 1);
   const float* cs = a.cos_tab + static_cast<long long>(pt) * half;
@@ -373,86 +378,72 @@ __global__ __launch_bounds__(256) void attn_prep_kernel(AttnPrepArgs a) {
   const bool keep = a.row_keep == nullptr || a.row_keep[row] != 0;
   const long long kv = a.row_kv ? a.row_kv[row] : -1;
   const int cslot = p % a.cap;
-  // normalised and rotated element d of head h of a section
-  auto value = [&](int col, const float* w, float r, int h, int d) {
-    const int c = h * a.D + d;
-    float u = src1(a.src, row, col + c) * r;
-    if (w) u *= w[c];
-    if (d < a.rot) {
-      const int i = d < half ? d : d - half, c2 = d < half ? c + half : c - half;
-      float o = src1(a.src, row, col + c2) * r;
-      if (w) o *= w[c2];
-      u = d < half ? u * cs[i] - o * sn[i] : u * cs[i] + o * sn[i];
-    }
-    return u;
-  };
-  T* q = static_cast<T*>(a.q_out) + row * qn;
-  if ((half & 7) == 0) {
-    // eight elements of a head at a time, with the eight they are paired with
-    auto value8 = [&](int col, const float* w, float r, int c, float (&u)[8]) {
-      const int d = c % a.D;
-      src8(a.src, row, col + c, u);
+  // normalised and rotated elements c .. c + 7 (of one head) of a section
+  auto value8 = [&](int col, int lds0, const float* w, float r, int c, float (&u)[8]) {
+    const int d = c % a.D;
+    auto raw1 = [&](int e) {
+      const float v = STAGED ? row_lds[lds0 + e] : src1(a.src, row, col + e);
+      return w ? v * r * w[e] : v * r;
+    };
+    auto raw8 = [&](int e, float (&v)[8]) {
+      if constexpr (STAGED) load8(row_lds + lds0 + e, v);
+      else src8(a.src, row, col + e, v);
       float g[8];
-      if (w) {
-        load8(w + c, g);
+      if (w) load8(w + e, g);
 #pragma unroll
-        for (int i = 0; i < 8; ++i) u[i] *= r * g[i];
-      }
-      if (d >= a.rot) return;
+      for (int i = 0; i < 8; ++i) v[i] *= w ? r * g[i] : r;
+    };
+    raw8(c, u);
+    if (d >= a.rot) return;
+    if ((half & 7) == 0) {
       const bool lo = d < half;
-      const int c2 = lo ? c + half : c - half, i0 = lo ? d : d - half;
+      const int i0 = lo ? d : d - half;
       float o[8], cc[8], ss[8];
-      src8(a.src, row, col + c2, o);
-      if (w) {
-        load8(w + c2, g);
-#pragma unroll
-        for (int i = 0; i < 8; ++i) o[i] *= r * g[i];
-      }
+      raw8(lo ? c + half : c - half, o);
       load8(cs + i0, cc);
       load8(sn + i0, ss);
 #pragma unroll
       for (int i = 0; i < 8; ++i) u[i] = lo ? u[i] * cc[i] - o[i] * ss[i] : u[i] * cc[i] + o[i] * ss[i];
-    };
-    for (int c = threadIdx.x * 8; c < qn; c += 2048) {
-      float u[8];
-      value8(a.q_col, a.qw, rq, c, u);
-      store8(q + c, u);
-    }
-    for (int c = threadIdx.x * 8; c < kn; c += 2048) {
-      float u[8], v[8];
-      value8(a.k_col, a.kw, rk, c, u);
-      src8(a.src, row, a.v_col + c, v);
-      if (kv >= 0) {
-        store8(static_cast<T*>(a.k_buf) + kv * kn + c, u);
-        store8(static_cast<T*>(a.v_buf) + kv * kn + c, v);
-      }
-      if (keep) {
-        const long long o = ((slot * a.Hkv + c / a.D) * a.cap + cslot) * a.D + c % a.D;
-        store8(static_cast<T*>(a.k_cache) + o, u);
-        store8(static_cast<T*>(a.v_cache) + o, v);
+    } else {
+#pragma unroll
+      for (int i = 0; i < 8; ++i) {
+        const int e = d + i;
+        if (e < half) u[i] = u[i] * cs[e] - raw1(c + i + half) * sn[e];
+        else if (e < a.rot) u[i] = u[i] * cs[e - half] + raw1(c + i - half) * sn[e - half];
       }
     }
-    return;
+  };
+  T* q = static_cast<T*>(a.q_out) + row * qn;
+  for (int c = threadIdx.x * 8; c < qn; c += 2048) {
+    float u[8];
+    value8(a.q_col, 0, a.qw, rq, c, u);
+    store8(q + c, u);
   }
-  for (int c = threadIdx.x; c < qn; c += 256) q[c] = from_f32<T>(value(a.q_col, a.qw, rq, c / a.D, c % a.D));
-  for (int c = threadIdx.x; c < kn; c += 256) {
-    const int h = c / a.D, d = c % a.D;
-    const T kk = from_f32<T>(value(a.k_col, a.kw, rk, h, d));
-    const T vv = from_f32<T>(src1(a.src, row, a.v_col + c));
+  for (int c = threadIdx.x * 8; c < kn; c += 2048) {
+    float u[8], v[8];
+    value8(a.k_col, qn, a.kw, rk, c, u);
+    src8(a.src, row, a.v_col + c, v);
     if (kv >= 0) {
-      static_cast<T*>(a.k_buf)[kv * kn + c] = kk;
-      static_cast<T*>(a.v_buf)[kv * kn + c] = vv;
+      store8(static_cast<T*>(a.k_buf) + kv * kn + c, u);
+      store8(static_cast<T*>(a.v_buf) + kv * kn + c, v);
     }
     if (keep) {
-      const long long o = ((slot * a.Hkv + h) * a.cap + cslot) * a.D + d;
-      static_cast<T*>(a.k_cache)[o] = kk;
-      static_cast<T*>(a.v_cache)[o] = vv;
+      const long long o = ((slot * a.Hkv + c / a.D) * a.cap + cslot) * a.D + c % a.D;
+      store8(static_cast<T*>(a.k_cache) + o, u);
+      store8(static_cast<T*>(a.v_cache) + o, v);
     }
   }
 }
 void launch_attn_prep(const AttnPrepArgs& a, bool f32, int rows, hipStream_t st) {
-  if (f32) hipLaunchKernelGGL(attn_prep_kernel<float>, dim3(rows), dim3(256), 0, st, a);
-  else hipLaunchKernelGGL(attn_prep_kernel<bf16_t>, dim3(rows), dim3(256), 0, st, a);
+  const size_t lds = static_cast<size_t>(a.Hq + a.Hkv) * a.D * 4;
+  const bool staged = lds <= 64 * 1024;
+  if (f32) {
+    if (staged) hipLaunchKernelGGL((attn_prep_kernel<float, true>), dim3(rows), dim3(256), lds, st, a);
+    else hipLaunchKernelGGL((attn_prep_kernel<float, false>), dim3(rows), dim3(256), 0, st, a);
+  } else {
+    if (staged) hipLaunchKernelGGL((attn_prep_kernel<bf16_t, true>), dim3(rows), dim3(256), lds, st, a);
+    else hipLaunchKernelGGL((attn_prep_kernel<bf16_t, false>), dim3(rows), dim3(256), 0, st, a);
+  }
 }
 
 template <typename T>

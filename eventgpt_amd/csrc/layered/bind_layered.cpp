@@ -198,14 +198,8 @@ Tensor group_norm_rows(const Tensor& y, const OptTensor& gate, int64_t gcol, int
                                   (int)v, (int)vp, (int)parts, (int)ld_out, (float)eps, cur_stream());
   return o;
 }
-void argmax_logits_(const Tensor& logits, const Tensor& out, int64_t vocab) {
-  TORCH_CHECK(logits.is_cuda() && logits.dim() == 2 && is_f32(logits) && logits.stride(1) == 1, "logits: fp32 [B, V]");
-  check_i(out, "out");
-  TORCH_CHECK(vocab >= 1 && vocab <= logits.size(1) && out.numel() >= logits.size(0), "argmax_logits: sizes");
-  evgpt::launch_argmax_logits(logits.data_ptr<float>(), logits.stride(0), out.data_ptr<int>(), (int)logits.size(0),
-                              (int)vocab, cur_stream());
-}
-void commit_rows_(const Tensor& sampled, const Tensor& embed, double scale, const Tensor& x, const Tensor& out_tokens,
+// logits [B, >= V] fp32: greedy, `sampled` receives the tokens; without: `sampled` holds them
+void commit_rows_(const OptTensor& logits, const Tensor& sampled, const Tensor& embed, double scale, const Tensor& x, const Tensor& out_tokens,
                   const Tensor& step, const Tensor& pos, const Tensor& done, const Tensor& cur, int64_t eos,
                   const OptTensor& active) {
   check_i(sampled, "sampled"); check_t(embed, "embed"); check_f(x, "x"); check_i(out_tokens, "out_tokens");
@@ -215,7 +209,10 @@ void commit_rows_(const Tensor& sampled, const Tensor& embed, double scale, cons
   TORCH_CHECK(sampled.numel() >= B && step.numel() >= B && pos.numel() >= B && done.numel() >= B && cur.numel() >= B &&
               out_tokens.dim() == 2 && out_tokens.size(0) >= B, "commit_rows: per-sequence buffers");
   if (active.has_value()) { check_i(*active, "active"); TORCH_CHECK(active->numel() >= B, "active"); }
-  evgpt::launch_commit_rows(sampled.data_ptr<int>(), embed.data_ptr(), is_f32(embed), (float)scale, x.data_ptr<float>(),
+  if (logits.has_value())
+    TORCH_CHECK(logits->is_cuda() && logits->dim() == 2 && is_f32(*logits) && logits->stride(1) == 1 && logits->size(0) == B &&
+                logits->size(1) >= embed.size(0), "commit_rows: logits [B, V] fp32");
+  evgpt::launch_commit_rows(fptr(logits), logits.has_value() ? logits->stride(0) : 0, sampled.data_ptr<int>(), embed.data_ptr(), is_f32(embed), (float)scale, x.data_ptr<float>(),
                             out_tokens.data_ptr<int>(), (int)out_tokens.size(1), step.data_ptr<int>(), pos.data_ptr<int>(),
                             done.data_ptr<int>(), cur.data_ptr<int>(), (int)eos, (int)B, (int)x.size(1),
                             (int)embed.size(0), iptr(active), cur_stream());
@@ -652,8 +649,7 @@ TORCH_LIBRARY(evlay, m) {
   m.def("merge_norm_rows_(Tensor(a!) x, Tensor a, Tensor b, Tensor wa, Tensor wb, Tensor? w, int n, float eps, bool f32) -> Tensor", &merge_norm_rows_);
   m.def("glu_rows(Tensor src, int act, bool f32) -> Tensor", &glu_rows);
   m.def("group_norm_rows(Tensor y, Tensor? gate, int gcol, int gate_mode, Tensor w, int heads, int v, int vp, int parts, int ld_out, float eps, bool f32) -> Tensor", &group_norm_rows);
-  m.def("argmax_logits_(Tensor logits, Tensor(a!) out, int vocab) -> ()", &argmax_logits_);
-  m.def("commit_rows_(Tensor sampled, Tensor embed, float scale, Tensor(a!) x, Tensor(b!) out_tokens, Tensor(c!) step, Tensor(d!) pos, Tensor(e!) done, Tensor(f!) cur_token, int eos, Tensor? active) -> ()", &commit_rows_);
+  m.def("commit_rows_(Tensor? logits, Tensor(g!) sampled, Tensor embed, float scale, Tensor(a!) x, Tensor(b!) out_tokens, Tensor(c!) step, Tensor(d!) pos, Tensor(e!) done, Tensor(f!) cur_token, int eos, Tensor? active) -> ()", &commit_rows_);
   m.def("sample_top_p(Tensor logits, Tensor(a!) out, float temperature, float top_p, int seed, Tensor step, int top_k=0) -> ()", &sample_top_p);
   m.def("attn_prep_(Tensor src, int q_col, int k_col, int v_col, Tensor? qw, Tensor? kw, int Hq, int Hkv, int D, int nq, int nk, float eps, Tensor cos, Tensor sin, Tensor? row_slot, Tensor row_pos, Tensor? row_kv, Tensor? row_keep, Tensor(a!)? k_buf, Tensor(b!)? v_buf, Tensor(c!) k_cache, Tensor(d!) v_cache) -> Tensor", &attn_prep_);
   m.def("chunk_keys_copy_(Tensor k_cache, Tensor v_cache, Tensor(a!) k_buf, Tensor(b!) v_buf, Tensor copies) -> ()", &chunk_keys_copy_);
@@ -667,6 +663,8 @@ TORCH_LIBRARY(evlay, m) {
   m.def("gemv_add_(Tensor(a!) x, Tensor w, Tensor h) -> ()", &gemv_add_);
   m.def("gemv_group_add_(Tensor(a!) x, Tensor w, Tensor y, Tensor norm, int heads, int v, int vp, int parts, float eps) -> ()", &gemv_group_add_);
   m.def("gemv_branches(Tensor wa, Tensor h, Tensor wb, Tensor y, Tensor gate, int gcol, Tensor norm, int heads, int v, int vp, float eps) -> Tensor", &gemv_branches);
+  m.def("gemv_blocks(int n) -> ()", [](int64_t n) { evgpt::row_gemv_blocks((int)n); });
+  m.def("scan_chunk(bool f32) -> int", [](bool f32) { return (int64_t)(f32 ? evgpt::SCAN_CHUNK_F32 : evgpt::SCAN_CHUNK_BF16); });
   m.def("gemv_rows_max() -> int", &gemv_rows_max);
   m.def("gemv_lds_bytes() -> int", &gemv_lds_bytes);
   m.def("mlstm_gates(Tensor src, int i_col, int f_col, Tensor ib, Tensor fb, float cap) -> (Tensor, Tensor)", &mlstm_gates);

@@ -42,8 +42,9 @@ void launch_glu_rows(const SrcRows& src, void* h, bool f32, int rows, int ip, in
 enum { GATE_NONE = 0, GATE_SILU_BEFORE = 1, GATE_SIGMOID_AFTER = 2 };
 void launch_group_norm_rows(const SrcRows& y, const SrcRows& gate, int gcol, int mode, const float* w, void* out, bool f32,
                             int rows, int heads, int v, int vp, int parts, int ld_out, float eps, hipStream_t st);
-void launch_argmax_logits(const float* logits, long long ld, int* out, int rows, int vocab, hipStream_t st);
-void launch_commit_rows(const int* sampled, const void* embed, bool f32, float scale, float* x, int* out_tokens,
+// Commit of one token per sequence: the first maximum of its logits, or sampled[b] when logits is null.  `sampled`
+// receives the token either way.
+void launch_commit_rows(const float* logits, long long ld_logits, int* sampled, const void* embed, bool f32, float scale, float* x, int* out_tokens,
                         int max_out, int* step, int* pos, int* done, int* cur_token, int eos, int B, int ld, int vocab,
                         const int* active, hipStream_t st);
 
@@ -103,7 +104,7 @@ struct ScanArgs {
   int slots;
 };
 struct ScanChunks {
-  // [C][4]: first row, rows (<= 64), slot, flags (bit 0: the sequence's last chunk, bit 1: parity of the next position)
+  // [C][4]: first row, rows (<= the chunk), slot, flags (bit 0: the sequence's last chunk, bit 1: parity of the next position)
   const int* chunks;
   // [nseq][4]: first chunk, chunks, slot, flags (bit 0: from position 0, bits 1 and 2: parities of start and end)
   const int* seqs;
@@ -113,7 +114,7 @@ struct ScanChunks {
   double* am; double* fl;          // [C][H]
   float* m0;                       // [C][H]
 };
-constexpr int SCAN_CHUNK = 64;
+constexpr int SCAN_CHUNK_BF16 = 128, SCAN_CHUNK_F32 = 64;      // tokens per chunk
 void launch_scan_prefill(const ScanArgs& a, const ScanChunks& c, bool f32, hipStream_t st);
 // log gates of the matrix memory: cap * tanh((x + b) / cap), and the log sigmoid of it for the forget gate
 void launch_mlstm_gates(const SrcRows& src, int i_col, int f_col, const float* ib, const float* fb, float cap, float* li,
@@ -182,6 +183,7 @@ struct GemvCall {
   void* h;                         // GLU: [B][N / 2] of T (W is [gate rows | up rows])
   int act;
 };
+void row_gemv_blocks(int n);       // workgroups of a launch (0: the default); for tuning runs
 constexpr int GEMV_ROWS_MAX = 4;
 size_t row_gemv_lds(const GemvCall& c, bool f32, int B);     // bytes of LDS the call needs
 void launch_row_gemv(const GemvCall& c, bool f32, int B, hipStream_t st);

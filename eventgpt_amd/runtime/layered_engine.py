@@ -52,6 +52,7 @@ class LayeredEngine(DecodeEngine):
         self.V = cfg.vocab_size
         # decode steps of up to this many sequences run on the weight-streaming kernels, more on the few-row GEMM
         self.gemv_rows = int(self.raw.gemv_rows_max())
+        self.scan_chunk = int(self.raw.scan_chunk(self.f32))
         self.gemv_lds = int(self.raw.gemv_lds_bytes())
         if self.wp * (4 if self.f32 else 2) * min(self.B, self.gemv_rows) > self.gemv_lds:
             self.gemv_rows = 0
@@ -113,13 +114,16 @@ class LayeredEngine(DecodeEngine):
         if not greedy or want_logits:
             self.logits.copy_(logits)
         if greedy:
-            self.raw.argmax_logits_(logits, self.sampled, self.V)
-            self._commit_sampled()
+            self._commit(logits)
 
     _stream: Optional[Stream] = None
 
     def _commit_sampled(self) -> None:
-        self.raw.commit_rows_(self.sampled, self.embed, self.cfg.embedding_scale, self.x, self.out_tokens, self.step,
+        self._commit(None)
+
+    def _commit(self, logits: Optional[torch.Tensor]) -> None:
+        """Commit ``sampled``, or the argmax of ``logits``, and stage the next token's embedding."""
+        self.raw.commit_rows_(logits, self.sampled, self.embed, self.cfg.embedding_scale, self.x, self.out_tokens, self.step,
                               self.pos, self.done, self.cur_token, self.eos, self.active)
 
     def _capture(self, fn):
@@ -149,7 +153,7 @@ class LayeredEngine(DecodeEngine):
             n += int(t.numel())
         flat = torch.cat([t.reshape(-1).to("cpu", torch.int32) if not t.is_cuda else t.reshape(-1).to(torch.int32) for t in ids])
         x = self.raw.embed_rows(flat.to(self.device).contiguous(), self.embed, self.cfg.embedding_scale)
-        stream = self._run_stages(RowBatch(self.device, False, seqs=seqs), x, collect)
+        stream = self._run_stages(RowBatch(self.device, False, seqs=seqs, scan_chunk=self.scan_chunk), x, collect)
         return stream.settle(), [s.row0 for s in seqs]
 
     def _packs(self, slots, ids, starts):

@@ -25,7 +25,6 @@ import torch
 
 from ..models.layered import AttentionSpec, DenseMLPSpec, MatrixMemorySpec, Mamba2Spec, ParallelSpec
 
-SCAN_CHUNK = 64          # tokens per chunk of the prefill kernels of the recurrences
 ATTN_TILE = 64           # query rows per work item of the chunk attention
 GATE_NONE, GATE_SILU_BEFORE, GATE_SIGMOID_AFTER = 0, 1, 2      # group_norm_rows
 
@@ -76,7 +75,8 @@ class RowBatch:
     shared by all layers."""
 
     def __init__(self, device, decode: bool, pos: Optional[torch.Tensor] = None, live: Optional[torch.Tensor] = None,
-                 seqs: Sequence[Sequence_] = ()):
+                 seqs: Sequence[Sequence_] = (), scan_chunk: int = 64):
+        """``scan_chunk``: tokens per chunk of the recurrences' prefill kernels (``raw.scan_chunk``)."""
         self.device, self.decode, self.live = device, decode, live
         self.seqs: List[Sequence_] = list(seqs)
         self._tables: Dict = {}
@@ -88,11 +88,11 @@ class RowBatch:
             slot += [s.slot] * s.rows
             ps += range(s.start, s.start + s.rows)
             first += [s.row0] * s.rows
-            n = -(-s.rows // SCAN_CHUNK)
+            n = -(-s.rows // scan_chunk)
             end = (s.start + s.rows) & 1
             seq_rows += [len(chunks) // 4, n, s.slot, int(s.start == 0) | (s.start & 1) << 1 | end << 2]
             for c in range(n):
-                chunks += [s.row0 + c * SCAN_CHUNK, min(SCAN_CHUNK, s.rows - c * SCAN_CHUNK), s.slot,
+                chunks += [s.row0 + c * scan_chunk, min(scan_chunk, s.rows - c * scan_chunk), s.slot,
                            int(c == n - 1) | end << 1]
             tails += [s.row0, s.rows, s.slot, s.start]
         self.slot, self.pos, self.first, self.chunks, self.scan_seqs, self.tails = self._upload(

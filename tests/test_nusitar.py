@@ -134,14 +134,14 @@ def test_chunk_tables_cover_every_query_once(size):
     assert all(n <= 64 for _, n, _, _ in items.tolist())
 
 
-def test_scan_tables():
+@pytest.mark.parametrize("L", [64, 128])
+def test_scan_tables(L):
     seqs = [Sequence_(3, 0, 130, 0), Sequence_(1, 130, 2, 50), Sequence_(0, 132, 64, 0)]
-    rb = RowBatch("cpu", False, seqs=seqs)
-    rb = RowBatch("cpu", False, seqs=seqs + [Sequence_(2, 196, 3, 7), Sequence_(4, 199, 1, 0)])
+    rb = RowBatch("cpu", False, seqs=seqs + [Sequence_(2, 196, 3, 7), Sequence_(4, 199, 1, 0)], scan_chunk=L)
     assert rb.tails.tolist() == [[0, 130, 3, 0], [130, 2, 1, 50], [132, 64, 0, 0], [196, 3, 2, 7], [199, 1, 4, 0]]
     assert rb.pos.tolist()[126:134] == [126, 127, 128, 129, 50, 51, 0, 1]
     # flags: first chunk from the zero state / last chunk of the sequence, and the parities of start and end
-    L, at = mixers.SCAN_CHUNK, 0
+    at = 0
     for (c0, n, slot, flags), s in zip(rb.scan_seqs.tolist(), rb.seqs):
         assert (c0, n, slot) == (at, -(-s.rows // L), s.slot)
         assert flags == int(s.start == 0) + 2 * (s.start % 2) + 4 * ((s.start + s.rows) % 2)
