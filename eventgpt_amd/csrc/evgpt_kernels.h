@@ -283,7 +283,8 @@ void launch_attn_prefill(const bf16_t* q, const bf16_t* k, const bf16_t* v, bf16
                          const long long* strides, const int* kv_len, int B, int Sq, int Sk,
                          int Hq, int Hkv, int D, int causal, int q_offset, int q_offset_from_len,
                          float scale, hipStream_t st, float* part_o = nullptr,
-                         float* part_ml = nullptr, int nsplit = 0, float* lse = nullptr);
+                         float* part_ml = nullptr, int nsplit = 0, float* lse = nullptr,
+                         bool wide_p = false);   // wide_p (causal): fp32 softmax weights in the second product
 
 // ---- attn_bwd.hip: flash-attention backward (recomputes P from the forward's LSE)
 // q/do/dq [B,Sq,Hq,D], k/v/dk/dv [B,Sk,Hkv,D], o [B,Sq,Hq,D], all contiguous bf16;

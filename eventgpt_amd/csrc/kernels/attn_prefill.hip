@@ -24,6 +24,11 @@
 
 namespace evgpt {
 
+// what rounding the pair to bf16 left out
+__device__ __forceinline__ unsigned int bf16_rest(float a, float b, unsigned int packed) {
+  return pack_bf16x2(a - bf16lo(packed), b - bf16hi(packed));
+}
+
 struct AttnParams {
   const bf16_t* q; const bf16_t* k; const bf16_t* v; bf16_t* o;
   long long q_sb, q_ss, q_sh;   // element strides: batch, sequence, head
@@ -48,7 +53,8 @@ struct AttnParams {
 // buffers, and group 1's running (max, sum, O) is merged into group 0's at the end through LDS.  A
 // few hundred query rows of a few heads are fewer blocks than CUs, each a serial chain over its key
 // tiles; two groups halve the chain and double the waves (used for the ViT, see launch_attn_prefill).
-template <int D, bool CAUSAL, bool SPLIT = false, int GROUPS = 1>
+// WP: the softmax weights enter the second product as two bf16 parts (16 mantissa bits) instead of one.
+template <int D, bool CAUSAL, bool SPLIT = false, int GROUPS = 1, bool WP = false>
 __global__ __launch_bounds__(256 * GROUPS) void attn_prefill_kernel(AttnParams p) {
   constexpr int CPR = D / 8;                  // 16-byte chunks per row
   constexpr int TILE_BYTES = TK * D * 2;
@@ -175,7 +181,7 @@ __global__ __launch_bounds__(256 * GROUPS) void attn_prefill_kernel(AttnParams p
     }
     const float ms = msafe * p.scale_log2e;
     float psum = 0.f;
-    unsigned int pk[4][2];
+    unsigned int pk[4][2], pl[4][2];
 #pragma unroll
     for (int n = 0; n < 4; ++n) {
       float e[4];
@@ -183,6 +189,10 @@ __global__ __launch_bounds__(256 * GROUPS) void attn_prefill_kernel(AttnParams p
       for (int r = 0; r < 4; ++r) { e[r] = __builtin_amdgcn_exp2f(fmaf(st[n][r], p.scale_log2e, -ms)); psum += e[r]; }
       pk[n][0] = pack_bf16x2(e[0], e[1]);
       pk[n][1] = pack_bf16x2(e[2], e[3]);
+      if constexpr (WP) {
+        pl[n][0] = bf16_rest(e[0], e[1], pk[n][0]);
+        pl[n][1] = bf16_rest(e[2], e[3], pk[n][1]);
+      }
     }
     l += psum;
 
@@ -192,6 +202,11 @@ __global__ __launch_bounds__(256 * GROUPS) void attn_prefill_kernel(AttnParams p
     for (int s = 0; s < 2; ++s) {
       u32x4_t pw = {pk[2 * s][0], pk[2 * s][1], pk[2 * s + 1][0], pk[2 * s + 1][1]};
       const bf16x8_t pf = __builtin_bit_cast(bf16x8_t, pw);
+      bf16x8_t pf_lo = pf;
+      if constexpr (WP) {
+        const u32x4_t lw = {pl[2 * s][0], pl[2 * s][1], pl[2 * s + 1][0], pl[2 * s + 1][1]};
+        pf_lo = __builtin_bit_cast(bf16x8_t, lw);
+      }
       const int q4 = fr >> 2, p4 = fr & 3;
       const int r0 = s * 32 + g * 4 + q4, r1 = r0 + 16;
 #pragma unroll
@@ -203,6 +218,8 @@ __global__ __launch_bounds__(256 * GROUPS) void attn_prefill_kernel(AttnParams p
             (s16x4_t __attribute__((address_space(3)))*)(v_lds + tile_off<D>(r1, ch) + 8 * (p4 & 1)));
         typedef __attribute__((ext_vector_type(8))) short s16x8_t;
         const s16x8_t vv = {lo[0], lo[1], lo[2], lo[3], hi[0], hi[1], hi[2], hi[3]};
+        if constexpr (WP)
+          o[dt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, vv), pf_lo, o[dt], 0, 0, 0);
         o[dt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, vv), pf,
                                                         o[dt], 0, 0, 0);
       }
@@ -302,7 +319,7 @@ constexpr int AW_STAGES = 4;   // K / V tiles in the LDS ring: three in flight w
 
 // AW_WAVES = 8: 256 query rows per block (long prompts); 4: 128 rows (a few hundred tokens, the ViT)
 // QT: 16-row query tiles per wave (2: every K / V fragment feeds two MFMAs; 1: twice the blocks)
-template <int D, bool CAUSAL, int AW_WAVES, int QT = 2>
+template <int D, bool CAUSAL, int AW_WAVES, int QT = 2, bool WP = false>
 __global__ __launch_bounds__(AW_WAVES * 64) void attn_prefill_wide_kernel(AttnParams p) {
   constexpr int CPR = D / 8;
   constexpr int TILE_BYTES = TK * D * 2;
@@ -381,7 +398,7 @@ __global__ __launch_bounds__(AW_WAVES * 64) void attn_prefill_wide_kernel(AttnPa
   // SIMD) run ONE BARRIER APART: while one half is in its MFMA phase the other is in its softmax,
   // so the SIMD's matrix and vector pipes work at the same time instead of taking turns.
   f32x4_t st[QT][4];
-  unsigned int pk[QT][4][2];
+  unsigned int pk[QT][4][2], pl[QT][WP ? 4 : 1][2];
   auto qk = [&](const unsigned char* k_lds) {
 #pragma unroll
     for (int n = 0; n < 4; ++n)
@@ -443,6 +460,10 @@ __global__ __launch_bounds__(AW_WAVES * 64) void attn_prefill_wide_kernel(AttnPa
         for (int r = 0; r < 4; ++r) { e[r] = __builtin_amdgcn_exp2f(fmaf(st[qt][n][r], p.scale_log2e, -ms)); psum += e[r]; }
         pk[qt][n][0] = pack_bf16x2(e[0], e[1]);
         pk[qt][n][1] = pack_bf16x2(e[2], e[3]);
+        if constexpr (WP) {
+          pl[qt][n][0] = bf16_rest(e[0], e[1], pk[qt][n][0]);
+          pl[qt][n][1] = bf16_rest(e[2], e[3], pk[qt][n][1]);
+        }
       }
       l[qt] += psum;
     }
@@ -450,9 +471,13 @@ __global__ __launch_bounds__(AW_WAVES * 64) void attn_prefill_wide_kernel(AttnPa
   auto pv = [&](const unsigned char* v_lds) {
 #pragma unroll
     for (int s2 = 0; s2 < 2; ++s2) {
-      bf16x8_t pf[QT];
+      bf16x8_t pf[QT], pf_lo[QT];
 #pragma unroll
       for (int qt = 0; qt < QT; ++qt) {
+        if constexpr (WP) {
+          const u32x4_t lw = {pl[qt][2 * s2][0], pl[qt][2 * s2][1], pl[qt][2 * s2 + 1][0], pl[qt][2 * s2 + 1][1]};
+          pf_lo[qt] = __builtin_bit_cast(bf16x8_t, lw);
+        }
         u32x4_t pw = {pk[qt][2 * s2][0], pk[qt][2 * s2][1], pk[qt][2 * s2 + 1][0], pk[qt][2 * s2 + 1][1]};
         pf[qt] = __builtin_bit_cast(bf16x8_t, pw);
       }
@@ -468,8 +493,11 @@ __global__ __launch_bounds__(AW_WAVES * 64) void attn_prefill_wide_kernel(AttnPa
         typedef __attribute__((ext_vector_type(8))) short s16x8_t;
         const s16x8_t vv = {lo[0], lo[1], lo[2], lo[3], hi[0], hi[1], hi[2], hi[3]};
 #pragma unroll
-        for (int qt = 0; qt < QT; ++qt)
+        for (int qt = 0; qt < QT; ++qt) {
+          if constexpr (WP)
+            o[qt][dt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, vv), pf_lo[qt], o[qt][dt], 0, 0, 0);
           o[qt][dt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, vv), pf[qt], o[qt][dt], 0, 0, 0);
+        }
       }
     }
   };
@@ -579,7 +607,7 @@ void launch_attn_prefill(const bf16_t* q, const bf16_t* k, const bf16_t* v, bf16
                          const long long* strides /*12: q,k,v,o x (b,s,h)*/, const int* kv_len,
                          int B, int Sq, int Sk, int Hq, int Hkv, int D, int causal, int q_offset,
                          int q_offset_from_len, float scale, hipStream_t st, float* part_o,
-                         float* part_ml, int nsplit, float* lse) {
+                         float* part_ml, int nsplit, float* lse, bool wide_p) {
   AttnParams p;
   p.part_o = part_o; p.part_ml = part_ml; p.nsplit = nsplit; p.lse = lse;
   p.q = q; p.k = k; p.v = v; p.o = o;
@@ -626,7 +654,10 @@ void launch_attn_prefill(const bf16_t* q, const bf16_t* k, const bf16_t* v, bf16
       }
       hipLaunchKernelGGL(kern, wgrid, wblock, smem, st, p);
     };
-    if (wide == 8) {
+    if (wide_p && causal) {
+      if (wide == 8) { if (D == 128) go(attn_prefill_wide_kernel<128, true, 8, qt, true>, 128); else go(attn_prefill_wide_kernel<64, true, 8, qt, true>, 64); }
+      else { if (D == 128) go(attn_prefill_wide_kernel<128, true, 4, qt, true>, 128); else go(attn_prefill_wide_kernel<64, true, 4, qt, true>, 64); }
+    } else if (wide == 8) {
       if (D == 128) { if (causal) go(attn_prefill_wide_kernel<128, true, 8>, 128); else go(attn_prefill_wide_kernel<128, false, 8>, 128); }
       else { if (causal) go(attn_prefill_wide_kernel<64, true, 8>, 64); else go(attn_prefill_wide_kernel<64, false, 8>, 64); }
     } else {
@@ -636,6 +667,11 @@ void launch_attn_prefill(const bf16_t* q, const bf16_t* k, const bf16_t* v, bf16
     return;
   }
   dim3 grid((Sq + 63) / 64, Hq, B);
+  if (wide_p && causal) {
+    if (D == 128) hipLaunchKernelGGL((attn_prefill_kernel<128, true, false, 1, true>), grid, block, 0, st, p);
+    else hipLaunchKernelGGL((attn_prefill_kernel<64, true, false, 1, true>), grid, block, 0, st, p);
+    return;
+  }
   // Two key-tile groups per block for the ViT's shape class -- head_dim 64, non-causal, so few blocks
   // that half the chip idles (577 tokens x 16 heads: 160) -- while all blocks are resident at once:
   // 12.3 -> 9.9 us per layer.  Causal head_dim-128 blocks do not gain (636 tokens x 32 heads: 23.9 ->

@@ -366,10 +366,14 @@ __global__ __launch_bounds__(256) void attn_prep_kernel(AttnPrepArgs a) {
     sk += sumsq8(t);
     if constexpr (STAGED) store8(row_lds + qn + c, t);
   }
-  // (the sums' barriers also publish the staged row)
-  const float rq = a.qw ? rsqrtf(block_sum(sq, red) / static_cast<float>(a.nq) + a.eps) : 1.f;
-  const float rk = a.kw ? rsqrtf(block_sum(sk, red) / static_cast<float>(a.nk) + a.eps) : 1.f;
-  __syncthreads();
+  float v0[8];                                   // the first values are on their way while the sums meet
+  if (threadIdx.x * 8 < static_cast<unsigned>(kn)) src8(a.src, row, a.v_col + threadIdx.x * 8, v0);
+  sq = wave_sum(sq);
+  sk = wave_sum(sk);
+  if ((threadIdx.x & 63) == 0) { red[threadIdx.x >> 6] = sq; red[8 + (threadIdx.x >> 6)] = sk; }
+  __syncthreads();                               // (publishes the staged row too)
+  const float rq = a.qw ? rsqrtf((red[0] + red[1] + red[2] + red[3]) / static_cast<float>(a.nq) + a.eps) : 1.f;
+  const float rk = a.kw ? rsqrtf((red[8] + red[9] + red[10] + red[11]) / static_cast<float>(a.nk) + a.eps) : 1.f;
   const int p = a.row_pos[row];
   const int pt = min(max(p, 0), a.max_pos - 1);
   const float* cs = a.cos_tab + static_cast<long long>(pt) * half;
@@ -422,7 +426,10 @@ __global__ __launch_bounds__(256) void attn_prep_kernel(AttnPrepArgs a) {
   for (int c = threadIdx.x * 8; c < kn; c += 2048) {
     float u[8], v[8];
     value8(a.k_col, qn, a.kw, rk, c, u);
-    src8(a.src, row, a.v_col + c, v);
+    if (c == static_cast<int>(threadIdx.x) * 8)
+#pragma unroll
+      for (int i = 0; i < 8; ++i) v[i] = v0[i];
+    else src8(a.src, row, a.v_col + c, v);
     if (kv >= 0) {
       store8(static_cast<T*>(a.k_buf) + kv * kn + c, u);
       store8(static_cast<T*>(a.v_buf) + kv * kn + c, v);

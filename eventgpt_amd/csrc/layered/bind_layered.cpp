@@ -322,7 +322,7 @@ void attn_runs_(const Tensor& q, const Tensor& k, const Tensor& v, const Tensor&
   const long long st[12] = {rows * Hq * D, Hq * D, D, rows * Hkv * D, Hkv * D, D, rows * Hkv * D, Hkv * D, D, rows * Hq * D, Hq * D, D};
   evgpt::launch_attn_prefill(bptr(q) + q0 * Hq * D, bptr(k) + kv0 * Hkv * D, bptr(v) + kv0 * Hkv * D, bptr_mut(o) + q0 * Hq * D,
                              st, nullptr, (int)n, (int)rows, (int)(off + rows), (int)Hq, (int)Hkv, (int)D, 1, (int)off, 0,
-                             (float)scale, cur_stream());
+                             (float)scale, cur_stream(), nullptr, nullptr, 0, nullptr, true);
 }
 // split-KV decode attention of the other models on the chunk cache (bf16, head size 64 or 128); part_o / part_ml: scratch
 Tensor attn_chunk_decode(const Tensor& q, const Tensor& k_cache, const Tensor& v_cache, const Tensor& pos, double scale,
