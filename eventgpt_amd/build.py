@@ -34,7 +34,7 @@ BUILD_DIR = os.path.join(os.path.dirname(PKG_DIR), "build", "evgpt_C")
 SO_PATH = os.path.join(PKG_DIR, "_C.so")
 LAYERED_SO_PATH = os.path.join(PKG_DIR, "_D.so")
 # kernels of the layered decoders alone, and the ones they share with the rest
-LAYERED_KERNELS = ("attn_chunk", "conv1d", "decode_step", "gemm_f32", "linear_scan", "row_gemv", "rowops")
+LAYERED_KERNELS = ("attn_chunk", "conv1d", "decode_step", "gemm_f32", "latent", "linear_scan", "moe", "row_gemv", "rowops")
 LAYERED_SHARED = ("attn_decode", "attn_prefill", "gemm", "sd")
 ARCH = "gfx950"
 

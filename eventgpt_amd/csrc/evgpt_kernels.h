@@ -102,6 +102,9 @@ void launch_gemm_bf16(const bf16_t* A, const bf16_t* W, bf16_t* C, float* Cf, co
                       hipStream_t st);
 void launch_gemm_glu(const bf16_t* A, const bf16_t* W, bf16_t* H, int M, int I, int K, int lda, int ldw, int ldc,
                      hipStream_t st, int glu_act = 0);   // 0: silu, 1: gelu (tanh form)
+// grouped product of experts; glu: 0 plain, otherwise 1 + the GLU activation of launch_gemm_glu
+void launch_gemm_grouped(const bf16_t* A, const bf16_t* W, bf16_t* C, const int* start, const int* perm, int top, int E,
+                         int a_rows, int rows, int N, int K, int glu, hipStream_t st);
 bool launch_gemm_qkv_rope(const bf16_t* A, const bf16_t* W, int M, int K, bf16_t* q_out, bf16_t* k_cache,
                           bf16_t* v_cache, const float* cos_tab, const float* sin_tab, const int* pos0, int Hq,
                           int Hkv, int l_max, hipStream_t st);
@@ -284,7 +287,8 @@ void launch_attn_prefill(const bf16_t* q, const bf16_t* k, const bf16_t* v, bf16
                          int Hq, int Hkv, int D, int causal, int q_offset, int q_offset_from_len,
                          float scale, hipStream_t st, float* part_o = nullptr,
                          float* part_ml = nullptr, int nsplit = 0, float* lse = nullptr,
-                         bool wide_p = false);   // wide_p (causal): fp32 softmax weights in the second product
+                         bool wide_p = false,    // (causal) fp32 softmax weights in the second product
+                         const bf16_t* gate = nullptr, int gate_ld = 0);   // [B * Sq][gate_ld]: o of head h times sigmoid(gate[row][h])
 
 // ---- attn_bwd.hip: flash-attention backward (recomputes P from the forward's LSE)
 // q/do/dq [B,Sq,Hq,D], k/v/dk/dv [B,Sk,Hkv,D], o [B,Sq,Hq,D], all contiguous bf16;

@@ -21,7 +21,7 @@ template <typename T>
 __global__ __launch_bounds__(256) void attn_chunk_kernel(const T* __restrict__ q, const T* __restrict__ k,
                                                          const T* __restrict__ v, T* __restrict__ o,
                                                          const int* __restrict__ items, int Hq, int Hkv, int D,
-                                                         float scale) {
+                                                         long long kld, float scale, const T* __restrict__ gate, int gate_ld) {
   __shared__ __attribute__((aligned(16))) T vt[64 * AC_TS];
   const int* it = items + blockIdx.x * 4;
   const int q0 = it[0], nq = min(it[1], 64), kv0 = it[2], off = it[3];
@@ -30,7 +30,6 @@ __global__ __launch_bounds__(256) void attn_chunk_kernel(const T* __restrict__ q
   const int t = wid * 16 + fr, tc = min(t, nq - 1);
   const int lim = off + tc;                       // this lane's last visible key
   const int k_end = off + nq;                     // keys the block needs
-  const long long kld = static_cast<long long>(Hkv) * D;
   const T* qp = q + (static_cast<long long>(q0 + tc) * Hq + h) * D;
   const T* kb = k + static_cast<long long>(kv0) * kld + hk * D;
   const T* vb = v + static_cast<long long>(kv0) * kld + hk * D + v0;
@@ -113,7 +112,8 @@ __global__ __launch_bounds__(256) void attn_chunk_kernel(const T* __restrict__ q
   l += __shfl_xor(l, 16, 64);
   l += __shfl_xor(l, 32, 64);
   if (t >= nq) return;
-  const float inv = 1.f / l;
+  float inv = 1.f / l;
+  if (gate) inv *= sigmoid_f(to_f32(gate[static_cast<long long>(q0 + t) * gate_ld + h]));
   T* op = o + (static_cast<long long>(q0 + t) * Hq + h) * D + v0;
 #pragma unroll
   for (int i = 0; i < 4; ++i)
@@ -121,16 +121,16 @@ __global__ __launch_bounds__(256) void attn_chunk_kernel(const T* __restrict__ q
 }
 
 void launch_attn_chunk(const void* q, const void* k, const void* v, void* o, const int* items, int n_items, bool f32,
-                       int Hq, int Hkv, int D, float scale, hipStream_t st) {
+                       int Hq, int Hkv, int D, long long kld, float scale, const void* gate, int gate_ld, hipStream_t st) {
   const dim3 grid(n_items, Hq, D / 64);
   if (f32)
     hipLaunchKernelGGL(attn_chunk_kernel<float>, grid, dim3(256), 0, st, static_cast<const float*>(q),
                        static_cast<const float*>(k), static_cast<const float*>(v), static_cast<float*>(o), items, Hq, Hkv, D,
-                       scale);
+                       kld, scale, static_cast<const float*>(gate), gate_ld);
   else
     hipLaunchKernelGGL(attn_chunk_kernel<bf16_t>, grid, dim3(256), 0, st, static_cast<const bf16_t*>(q),
                        static_cast<const bf16_t*>(k), static_cast<const bf16_t*>(v), static_cast<bf16_t*>(o), items, Hq, Hkv,
-                       D, scale);
+                       D, kld, scale, static_cast<const bf16_t*>(gate), gate_ld);
 }
 
 // One query per sequence.  Sixteen lanes per key: lane l holds elements 4 l .. 4 l + 3 of every run of 64, so a
@@ -138,7 +138,7 @@ void launch_attn_chunk(const void* q, const void* k, const void* v, void* o, con
 template <typename T, int E>
 __global__ __launch_bounds__(256) void attn_chunk_decode_kernel(const T* __restrict__ q, const T* __restrict__ kc,
                                                                 const T* __restrict__ vc, T* __restrict__ o,
-                                                                const int* __restrict__ pos, int Hq, int Hkv, int D,
+                                                                const int* __restrict__ row_slot, const int* __restrict__ pos, int Hq, int Hkv, int D,
                                                                 int cap, float scale) {
   __shared__ __attribute__((aligned(16))) float so[16][64 * E];
   __shared__ float sm[16], sl[16];
@@ -146,7 +146,7 @@ __global__ __launch_bounds__(256) void attn_chunk_decode_kernel(const T* __restr
   const int tid = threadIdx.x, l16 = tid & 15, grp = tid >> 4;
   const int len = max(pos[b], 0) % cap + 1;
   const T* qp = q + (static_cast<long long>(b) * Hq + h) * D + l16 * 4;
-  const long long base = (static_cast<long long>(b) * Hkv + hk) * cap * D + l16 * 4;
+  const long long base = (static_cast<long long>(row_slot ? row_slot[b] : b) * Hkv + hk) * cap * D + l16 * 4;
   f32x4_t qv[E], ov[E];
 #pragma unroll
   for (int e = 0; e < E; ++e) {
@@ -194,20 +194,20 @@ __global__ __launch_bounds__(256) void attn_chunk_decode_kernel(const T* __restr
 }
 
 template <typename T>
-static void launch_decode(const void* q, const void* kc, const void* vc, void* o, const int* pos, int B, int Hq,
+static void launch_decode(const void* q, const void* kc, const void* vc, void* o, const int* row_slot, const int* pos, int B, int Hq,
                           int Hkv, int D, int cap, float scale, hipStream_t st) {
   const dim3 grid(Hq, B), block(256);
   const T *qt = static_cast<const T*>(q), *kt = static_cast<const T*>(kc), *vt = static_cast<const T*>(vc);
   T* ot = static_cast<T*>(o);
-  if (D <= 64) hipLaunchKernelGGL((attn_chunk_decode_kernel<T, 1>), grid, block, 0, st, qt, kt, vt, ot, pos, Hq, Hkv, D, cap, scale);
-  else if (D <= 128) hipLaunchKernelGGL((attn_chunk_decode_kernel<T, 2>), grid, block, 0, st, qt, kt, vt, ot, pos, Hq, Hkv, D, cap, scale);
-  else if (D <= 256) hipLaunchKernelGGL((attn_chunk_decode_kernel<T, 4>), grid, block, 0, st, qt, kt, vt, ot, pos, Hq, Hkv, D, cap, scale);
-  else hipLaunchKernelGGL((attn_chunk_decode_kernel<T, 8>), grid, block, 0, st, qt, kt, vt, ot, pos, Hq, Hkv, D, cap, scale);
+  if (D <= 64) hipLaunchKernelGGL((attn_chunk_decode_kernel<T, 1>), grid, block, 0, st, qt, kt, vt, ot, row_slot, pos, Hq, Hkv, D, cap, scale);
+  else if (D <= 128) hipLaunchKernelGGL((attn_chunk_decode_kernel<T, 2>), grid, block, 0, st, qt, kt, vt, ot, row_slot, pos, Hq, Hkv, D, cap, scale);
+  else if (D <= 256) hipLaunchKernelGGL((attn_chunk_decode_kernel<T, 4>), grid, block, 0, st, qt, kt, vt, ot, row_slot, pos, Hq, Hkv, D, cap, scale);
+  else hipLaunchKernelGGL((attn_chunk_decode_kernel<T, 8>), grid, block, 0, st, qt, kt, vt, ot, row_slot, pos, Hq, Hkv, D, cap, scale);
 }
-void launch_attn_chunk_decode(const void* q, const void* k_cache, const void* v_cache, void* o, const int* pos,
+void launch_attn_chunk_decode(const void* q, const void* k_cache, const void* v_cache, void* o, const int* row_slot, const int* pos,
                               bool f32, int B, int Hq, int Hkv, int D, int cap, float scale, hipStream_t st) {
-  if (f32) launch_decode<float>(q, k_cache, v_cache, o, pos, B, Hq, Hkv, D, cap, scale, st);
-  else launch_decode<bf16_t>(q, k_cache, v_cache, o, pos, B, Hq, Hkv, D, cap, scale, st);
+  if (f32) launch_decode<float>(q, k_cache, v_cache, o, row_slot, pos, B, Hq, Hkv, D, cap, scale, st);
+  else launch_decode<bf16_t>(q, k_cache, v_cache, o, row_slot, pos, B, Hq, Hkv, D, cap, scale, st);
 }
 
 }  // namespace evgpt

@@ -46,7 +46,12 @@ struct AttnParams {
   int nsplit;
   float* lse;                   // optional [B][Hq][Sq]: log2 of the row's softmax denominator in the
                                 // scaled-log2 domain (max + log2(sum)); the backward recomputes P from it
+  const bf16_t* gate;           // optional [B * Sq][gate_ld]: head h's output is multiplied by sigmoid of column h
+  int gate_ld;
 };
+__device__ __forceinline__ float head_gate(const AttnParams& p, int b, int qi, int h) {
+  return 1.f / (1.f + __expf(-bf16_to_f32(p.gate[(static_cast<long long>(b) * p.Sq + qi) * p.gate_ld + h])));
+}
 
 // GROUPS = 2: the block is two such groups of 4 waves over the SAME 64 query rows; group 0 takes the
 // even key tiles of the block's range and group 1 the odd ones, each through its own K / V tile
@@ -289,7 +294,8 @@ __global__ __launch_bounds__(256 * GROUPS) void attn_prefill_kernel(AttnParams p
     }
     return;
   }
-  const float inv = l > 0.f ? 1.f / l : 0.f;
+  float inv = l > 0.f ? 1.f / l : 0.f;
+  if (p.gate && qi < p.Sq) inv *= head_gate(p, b, qi, h);
   if (p.lse && g == 0 && qi < p.Sq)
     p.lse[(static_cast<long long>(b) * p.Hq + h) * p.Sq + qi] = l > 0.f ? m * p.scale_log2e + log2f(l) : INFINITY;
   if (qi < p.Sq) {
@@ -548,8 +554,9 @@ __global__ __launch_bounds__(AW_WAVES * 64) void attn_prefill_wide_kernel(AttnPa
     float lt = l[qt];
     lt += __shfl_xor(lt, 16, 64);
     lt += __shfl_xor(lt, 32, 64);
-    const float inv = lt > 0.f ? 1.f / lt : 0.f;
+    float inv = lt > 0.f ? 1.f / lt : 0.f;
     if (qi[qt] >= p.Sq) continue;
+    if (p.gate) inv *= head_gate(p, b, qi[qt], h);
     if (p.lse && g == 0)
       p.lse[(static_cast<long long>(b) * p.Hq + h) * p.Sq + qi[qt]] = lt > 0.f ? m[qt] * p.scale_log2e + log2f(lt) : INFINITY;
     bf16_t* op = p.o + b * p.o_sb + static_cast<long long>(qi[qt]) * p.o_ss + h * p.o_sh;
@@ -607,8 +614,9 @@ void launch_attn_prefill(const bf16_t* q, const bf16_t* k, const bf16_t* v, bf16
                          const long long* strides /*12: q,k,v,o x (b,s,h)*/, const int* kv_len,
                          int B, int Sq, int Sk, int Hq, int Hkv, int D, int causal, int q_offset,
                          int q_offset_from_len, float scale, hipStream_t st, float* part_o,
-                         float* part_ml, int nsplit, float* lse, bool wide_p) {
+                         float* part_ml, int nsplit, float* lse, bool wide_p, const bf16_t* gate, int gate_ld) {
   AttnParams p;
+  p.gate = gate; p.gate_ld = gate_ld;
   p.part_o = part_o; p.part_ml = part_ml; p.nsplit = nsplit; p.lse = lse;
   p.q = q; p.k = k; p.v = v; p.o = o;
   p.q_sb = strides[0]; p.q_ss = strides[1]; p.q_sh = strides[2];

@@ -146,4 +146,29 @@ __device__ __forceinline__ int xcd_remap(int id, int n) {
   return base + (id >> 3);
 }
 
+// Tiles of a grouped product: group e has rows start[e] .. start[e + 1], cut into row tiles of `bm`, each with `tiles_n`
+// column tiles; groups follow each other.  The wave finds the group of `tile`, which becomes the tile's index within
+// it; returns -1 past the last tile.
+__device__ __forceinline__ int group_of_tile(const int* start, int groups, int bm, int tiles_n, int& tile) {
+  const int lane = threadIdx.x & 63;
+  for (int e0 = 0; e0 < groups; e0 += 64) {
+    const int e = e0 + lane;
+    const int mine = e < groups ? (start[e + 1] - start[e] + bm - 1) / bm * tiles_n : 0;
+    int sum = mine;                                     // inclusive scan
+#pragma unroll
+    for (int off = 1; off < 64; off <<= 1) {
+      const int t = __shfl_up(sum, off, 64);
+      if (lane >= off) sum += t;
+    }
+    const unsigned long long past = __builtin_amdgcn_ballot_w64(tile < sum);
+    if (past) {
+      const int l = __builtin_ctzll(past);
+      tile -= __builtin_amdgcn_readlane(sum - mine, l);
+      return e0 + l;
+    }
+    tile -= __builtin_amdgcn_readlane(sum, 63);
+  }
+  return -1;
+}
+
 }  // namespace evgpt

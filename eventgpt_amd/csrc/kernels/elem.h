@@ -116,5 +116,9 @@ __device__ __forceinline__ float softplus_f(float x) { return fmaxf(x, 0.f) + lo
 __device__ __forceinline__ float gelu_tanh_f(float x) {
   return 0.5f * x * (1.f + tanhf(0.7978845608028654f * (x + 0.044715f * x * x * x)));
 }
+__device__ __forceinline__ float soft_cap(float x, float scale, float cap) {
+  x *= scale;
+  return cap > 0.f ? cap * tanhf(x / cap) : x;
+}
 
 }  // namespace evgpt

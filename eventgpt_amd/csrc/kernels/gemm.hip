@@ -98,6 +98,12 @@ struct GemmParams {
   int rows_epilogue;   // 8-wave kernel: bf16 output stored as whole lines through LDS (set by launch_256)
   // 4-wave kernel with split K: workgroup index = split * tiles + tile instead of tile * splits + split
   int split_major;
+  // Grouped product (GRP instances of the 4-wave kernel): the rows are sorted into grp_count groups (group e: rows
+  // grp_start[e] .. grp_start[e + 1]), each with its own weights W + e * grp_wstride; row i is row grp_perm[i] / grp_top of
+  // A (grp_perm null: row i) and goes to row i of C.
+  const int* grp_start; const int* grp_perm;
+  int grp_count, grp_top;
+  long long grp_wstride;
 };
 
 // wait until at most `n` of this wave's direct-to-LDS loads are still in flight
@@ -429,8 +435,9 @@ __device__ __forceinline__ void gemm_rope_epilogue(const GemmParams& p, f32x4_t 
 }
 
 template <int BM, int BN, int WGM, int WGN, int STAGES, bool AT = false, bool BT = false, bool KT = false,
-          bool ROPE = false>
+          bool ROPE = false, bool GRP = false>
 __global__ __launch_bounds__(256) void gemm_bf16_kernel(GemmParams p) {
+  static_assert(!GRP || (!AT && !BT && !KT && !ROPE), "grouped products are plain ones");
   static_assert(!AT || BM == 64 || BM == 128, "K-strided A needs a 64- or 128-row tile");
   static_assert(!BT || BN == 64 || BN == 128, "K-strided W needs a 64- or 128-column tile");
   constexpr int WM = BM / WGM, WN = BN / WGN;  // per-wave tile
@@ -442,13 +449,26 @@ __global__ __launch_bounds__(256) void gemm_bf16_kernel(GemmParams p) {
 
   const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6;
   const int bn_out = p.glu_half ? BN / 2 : BN;      // output columns per tile
-  const int tiles_n = (p.N + bn_out - 1) / bn_out, tiles_m = (p.M + BM - 1) / BM;
-  const int bid = xcd_remap(blockIdx.x, tiles_m * tiles_n * p.splitk);
+  const int tiles_n = (p.N + bn_out - 1) / bn_out;
+  // bytes of each operand that exist in memory (everything past them reads as zero)
+  const long long bytes_a = 2ll * (AT ? p.ka_rows : p.M) * p.lda;
+  const long long bytes_w = 2ll * (BT ? p.kw_rows : (p.glu_half ? 2 * p.glu_half : p.N)) * p.ldw;
+  const int bid = xcd_remap(blockIdx.x, GRP ? gridDim.x : (p.M + BM - 1) / BM * tiles_n * p.splitk);
+  int grp_tile = bid, grp_first = 0;
+  if constexpr (GRP) {
+    const int e = group_of_tile(p.grp_start, p.grp_count, BM, tiles_n, grp_tile);
+    if (e < 0) return;
+    grp_first = p.grp_start[e];
+    p.M = p.grp_start[e + 1] - grp_first;
+    p.W += e * p.grp_wstride;
+    p.C += static_cast<size_t>(grp_first) * p.ldc;
+  }
+  const int tiles_m = (p.M + BM - 1) / BM;
   // split K: tile-major (the splits of a tile are neighbours) or split-major (an XCD works inside one K range:
   // with a few hundred rows that range of A stays in its L2 while the weights stream past)
   const int ntile = tiles_m * tiles_n;
-  const int tile = p.split_major ? bid % ntile : bid / p.splitk;
-  const int ksplit = p.split_major ? bid / ntile : bid % p.splitk;
+  const int tile = GRP ? grp_tile : p.split_major ? bid % ntile : bid / p.splitk;
+  const int ksplit = GRP ? 0 : p.split_major ? bid / ntile : bid % p.splitk;
   const int k_begin = ksplit * p.k_per_split;
   const int k_len = min(p.k_per_split, p.K - k_begin);
   // consecutive tiles walk down (a group of) M first: they share one weight panel
@@ -479,7 +499,12 @@ __global__ __launch_bounds__(256) void gemm_bf16_kernel(GemmParams p) {
     } else {
       const int row = rg * 8 + srow;
       const int c = schunk ^ ((row >> 1) & 7);
-      voff_a[i] = ((m0 + row) * p.lda + c * 8) * 2;
+      int src = m0 + row;
+      if constexpr (GRP) {
+        const int at = grp_first + min(src, p.M - 1);      // (rows past the group are not stored)
+        src = p.grp_perm ? p.grp_perm[at] / p.grp_top : at;
+      }
+      voff_a[i] = (src * p.lda + c * 8) * 2;
     }
   }
 #pragma unroll
@@ -501,9 +526,6 @@ __global__ __launch_bounds__(256) void gemm_bf16_kernel(GemmParams p) {
       voff_w[i] = (src * p.ldw + c * 8) * 2;
     }
   }
-  // bytes of each operand that exist in memory (everything past them reads as zero)
-  const long long bytes_a = 2ll * (AT ? p.ka_rows : p.M) * p.lda;
-  const long long bytes_w = 2ll * (BT ? p.kw_rows : (p.glu_half ? 2 * p.glu_half : p.N)) * p.ldw;
   auto stage = [&](int buf, int kt) {
     unsigned char* base = smem + buf * STAGE;
     const int k0 = k_begin + kt * BK;
@@ -1367,6 +1389,36 @@ int gemm_splitk_t(int M, int N, int K) {
   if (K < 8192 || t < 96 || t >= 256) return 1;
   const int s = static_cast<int>(512 / t);
   return s < 1 ? 1 : (s > 4 ? 4 : s);
+}
+
+// Grouped product (experts): row i of group e = rows grp_start[e] .. grp_start[e + 1] (`rows` of them in all groups) is row
+// perm[i] / top of A [a_rows][K] (perm null: row i) times W + e * N K (glu: [gate | up] rows, N = 2 * output columns), bf16 out.
+template <int BM, int BN, int WGM, int WGN, int STAGES>
+static void launch_grp(GemmParams p, int rows, hipStream_t st) {
+  const int bn_out = p.glu_half ? BN / 2 : BN;
+  const int tiles = (rows / BM + p.grp_count) * ((p.N + bn_out - 1) / bn_out);
+  constexpr size_t smem = static_cast<size_t>(STAGES) * (BM + BN) * BK * 2;
+  auto kern = gemm_bf16_kernel<BM, BN, WGM, WGN, STAGES, false, false, false, false, true>;
+  static const bool attr = [&] {
+    return smem <= 64 * 1024 || hipFuncSetAttribute(reinterpret_cast<const void*>(kern), hipFuncAttributeMaxDynamicSharedMemorySize,
+                                                    static_cast<int>(smem)) == hipSuccess;
+  }();
+  (void)attr;
+  p.group_m = g_group_m;
+  hipLaunchKernelGGL(kern, dim3(tiles), dim3(256), smem, st, p);
+}
+void launch_gemm_grouped(const bf16_t* A, const bf16_t* W, bf16_t* C, const int* start, const int* perm, int top, int E,
+                         int a_rows, int rows, int N, int K, int glu, hipStream_t st) {
+  const int cols = glu ? N / 2 : N;
+  GemmParams p{A, W, C, nullptr, nullptr, nullptr, a_rows, cols, K, K, K, cols, ACT_NONE, nullptr, nullptr, 1, K, nullptr, 0, K, K};
+  p.glu_half = glu ? cols : 0;
+  p.glu_act = glu - 1;
+  p.grp_start = start; p.grp_perm = perm; p.grp_top = top; p.grp_count = E;
+  p.grp_wstride = static_cast<long long>(N) * K;
+  const int per = rows / E;             // rows of an average group
+  if (per < 48) launch_grp<32, 128, 1, 4, 4>(p, rows, st);
+  else if (per < 192) launch_grp<64, 128, 2, 2, 3>(p, rows, st);
+  else launch_grp<128, 128, 2, 2, 2>(p, rows, st);
 }
 
 // H[M, I] = act(A · Wgate^T) * (A · Wup^T), act = silu or (glu_act) gelu, with W = [gate rows | up rows] ([2I, K]): the gate/up

@@ -4,12 +4,15 @@
 // (16-byte non-temporal loads, the next batch in flight while the current one is multiplied), the partial sums
 // meet in LDS.  Blocks walk the units, and the first unit's weights are requested before the block prepares its
 // input, which it keeps in LDS in the storage type:
-//   NORM   RMS norm of the stream;
+//   NORM   norm (RMS or layer norm) of the stream;
 //   MERGE  x + (rms(a) wa + rms(b) wb) / 2, its RMS norm, and (one block) the new stream;
+//   POST   x + norm(a) wa, its norm, and (one block) the new stream;
+//   ROWS   RMS norm of a run of columns of a projection's rows;
 //   GROUP  group norm of a recurrent mixer's output, with a sigmoid gate after it if asked for;
 //   PLAIN  a row that is already in the storage type, read from global memory.
-// Epilogues store fp32 rows, add to the stream, or multiply gate and up rows (GLU).  Two problems with the same
-// epilogue (the output projections of two branches) can share a launch.
+// Epilogues store fp32 rows (scaled and softly capped if asked for), add to the stream, or multiply gate and up
+// rows (GLU).  Two problems with the same epilogue (the output projections of two branches) can share a launch.  One more
+// block can norm another run of columns into a latent cache.
 #include "src_rows.h"
 
 namespace evgpt {
@@ -24,23 +27,100 @@ __device__ __forceinline__ float dot16(const u32x4_t& w, const u32x4_t& x, float
   return acc;
 }
 
+constexpr int GV_KEEP = 2;     // chunks of eight a thread keeps while it norms a row (4096 columns)
+
 template <typename T>
-__device__ void prepare_norm(const GemvInput& in, int b, int K, T* xs, float* red) {
+__device__ void prepare_norm(const GemvInput& in, int b, int K, T* xs, float* red, bool lead) {
   const float* x = static_cast<const float*>(in.x) + static_cast<long long>(b) * K;
-  float ss = 0.f;
-  for (int c = threadIdx.x * 8; c < K; c += 2048) {
-    float v[8];
-    load8(x + c, v);
-    ss += sumsq8(v);
+  const bool rows = in.kind == GV_ROWS;
+  float keep[GV_KEEP][8];
+  auto value = [&](int c, float (&v)[8]) {
+    if (!rows) { load8(x + c, v); return; }
+    if (c + 8 <= in.n) { src8(in.gate, b, in.gcol + c, v); return; }
+#pragma unroll
+    for (int i = 0; i < 8; ++i) v[i] = c + i < in.n ? src1(in.gate, b, in.gcol + c + i) : 0.f;
+  };
+#pragma unroll
+  for (int k = 0; k < GV_KEEP; ++k) {
+    const int c = (threadIdx.x + k * 256) * 8;
+    if (c < K) value(c, keep[k]);
   }
-  const float r = rsqrtf(block_sum(ss, red) / static_cast<float>(in.n) + in.eps);
-  for (int c = threadIdx.x * 8; c < K; c += 2048) {
-    float v[8], w[8];
-    load8(x + c, v);
+  const RowStat st = row_stat<GV_KEEP>(keep, in.n, K, in.eps, in.layer != 0, red, value);
+  auto put = [&](int c, const float (&v)[8]) {
+    float w[8];
     load8(in.w + c, w);
 #pragma unroll
-    for (int i = 0; i < 8; ++i) v[i] *= r * w[i];
-    store8(xs + c, v);
+    for (int i = 0; i < 8; ++i) w[i] *= (v[i] - st.mean) * st.r;
+    store8(xs + c, w);
+    if (lead && in.xn_out) store8(static_cast<T*>(in.xn_out) + static_cast<long long>(b) * K + c, w);
+  };
+#pragma unroll
+  for (int k = 0; k < GV_KEEP; ++k) {
+    const int c = (threadIdx.x + k * 256) * 8;
+    if (c < K) put(c, keep[k]);
+  }
+  for (int c = (threadIdx.x + GV_KEEP * 256) * 8; c < K; c += 2048) {
+    float v[8];
+    value(c, v);
+    put(c, v);
+  }
+}
+
+template <typename T>
+__device__ void prepare_post(const GemvInput& in, int b, int K, T* xs, float* red, bool lead) {
+  const long long o = static_cast<long long>(b) * K;
+  const float* x = static_cast<const float*>(in.x) + o;
+  float keep[GV_KEEP][8];
+  auto branch = [&](int c, float (&v)[8]) { load8(in.a + o + c, v); };
+#pragma unroll
+  for (int k = 0; k < GV_KEEP; ++k) {
+    const int c = (threadIdx.x + k * 256) * 8;
+    if (c < K) branch(c, keep[k]);
+  }
+  const RowStat sa = row_stat<GV_KEEP>(keep, in.n, K, in.eps, in.layer != 0, red, branch);
+  auto add = [&](int c, float (&v)[8]) {           // branch values -> the new stream
+    float u[8], p[8];
+    load8(x + c, u);
+    load8(in.wa + c, p);
+#pragma unroll
+    for (int i = 0; i < 8; ++i) v[i] = u[i] + (v[i] - sa.mean) * sa.r * p[i];
+  };
+  auto value = [&](int c, float (&v)[8]) { branch(c, v); add(c, v); };
+#pragma unroll
+  for (int k = 0; k < GV_KEEP; ++k) {
+    const int c = (threadIdx.x + k * 256) * 8;
+    if (c < K) add(c, keep[k]);
+  }
+  const RowStat st = row_stat<GV_KEEP>(keep, in.n, K, in.eps, in.layer != 0, red, value);
+  auto put = [&](int c, const float (&v)[8]) {
+    if (lead) store8(in.x_out + o + c, v);
+    float w[8];
+    load8(in.w + c, w);
+#pragma unroll
+    for (int i = 0; i < 8; ++i) w[i] *= (v[i] - st.mean) * st.r;
+    store8(xs + c, w);
+    if (lead && in.xn_out) store8(static_cast<T*>(in.xn_out) + o + c, w);
+  };
+#pragma unroll
+  for (int k = 0; k < GV_KEEP; ++k) {
+    const int c = (threadIdx.x + k * 256) * 8;
+    if (c < K) put(c, keep[k]);
+  }
+  for (int c = (threadIdx.x + GV_KEEP * 256) * 8; c < K; c += 2048) {
+    float v[8];
+    value(c, v);
+    put(c, v);
+  }
+}
+
+// The block past the units: RMS norm of the latent columns of every row into the row's cache, a wave per row.
+template <typename T>
+__device__ void store_latents(const LatentStore& s, int B) {
+  const int lane = threadIdx.x & 63;
+  for (int b = threadIdx.x >> 6; b < B; b += 4) {
+    if (s.live && !s.live[b]) continue;
+    const int p = min(max(s.pos[b], 0), s.cap - 1);
+    latent_row(s.src, b, s.col, s.n, s.R, s.w, s.eps, static_cast<T*>(s.cache) + (static_cast<long long>(b) * s.cap + p) * s.R, lane);
   }
 }
 
@@ -143,10 +223,14 @@ __global__ __launch_bounds__(256) void row_gemv_kernel(GemvCall call, int blocks
   constexpr int CE = 16 / sizeof(T);                      // elements per 16-byte chunk
   __shared__ float part[2][4][GV_R * B];
   __shared__ float red[16];
+  if (call.latent.cache && blockIdx.x + 1 == gridDim.x) {
+    store_latents<T>(call.latent, B);
+    return;
+  }
   const bool second = call.count == 2 && static_cast<int>(blockIdx.x) >= blocks0;
   const GemvProblem& p = call.p[second ? 1 : 0];
   const int blk = second ? blockIdx.x - blocks0 : blockIdx.x;
-  const int nblk = call.count == 2 ? (second ? gridDim.x - blocks0 : blocks0) : gridDim.x;
+  const int nblk = call.count == 2 ? (second ? gridDim.x - blocks0 : blocks0) : blocks0;
   const int K = p.K, nchunk = K / CE, nit = (nchunk + 255) / 256;
   const int units = EPI == GV_GLU ? p.N / 4 : p.N / GV_R;
   const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6;
@@ -170,7 +254,8 @@ __global__ __launch_bounds__(256) void row_gemv_kernel(GemvCall call, int blocks
   if constexpr (!PLAIN) {
     for (int b = 0; b < B; ++b) {
       T* xb = xs + static_cast<long long>(b) * K;
-      if (p.in.kind == GV_NORM) prepare_norm(p.in, b, K, xb, red);
+      if (p.in.kind == GV_NORM || p.in.kind == GV_ROWS) prepare_norm(p.in, b, K, xb, red, blk == 0);
+      else if (p.in.kind == GV_POST) prepare_post(p.in, b, K, xb, red, blk == 0);
       else if (p.in.kind == GV_MERGE) prepare_merge(p.in, b, K, xb, red, blk == 0);
       else if (p.in.kind == GV_GROUP) prepare_group(p.in, b, K, xb, reinterpret_cast<float*>(smem + static_cast<long long>(B) * K * sizeof(T)));
       else
@@ -230,7 +315,7 @@ __global__ __launch_bounds__(256) void row_gemv_kernel(GemvCall call, int blocks
         const int r = tid / B, b = tid % B;
         float* y = p.y + static_cast<long long>(b) * p.ldy + u * GV_R + r;
         if constexpr (EPI == GV_ADD) *y += total(r * B + b);
-        else *y = total(r * B + b);
+        else *y = call.finish ? soft_cap(total(r * B + b), call.scale, call.cap) : total(r * B + b);
       }
     }
     flip ^= 1;       // the next unit's partial sums go to the other buffer: one barrier per unit
@@ -261,9 +346,9 @@ static void launch_b(const GemvCall& c, size_t lds, hipStream_t st) {
   // 45.8 / 33.4 / 35.4 / 40.2 / 42.0, two output projections 19.8 / 18.3 / 15.9 / 18.0 / 21.3; four rows, norm + 18560 rows
   // 58.9 / 38.8 / 34.6 / 41.6 / 47.4
   const int kind = c.p[0].in.kind;
-  const int budget = g_blocks ? g_blocks : (B == 1 && c.count == 1 && (kind == GV_NORM || kind == GV_MERGE) ? 512 : 768);
+  const int budget = g_blocks ? g_blocks : (B == 1 && c.count == 1 && (kind == GV_NORM || kind == GV_MERGE || kind == GV_POST) ? 512 : 768);
   const int b0 = blocks_of(c.p[0], c.count == 2 ? budget / 2 : budget), b1 = c.count == 2 ? blocks_of(c.p[1], budget / 2) : 0;
-  const dim3 grid(b0 + b1), block(256);
+  const dim3 grid(b0 + b1 + (c.latent.cache ? 1 : 0)), block(256);
   const bool plain = c.count == 1 && c.p[0].in.kind == GV_PLAIN;
 #define EVGPT_GEMV(E)                                                                              \
   if (plain) hipLaunchKernelGGL((row_gemv_kernel<T, B, E, true>), grid, block, 0, st, c, b0);      \

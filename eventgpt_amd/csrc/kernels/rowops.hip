@@ -32,19 +32,40 @@ void launch_embed_rows(const int* tok, const void* embed, bool f32, float scale,
                        static_cast<const bf16_t*>(embed), scale, x, ld, vocab);
 }
 
-// The three residual kernels.  MODE 0: xn = norm(x).  MODE 1: x += a first.  MODE 2: x += (norm(a) wa +
-// norm(b) wb) / 2 first.  A thread keeps its first NC chunks of eight in registers between the passes.
-template <typename T, int MODE>
+// The residual kernels.  MODE 0: xn = norm(x).  MODE 1: x += a first.  MODE 2: x += (norm(a) wa + norm(b) wb) / 2
+// first.  MODE 3: x += norm(a) wa first.  MODE 4: the same (or x += y without wa) with y the weighted sum of a few
+// rows of another matrix.  norm: RMS, or layer norm (LN).  A thread keeps its first NC chunks of eight in registers
+// between the passes.
+template <typename T, int MODE, bool LN>
 __global__ __launch_bounds__(256) void residual_norm_kernel(float* __restrict__ x, const int* __restrict__ sel,
-                                                            SrcRows a, SrcRows b, const float* __restrict__ wa,
+                                                            SrcRows a, SrcRows b, MixRows mix, const float* __restrict__ wa,
                                                             const float* __restrict__ wb, const float* __restrict__ w,
                                                             T* __restrict__ xn, int n, int ld, float eps) {
   __shared__ float red[16];
   const long long row = blockIdx.x, xrow = MODE == 0 && sel ? sel[row] : row;
-  const float inv_n = 1.f / static_cast<float>(n);
   float* xr = x + xrow * ld;
+  constexpr int NC = 4;       // 8192 columns stay in registers
+  float keep[NC][8];
   float ra = 0.f, rb = 0.f;
+  RowStat sy{0.f, 1.f};
+  auto branch = [&](int c, float (&v)[8]) {          // MODE 3 and 4: the sublayer's output
+    if constexpr (MODE == 3) src8(a, row, c, v);
+    if constexpr (MODE == 4) {
+      const int* pick = mix.pick + row * mix.top;
+      const float* pw = mix.w + row * mix.top;
+#pragma unroll
+      for (int i = 0; i < 8; ++i) v[i] = 0.f;
+      for (int k = 0; k < mix.top; ++k) {
+        float t[8];
+        load8(static_cast<const T*>(mix.y) + static_cast<long long>(pick[k]) * mix.ld + c, t);
+        const float f = pw[k];
+#pragma unroll
+        for (int i = 0; i < 8; ++i) v[i] += f * t[i];
+      }
+    }
+  };
   if constexpr (MODE == 2) {
+    const float inv_n = 1.f / static_cast<float>(n);
     float sa = 0.f, sb = 0.f;
     for (int c = threadIdx.x * 8; c < ld; c += 2048) {
       float t[8];
@@ -56,11 +77,30 @@ __global__ __launch_bounds__(256) void residual_norm_kernel(float* __restrict__ 
     ra = 0.5f * rsqrtf(block_sum(sa, red) * inv_n + eps);
     rb = 0.5f * rsqrtf(block_sum(sb, red) * inv_n + eps);
   }
-  constexpr int NC = 4;       // 8192 columns stay in registers
-  float keep[NC][8];
-  float ss = 0.f;
+  if constexpr (MODE >= 3) {
+#pragma unroll
+    for (int k = 0; k < NC; ++k) {
+      const int c = (threadIdx.x + k * 256) * 8;
+      if (c < ld) branch(c, keep[k]);
+    }
+    if (MODE == 3 || wa) sy = row_stat<NC>(keep, n, ld, eps, LN, red, branch);
+  }
+  // the new stream: v holds the branch's values (MODE 3 and 4) on entry
   auto value = [&](int c, float (&v)[8]) {
-    load8(xr + c, v);
+    if constexpr (MODE >= 3) {
+      float p[8], u[8];
+      load8(xr + c, u);
+      if (MODE == 3 || wa) {
+        load8(wa + c, p);       // (zero in the padding)
+#pragma unroll
+        for (int i = 0; i < 8; ++i) v[i] = u[i] + (v[i] - sy.mean) * sy.r * p[i];
+      } else {
+#pragma unroll
+        for (int i = 0; i < 8; ++i) v[i] += u[i];
+      }
+    } else {
+      load8(xr + c, v);
+    }
     if constexpr (MODE == 1) {
       float t[8];
       src8(a, row, c, t);
@@ -77,25 +117,27 @@ __global__ __launch_bounds__(256) void residual_norm_kernel(float* __restrict__ 
       for (int i = 0; i < 8; ++i) v[i] += t[i] * ra * p[i] + u[i] * rb * q[i];
     }
     if constexpr (MODE != 0) store8(xr + c, v);
-    ss += sumsq8(v);
   };
 #pragma unroll
   for (int k = 0; k < NC; ++k) {
     const int c = (threadIdx.x + k * 256) * 8;
     if (c < ld) value(c, keep[k]);
   }
-  for (int c = (threadIdx.x + NC * 256) * 8; c < ld; c += 2048) {
-    float v[8];
-    value(c, v);
-  }
+  if constexpr (MODE != 0)
+    for (int c = (threadIdx.x + NC * 256) * 8; c < ld; c += 2048) {
+      float v[8];
+      branch(c, v);
+      value(c, v);
+    }
   if (w == nullptr) return;
-  const float r = rsqrtf(block_sum(ss, red) * inv_n + eps);
+  // each thread re-reads what it wrote
+  const RowStat st = row_stat<NC>(keep, n, ld, eps, LN, red, [&](int c, float (&v)[8]) { load8(xr + c, v); });
   T* o = xn + row * ld;
   auto put = [&](int c, const float (&v)[8]) {
     float g[8];
     load8(w + c, g);
 #pragma unroll
-    for (int i = 0; i < 8; ++i) g[i] *= v[i] * r;
+    for (int i = 0; i < 8; ++i) g[i] *= (v[i] - st.mean) * st.r;
     store8(o + c, g);
   };
 #pragma unroll
@@ -103,34 +145,56 @@ __global__ __launch_bounds__(256) void residual_norm_kernel(float* __restrict__ 
     const int c = (threadIdx.x + k * 256) * 8;
     if (c < ld) put(c, keep[k]);
   }
-  for (int c = (threadIdx.x + NC * 256) * 8; c < ld; c += 2048) {   // each thread re-reads what it wrote
+  for (int c = (threadIdx.x + NC * 256) * 8; c < ld; c += 2048) {
     float v[8];
     load8(xr + c, v);
     put(c, v);
   }
 }
 template <int MODE>
-static void launch_residual(float* x, const int* sel, const SrcRows& a, const SrcRows& b, const float* wa,
+static void launch_residual(float* x, const int* sel, const SrcRows& a, const SrcRows& b, const MixRows& mix, const float* wa,
                             const float* wb, const float* w, void* xn, bool f32, int rows, int n, int ld, float eps,
-                            hipStream_t st) {
-  if (f32)
-    hipLaunchKernelGGL((residual_norm_kernel<float, MODE>), dim3(rows), dim3(256), 0, st, x, sel, a, b, wa, wb, w,
-                       static_cast<float*>(xn), n, ld, eps);
-  else
-    hipLaunchKernelGGL((residual_norm_kernel<bf16_t, MODE>), dim3(rows), dim3(256), 0, st, x, sel, a, b, wa, wb, w,
-                       static_cast<bf16_t*>(xn), n, ld, eps);
+                            bool layer, hipStream_t st) {
+#define EVGPT_RES(T, LN) \
+  hipLaunchKernelGGL((residual_norm_kernel<T, MODE, LN>), dim3(rows), dim3(256), 0, st, x, sel, a, b, mix, wa, wb, w, \
+                     static_cast<T*>(xn), n, ld, eps)
+  if (layer) { if (f32) EVGPT_RES(float, true); else EVGPT_RES(bf16_t, true); }
+  else { if (f32) EVGPT_RES(float, false); else EVGPT_RES(bf16_t, false); }
+#undef EVGPT_RES
 }
 void launch_norm_rows(const float* x, const int* sel, const float* w, void* xn, bool f32, int rows, int n, int ld,
-                      float eps, hipStream_t st) {
-  launch_residual<0>(const_cast<float*>(x), sel, SrcRows{}, SrcRows{}, nullptr, nullptr, w, xn, f32, rows, n, ld, eps, st);
+                      float eps, bool layer, hipStream_t st) {
+  launch_residual<0>(const_cast<float*>(x), sel, SrcRows{}, SrcRows{}, MixRows{}, nullptr, nullptr, w, xn, f32, rows, n, ld, eps, layer, st);
 }
 void launch_add_norm_rows(float* x, const SrcRows& y, const float* w, void* xn, bool f32, int rows, int n, int ld,
-                          float eps, hipStream_t st) {
-  launch_residual<1>(x, nullptr, y, SrcRows{}, nullptr, nullptr, w, xn, f32, rows, n, ld, eps, st);
+                          float eps, bool layer, hipStream_t st) {
+  launch_residual<1>(x, nullptr, y, SrcRows{}, MixRows{}, nullptr, nullptr, w, xn, f32, rows, n, ld, eps, layer, st);
 }
 void launch_merge_norm_rows(float* x, const SrcRows& a, const SrcRows& b, const float* wa, const float* wb,
                             const float* w, void* xn, bool f32, int rows, int n, int ld, float eps, hipStream_t st) {
-  launch_residual<2>(x, nullptr, a, b, wa, wb, w, xn, f32, rows, n, ld, eps, st);
+  launch_residual<2>(x, nullptr, a, b, MixRows{}, wa, wb, w, xn, f32, rows, n, ld, eps, false, st);
+}
+void launch_post_norm_rows(float* x, const SrcRows& y, const float* wy, const float* w, void* xn, bool f32, int rows, int n,
+                           int ld, float eps, bool layer, hipStream_t st) {
+  launch_residual<3>(x, nullptr, y, SrcRows{}, MixRows{}, wy, nullptr, w, xn, f32, rows, n, ld, eps, layer, st);
+}
+void launch_mix_norm_rows(float* x, const MixRows& y, const float* wy, const float* w, void* xn, bool f32, int rows, int n,
+                          int ld, float eps, bool layer, hipStream_t st) {
+  launch_residual<4>(x, nullptr, SrcRows{}, SrcRows{}, y, wy, nullptr, w, xn, f32, rows, n, ld, eps, layer, st);
+}
+
+// logits = cap * tanh(scale * logits / cap); cap 0: scale alone
+__global__ __launch_bounds__(256) void cap_logits_kernel(float* __restrict__ x, long long n, float scale, float cap) {
+  for (long long i = (blockIdx.x * 256ll + threadIdx.x) * 4; i < n; i += gridDim.x * 1024ll) {
+    f32x4_t v = load4(x + i);
+#pragma unroll
+    for (int k = 0; k < 4; ++k) v[k] = soft_cap(v[k], scale, cap);
+    *reinterpret_cast<f32x4_t*>(x + i) = v;
+  }
+}
+void launch_cap_logits(float* x, long long n, float scale, float cap, hipStream_t st) {
+  const long long want = (n + 1023) / 1024;
+  hipLaunchKernelGGL(cap_logits_kernel, dim3(static_cast<unsigned>(want < 4096 ? want : 4096)), dim3(256), 0, st, x, n, scale, cap);
 }
 
 template <typename T, int ACT>

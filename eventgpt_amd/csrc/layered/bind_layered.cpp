@@ -128,7 +128,7 @@ void check_stream(const Tensor& x, int64_t n) {
   check_f(x, "x");
   TORCH_CHECK(x.dim() == 2 && x.size(1) % 64 == 0 && n >= 1 && n <= x.size(1), "x: [M, padded width]");
 }
-Tensor norm_rows(const Tensor& x, const OptTensor& sel, const Tensor& w, int64_t n, double eps, bool f32) {
+Tensor norm_rows(const Tensor& x, const OptTensor& sel, const Tensor& w, int64_t n, double eps, bool f32, bool layer) {
   check_stream(x, n); check_f(w, "w");
   TORCH_CHECK(w.numel() == x.size(1), "norm_rows: weight size");
   if (sel.has_value()) check_i(*sel, "sel");
@@ -136,7 +136,7 @@ Tensor norm_rows(const Tensor& x, const OptTensor& sel, const Tensor& w, int64_t
   Tensor xn = at::empty({M, x.size(1)}, x.options().dtype(t_of(f32)));
   if (M > 0)
     evgpt::launch_norm_rows(x.data_ptr<float>(), iptr(sel), w.data_ptr<float>(), xn.data_ptr(), f32, (int)M, (int)n,
-                            (int)x.size(1), (float)eps, cur_stream());
+                            (int)x.size(1), (float)eps, layer, cur_stream());
   return xn;
 }
 SrcRows stream_src(const Tensor& y, const Tensor& x, const char* name) {
@@ -151,13 +151,45 @@ Tensor xn_of(const Tensor& x, const OptTensor& w, bool f32) {
   TORCH_CHECK(w->numel() == x.size(1), "norm weight size");
   return at::empty({x.size(0), x.size(1)}, x.options().dtype(t_of(f32)));
 }
-Tensor add_norm_rows_(const Tensor& x, const Tensor& y, const OptTensor& w, int64_t n, double eps, bool f32) {
+Tensor add_norm_rows_(const Tensor& x, const Tensor& y, const OptTensor& w, int64_t n, double eps, bool f32, bool layer) {
   check_stream(x, n);
   const SrcRows s = stream_src(y, x, "y");
   Tensor xn = xn_of(x, w, f32);
   evgpt::launch_add_norm_rows(x.data_ptr<float>(), s, fptr(w), xn.data_ptr(), f32, (int)x.size(0), (int)n, (int)x.size(1),
-                              (float)eps, cur_stream());
+                              (float)eps, layer, cur_stream());
   return xn;
+}
+// x += norm(y) * wy; norm of the new x * w
+Tensor post_norm_rows_(const Tensor& x, const Tensor& y, const Tensor& wy, const OptTensor& w, int64_t n, double eps, bool f32,
+                       bool layer) {
+  check_stream(x, n); check_f(wy, "wy");
+  TORCH_CHECK(wy.numel() == x.size(1), "post_norm_rows: weight size");
+  const SrcRows s = stream_src(y, x, "y");
+  Tensor xn = xn_of(x, w, f32);
+  if (x.size(0) > 0)
+    evgpt::launch_post_norm_rows(x.data_ptr<float>(), s, wy.data_ptr<float>(), fptr(w), xn.data_ptr(), f32, (int)x.size(0), (int)n,
+                                 (int)x.size(1), (float)eps, layer, cur_stream());
+  return xn;
+}
+// the same with y[row] = sum_k weights[row][k] * y[pick[row][k]] (without wy: x += y)
+Tensor mix_norm_rows_(const Tensor& x, const Tensor& y, const Tensor& pick, const Tensor& weights, const OptTensor& wy,
+                      const OptTensor& w, int64_t n, double eps, bool f32, bool layer) {
+  check_stream(x, n); check_t(y, "y"); check_i(pick, "pick"); check_f(weights, "weights");
+  TORCH_CHECK(y.dim() == 2 && y.size(1) >= x.size(1) && y.size(1) % 8 == 0 && is_f32(y) == f32, "mix_norm_rows: y [rows, width]");
+  TORCH_CHECK(weights.dim() == 2 && weights.size(0) == x.size(0) && weights.size(1) >= 1 && pick.numel() == weights.numel(),
+              "mix_norm_rows: pick, weights [M, top]");
+  if (wy.has_value()) { check_f(*wy, "wy"); TORCH_CHECK(wy->numel() == x.size(1), "mix_norm_rows: weight size"); }
+  Tensor xn = xn_of(x, w, f32);
+  const evgpt::MixRows m{y.data_ptr(), pick.data_ptr<int>(), weights.data_ptr<float>(), (int)weights.size(1), (int)y.size(1)};
+  if (x.size(0) > 0)
+    evgpt::launch_mix_norm_rows(x.data_ptr<float>(), m, fptr(wy), fptr(w), xn.data_ptr(), f32, (int)x.size(0), (int)n,
+                                (int)x.size(1), (float)eps, layer, cur_stream());
+  return xn;
+}
+void cap_logits_(const Tensor& x, double scale, double cap) {
+  check_f(x, "logits");
+  TORCH_CHECK(x.numel() % 4 == 0 && cap >= 0, "cap_logits: a multiple of four values, cap >= 0");
+  if (x.numel() > 0) evgpt::launch_cap_logits(x.data_ptr<float>(), x.numel(), (float)scale, (float)cap, cur_stream());
 }
 Tensor merge_norm_rows_(const Tensor& x, const Tensor& a, const Tensor& b, const Tensor& wa, const Tensor& wb,
                         const OptTensor& w, int64_t n, double eps, bool f32) {
@@ -295,34 +327,55 @@ void chunk_keys_copy_(const Tensor& k_cache, const Tensor& v_cache, const Tensor
                                   copies.data_ptr<int>(), (int)copies.size(0), is_f32(k_cache), (int)k_cache.size(1),
                                   (int)k_cache.size(2), (int)k_cache.size(3), cur_stream());
 }
+// k, v: rows of [Hkv][D]; the rows may be strided (columns of a wider matrix)
 void check_qkv(const Tensor& q, const Tensor& k, const Tensor& v) {
-  check_t(q, "q"); check_t(k, "k"); check_t(v, "v");
+  check_t(q, "q");
   TORCH_CHECK(q.dim() == 3 && k.dim() == 3 && k.sizes() == v.sizes() && q.size(2) == k.size(2) && q.size(1) % k.size(1) == 0 &&
               q.scalar_type() == k.scalar_type() && q.scalar_type() == v.scalar_type(), "attention: q [M, Hq, D], k / v [R, Hkv, D]");
   TORCH_CHECK(q.size(2) % 64 == 0 && q.size(2) <= 512, "attention: head size a multiple of 64 up to 512");
+  for (const Tensor* t : {&k, &v})
+    TORCH_CHECK(t->is_cuda() && t->stride(2) == 1 && (t->size(1) == 1 || t->stride(1) == t->size(2)) && t->stride(0) % 8 == 0 &&
+                t->stride(0) >= t->size(1) * t->size(2) && t->stride(0) == k.stride(0) &&
+                (reinterpret_cast<uintptr_t>(t->data_ptr()) & 15) == 0, "attention: k, v: aligned rows of heads");
 }
-Tensor attn_chunk(const Tensor& q, const Tensor& k, const Tensor& v, const Tensor& items, double scale) {
+// rows of a matrix of q's type whose columns gcol .. gcol + Hq gate the heads
+const void* head_gates(const OptTensor& gate, int64_t gcol, const Tensor& q, int64_t* ld) {
+  *ld = 0;
+  if (!gate.has_value()) return nullptr;
+  TORCH_CHECK(gate->is_cuda() && gate->dim() == 2 && gate->stride(1) == 1 && gate->scalar_type() == q.scalar_type() &&
+              gate->size(0) == q.size(0) && gcol >= 0 && gcol + q.size(1) <= gate->size(1), "attention: gate [M, N]");
+  *ld = gate->stride(0);
+  return static_cast<const char*>(gate->data_ptr()) + gcol * (is_f32(q) ? 4 : 2);
+}
+Tensor attn_chunk(const Tensor& q, const Tensor& k, const Tensor& v, const Tensor& items, double scale, const OptTensor& gate,
+                  int64_t gcol) {
   check_qkv(q, k, v); check_i(items, "items");
   TORCH_CHECK(items.dim() == 2 && items.size(1) == 4, "attn_chunk: items [n, 4]");
+  int64_t gld;
+  const void* g = head_gates(gate, gcol, q, &gld);
   Tensor o = at::empty_like(q);
   if (items.size(0) > 0)
     evgpt::launch_attn_chunk(q.data_ptr(), k.data_ptr(), v.data_ptr(), o.data_ptr(), items.data_ptr<int>(), (int)items.size(0),
-                             is_f32(q), (int)q.size(1), (int)k.size(1), (int)q.size(2), (float)scale, cur_stream());
+                             is_f32(q), (int)q.size(1), (int)k.size(1), (int)q.size(2), k.stride(0), (float)scale, g, (int)gld,
+                             cur_stream());
   return o;
 }
 // `n` equal runs of `rows` query rows starting at q0, each with its keys `stride` key rows after the one before, the
 // run's first query at position `off` of its chunk, on the flash kernel (bf16, head size 64 or 128)
 void attn_runs_(const Tensor& q, const Tensor& k, const Tensor& v, const Tensor& o, int64_t q0, int64_t rows, int64_t kv0,
-                int64_t off, int64_t n, double scale) {
+                int64_t off, int64_t n, double scale, const OptTensor& gate, int64_t gcol) {
   check_qkv(q, k, v); check_t(o, "o");
   const int64_t Hq = q.size(1), Hkv = k.size(1), D = q.size(2);
   TORCH_CHECK(!is_f32(q) && (D == 64 || D == 128) && o.sizes() == q.sizes() && !is_f32(o), "attn_runs: bf16, head size 64 or 128");
   TORCH_CHECK(rows >= 1 && n >= 1 && q0 >= 0 && kv0 >= 0 && off >= 0 && (n == 1 || off == 0) && q0 + n * rows <= q.size(0) &&
               kv0 + off + n * rows <= k.size(0), "attn_runs: rows");
-  const long long st[12] = {rows * Hq * D, Hq * D, D, rows * Hkv * D, Hkv * D, D, rows * Hkv * D, Hkv * D, D, rows * Hq * D, Hq * D, D};
-  evgpt::launch_attn_prefill(bptr(q) + q0 * Hq * D, bptr(k) + kv0 * Hkv * D, bptr(v) + kv0 * Hkv * D, bptr_mut(o) + q0 * Hq * D,
+  const long long ks = k.stride(0);
+  int64_t gld;
+  const evgpt::bf16_t* g = static_cast<const evgpt::bf16_t*>(head_gates(gate, gcol, q, &gld));
+  const long long st[12] = {rows * Hq * D, Hq * D, D, rows * ks, ks, D, rows * ks, ks, D, rows * Hq * D, Hq * D, D};
+  evgpt::launch_attn_prefill(bptr(q) + q0 * Hq * D, bptr(k) + kv0 * ks, bptr(v) + kv0 * ks, bptr_mut(o) + q0 * Hq * D,
                              st, nullptr, (int)n, (int)rows, (int)(off + rows), (int)Hq, (int)Hkv, (int)D, 1, (int)off, 0,
-                             (float)scale, cur_stream(), nullptr, nullptr, 0, nullptr, true);
+                             (float)scale, cur_stream(), nullptr, nullptr, 0, nullptr, true, g ? g + q0 * gld : nullptr, (int)gld);
 }
 // split-KV decode attention of the other models on the chunk cache (bf16, head size 64 or 128); part_o / part_ml: scratch
 Tensor attn_chunk_decode(const Tensor& q, const Tensor& k_cache, const Tensor& v_cache, const Tensor& pos, double scale,
@@ -342,7 +395,7 @@ Tensor attn_chunk_decode(const Tensor& q, const Tensor& k_cache, const Tensor& v
                               cur_stream(), 1);
     return o;
   }
-  evgpt::launch_attn_chunk_decode(q.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(), o.data_ptr(), pos.data_ptr<int>(),
+  evgpt::launch_attn_chunk_decode(q.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(), o.data_ptr(), nullptr, pos.data_ptr<int>(),
                                   is_f32(q), (int)B, (int)Hq, (int)Hkv, (int)D, (int)cap, (float)scale, cur_stream());
   return o;
 }
@@ -470,14 +523,22 @@ void check_gemv_w(const Tensor& w, int64_t B, int64_t K, const char* name) {
   TORCH_CHECK(B >= 1 && B <= evgpt::GEMV_ROWS_MAX, "row_gemv: one to four rows");
 }
 evgpt::GemvInput stream_input(const Tensor& x, const Tensor& w, int64_t n, double eps, const OptTensor& a, const OptTensor& b,
-                              const OptTensor& wa, const OptTensor& wb, const OptTensor& x_out) {
+                              const OptTensor& wa, const OptTensor& wb, const OptTensor& x_out, bool layer) {
   check_stream(x, n); check_f(w, "norm");
   const int64_t K = x.size(1);
   TORCH_CHECK(w.numel() == K, "row_gemv: norm weight size");
   evgpt::GemvInput in{};
   in.kind = evgpt::GV_NORM;
-  in.x = x.data_ptr(); in.w = w.data_ptr<float>(); in.n = (int)n; in.eps = (float)eps;
-  if (a.has_value()) {
+  in.x = x.data_ptr(); in.w = w.data_ptr<float>(); in.n = (int)n; in.eps = (float)eps; in.layer = layer;
+  if (a.has_value() && !b.has_value()) {
+    TORCH_CHECK(wa.has_value() && x_out.has_value(), "row_gemv: post norm");
+    check_f(*a, "a"); check_f(*wa, "wa"); check_f(*x_out, "x_out");
+    TORCH_CHECK(a->numel() == x.numel() && wa->numel() == K && x_out->numel() == x.numel() && x_out->data_ptr() != x.data_ptr(),
+                "row_gemv: post norm sizes");
+    in.kind = evgpt::GV_POST;
+    in.a = a->data_ptr<float>(); in.wa = wa->data_ptr<float>(); in.x_out = x_out->data_ptr<float>();
+  } else if (a.has_value()) {
+    TORCH_CHECK(!layer, "row_gemv: branches are merged with RMS norms");
     TORCH_CHECK(b.has_value() && wa.has_value() && wb.has_value() && x_out.has_value(), "row_gemv: branches");
     check_f(*a, "a"); check_f(*b, "b"); check_f(*wa, "wa"); check_f(*wb, "wb"); check_f(*x_out, "x_out");
     TORCH_CHECK(a->numel() == x.numel() && b->numel() == x.numel() && wa->numel() == K && wb->numel() == K &&
@@ -493,12 +554,23 @@ void run_gemv(const evgpt::GemvCall& c, bool f32, int64_t B) {
   evgpt::launch_row_gemv(c, f32, (int)B, cur_stream());
 }
 // W · norm(x): fp32 [B, N], or with act >= 0 act(gate) * up of [gate | up] rows in the storage type.  With branches a, b: x +
-// (rms(a) wa + rms(b) wb) / 2 takes x's place and is stored to x_out.
+// (rms(a) wa + rms(b) wb) / 2 takes x's place and is stored to x_out; with a alone: x + norm(a) wa.  xn_out also gets the
+// normed rows.  scale: the fp32 rows are cap * tanh(scale * y / cap) (cap 0: scale * y).
 Tensor gemv_norm(const Tensor& x, const Tensor& norm, int64_t n, double eps, const Tensor& w, int64_t act, const OptTensor& a,
-                 const OptTensor& b, const OptTensor& wa, const OptTensor& wb, const OptTensor& x_out) {
+                 const OptTensor& b, const OptTensor& wa, const OptTensor& wb, const OptTensor& x_out, bool layer, const OptTensor& xn_out,
+                 c10::optional<double> scale, double cap) {
   evgpt::GemvCall c{};
   c.count = 1;
-  c.p[0].in = stream_input(x, norm, n, eps, a, b, wa, wb, x_out);
+  c.p[0].in = stream_input(x, norm, n, eps, a, b, wa, wb, x_out, layer);
+  if (xn_out.has_value()) {
+    check_t(*xn_out, "xn_out");
+    TORCH_CHECK(xn_out->numel() == x.numel() && xn_out->scalar_type() == w.scalar_type() && c.p[0].in.kind != evgpt::GV_MERGE, "gemv_norm: xn_out");
+    c.p[0].in.xn_out = xn_out->data_ptr();
+  }
+  if (scale.has_value()) {
+    TORCH_CHECK(act < 0 && cap >= 0, "gemv_norm: scaled rows");
+    c.finish = 1; c.scale = (float)*scale; c.cap = (float)cap;
+  }
   const int64_t B = x.size(0), N = w.size(0);
   check_gemv_w(w, B, x.size(1), "w");
   c.p[0].W = w.data_ptr(); c.p[0].N = (int)N; c.p[0].K = (int)x.size(1);
@@ -511,6 +583,62 @@ Tensor gemv_norm(const Tensor& x, const Tensor& norm, int64_t n, double eps, con
     y = at::empty({B, N}, x.options());
     c.epilogue = evgpt::GV_STORE; c.p[0].y = y.data_ptr<float>(); c.p[0].ldy = (int)N;
   }
+  run_gemv(c, is_f32(w), B);
+  return y;
+}
+// the latent columns of projection rows `src` -> cache [slots, cap, R] at pos (rows whose `live` is 0 are left out)
+struct LatentCols { SrcRows s; int64_t rows; };
+LatentCols check_latent(const Tensor& src, int64_t col, int64_t n, const Tensor& w, const Tensor& cache, const Tensor& pos,
+                        const OptTensor& live, bool f32) {
+  LatentCols l;
+  int64_t N;
+  l.s = src_of(src, "src", &l.rows, &N);
+  check_f(w, "latent weight"); check_t(cache, "cache"); check_i(pos, "pos");
+  TORCH_CHECK(cache.dim() == 3 && cache.size(1) >= 1 && cache.size(2) % 64 == 0 && cache.size(2) == w.numel() && is_f32(cache) == f32 &&
+              n >= 1 && n <= cache.size(2) && col >= 0 && col % 8 == 0 && col + n <= N && pos.numel() >= l.rows, "latent: columns, cache [slots, cap, R]");
+  if (live.has_value()) { check_i(*live, "live"); TORCH_CHECK(live->numel() >= l.rows, "latent: live"); }
+  return l;
+}
+// fp32 [B, N] = W · rms(src[:, col .. col + n)); with a cache, the latent columns of the same rows go into it
+Tensor gemv_rows(const Tensor& src, int64_t col, int64_t n, const Tensor& norm, double eps, const Tensor& w, int64_t c_col, int64_t c_n,
+                 const OptTensor& c_norm, const OptTensor& cache, const OptTensor& pos, const OptTensor& live) {
+  int64_t B, cols;
+  evgpt::GemvCall c{};
+  c.count = 1;
+  evgpt::GemvInput& in = c.p[0].in;
+  in.kind = evgpt::GV_ROWS;
+  in.gate = src_of(src, "src", &B, &cols);
+  check_f(norm, "norm");
+  const int64_t K = norm.numel(), N = w.size(0);
+  TORCH_CHECK(n >= 1 && n <= K && col >= 0 && col % 8 == 0 && col + n <= cols, "gemv_rows: columns");
+  check_gemv_w(w, B, K, "w");
+  in.gcol = (int)col; in.n = (int)n; in.eps = (float)eps; in.w = norm.data_ptr<float>();
+  if (cache.has_value()) {
+    TORCH_CHECK(c_norm.has_value() && pos.has_value(), "gemv_rows: latents");
+    const LatentCols l = check_latent(src, c_col, c_n, *c_norm, *cache, *pos, live, is_f32(w));
+    TORCH_CHECK(cache->size(0) >= B, "gemv_rows: slots");
+    c.latent = evgpt::LatentStore{l.s, (int)c_col, (int)c_n, (int)cache->size(2), c_norm->data_ptr<float>(), (float)eps, cache->data_ptr(),
+                                  (int)cache->size(1), pos->data_ptr<int>(), iptr(live)};
+  }
+  Tensor y = at::empty({B, N}, norm.options());
+  c.p[0].W = w.data_ptr(); c.p[0].N = (int)N; c.p[0].K = (int)K;
+  c.epilogue = evgpt::GV_STORE; c.p[0].y = y.data_ptr<float>(); c.p[0].ldy = (int)N;
+  run_gemv(c, is_f32(w), B);
+  return y;
+}
+// fp32 [B, N] = W · h for rows h of the storage type
+Tensor gemv_plain(const Tensor& w, const Tensor& h) {
+  check_t(h, "h");
+  TORCH_CHECK(h.dim() == 2 && h.scalar_type() == w.scalar_type(), "gemv_plain: h [B, K]");
+  const int64_t B = h.size(0), N = w.size(0);
+  check_gemv_w(w, B, h.size(1), "w");
+  Tensor y = at::empty({B, N}, h.options().dtype(at::kFloat));
+  evgpt::GemvCall c{};
+  c.count = 1;
+  c.epilogue = evgpt::GV_STORE;
+  c.p[0].W = w.data_ptr(); c.p[0].N = (int)N; c.p[0].K = (int)w.size(1);
+  c.p[0].in.kind = evgpt::GV_PLAIN; c.p[0].in.x = h.data_ptr();
+  c.p[0].y = y.data_ptr<float>(); c.p[0].ldy = (int)N;
   run_gemv(c, is_f32(w), B);
   return y;
 }
@@ -583,6 +711,183 @@ Tensor gemv_branches(const Tensor& wa, const Tensor& h, const Tensor& wb, const 
   run_gemv(c, is_f32(wa), B);
   return o;
 }
+
+// ---------------------------------------------------------------- latent attention
+// Query latents [M, Q] in the storage type (q_norm given) from columns of `src`, key / value latents into `cache` (given)
+Tensor latent_prep_(const Tensor& src, int64_t q_col, int64_t nq, const OptTensor& q_norm, int64_t c_col, int64_t nc, const OptTensor& c_norm,
+                    const OptTensor& cache, const OptTensor& row_slot, const Tensor& row_pos, const OptTensor& live, double eps, bool f32) {
+  int64_t M, N;
+  evgpt::LatentPrepArgs a{};
+  a.src = src_of(src, "src", &M, &N);
+  a.eps = (float)eps;
+  check_i(row_pos, "row_pos");
+  TORCH_CHECK(row_pos.numel() >= M, "latent_prep: row_pos");
+  a.row_pos = row_pos.data_ptr<int>();
+  if (row_slot.has_value()) { check_i(*row_slot, "row_slot"); TORCH_CHECK(row_slot->numel() >= M, "latent_prep: row_slot"); a.row_slot = iptr(row_slot); }
+  Tensor q;
+  if (q_norm.has_value()) {
+    check_f(*q_norm, "q_norm");
+    const int64_t Q = q_norm->numel();
+    TORCH_CHECK(Q % 8 == 0 && nq >= 1 && nq <= Q && q_col >= 0 && q_col % 8 == 0 && q_col + nq <= N, "latent_prep: query columns");
+    q = at::empty({M, Q}, q_norm->options().dtype(t_of(f32)));
+    a.q_col = (int)q_col; a.nq = (int)nq; a.Q = (int)Q; a.qw = q_norm->data_ptr<float>(); a.q_out = q.data_ptr();
+  } else {
+    q = at::empty({0}, src.options().dtype(t_of(f32)));
+  }
+  if (cache.has_value()) {
+    TORCH_CHECK(c_norm.has_value(), "latent_prep: c_norm");
+    check_latent(src, c_col, nc, *c_norm, *cache, row_pos, live, f32);
+    if (!row_slot.has_value()) TORCH_CHECK(cache->size(0) >= M, "latent_prep: slots");
+    a.c_col = (int)c_col; a.nc = (int)nc; a.R = (int)cache->size(2); a.cw = c_norm->data_ptr<float>(); a.cache = cache->data_ptr();
+    a.cap = (int)cache->size(1); a.live = iptr(live);
+  }
+  if (M > 0) evgpt::launch_latent_prep(a, f32, (int)M, cur_stream());
+  return q;
+}
+// cached rows into a buffer [rows, R]; copies [n, 4] of {slot, first position, first buffer row, count}
+Tensor latent_gather(const Tensor& cache, const Tensor& copies, int64_t rows) {
+  check_t(cache, "cache"); check_i(copies, "copies");
+  TORCH_CHECK(cache.dim() == 3 && cache.size(2) % 8 == 0 && copies.dim() == 2 && copies.size(1) == 4 && copies.size(0) < 65536 && rows >= 0,
+              "latent_gather: cache [slots, cap, R], copies [n, 4]");
+  Tensor buf = at::empty({rows, cache.size(2)}, cache.options());
+  if (rows > 0 && copies.size(0) > 0)
+    evgpt::launch_latent_gather(cache.data_ptr(), buf.data_ptr(), copies.data_ptr<int>(), (int)copies.size(0), is_f32(cache),
+                                (int)cache.size(1), (int)cache.size(2), cur_stream());
+  return buf;
+}
+// rows of heads: x [M, H * K] (any SrcRows) -> [M, H, N] in w's type, w [H, N, K]; with a gate, times sigmoid of its column gcol + h
+Tensor head_linear(const Tensor& x, const Tensor& w, const OptTensor& gate, int64_t gcol) {
+  check_t(w, "w");
+  int64_t M, cols;
+  evgpt::HeadLinearArgs a{};
+  a.x = src_of(x, "x", &M, &cols);
+  TORCH_CHECK(w.dim() == 3 && w.size(2) % 64 == 0 && w.size(1) % 64 == 0 && w.size(2) <= 512 && cols >= w.size(0) * w.size(2) &&
+              w.size(0) < 65536 && M < 16 * 65535, "head_linear: w [H, N, K]");
+  a.w = w.data_ptr(); a.H = (int)w.size(0); a.N = (int)w.size(1); a.K = (int)w.size(2);
+  if (gate.has_value()) {
+    int64_t gm, gn;
+    a.gate = src_of(*gate, "gate", &gm, &gn);
+    TORCH_CHECK(gm == M && gcol >= 0 && gcol + a.H <= gn, "head_linear: gate");
+    a.gcol = (int)gcol;
+  }
+  Tensor y = at::empty({M, w.size(0), w.size(1)}, w.options());
+  a.y = y.data_ptr();
+  if (M > 0) evgpt::launch_head_linear(a, is_f32(w), (int)M, cur_stream());
+  return y;
+}
+// Attention of queries q [M, H, R] in the latent space over positions 0 .. pos[row] of each row's cache, the attended latents
+// taken out of it by w_v [H, D, R], heads gated: [M, H, D]
+Tensor latent_attend(const Tensor& q, const Tensor& cache, const OptTensor& row_slot, const Tensor& pos, double scale, int64_t nsplit,
+                     const Tensor& w_v, const Tensor& gate, int64_t gcol) {
+  check_t(q, "q"); check_t(cache, "cache"); check_i(pos, "pos"); check_t(w_v, "w_v");
+  const bool f32 = is_f32(q);
+  const int64_t M = q.size(0), H = q.size(1), R = q.size(2);
+  TORCH_CHECK(q.dim() == 3 && cache.dim() == 3 && cache.size(2) == R && R % 64 == 0 && R <= evgpt::LATENT_MAX && cache.size(1) >= 1 &&
+              is_f32(cache) == f32 && is_f32(w_v) == f32 && pos.numel() >= M && M < 65536 && scale > 0, "latent_attend: q [M, H, R], cache [slots, cap, R]");
+  if (row_slot.has_value()) { check_i(*row_slot, "row_slot"); TORCH_CHECK(row_slot->numel() >= M, "latent_attend: row_slot"); }
+  else TORCH_CHECK(cache.size(0) >= M, "latent_attend: slots");
+  TORCH_CHECK(w_v.dim() == 3 && w_v.size(0) == H && w_v.size(1) % 64 == 0 && w_v.size(2) == R, "latent_attend: w_v [H, D, R]");
+  if (M == 0) return at::empty({0, H, w_v.size(1)}, q.options());
+  const int64_t cap = cache.size(1);
+  if (f32) {
+    Tensor o = at::empty_like(q);
+    evgpt::launch_attn_chunk_decode(q.data_ptr(), cache.data_ptr(), cache.data_ptr(), o.data_ptr(), iptr(row_slot), pos.data_ptr<int>(),
+                                    true, (int)M, (int)H, 1, (int)R, (int)cap, (float)scale, cur_stream());
+    return head_linear(o.view({M, H * R}), w_v, gate, gcol);
+  }
+  TORCH_CHECK(R == 64 || R % 128 == 0, "latent_attend: R 64 or a multiple of 128");
+  nsplit = std::min<int64_t>(std::max<int64_t>(nsplit, 1), 256);
+  Tensor po = at::empty({M, H, nsplit, R}, q.options().dtype(at::kFloat)), pm = at::empty({M, H, nsplit, 2}, q.options().dtype(at::kFloat));
+  evgpt::launch_latent_attend(bptr(q), bptr(cache), po.data_ptr<float>(), pm.data_ptr<float>(), iptr(row_slot), pos.data_ptr<int>(), (int)M,
+                              (int)H, (int)R, (int)cap, (int)nsplit, (float)scale, cur_stream());
+  evgpt::HeadLinearArgs a{};
+  int64_t gm, gn;
+  a.gate = src_of(gate, "gate", &gm, &gn);
+  TORCH_CHECK(gm == M && gcol >= 0 && gcol + H <= gn, "latent_attend: gate");
+  a.gcol = (int)gcol;
+  a.part_o = po.data_ptr<float>(); a.part_ml = pm.data_ptr<float>(); a.pos = pos.data_ptr<int>(); a.cap = (int)cap; a.nsplit = (int)nsplit;
+  a.w = w_v.data_ptr(); a.H = (int)H; a.N = (int)w_v.size(1); a.K = (int)R;
+  Tensor y = at::empty({M, H, w_v.size(1)}, q.options());
+  a.y = y.data_ptr();
+  evgpt::launch_head_linear(a, false, (int)M, cur_stream());
+  return y;
+}
+
+// ---------------------------------------------------------------- experts
+evgpt::MoeRoute route_of(const Tensor& logits, const Tensor& bias, int64_t top, int64_t* rows) {
+  int64_t N;
+  evgpt::MoeRoute r{};
+  r.z = src_of(logits, "router logits", rows, &N);
+  check_f(bias, "bias");
+  TORCH_CHECK(is_f32(logits) && bias.numel() >= 1 && bias.numel() <= 2048 && N >= bias.numel() && top >= 1 && top <= bias.numel() && top <= 64,
+              "router: fp32 logits [M, >= E], up to 2048 experts and 64 chosen");
+  r.bias = bias.data_ptr<float>(); r.E = (int)bias.numel(); r.top = (int)top;
+  return r;
+}
+// {experts [M, top], weights [M, top]}
+std::tuple<Tensor, Tensor> moe_route(const Tensor& logits, const Tensor& bias, int64_t top) {
+  int64_t M;
+  const evgpt::MoeRoute r = route_of(logits, bias, top, &M);
+  Tensor idx = at::empty({M, top}, bias.options().dtype(at::kInt)), w = at::empty({M, top}, bias.options());
+  if (M > 0) evgpt::launch_moe_route(r, idx.data_ptr<int>(), w.data_ptr<float>(), (int)M, cur_stream());
+  return {idx, w};
+}
+// entries of idx [M, top] sorted by expert: {perm, inverse, start [E + 1]}.  idx holds what moe_route wrote: 0 .. E - 1.
+std::tuple<Tensor, Tensor, Tensor> moe_group(const Tensor& idx, int64_t E) {
+  check_i(idx, "idx");
+  TORCH_CHECK(idx.dim() == 2 && E >= 1 && E < 65536 && idx.numel() > 0 && idx.numel() < (1 << 30), "moe_group: idx [M, top]");
+  Tensor perm = at::empty({idx.numel()}, idx.options()), inv = at::empty_like(idx), start = at::empty({E + 1}, idx.options());
+  evgpt::launch_moe_group(idx.data_ptr<int>(), perm.data_ptr<int>(), inv.data_ptr<int>(), start.data_ptr<int>(), (int)idx.numel(), (int)E, cur_stream());
+  return {perm, inv, start};
+}
+// Rows sorted by expert times each expert's matrix w [E, N, K]: row i is x[perm[i] / top] (gather) or x[i].  act >= 0: w's
+// rows are [gate | up] and the result is act(gate) * up [rows, N / 2].
+Tensor moe_linear(const Tensor& x, const Tensor& w, const Tensor& start, const OptTensor& perm, int64_t top, int64_t act) {
+  check_t(x, "x"); check_t(w, "w"); check_i(start, "start");
+  TORCH_CHECK(x.dim() == 2 && w.dim() == 3 && x.scalar_type() == w.scalar_type() && w.size(2) == x.size(1) && start.numel() == w.size(0) + 1,
+              "moe_linear: x [M, K], w [E, N, K], start [E + 1]");
+  const int64_t E = w.size(0), N = w.size(1), K = w.size(2), A = x.size(0);
+  int64_t rows = A;
+  if (perm.has_value()) {
+    check_i(*perm, "perm");
+    rows = perm->numel();
+    TORCH_CHECK(top >= 1 && rows == A * top, "moe_linear: perm has top entries per row");
+  }
+  TORCH_CHECK(rows >= 1 && K % 64 == 0 && K > 0 && N % 64 == 0 && act <= evgpt::GLU_SILU, "moe_linear: K % 64 == 0, N % 64 == 0");
+  TORCH_CHECK(A * K < (1ll << 30) && N * K < (1ll << 30) && rows * N < (1ll << 31), "moe_linear: operands are addressed with 32-bit offsets");
+  const int* pp = iptr(perm);
+  if (is_f32(x)) {
+    Tensor y = at::empty({rows, N}, x.options());
+    evgpt::launch_gemm_f32_grouped(x.data_ptr<float>(), w.data_ptr<float>(), y.data_ptr<float>(), start.data_ptr<int>(), pp, (int)top,
+                                   (int)E, (int)rows, (int)N, (int)K, (int)K, (int)N, cur_stream());
+    if (act < 0) return y;
+    return glu_rows(y, act, true);
+  }
+  Tensor y = at::empty({rows, act < 0 ? N : N / 2}, x.options());
+  // (the tile's activation: 0 silu, 1 gelu)
+  evgpt::launch_gemm_grouped(bptr(x), bptr(w), bptr_mut(y), start.data_ptr<int>(), pp, (int)top, (int)E, (int)A, (int)rows, (int)N, (int)K,
+                             act < 0 ? 0 : (act == evgpt::GLU_SILU ? 1 : 2), cur_stream());
+  return y;
+}
+// Up to four rows x [B, K]: fp32 [B, N] = sum_k weight_k Wd_k (act(Wg_k x) * (Wu_k x)) over the chosen experts
+Tensor moe_step(const Tensor& x, const Tensor& logits, const Tensor& bias, int64_t top, const Tensor& w_gate_up, const Tensor& w_down, int64_t act) {
+  check_t(x, "x"); check_t(w_gate_up, "w_gate_up"); check_t(w_down, "w_down");
+  int64_t B;
+  evgpt::MoeStep s{};
+  s.route = route_of(logits, bias, top, &B);
+  const int64_t E = bias.numel(), K = x.size(1), F = w_down.size(2), N = w_down.size(1);
+  TORCH_CHECK(x.dim() == 2 && x.size(0) == B && w_gate_up.dim() == 3 && w_down.dim() == 3 && w_gate_up.size(0) == E && w_down.size(0) == E &&
+              w_gate_up.size(1) == 2 * F && w_gate_up.size(2) == K && x.scalar_type() == w_gate_up.scalar_type() &&
+              x.scalar_type() == w_down.scalar_type() && K % 8 == 0 && F % 8 == 0 && N % 8 == 0 && B >= 1 && B < 65536 &&
+              (act == evgpt::GLU_GELU_TANH || act == evgpt::GLU_SILU), "moe_step: x [B, K], w_gate_up [E, 2 F, K], w_down [E, N, F]");
+  Tensor h = at::empty({B, top, F}, x.options()), y = at::empty({B, N}, bias.options());
+  s.K = (int)K; s.F = (int)F; s.N = (int)N; s.act = (int)act;
+  s.x = x.data_ptr(); s.w = w_gate_up.data_ptr(); s.h = h.data_ptr();
+  evgpt::launch_moe_step_up(s, is_f32(x), (int)B, cur_stream());
+  s.x = h.data_ptr(); s.w = w_down.data_ptr(); s.y = y.data_ptr<float>();
+  evgpt::launch_moe_step_down(s, is_f32(x), (int)B, cur_stream());
+  return y;
+}
 int64_t gemv_rows_max() { return evgpt::GEMV_ROWS_MAX; }
 int64_t gemv_lds_bytes() { return GEMV_LDS; }
 
@@ -644,8 +949,22 @@ TORCH_LIBRARY(evlay, m) {
   m.def("linear_slabs(Tensor x, Tensor w) -> Tensor", &linear_slabs);
   m.def("linear_glu(Tensor x, Tensor w_gate_up, int act) -> Tensor", &linear_glu);
   m.def("embed_rows(Tensor tok, Tensor embed, float scale) -> Tensor", &embed_rows);
-  m.def("norm_rows(Tensor x, Tensor? sel, Tensor w, int n, float eps, bool f32) -> Tensor", &norm_rows);
-  m.def("add_norm_rows_(Tensor(a!) x, Tensor y, Tensor? w, int n, float eps, bool f32) -> Tensor", &add_norm_rows_);
+  m.def("norm_rows(Tensor x, Tensor? sel, Tensor w, int n, float eps, bool f32, bool layer=False) -> Tensor", &norm_rows);
+  m.def("add_norm_rows_(Tensor(a!) x, Tensor y, Tensor? w, int n, float eps, bool f32, bool layer=False) -> Tensor", &add_norm_rows_);
+  m.def("post_norm_rows_(Tensor(a!) x, Tensor y, Tensor wy, Tensor? w, int n, float eps, bool f32, bool layer) -> Tensor", &post_norm_rows_);
+  m.def("mix_norm_rows_(Tensor(a!) x, Tensor y, Tensor pick, Tensor weights, Tensor? wy, Tensor? w, int n, float eps, bool f32, bool layer) -> Tensor", &mix_norm_rows_);
+  m.def("cap_logits_(Tensor(a!) x, float scale, float cap) -> ()", &cap_logits_);
+  m.def("gemv_rows(Tensor src, int col, int n, Tensor norm, float eps, Tensor w, int c_col, int c_n, Tensor? c_norm, Tensor(a!)? cache, Tensor? pos, Tensor? live) -> Tensor", &gemv_rows);
+  m.def("gemv_plain(Tensor w, Tensor h) -> Tensor", &gemv_plain);
+  m.def("latent_prep_(Tensor src, int q_col, int nq, Tensor? q_norm, int c_col, int nc, Tensor? c_norm, Tensor(a!)? cache, Tensor? row_slot, Tensor row_pos, Tensor? live, float eps, bool f32) -> Tensor", &latent_prep_);
+  m.def("latent_gather(Tensor cache, Tensor copies, int rows) -> Tensor", &latent_gather);
+  m.def("head_linear(Tensor x, Tensor w, Tensor? gate, int gcol) -> Tensor", &head_linear);
+  m.def("latent_attend(Tensor q, Tensor cache, Tensor? row_slot, Tensor pos, float scale, int nsplit, Tensor w_v, Tensor gate, int gcol) -> Tensor", &latent_attend);
+  m.def("latent_max() -> int", []() { return (int64_t)evgpt::LATENT_MAX; });
+  m.def("moe_route(Tensor logits, Tensor bias, int top) -> (Tensor, Tensor)", &moe_route);
+  m.def("moe_group(Tensor idx, int E) -> (Tensor, Tensor, Tensor)", &moe_group);
+  m.def("moe_linear(Tensor x, Tensor w, Tensor start, Tensor? perm, int top, int act) -> Tensor", &moe_linear);
+  m.def("moe_step(Tensor x, Tensor logits, Tensor bias, int top, Tensor w_gate_up, Tensor w_down, int act) -> Tensor", &moe_step);
   m.def("merge_norm_rows_(Tensor(a!) x, Tensor a, Tensor b, Tensor wa, Tensor wb, Tensor? w, int n, float eps, bool f32) -> Tensor", &merge_norm_rows_);
   m.def("glu_rows(Tensor src, int act, bool f32) -> Tensor", &glu_rows);
   m.def("group_norm_rows(Tensor y, Tensor? gate, int gcol, int gate_mode, Tensor w, int heads, int v, int vp, int parts, int ld_out, float eps, bool f32) -> Tensor", &group_norm_rows);
@@ -653,13 +972,13 @@ TORCH_LIBRARY(evlay, m) {
   m.def("sample_top_p(Tensor logits, Tensor(a!) out, float temperature, float top_p, int seed, Tensor step, int top_k=0) -> ()", &sample_top_p);
   m.def("attn_prep_(Tensor src, int q_col, int k_col, int v_col, Tensor? qw, Tensor? kw, int Hq, int Hkv, int D, int nq, int nk, float eps, Tensor cos, Tensor sin, Tensor? row_slot, Tensor row_pos, Tensor? row_kv, Tensor? row_keep, Tensor(a!)? k_buf, Tensor(b!)? v_buf, Tensor(c!) k_cache, Tensor(d!) v_cache) -> Tensor", &attn_prep_);
   m.def("chunk_keys_copy_(Tensor k_cache, Tensor v_cache, Tensor(a!) k_buf, Tensor(b!) v_buf, Tensor copies) -> ()", &chunk_keys_copy_);
-  m.def("attn_chunk(Tensor q, Tensor k, Tensor v, Tensor items, float scale) -> Tensor", &attn_chunk);
-  m.def("attn_runs_(Tensor q, Tensor k, Tensor v, Tensor(a!) o, int q0, int rows, int kv0, int off, int n, float scale) -> ()", &attn_runs_);
+  m.def("attn_chunk(Tensor q, Tensor k, Tensor v, Tensor items, float scale, Tensor? gate=None, int gcol=0) -> Tensor", &attn_chunk);
+  m.def("attn_runs_(Tensor q, Tensor k, Tensor v, Tensor(a!) o, int q0, int rows, int kv0, int off, int n, float scale, Tensor? gate=None, int gcol=0) -> ()", &attn_runs_);
   m.def("attn_chunk_decode(Tensor q, Tensor k_cache, Tensor v_cache, Tensor pos, float scale, int nsplit) -> Tensor", &attn_chunk_decode);
   m.def("scan_prefill_(Tensor q, Tensor k, Tensor v, int H, int per_group, int N, int V, float qscale, Tensor log_decay, Tensor? log_in, Tensor? scale_in, Tensor? skip, Tensor(a!) S, Tensor(b!)? n, Tensor(c!)? m, Tensor chunks, Tensor seqs) -> Tensor", &scan_prefill_);
   m.def("parallel_step_(Tensor src, int[] attn, Tensor? qw, Tensor? kw, float eps, Tensor cos, Tensor sin, Tensor(a!) k_cache, Tensor(b!) v_cache, int[] mem, Tensor ib, Tensor fb, float cap, float qscale, Tensor(c!) S, Tensor(d!) n, Tensor(e!) m, Tensor pos, Tensor? live) -> (Tensor, Tensor)", &parallel_step_);
   m.def("ssd_step_(Tensor src, int[] dims, Tensor conv_w, Tensor conv_b, Tensor(a!) ring, Tensor dt_bias, Tensor a_log, Tensor skip, Tensor(b!) S, Tensor pos, Tensor? live) -> Tensor", &ssd_step_);
-  m.def("gemv_norm(Tensor x, Tensor norm, int n, float eps, Tensor w, int act, Tensor? a, Tensor? b, Tensor? wa, Tensor? wb, Tensor(a!)? x_out) -> Tensor", &gemv_norm);
+  m.def("gemv_norm(Tensor x, Tensor norm, int n, float eps, Tensor w, int act, Tensor? a, Tensor? b, Tensor? wa, Tensor? wb, Tensor(a!)? x_out, bool layer=False, Tensor(b!)? xn_out=None, float? scale=None, float cap=0.0) -> Tensor", &gemv_norm);
   m.def("gemv_add_(Tensor(a!) x, Tensor w, Tensor h) -> ()", &gemv_add_);
   m.def("gemv_group_add_(Tensor(a!) x, Tensor w, Tensor y, Tensor norm, int heads, int v, int vp, int parts, float eps) -> ()", &gemv_group_add_);
   m.def("gemv_branches(Tensor wa, Tensor h, Tensor wb, Tensor y, Tensor gate, int gcol, Tensor norm, int heads, int v, int vp, float eps) -> Tensor", &gemv_branches);

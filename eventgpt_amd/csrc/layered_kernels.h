@@ -17,6 +17,14 @@ struct SrcRows {
   int f32;
 };
 
+// Rows that are weighted sums of rows of another matrix: row = sum over k < top of w[row][k] * y[pick[row][k]].
+struct MixRows {
+  const void* y;    // [..][ld], T
+  const int* pick;  // [rows][top]
+  const float* w;   // [rows][top]
+  int top, ld;
+};
+
 // ---- gemm_f32.hip
 void launch_gemm_f32(const float* A, const float* W, float* C, int M, int N, int K, int lda, int ldw, int ldc,
                      hipStream_t st);
@@ -25,12 +33,21 @@ void launch_gemm_f32(const float* A, const float* W, float* C, int M, int N, int
 enum { GLU_GELU_TANH = 0, GLU_SILU = 1 };
 void launch_embed_rows(const int* tok, const void* embed, bool f32, float scale, float* x, int rows, int ld, int vocab,
                        hipStream_t st);
-// xn[i] = RMS norm of x[sel ? sel[i] : i] * w
+// `layer`: layer norm (mean taken off), otherwise RMS norm.
+// xn[i] = norm of x[sel ? sel[i] : i] * w
 void launch_norm_rows(const float* x, const int* sel, const float* w, void* xn, bool f32, int rows, int n, int ld,
-                      float eps, hipStream_t st);
-// x += y; xn = RMS norm of x * w (skipped when w is null)
+                      float eps, bool layer, hipStream_t st);
+// x += y; xn = norm of x * w (skipped when w is null, here and below)
 void launch_add_norm_rows(float* x, const SrcRows& y, const float* w, void* xn, bool f32, int rows, int n, int ld,
-                          float eps, hipStream_t st);
+                          float eps, bool layer, hipStream_t st);
+// x += norm(y) * wy; xn = norm of x * w
+void launch_post_norm_rows(float* x, const SrcRows& y, const float* wy, const float* w, void* xn, bool f32, int rows, int n,
+                           int ld, float eps, bool layer, hipStream_t st);
+// the same with y the weighted sum of picked rows (without wy: x += y)
+void launch_mix_norm_rows(float* x, const MixRows& y, const float* wy, const float* w, void* xn, bool f32, int rows, int n,
+                          int ld, float eps, bool layer, hipStream_t st);
+// x[i] = cap * tanh(scale * x[i] / cap) (cap 0: scale * x[i]); n % 4 == 0
+void launch_cap_logits(float* x, long long n, float scale, float cap, hipStream_t st);
 // x += (rms(a) * wa + rms(b) * wb) / 2; xn = RMS norm of x * w (skipped when w is null)
 void launch_merge_norm_rows(float* x, const SrcRows& a, const SrcRows& b, const float* wa, const float* wb,
                             const float* w, void* xn, bool f32, int rows, int n, int ld, float eps, hipStream_t st);
@@ -80,11 +97,74 @@ void launch_chunk_keys_copy(const void* k_cache, const void* v_cache, void* k_bu
 // ---- attn_chunk.hip (D a multiple of 64, up to 512; any number of query heads per key head)
 // items [n][4]: {first query row, query rows (<= 64), key buffer row of the chunk's first key, position of the
 // first query within the chunk}
+// kld: elements between rows of k and of v; gate: rows of T whose column h gates head h of the output; or null
 void launch_attn_chunk(const void* q, const void* k, const void* v, void* o, const int* items, int n_items, bool f32,
-                       int Hq, int Hkv, int D, float scale, hipStream_t st);
-// keys 0 .. pos % cap of every sequence's cache
-void launch_attn_chunk_decode(const void* q, const void* k_cache, const void* v_cache, void* o, const int* pos,
+                       int Hq, int Hkv, int D, long long kld, float scale, const void* gate, int gate_ld, hipStream_t st);
+// keys 0 .. pos % cap of every sequence's cache (row b: cache row_slot[b], or b)
+void launch_attn_chunk_decode(const void* q, const void* k_cache, const void* v_cache, void* o, const int* row_slot, const int* pos,
                               bool f32, int B, int Hq, int Hkv, int D, int cap, float scale, hipStream_t st);
+
+// ---- latent.hip: one cached row of R (padded) columns per token, keys and values of all heads linear in it
+constexpr int LATENT_MAX = 512;
+struct LatentPrepArgs {
+  SrcRows src;
+  int q_col, nq, Q;                // query latent: first column, true and padded size; q_out null: none
+  const float* qw;                 // [Q], zero in the padding
+  void* q_out;                     // [rows][Q]
+  int c_col, nc, R;                // key / value latent; cache null: none
+  const float* cw;                 // [R]
+  void* cache;                     // [slots][cap][R]
+  int cap;
+  const int* row_slot;             // [rows] or null: the row's index
+  const int* row_pos;              // [rows]
+  const int* live;                 // [rows]: 0 keeps the row out of the cache; or null
+  float eps;
+};
+void launch_latent_prep(const LatentPrepArgs& a, bool f32, int rows, hipStream_t st);
+// cached rows into a buffer: copies [n][4] of {slot, first position, first buffer row, count}
+void launch_latent_gather(const void* cache, void* buf, const int* copies, int n, bool f32, int cap, int R, hipStream_t st);
+// y[row][h][0 .. N) = W[h] x[row][h][0 .. K), times sigmoid(gate[row][gcol + h]) with a gate; K % 32 == 0, N % 16 == 0
+struct HeadLinearArgs {
+  SrcRows x; int x_col;            // input rows: head h at columns x_col + h * K
+  const float* part_o; const float* part_ml;   // or (bf16) the splits of attend, merged: part_o not null
+  const int* pos; int cap, nsplit;
+  const void* w;                   // [H][N][K]
+  SrcRows gate; int gcol;          // gate.p null: none
+  void* y;                         // [rows][H][N]
+  int H, N, K;
+};
+void launch_head_linear(const HeadLinearArgs& a, bool f32, int rows, hipStream_t st);
+// partial attention of q [rows][H][R] over positions 0 .. pos[row] of the rows' caches: part_o [rows][H][nsplit][R],
+// part_ml [rows][H][nsplit][2] (maximum in log2 units, sum).  R: 64, 128, 256, 384 or 512
+void launch_latent_attend(const bf16_t* q, const bf16_t* cache, float* part_o, float* part_ml, const int* row_slot,
+                          const int* pos, int rows, int H, int R, int cap, int nsplit, float scale, hipStream_t st);
+
+// ---- moe.hip
+// Router logits [rows][>= E] + bias -> the `top` largest in order (the first of equals) and their softmax weights
+struct MoeRoute {
+  SrcRows z;
+  const float* bias;               // [E]
+  int E, top;
+};
+void launch_moe_route(const MoeRoute& r, int* idx, float* w, int rows, hipStream_t st);      // idx, w [rows][top]
+// Entries (row * top + k) sorted by expert: perm [n], its inverse inv [n], start [E + 1]
+void launch_moe_group(const int* idx, int* perm, int* inv, int* start, int n, int E, hipStream_t st);
+// Up to four rows, weights of the chosen experts streamed: h[b][k] = act(Wg x) * (Wu x), y[b] = sum_k w_k Wd h[b][k].
+// w_gate_up [E][2 F][K], w_down [E][N][F]
+struct MoeStep {
+  MoeRoute route;
+  const void* x;                   // up: [B][K]; down: h [B][top][F]
+  const void* w;
+  void* h;                         // up
+  float* y;                        // down: [B][N]
+  int K, F, N, act;
+};
+void launch_moe_step_up(const MoeStep& a, bool f32, int B, hipStream_t st);
+void launch_moe_step_down(const MoeStep& a, bool f32, int B, hipStream_t st);
+// fp32 grouped product (gemm_f32.hip): row i of expert e's group (rows start[e] .. start[e + 1]) is A row perm[i] / top
+// (perm null: i) times W[e] [N][K] -> C row i
+void launch_gemm_f32_grouped(const float* A, const float* W, float* C, const int* start, const int* perm, int top, int E,
+                             int rows, int N, int K, int lda, int ldc, hipStream_t st);
 
 // ---- linear_scan.hip: S_t = exp(a_t) S_(t-1) + b_t v_t k_t^T per head, y_t = S_t q_t
 struct ScanArgs {
@@ -154,19 +234,21 @@ struct StepSsd {
 void launch_ssd_step(const StepSsd& a, const int* pos, const int* live, bool f32, int B, hipStream_t st);
 
 // ---- row_gemv.hip: up to four rows, weights streamed once, the input prepared and the output finished in the launch
-enum { GV_PLAIN = 0, GV_NORM = 1, GV_MERGE = 2, GV_GROUP = 3 };
+enum { GV_PLAIN = 0, GV_NORM = 1, GV_MERGE = 2, GV_GROUP = 3, GV_POST = 4, GV_ROWS = 5 };
 enum { GV_STORE = 0, GV_ADD = 1, GV_GLU = 2 };
 struct GemvInput {
   int kind;
-  const void* x;                   // PLAIN: [B][K] of T; NORM, MERGE: the fp32 stream [B][K]
-  const float* a; const float* b;  // MERGE: branch outputs [B][K], x + (rms(a) wa + rms(b) wb) / 2
+  const void* x;                   // PLAIN: [B][K] of T; NORM, MERGE, POST: the fp32 stream [B][K]
+  const float* a; const float* b;  // MERGE: branch outputs [B][K], x + (rms(a) wa + rms(b) wb) / 2; POST: x + norm(a) wa
   const float* wa; const float* wb;
-  float* x_out;                    // MERGE: the merged stream [B][K]
-  const float* w;                  // NORM, MERGE, GROUP: norm weights [K]
+  float* x_out;                    // MERGE, POST: the new stream [B][K]
+  void* xn_out;                    // NORM, POST: the normed rows [B][K] of T as well; or null
+  const float* w;                  // norm weights [K]
   int n;                           // true width
   float eps;
+  int layer;                       // NORM, POST: layer norm
   const float* y;                  // GROUP: [B][heads * vp] fp32
-  SrcRows gate;
+  SrcRows gate;                    // GROUP: the gate's rows; ROWS: the input rows, from column gcol on
   int gcol, gate_mode;
   int heads, v, vp, parts;
 };
@@ -176,7 +258,19 @@ struct GemvProblem {
   GemvInput in;
   float* y; int ldy;               // STORE: [B][ldy] fp32; ADD: the stream, accumulated
 };
+struct LatentStore {               // latent row b = RMS norm of n columns of src -> cache[b][pos[b]], R columns
+  SrcRows src;
+  int col, n, R;
+  const float* w;                  // [R]
+  float eps;
+  void* cache;                     // [slots][cap][R] of T; null: nothing to do
+  int cap;
+  const int* pos; const int* live;
+};
 struct GemvCall {
+  LatentStore latent;
+  int finish;                      // STORE: y = cap * tanh(scale * y / cap) (cap 0: scale * y)
+  float scale, cap;
   GemvProblem p[2];
   int count;                       // problems in this launch (same epilogue)
   int epilogue;

@@ -11,6 +11,9 @@ Designs built from these parts:
 * **Nusitar** -- layers of type ``parallel`` (a chunk-masked softmax attention and an mLSTM matrix memory
   side by side on the same input) and ``mamba2`` (state-space duality with a short convolution), an fp32
   residual stream, gelu-gated feed-forwards.
+* **Zapipel** -- layers of type ``latent_attention`` (one cached latent per token, which layers can share),
+  layer norms before and after every sublayer, silu-gated feed-forwards that are dense or a mixture of
+  experts, logits scaled and softly capped.
 """
 from __future__ import annotations
 
@@ -145,61 +148,168 @@ class Mamba2Spec:
 
 
 @dataclasses.dataclass(frozen=True)
-class DenseMLPSpec:
-    """``W_down(gelu_tanh(W_gate h) * W_up h)``."""
-    ff: int
-    act: str = "gelu_tanh"
+class LatentAttentionSpec:
+    """Softmax attention whose keys and values are linear in one RMS-normed latent per token, the only thing
+    that is cached.  Queries go through a latent of their own; every head has a sigmoid output gate; there are no
+    positions.  ``kv_from``: the layer whose latents this one reads instead of having its own."""
+    heads: int
+    dim: int
+    vdim: int
+    kv_rank: int
+    q_rank: int
+    scale: float
+    kv_from: Optional[int] = None
 
     @classmethod
-    def from_dict(cls, d, where) -> "DenseMLPSpec":
-        kind, ff = _take(d, where, "kind", "ff")
-        if kind != "dense":
-            raise ValueError(f"{where}.kind {kind!r} is not supported")
+    def from_dict(cls, d, where) -> "LatentAttentionSpec":
+        heads, dim, vdim, kv_rank, q_rank, scale, src = _take(d, where, "heads", "dim", "vdim", "kv_rank", "q_rank", "scale",
+                                                              kv_from=None)
+        _positive(where, heads=heads, dim=dim, vdim=vdim, kv_rank=kv_rank, q_rank=q_rank)
+        if not scale > 0:
+            raise ValueError(f"{where}.scale must be positive")
+        return cls(heads, dim, vdim, kv_rank, q_rank, float(scale), src)
+
+    def check(self, index: int, earlier: List["LayerSpec"], where: str) -> None:
+        """``kv_from`` names an earlier layer with latents of its own and of this size."""
+        j = self.kv_from
+        if j is None:
+            return
+        if not isinstance(j, int) or not 0 <= j < index:
+            raise ValueError(f"{where}.kv_from {j!r} is not an earlier layer")
+        other = earlier[j].mixer
+        if not isinstance(other, LatentAttentionSpec) or other.kv_from is not None or other.kv_rank != self.kv_rank:
+            raise ValueError(f"{where}.kv_from: layer {j} has no latents of its own of size {self.kv_rank}")
+
+    def shapes(self, p: str, width: int) -> Shapes:
+        h = self.heads
+        out = {p + "dq": (self.q_rank, width), p + "dq.norm": (self.q_rank,), p + "uq": (h * self.dim, self.q_rank),
+               p + "uk": (h * self.dim, self.kv_rank), p + "uv": (h * self.vdim, self.kv_rank), p + "g": (h, width),
+               p + "o": (width, h * self.vdim)}
+        if self.kv_from is None:
+            out.update({p + "dkv": (self.kv_rank, width), p + "dkv.norm": (self.kv_rank,)})
+        return out
+
+
+@dataclasses.dataclass(frozen=True)
+class DenseMLPSpec:
+    """``W_down(act(W_gate h) * W_up h)``."""
+    ff: int
+    act: str
+
+    @classmethod
+    def from_dict(cls, d, where, act) -> "DenseMLPSpec":
+        _, ff = _take(d, where, "kind", "ff")
         _positive(where, ff=ff)
-        return cls(ff)
+        return cls(ff, act)
 
     def shapes(self, p: str, width: int) -> Shapes:
         return {p + "gate": (self.ff, width), p + "up": (self.ff, width), p + "down": (width, self.ff)}
 
 
-MIXER_SPECS = {"parallel": ParallelSpec, "mamba2": Mamba2Spec}
+@dataclasses.dataclass(frozen=True)
+class MoESpec:
+    """Mixture of ``experts`` gated units of ``ff``: a token uses the ``top`` ones with the largest router logits,
+    weighted by the softmax over those logits."""
+    experts: int
+    top: int
+    ff: int
+    act: str
+
+    @classmethod
+    def from_dict(cls, d, where, act) -> "MoESpec":
+        _, expert, router = _take(d, where, "kind", "expert", "router")
+        (ff,) = _take(expert, where + ".expert", "ff")
+        experts, top = _take(router, where + ".router", "experts", "top")
+        _positive(where, ff=ff, experts=experts, top=top)
+        if top > experts:
+            raise ValueError(f"{where}.router: {top} of {experts} experts")
+        return cls(experts, top, ff, act)
+
+    def shapes(self, p: str, width: int) -> Shapes:
+        out = {p + "router": (self.experts, width), p + "router.b": (self.experts,)}
+        for i in range(self.experts):
+            out.update(DenseMLPSpec(self.ff, self.act).shapes(f"{p}e{i}.", width))
+        return out
+
+
+MIXER_SPECS = {"parallel": ParallelSpec, "mamba2": Mamba2Spec, "latent_attention": LatentAttentionSpec}
+MLP_SPECS = {"dense": DenseMLPSpec, "moe": MoESpec}
+
+
+@dataclasses.dataclass(frozen=True)
+class Design:
+    """What an architecture fixes: its layer types and feed-forwards, the gated units' activation, the kind of norm and
+    where it stands, and the keys its configuration has besides the common ones."""
+    mixers: Tuple[str, ...]
+    mlps: Tuple[str, ...]
+    act: str
+    norm: str = "rms"              # "rms" or "layer"
+    post_norm: bool = False        # a norm of every sublayer's output as well
+    keys: Tuple[str, ...] = ()
+
+
+DESIGNS = {
+    "Nusitar": Design(("parallel", "mamba2"), ("dense",), "gelu_tanh", keys=("embedding",)),
+    "Zapipel": Design(("latent_attention",), ("dense", "moe"), "silu", norm="layer", post_norm=True,
+                      keys=("logit_scale", "logit_softcap")),
+}
 
 
 @dataclasses.dataclass(frozen=True)
 class LayerSpec:
     type: str
     mixer: Any
-    mlp: Optional[DenseMLPSpec]
+    mlp: Any                       # DenseMLPSpec, MoESpec or None
+    post_norm: bool = False
 
     def shapes(self, p: str, width: int) -> Shapes:
         out = {p + "norm1": (width,), **self.mixer.shapes(p + "mix.", width)}
+        if self.post_norm:
+            out[p + "norm1b"] = (width,)
         if self.mlp is not None:
             out[p + "norm2"] = (width,)
+            if self.post_norm:
+                out[p + "norm2b"] = (width,)
             out.update(self.mlp.shapes(p + "mlp.", width))
         return out
 
 
 class LayeredConfig:
-    """Configuration of a layered decoder (``architecture``, ``vocab``, ``width``, ``norm.eps``,
-    ``embedding.scale`` and the list of ``layers``)."""
+    """Configuration of a layered decoder: ``architecture``, ``vocab``, ``width``, ``norm.eps``, the list of ``layers``
+    and what the architecture has besides (``embedding.scale``; ``logit_scale``, ``logit_softcap``)."""
 
     def __init__(self, d: Dict[str, Any]):
         self.raw = copy.deepcopy(d)
-        known = ("architecture", "vocab", "width", "norm", "embedding", "layers")
-        arch, vocab, width, norm, emb, layers = _take({k: d[k] for k in known if k in d}, "config", *known)
-        self.architecture = arch
+        arch = d.get("architecture")
+        if arch not in DESIGNS:
+            raise ValueError(f"architecture {arch!r}: known are {sorted(DESIGNS)}")
+        self.architecture, self.design = arch, DESIGNS[arch]
+        known = ("vocab", "width", "norm", "layers") + self.design.keys
+        vocab, width, norm, layers, *_ = _take({k: d[k] for k in known if k in d}, "config", *known)
         _positive("config", vocab=vocab, width=width)
         self.vocab_size, self.hidden_size = vocab, width
         self.norm_eps = float(_take(norm, "norm", "eps")[0])
-        self.embedding_scale = float(_take(emb, "embedding", "scale")[0])
+        has = self.design.keys
+        self.embedding_scale = float(_take(d["embedding"], "embedding", "scale")[0]) if "embedding" in has else 1.0
+        self.logit_scale = float(d["logit_scale"]) if "logit_scale" in has else 1.0
+        #: logits are ``cap * tanh(logits / cap)``; None: they are not capped
+        cap = d["logit_softcap"] if "logit_softcap" in has else None
+        if cap is not None and not cap > 0:
+            raise ValueError("config.logit_softcap must be positive")
+        self.logit_softcap = None if cap is None else float(cap)
         self.eos_token_id = d.get("eos_token_id")
         self.layers: List[LayerSpec] = []
         for i, e in enumerate(layers):
             kind, mixer, mlp = _take(e, f"layers[{i}]", "type", "mixer", "mlp")
-            if kind not in MIXER_SPECS:
-                raise ValueError(f"layers[{i}].type {kind!r}: known are {sorted(MIXER_SPECS)}")
-            self.layers.append(LayerSpec(kind, MIXER_SPECS[kind].from_dict(mixer, f"layers[{i}].mixer"),
-                                         None if mlp is None else DenseMLPSpec.from_dict(mlp, f"layers[{i}].mlp")))
+            if kind not in self.design.mixers:
+                raise ValueError(f"layers[{i}].type {kind!r}: {arch} has {sorted(self.design.mixers)}")
+            spec = MIXER_SPECS[kind].from_dict(mixer, f"layers[{i}].mixer")
+            if isinstance(spec, LatentAttentionSpec):
+                spec.check(i, self.layers, f"layers[{i}].mixer")
+            if mlp is not None and mlp.get("kind") not in self.design.mlps:
+                raise ValueError(f"layers[{i}].mlp.kind {mlp.get('kind')!r}: {arch} has {sorted(self.design.mlps)}")
+            ff = None if mlp is None else MLP_SPECS[mlp["kind"]].from_dict(mlp, f"layers[{i}].mlp", self.design.act)
+            self.layers.append(LayerSpec(kind, spec, ff, self.design.post_norm))
         if not self.layers:
             raise ValueError("config: no layers")
 
@@ -270,6 +380,8 @@ class LayeredDecoder:
                 z = z + 3
             elif name.endswith(".i.b"):
                 z = z - 3
+            elif name.endswith("router.b"):
+                z = 0.1 * z
             elif t.dim() == 2:
                 z = z / t.shape[1] ** 0.5
             t.copy_(z)

@@ -22,6 +22,7 @@ class ModelEntry(NamedTuple):
 REGISTRY: Dict[str, ModelEntry] = {
     EventChatConfig.model_type: ModelEntry(EventChatConfig, EventChatModel, "event"),
     "Nusitar": ModelEntry(LayeredConfig, LayeredDecoder, "text"),
+    "Zapipel": ModelEntry(LayeredConfig, LayeredDecoder, "text"),
 }
 
 

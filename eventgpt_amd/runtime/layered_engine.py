@@ -6,8 +6,8 @@ it adds is the stack of mixers (``runtime/mixers.py``) over an fp32 residual str
 
 * a prompt is token ids; several prompts prefill as one pack without padding, long ones in portions;
 * what a sequence keeps depends on the layer -- the current chunk's keys, a recurrent state, the last inputs
-  of a convolution -- and is held per slot in static buffers, so a decode step is one captured graph whose
-  cost and memory do not grow with the context;
+  of a convolution, a latent per token (which several layers may read) -- and is held per slot in static
+  buffers, so a decode step is one captured graph;
 * ``active`` masks a slot's state updates as well as its commit: a recurrent state, unlike a cache row, may
   not be written twice for the same token.
 
@@ -20,14 +20,14 @@ from typing import Dict, List, Optional, Sequence, Tuple
 import torch
 
 from .engine import DecodeEngine, GenerationEngine, persistent_state
-from .mixers import MIXERS, DenseMLP, RowBatch, Sequence_, Stream, pad, pad_to
+from .mixers import MIXERS, MLPS, RowBatch, Sequence_, Stream, pad, pad_to
 
 
 class _Stage:
-    """One residual sublayer and the norm weights that lead into it."""
+    """One residual sublayer, the norm weights that lead into it and those of the norm after it (or None)."""
 
-    def __init__(self, block, norm):
-        self.block, self.norm = block, norm
+    def __init__(self, block, norm, post):
+        self.block, self.norm, self.post = block, norm, post
 
 
 class LayeredEngine(DecodeEngine):
@@ -50,6 +50,9 @@ class LayeredEngine(DecodeEngine):
         self.f32 = self.dtype == torch.float32
         self.width, self.wp, self.eps = cfg.hidden_size, pad(cfg.hidden_size, 64), cfg.norm_eps
         self.V = cfg.vocab_size
+        self.layer_norm = cfg.design.norm == "layer"
+        # logits = cap tanh(scale * logits / cap), or None
+        self._finish = None if cfg.logit_scale == 1.0 and cfg.logit_softcap is None else (cfg.logit_scale, cfg.logit_softcap or 0.0)
         # decode steps of up to this many sequences run on the weight-streaming kernels, more on the few-row GEMM
         self.gemv_rows = int(self.raw.gemv_rows_max())
         self.scan_chunk = int(self.raw.scan_chunk(self.f32))
@@ -66,11 +69,17 @@ class LayeredEngine(DecodeEngine):
         self.final_norm = norm("final.norm")
         self.stages: List[_Stage] = []
         self.layer_ends: List[int] = []      # number of stages after each layer
+        self.mixers: List = []               # one per layer; a layer may read an earlier one's cache
         for i, layer in enumerate(cfg.layers):
             p = f"l{i}."
-            self.stages.append(_Stage(MIXERS[layer.type](self, layer.mixer, lambda n, p=p: t[p + "mix." + n]), norm(p + "norm1")))
+
+            def post(n):
+                return norm(p + n) if layer.post_norm else None
+            self.mixers.append(MIXERS[layer.type](self, layer.mixer, lambda n: t[p + "mix." + n]))
+            self.stages.append(_Stage(self.mixers[-1], norm(p + "norm1"), post("norm1b")))
             if layer.mlp is not None:
-                self.stages.append(_Stage(DenseMLP(self, layer.mlp, lambda n, p=p: t[p + "mlp." + n]), norm(p + "norm2")))
+                block = MLPS[type(layer.mlp)](self, layer.mlp, lambda n: t[p + "mlp." + n])
+                self.stages.append(_Stage(block, norm(p + "norm2"), post("norm2b")))
             self.layer_ends.append(len(self.stages))
         self._init_decode_state(torch.zeros(self.B, self.wp, dtype=torch.float32, device=self.device), cfg.eos_token_id)
         self.active = torch.ones(self.B, dtype=torch.int32, device=self.device)
@@ -91,13 +100,17 @@ class LayeredEngine(DecodeEngine):
         """All layers over the residual rows ``x`` (updated in place, or replaced in the stream that is returned)."""
         stream = Stream(self, x, rows.decode)
         for i, st in enumerate(self.stages):
+            stream.post = st.post
             st.block.forward(rows, stream, st.norm)
             if collect is not None and i + 1 in self.layer_ends:
                 collect.append(stream.settle()[:, :self.width].clone())
         return stream
 
     def _logits(self, xn: torch.Tensor) -> torch.Tensor:
-        return self.raw.linear(xn, self.head, True)[:, :self.V]
+        logits = self.raw.linear(xn, self.head, True)
+        if self._finish:
+            self.raw.cap_logits_(logits, *self._finish)
+        return logits[:, :self.V]
 
     def _layers_step(self) -> None:
         rows = RowBatch(self.device, True, pos=self.pos, live=self.active)
@@ -108,7 +121,7 @@ class LayeredEngine(DecodeEngine):
         if stream is None:                   # after a prefill: ``x`` holds the last rows' residual stream
             stream = Stream(self, self.x, True)
         if stream.few:
-            logits = stream.gemv(self.final_norm, self.head)[:, :self.V]
+            logits = stream.gemv(self.final_norm, self.head, -1, None, *(self._finish or (None, 0.0)))[:, :self.V]
         else:
             logits = self._logits(stream.normed(self.final_norm))
         if not greedy or want_logits:
@@ -194,7 +207,8 @@ class LayeredEngine(DecodeEngine):
                         keys.append((i, w))
             if sel:
                 picked = torch.tensor(sel, dtype=torch.int32).to(self.device)
-                lg = self._logits(self.raw.norm_rows(x, picked, self.final_norm, self.width, self.eps, self.f32))
+                lg = self._logits(self.raw.norm_rows(x, picked, self.final_norm, self.width, self.eps, self.f32,
+                                                       self.layer_norm))
                 rows.update(zip(keys, lg))
         logits = None
         if want is not None and any(len(w) for w in want):

@@ -23,7 +23,8 @@ from typing import Dict, List, Optional, Sequence, Tuple
 
 import torch
 
-from ..models.layered import AttentionSpec, DenseMLPSpec, MatrixMemorySpec, Mamba2Spec, ParallelSpec
+from ..models.layered import (AttentionSpec, DenseMLPSpec, LatentAttentionSpec, MatrixMemorySpec, Mamba2Spec, MoESpec,
+                              ParallelSpec)
 
 ATTN_TILE = 64           # query rows per work item of the chunk attention
 GATE_NONE, GATE_SILU_BEFORE, GATE_SIGMOID_AFTER = 0, 1, 2      # group_norm_rows
@@ -41,6 +42,11 @@ def pad_value(n: int) -> int:
 def pad_attn_head(n: int) -> int:
     """Padded head size of the attention kernels: 64 and 128 have the flash kernels, larger ones the general one."""
     return 64 if n <= 64 else 128 if n <= 128 else pad(n, 64)
+
+
+def pad_latent(n: int) -> int:
+    """Padded latent size: 64, or a multiple of 128."""
+    return 64 if n <= 64 else pad(n, 128)
 
 
 def pad_rows(w: torch.Tensor, groups: int, size: int, padded: int) -> torch.Tensor:
@@ -141,41 +147,90 @@ class RowBatch:
         self._tables[size] = t
         return t
 
+    def causal_tables(self):
+        """For plain causal attention: ``(runs, items, copies, kv_rows)`` of ``chunk_tables``, where a buffer holds
+        every key of every sequence and ``copies`` brings all of them from the caches."""
+        t = self._tables.get("causal")
+        if t is None:
+            runs: List[Tuple[int, int, int, int, int]] = []
+            items: List[int] = []
+            copies: List[int] = []
+            kv = 0
+            for s in self.seqs:
+                runs.append((s.row0, s.rows, kv, s.start, 1))
+                for a in range(0, s.rows, ATTN_TILE):
+                    items += [s.row0 + a, min(ATTN_TILE, s.rows - a), kv, s.start + a]
+                copies += [s.slot, 0, kv, s.start + s.rows]
+                kv += s.start + s.rows
+            items_d, copies_d = self._upload(items, copies)
+            t = self._tables["causal"] = (runs, items_d.view(-1, 4), copies_d.view(-1, 4), kv)
+        return t
+
+    def latents(self, cache: torch.Tensor, gather) -> torch.Tensor:
+        """All cached rows of the pack's sequences, in the order of ``causal_tables``; shared by the layers that read
+        this cache.  ``gather(cache, copies, rows)`` copies them where they are not already one run of the cache."""
+        key = ("latents", cache.data_ptr())
+        t = self._tables.get(key)
+        if t is None:
+            _, _, copies, kv = self.causal_tables()
+            one = self.seqs[0]
+            t = cache[one.slot, :kv] if len(self.seqs) == 1 else gather(cache, copies, kv)
+            self._tables[key] = t
+        return t
+
 
 class Stream:
-    """The fp32 residual rows, with the last sublayer's contribution possibly still to be added: ``pending`` is None,
-    ``(y,)`` (add the rows or slabs ``y``) or ``(a, b, wa, wb)`` (add the mean of the two normed branches)."""
+    """The fp32 residual rows, with the last sublayer's contribution possibly still to be added.  ``pending`` is None or
+    names how: ``("add", y)`` the rows or slabs ``y``; ``("merge", a, b, wa, wb)`` the mean of two normed branches;
+    ``("post", y, w)`` the normed ``y``; ``("mix", y, pick, weights, w)`` the weighted sum of picked rows of ``y``, normed
+    if there is a ``w``.  ``post`` is the weight of the norm after the current sublayer, or None."""
 
     def __init__(self, engine, x: torch.Tensor, decode: bool):
         self.raw, self.n, self.eps, self.f32 = engine.raw, engine.width, engine.eps, engine.dtype == torch.float32
-        self.x, self.pending = x, None
+        self.layer = engine.layer_norm
+        self.x, self.pending, self.post = x, None, None
         self.few = decode and x.shape[0] <= engine.gemv_rows
 
+    def leave(self, y: torch.Tensor) -> None:
+        """The current sublayer's output, to be added."""
+        self.pending = ("add", y) if self.post is None else ("post", y, self.post)
+
     def normed(self, norm: Optional[torch.Tensor]) -> torch.Tensor:
-        """RMS norm of the stream in the storage type, pending contribution included (None: just add it)."""
+        """Norm of the stream in the storage type, pending contribution included (None: just add it)."""
         pending, self.pending = self.pending, None
+        last = (norm, self.n, self.eps, self.f32)
         if pending is None:
-            return self.raw.norm_rows(self.x, None, norm, self.n, self.eps, self.f32) if norm is not None else None
-        if len(pending) == 1:
-            return self.raw.add_norm_rows_(self.x, pending[0], norm, self.n, self.eps, self.f32)
-        return self.raw.merge_norm_rows_(self.x, *pending, norm, self.n, self.eps, self.f32)
+            return self.raw.norm_rows(self.x, None, *last, self.layer) if norm is not None else None
+        kind, *args = pending
+        if kind == "add":
+            return self.raw.add_norm_rows_(self.x, *args, *last, self.layer)
+        if kind == "post":
+            return self.raw.post_norm_rows_(self.x, *args, *last, self.layer)
+        if kind == "mix":
+            return self.raw.mix_norm_rows_(self.x, *args, *last, self.layer)
+        return self.raw.merge_norm_rows_(self.x, *args, *last)
 
     def settle(self) -> torch.Tensor:
         if self.pending is not None:
             self.normed(None)
         return self.x
 
-    def gemv(self, norm: torch.Tensor, w: torch.Tensor, act: int = -1) -> torch.Tensor:
-        """``w`` times the normed stream in one launch (a few rows): fp32 rows, or ``act(gate) * up``."""
+    def gemv(self, norm: torch.Tensor, w: torch.Tensor, act: int = -1, xn: Optional[torch.Tensor] = None,
+             scale: Optional[float] = None, cap: float = 0.0) -> torch.Tensor:
+        """``w`` times the normed stream in one launch (a few rows): fp32 rows, or ``act(gate) * up``.  ``xn`` also gets the
+        normed rows; ``scale`` and ``cap``: the rows are ``cap tanh(scale y / cap)``."""
         pending, self.pending = self.pending, None
-        if pending is not None and len(pending) == 1:
+        if pending is not None and pending[0] in ("add", "mix"):
             self.pending = pending
             self.settle()
             pending = None
+        last = (self.layer, xn, scale, cap)
         if pending is None:
-            return self.raw.gemv_norm(self.x, norm, self.n, self.eps, w, act, None, None, None, None, None)
+            return self.raw.gemv_norm(self.x, norm, self.n, self.eps, w, act, None, None, None, None, None, *last)
         out = torch.empty_like(self.x)       # blocks read the old stream while one of them writes the new one
-        y = self.raw.gemv_norm(self.x, norm, self.n, self.eps, w, act, *pending, out)
+        kind, *args = pending
+        a, b, wa, wb = args if kind == "merge" else (args[0], None, args[1], None)
+        y = self.raw.gemv_norm(self.x, norm, self.n, self.eps, w, act, a, b, wa, wb, out, *last)
         self.x = out
         return y
 
@@ -210,7 +265,7 @@ class Projection:
     def prompt(self, stream: Stream, norm: torch.Tensor):
         """``(sections in the storage type, gate sections in fp32)``."""
         xn = stream.normed(norm)
-        return self.raw.linear(xn, self.w_main, False), self.raw.linear(xn, self.w_gate, True)
+        return self.raw.linear(xn, self.w_main, False), self.raw.linear(xn, self.w_gate, True) if self.w_gate.shape[0] else None
 
     def gate_col(self, name: str) -> int:
         return self.col[name] - self.n_main
@@ -349,7 +404,7 @@ class ParallelMixer(Mixer):
             src, gates = self.proj.prompt(stream, norm)
             a = raw.linear(left.prompt(rows, src, col), left.w_o, True)
             b = raw.linear(right.prompt(rows, src, gates, self.proj), right.w_o, True)
-        stream.pending = (a, b, self.w_left, self.w_right)
+        stream.pending = ("merge", a, b, self.w_left, self.w_right)
 
 
 class Mamba2Mixer(Mixer):
@@ -381,11 +436,11 @@ class Mamba2Mixer(Mixer):
             src = self.proj.step(stream, norm)
             y = raw.ssd_step_(src, [col["z"], col["x"], col["dt"], H, G, N, V], self.conv_w, self.conv_b, self.ring,
                               self.dt_bias, self.a_log, self.skip, self.S, rows.pos, rows.live)
-            if self.few(stream, self.kp):
+            if self.few(stream, self.kp) and stream.post is None:
                 raw.gemv_group_add_(stream.settle(), self.w_o, y, *head_norm, self.eps)
                 return
             y = raw.group_norm_rows(y, None, 0, GATE_NONE, *head_norm, self.kp, self.eps, self.f32)
-            stream.pending = (raw.linear_slabs(y, self.w_o),)
+            stream.leave(raw.linear_slabs(y, self.w_o))
             return
         src, gates = self.proj.prompt(stream, norm)
         log_decay, dt = raw.ssd_gates(gates, self.proj.gate_col("dt"), self.dt_bias, self.a_log)
@@ -395,7 +450,95 @@ class Mamba2Mixer(Mixer):
         y = raw.scan_prefill_(c, b, xs, H, H // G, N, V, 1.0, log_decay, None, dt, self.skip, self.S, None, None, rows.chunks,
                               rows.scan_seqs)
         y = raw.group_norm_rows(y, src, col["z"], GATE_SILU_BEFORE, *head_norm, self.kp, self.eps, self.f32)
-        stream.pending = (raw.linear(y, self.w_o, True),)
+        stream.leave(raw.linear(y, self.w_o, True))
+
+
+class LatentAttentionMixer(Mixer):
+    """A prompt expands the latents of its keys to keys and values of every head and runs the causal attention kernels on
+    them; a decode step (and a short portion of a long sequence) takes its queries into the latent space instead and
+    attends over the cached rows themselves."""
+
+    def __init__(self, engine, spec: LatentAttentionSpec, t):
+        super().__init__(engine)
+        self.spec = s = spec
+        self.D = D = pad_attn_head(max(s.dim, s.vdim))
+        self.R = R = pad_latent(s.kv_rank)
+        self.Q = Q = pad(s.q_rank, 64)
+        if D > 512 or R > self.raw.latent_max():
+            raise ValueError(f"heads of {max(s.dim, s.vdim)} and latents of {s.kv_rank} elements (at most 512, {self.raw.latent_max()})")
+        H = s.heads
+        sections = [("q", pad_to(t("dq"), Q, self.width))]
+        self.cache = None
+        if s.kv_from is None:
+            sections.append(("c", pad_to(t("dkv"), R, self.width)))
+            self.c_norm = pad_to(self._w32(t("dkv.norm")), R)
+            self.cache = torch.zeros(self.slots, engine.l_max, R, dtype=self.dtype, device=self.device)
+        sections.append(("g", pad_to(t("g"), pad(H, 8), self.width)))
+        self.owner = self if s.kv_from is None else engine.mixers[s.kv_from]
+        self.proj = Projection(engine.raw, sections, [], self.wp)
+        self.q_norm = pad_to(self._w32(t("dq.norm")), Q)
+        self.w_uq = pad_to(pad_rows(t("uq"), H, s.dim, D), H * D, Q)
+        uk, uv = pad_to(pad_rows(t("uk"), H, s.dim, D), H * D, R), pad_to(pad_rows(t("uv"), H, s.vdim, D), H * D, R)
+        self.w_ukv = torch.cat([uk, uv])                                   # a prompt's keys and values
+        self.w_absorb = uk.view(H, D, R).transpose(1, 2).contiguous()      # queries into the latent space [H, R, D]
+        self.w_value = self.w_ukv[H * D:].view(H, D, R)                    # attended latents out of it
+        self.w_o = pad_to(pad_cols(t("o"), H, s.vdim, D), self.wp, H * D)
+
+    def splits(self, rows: int) -> int:
+        """Key splits of the attention over the cache: about one workgroup per CU."""
+        tiles = -(-self.spec.heads // 16)
+        return max(1, min(64, 256 // max(1, rows * tiles)))
+
+    def absorbs(self, rows: RowBatch) -> bool:
+        """Whether a pack's queries attend over the cached rows: few of them per key, so that expanding every key costs
+        more.  (Work per head in multiply-adds; a quarter of the rate of the prompt kernels.)"""
+        if any(s.start == 0 for s in rows.seqs):
+            return False
+        R, D, expand, direct = self.R, self.D, 0, 0
+        for s in rows.seqs:
+            keys = s.start + s.rows
+            expand += 2 * keys * D * (R + s.rows)
+            direct += 2 * s.rows * (keys * R * 4 + D * R)
+        return direct < expand
+
+    def attend(self, rows: RowBatch, q: torch.Tensor, src: torch.Tensor) -> torch.Tensor:
+        """Gated attention outputs of query rows ``[M, H * D]``, over the cache."""
+        raw, s = self.raw, self.spec
+        ql = raw.head_linear(q, self.w_absorb, None, 0)
+        o = raw.latent_attend(ql, self.owner.cache, rows.slot, rows.pos, s.scale, self.splits(ql.shape[0]), self.w_value, src,
+                              self.proj.col["g"])
+        return o.view(o.shape[0], -1)
+
+    def prompt_attention(self, rows: RowBatch, q: torch.Tensor, src: torch.Tensor) -> torch.Tensor:
+        raw, s, D = self.raw, self.spec, self.D
+        H = s.heads
+        runs, items, _, kv_rows = rows.causal_tables()
+        kv = raw.linear(rows.latents(self.owner.cache, raw.latent_gather), self.w_ukv, False)
+        q, k, v = q.view(-1, H, D), kv[:, :H * D].unflatten(1, (H, D)), kv[:, H * D:].unflatten(1, (H, D))
+        gate = (src, self.proj.col["g"])
+        if not self.f32 and D <= 128 and max(r[1] for r in runs) > 256:
+            o = torch.empty_like(q)
+            for q0, n, key0, off, reps in runs:
+                raw.attn_runs_(q, k, v, o, q0, n, key0, off, reps, s.scale, *gate)
+        else:
+            o = raw.attn_chunk(q, k, v, items, s.scale, *gate)
+        return o.view(o.shape[0], -1)
+
+    def forward(self, rows: RowBatch, stream: Stream, norm: torch.Tensor) -> None:
+        raw, s, col = self.raw, self.spec, self.proj.col
+        store = (col["c"], s.kv_rank, self.c_norm, self.cache) if self.cache is not None else (0, 0, None, None)
+        src = self.proj.step(stream, norm) if rows.decode else self.proj.prompt(stream, norm)[0]
+        if rows.decode and self.few(stream, self.Q):
+            q = raw.gemv_rows(src, col["q"], s.q_rank, self.q_norm, self.eps, self.w_uq, *store, rows.pos, rows.live)
+        else:
+            cq = raw.latent_prep_(src, col["q"], s.q_rank, self.q_norm, *store, rows.slot, rows.pos, rows.live, self.eps, self.f32)
+            q = raw.linear_slabs(cq, self.w_uq) if rows.decode else raw.linear(cq, self.w_uq, False)
+        if rows.decode or self.absorbs(rows):
+            o = self.attend(rows, q, src)
+        else:
+            o = self.prompt_attention(rows, q, src)
+        stream.leave(raw.gemv_plain(self.w_o, o) if stream.few else
+                     raw.linear_slabs(o, self.w_o) if rows.decode else raw.linear(o, self.w_o, True))
 
 
 class DenseMLP(Mixer):
@@ -411,10 +554,46 @@ class DenseMLP(Mixer):
         raw = self.raw
         if stream.few:
             h = stream.gemv(norm, self.w_gate_up, self.act)
-            raw.gemv_add_(stream.settle(), self.w_down, h)
+            if stream.post is None:
+                raw.gemv_add_(stream.settle(), self.w_down, h)
+            else:
+                stream.leave(raw.gemv_plain(self.w_down, h))
             return
         h = raw.linear_glu(stream.normed(norm), self.w_gate_up, self.act)
-        stream.pending = (raw.linear_slabs(h, self.w_down) if rows.decode else raw.linear(h, self.w_down, True),)
+        stream.leave(raw.linear_slabs(h, self.w_down) if rows.decode else raw.linear(h, self.w_down, True))
 
 
-MIXERS = {"parallel": ParallelMixer, "mamba2": Mamba2Mixer}
+class MoE(Mixer):
+    """Mixture of experts.  A few rows stream the weights of their own experts; more rows are sorted by expert and go through
+    grouped products, and the residual kernel sums each row's share of them."""
+
+    def __init__(self, engine, spec: MoESpec, t):
+        super().__init__(engine)
+        from ..ops.layered import GLU_ACTS
+        self.spec, self.act = spec, GLU_ACTS[spec.act]
+        fp, E = pad(spec.ff, 64), spec.experts
+        self.w_router = pad_to(t("router"), pad(E, 8), self.wp)
+        self.bias = self._w32(t("router.b"))
+        self.w_gate_up = torch.stack([torch.cat([pad_to(t(f"e{e}.gate"), fp, self.wp), pad_to(t(f"e{e}.up"), fp, self.wp)])
+                                      for e in range(E)])
+        self.w_down = torch.stack([pad_to(t(f"e{e}.down"), self.wp, fp) for e in range(E)])
+
+    def forward(self, rows: RowBatch, stream: Stream, norm: torch.Tensor) -> None:
+        raw, top = self.raw, self.spec.top
+        if stream.few:
+            xn = torch.empty(stream.x.shape, dtype=self.dtype, device=self.device)
+            logits = stream.gemv(norm, self.w_router, xn=xn)
+            y = raw.moe_step(xn, logits, self.bias, top, self.w_gate_up, self.w_down, self.act)
+            stream.leave(y)
+            return
+        xn = stream.normed(norm)
+        logits = raw.linear(xn, self.w_router, True)
+        idx, weights = raw.moe_route(logits, self.bias, top)
+        perm, inv, start = raw.moe_group(idx, self.spec.experts)
+        h = raw.moe_linear(xn, self.w_gate_up, start, perm, top, self.act)
+        y = raw.moe_linear(h, self.w_down, start, None, 1, -1)
+        stream.pending = ("mix", y, inv, weights, stream.post)
+
+
+MIXERS = {"parallel": ParallelMixer, "mamba2": Mamba2Mixer, "latent_attention": LatentAttentionMixer}
+MLPS = {DenseMLPSpec: DenseMLP, MoESpec: MoE}
