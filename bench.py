@@ -101,9 +101,11 @@ def parse_args(argv=None):
     ap.add_argument("--weight-format", choices=["bf16", "nf4", "fp4"], default="bf16",
                     help="nf4/fp4: the reference's 4-bit rows (bitsandbytes load_in_4bit); not the headline config")
     ap.add_argument("--layered", default=None, metavar="SIZES",
-                    help="instead of the headline: prefill and decode of a layered decoder (Nusitar) beside a LLaMA decoder "
+                    help="instead of the headline: prefill and decode of a layered decoder beside a LLaMA decoder "
                          "of equal size, one JSON line per pass (1b, 7b or both with a comma); one GPU")
-    ap.add_argument("--layered-only", choices=["both", "nusitar", "llama"], default="both", help="measure one of the two models")
+    ap.add_argument("--layered-design", choices=["nusitar", "zapipel"], default="nusitar", help="which layered decoder")
+    ap.add_argument("--layered-only", choices=["both", "nusitar", "zapipel", "llama"], default="both",
+                    help="measure one of the two models")
     ap.add_argument("--layered-pass", default=None, metavar="PASS",
                     help="one pass only, e.g. prefill:1x4096 or decode:8 (for profiling)")
     ap.add_argument("--rehearsal", action="store_true",
@@ -247,7 +249,7 @@ def layered_main(args) -> None:
         else:
             b, n = (int(v) for v in what.split("x"))
             kw.update({"prompts": (n,)} if b == 1 else {"packs": ((b, n),)})
-    layered_bench.run(sizes=tuple(args.layered.split(",")), only=args.layered_only, emit=lambda s: print(s, flush=True), **kw)
+    layered_bench.run(sizes=tuple(args.layered.split(",")), only=args.layered_only, design=args.layered_design, emit=lambda s: print(s, flush=True), **kw)
 
 
 def build_model(args, dev):

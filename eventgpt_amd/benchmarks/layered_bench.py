@@ -1,22 +1,26 @@
 """Prefill and decode throughput of a layered decoder beside a LLaMA decoder of equal size.
 
-``bench.py --layered [1b,7b]`` runs this; weights are random, layers have the sizes of real models of that
-width, the stack is ``2 n`` layers (``mamba2``, ``parallel``, ...) and the LLaMA stack has the number of
-layers that comes closest in parameters.  Every row prints both models' time and what it means against the
-bound of that pass: decoder weights over time for decode steps, 2 x parameters x tokens over time for prompts.
+``bench.py --layered 1b,7b [--layered-design nusitar|zapipel]`` runs this; weights are random, layers have the
+sizes of real models of that width, the stack is ``2 n`` layers (Nusitar: ``mamba2``, ``parallel``, ...;
+Zapipel: latent attention with a dense feed-forward, then on the same latents with experts, ...) and the LLaMA
+stack has the number of layers that comes closest in the parameters a token uses.  Every row prints both models'
+time and what it means against the bound of that pass: decoder weights over time for decode steps, 2 x parameters
+x tokens over time for prompts.
 """
 from __future__ import annotations
 
 import json
+import re
 import time
 from typing import Dict, List
 
 import torch
 
 SIZES: Dict[str, Dict[str, int]] = {
-    "1b": dict(width=2048, ff=5632, heads=16, kv_heads=4, memory_heads=4, mamba_heads=64, groups=4),
-    "7b": dict(width=4096, ff=11008, heads=32, kv_heads=8, memory_heads=8, mamba_heads=128, groups=8),
+    "1b": dict(width=2048, ff=5632, heads=16, kv_heads=4, memory_heads=4, mamba_heads=64, groups=4, q_rank=768, expert_ff=2816),
+    "7b": dict(width=4096, ff=11008, heads=32, kv_heads=8, memory_heads=8, mamba_heads=128, groups=8, q_rank=1536, expert_ff=5504),
 }
+KV_RANK, EXPERTS, TOP = 512, 8, 2
 
 
 def layered_config(size: str, pairs: int, vocab: int = 32000) -> dict:
@@ -31,11 +35,27 @@ def layered_config(size: str, pairs: int, vocab: int = 32000) -> dict:
             "embedding": {"scale": 1.0}, "layers": [mam, par] * pairs}
 
 
+def latent_config(size: str, pairs: int, vocab: int = 32000) -> dict:
+    s = SIZES[size]
+    mix = {"heads": s["heads"], "dim": 128, "vdim": 128, "kv_rank": KV_RANK, "q_rank": s["q_rank"], "scale": 128 ** -0.5}
+    layers = []
+    for i in range(pairs):
+        layers.append({"type": "latent_attention", "mixer": mix, "mlp": {"kind": "dense", "ff": s["ff"]}})
+        layers.append({"type": "latent_attention", "mixer": {**mix, "kv_from": 2 * i},
+                       "mlp": {"kind": "moe", "expert": {"ff": s["expert_ff"]}, "router": {"experts": EXPERTS, "top": TOP}}})
+    return {"architecture": "Zapipel", "vocab": vocab, "width": s["width"], "norm": {"eps": 1e-6}, "logit_scale": 1.0,
+            "logit_softcap": 30.0, "layers": layers}
+
+
+CONFIGS = {"nusitar": layered_config, "zapipel": latent_config}
+
+
 def layer_params(model) -> int:
-    """Matrix parameters of the decoder layers (no embedding, no head)."""
+    """Matrix parameters of the decoder layers that a token uses (no embedding, no head; the chosen experts)."""
     named = model.tensors.items() if hasattr(model, "tensors") else ((n, p) for n, p in model.model.named_parameters())
     skip = ("embed", "head", "visual", "feature")
-    return sum(t.numel() for n, t in named if t.dim() == 2 and not any(k in n for k in skip))
+    return sum(t.numel() * (TOP / EXPERTS if re.search(r"mlp\.e\d+\.", n) else 1)
+               for n, t in named if t.dim() == 2 and not any(k in n for k in skip))
 
 
 def llama_like(size: str, params: int, vocab: int, dev):
@@ -85,7 +105,7 @@ def decode_ms(engine, prompts, n: int) -> float:
 
 
 def run(sizes=("1b", "7b"), pairs: int = 4, prompts=(512, 4096), packs=((8, 512),), streams=(1, 8, 32), context: int = 1024,
-        steps: int = 40, only: str = "both", emit=print) -> List[dict]:
+        steps: int = 40, only: str = "both", design: str = "nusitar", emit=print) -> List[dict]:
     from ..models import LayeredConfig, LayeredDecoder
     from ..parallel.tp import TensorParallelEngine
     from ..runtime.layered_engine import LayeredEngine
@@ -93,12 +113,12 @@ def run(sizes=("1b", "7b"), pairs: int = 4, prompts=(512, 4096), packs=((8, 512)
     vocab = 32000
     out: List[dict] = []
     for size in sizes:
-        cfg = layered_config(size, pairs, vocab)
+        cfg = CONFIGS[design](size, pairs, vocab)
         model = LayeredDecoder.from_config(LayeredConfig(cfg), torch.bfloat16, dev, seed=0)
-        llama = llama_like(size, layer_params(model), vocab, dev)
+        llama = llama_like(size, int(layer_params(model)), vocab, dev)
         width = cfg["width"]
-        models = {"nusitar": model, "llama": llama}
-        params = {k: layer_params(m) + vocab * width for k, m in models.items()}
+        models = {design: model, "llama": llama}
+        params = {k: int(layer_params(m)) + vocab * width for k, m in models.items()}
         which = [k for k in models if only in ("both", k)]
 
         def ids(n):
@@ -109,7 +129,7 @@ def run(sizes=("1b", "7b"), pairs: int = 4, prompts=(512, 4096), packs=((8, 512)
 
         def engine(k, batch, length):
             kw = dict(max_len=length + 256, max_batch=batch, max_new_tokens=512)
-            if k == "nusitar":
+            if k == design:
                 return LayeredEngine(model, **kw)
             return llama.engine(max_len=length + 256, max_new_tokens=512) if batch == 1 else TensorParallelEngine(llama, None, **kw)
 
@@ -118,7 +138,7 @@ def run(sizes=("1b", "7b"), pairs: int = 4, prompts=(512, 4096), packs=((8, 512)
             for k in which:
                 llama._engine = None
                 e = engine(k, batch, length)
-                ms = fn(e, [(ids if k == "nusitar" else emb)(length) for _ in range(batch)])
+                ms = fn(e, [(ids if k == design else emb)(length) for _ in range(batch)])
                 work = params[k] * 2
                 if kind == "prefill":
                     r[k] = {"ms": round(ms, 3), "tok_s": round(batch * length / ms * 1e3),
@@ -135,7 +155,7 @@ def run(sizes=("1b", "7b"), pairs: int = 4, prompts=(512, 4096), packs=((8, 512)
             row("prefill", b, n, lambda e, p: prefill_ms(e, p, 8))
         for b in streams:
             row("decode", b, context, lambda e, p: decode_ms(e, p, steps))
-        emit(json.dumps({"size": size, "layers": {"nusitar": 2 * pairs, "llama": llama.config.num_hidden_layers},
+        emit(json.dumps({"size": size, "layers": {design: 2 * pairs, "llama": llama.config.num_hidden_layers},
                          "params": {k: v for k, v in params.items()}}))
         del model, llama, models
         torch.cuda.empty_cache()
