@@ -29,87 +29,76 @@ __device__ __forceinline__ float dot16(const u32x4_t& w, const u32x4_t& x, float
 
 constexpr int GV_KEEP = 2;     // chunks of eight a thread keeps while it norms a row (4096 columns)
 
+// f(k, c) for the thread's kept chunks of a row of K columns
+template <typename F> __device__ __forceinline__ void kept_chunks(int K, F f) {
+#pragma unroll
+  for (int k = 0; k < GV_KEEP; ++k) {
+    const int c = (threadIdx.x + k * 256) * 8;
+    if (c < K) f(k, c);
+  }
+}
+
 template <typename T>
 __device__ void prepare_norm(const GemvInput& in, int b, int K, T* xs, float* red, bool lead) {
   const float* x = static_cast<const float*>(in.x) + static_cast<long long>(b) * K;
   const bool rows = in.kind == GV_ROWS;
-  float keep[GV_KEEP][8];
+  float keep[GV_KEEP][8], wk[GV_KEEP][8];
   auto value = [&](int c, float (&v)[8]) {
-    if (!rows) { load8(x + c, v); return; }
-    if (c + 8 <= in.n) { src8(in.gate, b, in.gcol + c, v); return; }
-#pragma unroll
-    for (int i = 0; i < 8; ++i) v[i] = c + i < in.n ? src1(in.gate, b, in.gcol + c + i) : 0.f;
+    if (!rows) load8(x + c, v);
+    else section8(in.gate, b, in.gcol, in.n, c, v);
   };
-#pragma unroll
-  for (int k = 0; k < GV_KEEP; ++k) {
-    const int c = (threadIdx.x + k * 256) * 8;
-    if (c < K) value(c, keep[k]);
-  }
+  kept_chunks(K, [&](int k, int c) { value(c, keep[k]); load8(in.w + c, wk[k]); });
   const RowStat st = row_stat<GV_KEEP>(keep, in.n, K, in.eps, in.layer != 0, red, value);
-  auto put = [&](int c, const float (&v)[8]) {
-    float w[8];
-    load8(in.w + c, w);
+  auto put = [&](int c, const float (&v)[8], float (&w)[8]) {
 #pragma unroll
     for (int i = 0; i < 8; ++i) w[i] *= (v[i] - st.mean) * st.r;
     store8(xs + c, w);
     if (lead && in.xn_out) store8(static_cast<T*>(in.xn_out) + static_cast<long long>(b) * K + c, w);
   };
-#pragma unroll
-  for (int k = 0; k < GV_KEEP; ++k) {
-    const int c = (threadIdx.x + k * 256) * 8;
-    if (c < K) put(c, keep[k]);
-  }
+  kept_chunks(K, [&](int k, int c) { put(c, keep[k], wk[k]); });
   for (int c = (threadIdx.x + GV_KEEP * 256) * 8; c < K; c += 2048) {
-    float v[8];
+    float v[8], w[8];
     value(c, v);
-    put(c, v);
+    load8(in.w + c, w);
+    put(c, v, w);
   }
 }
 
+// (every operand of the kept chunks is requested before the first sum)
 template <typename T>
 __device__ void prepare_post(const GemvInput& in, int b, int K, T* xs, float* red, bool lead) {
   const long long o = static_cast<long long>(b) * K;
   const float* x = static_cast<const float*>(in.x) + o;
-  float keep[GV_KEEP][8];
+  float keep[GV_KEEP][8], xk[GV_KEEP][8], ak[GV_KEEP][8], wk[GV_KEEP][8];
   auto branch = [&](int c, float (&v)[8]) { load8(in.a + o + c, v); };
-#pragma unroll
-  for (int k = 0; k < GV_KEEP; ++k) {
-    const int c = (threadIdx.x + k * 256) * 8;
-    if (c < K) branch(c, keep[k]);
-  }
+  kept_chunks(K, [&](int k, int c) { branch(c, keep[k]); load8(x + c, xk[k]); load8(in.wa + c, ak[k]); load8(in.w + c, wk[k]); });
   const RowStat sa = row_stat<GV_KEEP>(keep, in.n, K, in.eps, in.layer != 0, red, branch);
-  auto add = [&](int c, float (&v)[8]) {           // branch values -> the new stream
-    float u[8], p[8];
-    load8(x + c, u);
-    load8(in.wa + c, p);
+  auto add = [&](float (&v)[8], const float (&u)[8], const float (&p)[8]) {           // branch values -> the new stream
 #pragma unroll
     for (int i = 0; i < 8; ++i) v[i] = u[i] + (v[i] - sa.mean) * sa.r * p[i];
   };
-  auto value = [&](int c, float (&v)[8]) { branch(c, v); add(c, v); };
-#pragma unroll
-  for (int k = 0; k < GV_KEEP; ++k) {
-    const int c = (threadIdx.x + k * 256) * 8;
-    if (c < K) add(c, keep[k]);
-  }
+  auto value = [&](int c, float (&v)[8]) {
+    float u[8], p[8];
+    branch(c, v);
+    load8(x + c, u);
+    load8(in.wa + c, p);
+    add(v, u, p);
+  };
+  kept_chunks(K, [&](int k, int) { add(keep[k], xk[k], ak[k]); });
   const RowStat st = row_stat<GV_KEEP>(keep, in.n, K, in.eps, in.layer != 0, red, value);
-  auto put = [&](int c, const float (&v)[8]) {
+  auto put = [&](int c, const float (&v)[8], float (&w)[8]) {
     if (lead) store8(in.x_out + o + c, v);
-    float w[8];
-    load8(in.w + c, w);
 #pragma unroll
     for (int i = 0; i < 8; ++i) w[i] *= (v[i] - st.mean) * st.r;
     store8(xs + c, w);
     if (lead && in.xn_out) store8(static_cast<T*>(in.xn_out) + o + c, w);
   };
-#pragma unroll
-  for (int k = 0; k < GV_KEEP; ++k) {
-    const int c = (threadIdx.x + k * 256) * 8;
-    if (c < K) put(c, keep[k]);
-  }
+  kept_chunks(K, [&](int k, int c) { put(c, keep[k], wk[k]); });
   for (int c = (threadIdx.x + GV_KEEP * 256) * 8; c < K; c += 2048) {
-    float v[8];
+    float v[8], w[8];
     value(c, v);
-    put(c, v);
+    load8(in.w + c, w);
+    put(c, v, w);
   }
 }
 

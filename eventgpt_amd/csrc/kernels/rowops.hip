@@ -35,8 +35,8 @@ void launch_embed_rows(const int* tok, const void* embed, bool f32, float scale,
 // The residual kernels.  MODE 0: xn = norm(x).  MODE 1: x += a first.  MODE 2: x += (norm(a) wa + norm(b) wb) / 2
 // first.  MODE 3: x += norm(a) wa first.  MODE 4: the same (or x += y without wa) with y the weighted sum of a few
 // rows of another matrix.  norm: RMS, or layer norm (LN).  A thread keeps its first NC chunks of eight in registers
-// between the passes.
-template <typename T, int MODE, bool LN>
+// between the passes; MODE 3 and 4 request the stream and the branch's weights with the branch.
+template <typename T, int MODE, bool LN, int NC>
 __global__ __launch_bounds__(256) void residual_norm_kernel(float* __restrict__ x, const int* __restrict__ sel,
                                                             SrcRows a, SrcRows b, MixRows mix, const float* __restrict__ wa,
                                                             const float* __restrict__ wb, const float* __restrict__ w,
@@ -44,8 +44,9 @@ __global__ __launch_bounds__(256) void residual_norm_kernel(float* __restrict__ 
   __shared__ float red[16];
   const long long row = blockIdx.x, xrow = MODE == 0 && sel ? sel[row] : row;
   float* xr = x + xrow * ld;
-  constexpr int NC = 4;       // 8192 columns stay in registers
   float keep[NC][8];
+  constexpr int NX = MODE >= 3 ? NC : 1;
+  float xk[NX][8], ak[NX][8];
   float ra = 0.f, rb = 0.f;
   RowStat sy{0.f, 1.f};
   auto branch = [&](int c, float (&v)[8]) {          // MODE 3 and 4: the sublayer's output
@@ -81,26 +82,20 @@ __global__ __launch_bounds__(256) void residual_norm_kernel(float* __restrict__ 
 #pragma unroll
     for (int k = 0; k < NC; ++k) {
       const int c = (threadIdx.x + k * 256) * 8;
-      if (c < ld) branch(c, keep[k]);
+      if (c < ld) {
+        branch(c, keep[k]);
+        load8(xr + c, xk[k]);
+        if (MODE == 3 || wa) load8(wa + c, ak[k]);       // (zero in the padding)
+      }
     }
     if (MODE == 3 || wa) sy = row_stat<NC>(keep, n, ld, eps, LN, red, branch);
   }
-  // the new stream: v holds the branch's values (MODE 3 and 4) on entry
+  auto post = [&](float (&v)[8], const float (&u)[8], const float (&p)[8]) {       // branch values -> the new stream
+#pragma unroll
+    for (int i = 0; i < 8; ++i) v[i] = MODE == 3 || wa ? u[i] + (v[i] - sy.mean) * sy.r * p[i] : u[i] + v[i];
+  };
   auto value = [&](int c, float (&v)[8]) {
-    if constexpr (MODE >= 3) {
-      float p[8], u[8];
-      load8(xr + c, u);
-      if (MODE == 3 || wa) {
-        load8(wa + c, p);       // (zero in the padding)
-#pragma unroll
-        for (int i = 0; i < 8; ++i) v[i] = u[i] + (v[i] - sy.mean) * sy.r * p[i];
-      } else {
-#pragma unroll
-        for (int i = 0; i < 8; ++i) v[i] += u[i];
-      }
-    } else {
-      load8(xr + c, v);
-    }
+    load8(xr + c, v);
     if constexpr (MODE == 1) {
       float t[8];
       src8(a, row, c, t);
@@ -121,13 +116,27 @@ __global__ __launch_bounds__(256) void residual_norm_kernel(float* __restrict__ 
 #pragma unroll
   for (int k = 0; k < NC; ++k) {
     const int c = (threadIdx.x + k * 256) * 8;
-    if (c < ld) value(c, keep[k]);
+    if (c >= ld) continue;
+    if constexpr (MODE >= 3) {
+      post(keep[k], xk[k], ak[k]);
+      store8(xr + c, keep[k]);
+    } else {
+      value(c, keep[k]);
+    }
   }
   if constexpr (MODE != 0)
     for (int c = (threadIdx.x + NC * 256) * 8; c < ld; c += 2048) {
       float v[8];
-      branch(c, v);
-      value(c, v);
+      if constexpr (MODE >= 3) {
+        float u[8], p[8];
+        branch(c, v);
+        load8(xr + c, u);
+        if (MODE == 3 || wa) load8(wa + c, p);
+        post(v, u, p);
+        store8(xr + c, v);
+      } else {
+        value(c, v);
+      }
     }
   if (w == nullptr) return;
   // each thread re-reads what it wrote
@@ -156,10 +165,12 @@ static void launch_residual(float* x, const int* sel, const SrcRows& a, const Sr
                             const float* wb, const float* w, void* xn, bool f32, int rows, int n, int ld, float eps,
                             bool layer, hipStream_t st) {
 #define EVGPT_RES(T, LN) \
-  hipLaunchKernelGGL((residual_norm_kernel<T, MODE, LN>), dim3(rows), dim3(256), 0, st, x, sel, a, b, mix, wa, wb, w, \
-                     static_cast<T*>(xn), n, ld, eps)
-  if (layer) { if (f32) EVGPT_RES(float, true); else EVGPT_RES(bf16_t, true); }
-  else { if (f32) EVGPT_RES(float, false); else EVGPT_RES(bf16_t, false); }
+  if (ld <= 4096) hipLaunchKernelGGL((residual_norm_kernel<T, MODE, LN, 2>), dim3(rows), dim3(256), 0, st, x, sel, a, b, mix, wa, wb, w, \
+                                     static_cast<T*>(xn), n, ld, eps); \
+  else hipLaunchKernelGGL((residual_norm_kernel<T, MODE, LN, 4>), dim3(rows), dim3(256), 0, st, x, sel, a, b, mix, wa, wb, w, \
+                          static_cast<T*>(xn), n, ld, eps)
+  if (layer) { if (f32) { EVGPT_RES(float, true); } else { EVGPT_RES(bf16_t, true); } }
+  else { if (f32) { EVGPT_RES(float, false); } else { EVGPT_RES(bf16_t, false); } }
 #undef EVGPT_RES
 }
 void launch_norm_rows(const float* x, const int* sel, const float* w, void* xn, bool f32, int rows, int n, int ld,

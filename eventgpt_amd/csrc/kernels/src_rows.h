@@ -56,19 +56,20 @@ __device__ __forceinline__ float sumsq8(const float (&v)[8]) {
   return s;
 }
 
+// eight columns of a section of `n` true columns; zeros past them
+__device__ __forceinline__ void section8(const SrcRows& s, long long row, int col, int n, int c, float (&v)[8]) {
+  if (c + 8 <= n) { src8(s, row, col + c, v); return; }
+#pragma unroll
+  for (int i = 0; i < 8; ++i) v[i] = c + i < n ? src1(s, row, col + c + i) : 0.f;
+}
 // RMS norm of `n` columns of a projection row by one wave, stored with zeros up to `ld` columns
 template <typename T>
 __device__ __forceinline__ void latent_row(const SrcRows& s, long long row, int col, int n, int ld, const float* w, float eps,
                                            T* out, int lane) {
-  auto value = [&](int c, float (&v)[8]) {
-    if (c + 8 <= n) { src8(s, row, col + c, v); return; }
-#pragma unroll
-    for (int i = 0; i < 8; ++i) v[i] = c + i < n ? src1(s, row, col + c + i) : 0.f;
-  };
   float v0[8], ss = 0.f;
   for (int c = lane * 8; c < ld; c += 512) {
     float v[8];
-    value(c, v);
+    section8(s, row, col, n, c, v);
     ss += sumsq8(v);
     if (c == lane * 8)
 #pragma unroll
@@ -81,7 +82,7 @@ __device__ __forceinline__ void latent_row(const SrcRows& s, long long row, int 
 #pragma unroll
       for (int i = 0; i < 8; ++i) v[i] = v0[i];
     } else {
-      value(c, v);
+      section8(s, row, col, n, c, v);
     }
     load8(w + c, g);
 #pragma unroll
@@ -91,47 +92,60 @@ __device__ __forceinline__ void latent_row(const SrcRows& s, long long row, int 
 }
 // Mean (0 for an RMS norm) and reciprocal root of the mean square (of the deviations) of a row of `n` true
 // columns, `ld` padded ones, by a block of 256 threads.  keep: the thread's first NC chunks of eight columns, chunk
-// (threadIdx.x + k * 256) * 8; far(c, v) gives a chunk past them again.  Padding columns hold zeros.
+// (threadIdx.x + k * 256) * 8; far(c, v) gives a chunk past them again.  Padding columns hold zeros.  Layer norm: every
+// wave takes the squares about its own mean, and the four waves' counts, means and squares are put together.
 struct RowStat { float mean, r; };
 template <int NC, typename Far>
 __device__ __forceinline__ RowStat row_stat(const float (&keep)[NC][8], int n, int ld, float eps, bool layer, float* red,
                                             Far far) {
-  const float inv_n = 1.f / static_cast<float>(n);
-  float mean = 0.f;
-  if (layer) {
-    float s = 0.f;
+  auto each = [&](auto f) {
 #pragma unroll
-    for (int k = 0; k < NC; ++k)
-      if (static_cast<int>(threadIdx.x + k * 256) * 8 < ld)
-#pragma unroll
-        for (int i = 0; i < 8; ++i) s += keep[k][i];
+    for (int k = 0; k < NC; ++k) {
+      const int c = (threadIdx.x + k * 256) * 8;
+      if (c < ld) f(c, keep[k]);
+    }
     for (int c = (threadIdx.x + NC * 256) * 8; c < ld; c += 2048) {
       float v[8];
       far(c, v);
-#pragma unroll
-      for (int i = 0; i < 8; ++i) s += v[i];
-    }
-    mean = block_sum(s, red) * inv_n;
-  }
-  float ss = 0.f;
-  auto add = [&](int c, const float (&v)[8]) {
-#pragma unroll
-    for (int i = 0; i < 8; ++i) {
-      const float d = layer && c + i >= n ? 0.f : v[i] - mean;
-      ss += d * d;
+      f(c, v);
     }
   };
+  if (!layer) {
+    float ss = 0.f;
+    each([&](int, const float (&v)[8]) { ss += sumsq8(v); });
+    return {0.f, rsqrtf(block_sum(ss, red) / static_cast<float>(n) + eps)};
+  }
+  float s = 0.f, cnt = 0.f;
+  each([&](int c, const float (&v)[8]) {
 #pragma unroll
-  for (int k = 0; k < NC; ++k) {
-    const int c = (threadIdx.x + k * 256) * 8;
-    if (c < ld) add(c, keep[k]);
+    for (int i = 0; i < 8; ++i) s += v[i];
+    cnt += static_cast<float>(min(max(n - c, 0), 8));
+  });
+  cnt = wave_sum(cnt);
+  const float mw = wave_sum(s) / fmaxf(cnt, 1.f);
+  float ss = 0.f;
+  each([&](int c, const float (&v)[8]) {
+#pragma unroll
+    for (int i = 0; i < 8; ++i) {
+      const float d = c + i < n ? v[i] - mw : 0.f;
+      ss += d * d;
+    }
+  });
+  ss = wave_sum(ss);
+  const int wid = threadIdx.x >> 6;
+  __syncthreads();
+  if ((threadIdx.x & 63) == 0) { red[wid] = cnt; red[4 + wid] = mw; red[8 + wid] = ss; }
+  __syncthreads();
+  float mean = 0.f, sq = 0.f;
+#pragma unroll
+  for (int w = 0; w < 4; ++w) mean += red[w] * red[4 + w];
+  mean /= static_cast<float>(n);
+#pragma unroll
+  for (int w = 0; w < 4; ++w) {
+    const float d = red[4 + w] - mean;
+    sq += red[8 + w] + red[w] * d * d;
   }
-  for (int c = (threadIdx.x + NC * 256) * 8; c < ld; c += 2048) {
-    float v[8];
-    far(c, v);
-    add(c, v);
-  }
-  return {mean, rsqrtf(block_sum(ss, red) * inv_n + eps)};
+  return {mean, rsqrtf(sq / static_cast<float>(n) + eps)};
 }
 
 }  // namespace evgpt

@@ -486,7 +486,7 @@ class LatentAttentionMixer(Mixer):
 
     def splits(self, rows: int) -> int:
         """Key splits of the attention over the cache: about one workgroup per CU."""
-        tiles = -(-self.spec.heads // 16)
+        tiles = -(-self.spec.heads // 32)
         return max(1, min(64, 256 // max(1, rows * tiles)))
 
     def absorbs(self, rows: RowBatch) -> bool:
@@ -587,7 +587,7 @@ class MoE(Mixer):
             stream.leave(y)
             return
         xn = stream.normed(norm)
-        logits = raw.linear(xn, self.w_router, True)
+        logits = raw.linear_slabs(xn, self.w_router) if rows.decode else raw.linear(xn, self.w_router, True)
         idx, weights = raw.moe_route(logits, self.bias, top)
         perm, inv, start = raw.moe_group(idx, self.spec.experts)
         h = raw.moe_linear(xn, self.w_gate_up, start, perm, top, self.act)
