@@ -146,6 +146,11 @@ __device__ __forceinline__ int xcd_remap(int id, int n) {
   return base + (id >> 3);
 }
 
+__device__ __forceinline__ int wave_sum_int(int v) {
+#pragma unroll
+  for (int off = 32; off > 0; off >>= 1) v += __shfl_xor(v, off, 64);
+  return v;
+}
 // Tiles of a grouped product: group e has rows start[e] .. start[e + 1], cut into row tiles of `bm`, each with `tiles_n`
 // column tiles; groups follow each other.  The wave finds the group of `tile`, which becomes the tile's index within
 // it; returns -1 past the last tile.
@@ -169,6 +174,12 @@ __device__ __forceinline__ int group_of_tile(const int* start, int groups, int b
     tile -= __builtin_amdgcn_readlane(sum, 63);
   }
   return -1;
+}
+// how many there are
+__device__ __forceinline__ int group_tiles(const int* start, int groups, int bm, int tiles_n) {
+  int n = 0;
+  for (int e = threadIdx.x & 63; e < groups; e += 64) n += (start[e + 1] - start[e] + bm - 1) / bm * tiles_n;
+  return __builtin_amdgcn_readfirstlane(wave_sum_int(n));
 }
 
 }  // namespace evgpt

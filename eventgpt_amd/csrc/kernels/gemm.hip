@@ -781,8 +781,9 @@ static void launch_fewrow(const GemmParams& p, hipStream_t st) {
 // into zero fills of images nobody reads, which keeps the vmcnt arithmetic uniform.
 // BMT = 128: the same schedule on a 128 x 256 tile (each wave 64 x 64; the A images are 64 rows, one staging
 // instruction per wave; 8 MFMAs per phase) for row counts that fill 256-row tiles badly.  K-contiguous A only.
-template <bool AT, bool BT, int BMT = 256>
+template <bool AT, bool BT, int BMT = 256, bool GRP = false>
 __global__ __launch_bounds__(512) void gemm256_kernel(GemmParams p) {
+  static_assert(!GRP || (!AT && !BT && BMT == 256), "grouped products: K-contiguous operands, 256-row tiles");
   static_assert(BMT == 256 || (BMT == 128 && !AT), "128-row variant: K-contiguous A");
   constexpr int BM = BMT, BN = 256, A_HALF = BM * 64, W_HALF = 16384, TILE = 2 * A_HALF + 2 * W_HALF;
   constexpr int IS = BM / 64;          // 16-row tiles of one wave in one A image
@@ -795,7 +796,11 @@ __global__ __launch_bounds__(512) void gemm256_kernel(GemmParams p) {
   const int wr = wid >> 2, wc = wid & 3;
   const int bn_out = p.glu_half ? BN / 2 : BN;      // gated mode: W-sub0 holds gate rows, W-sub1 the up rows
   const int tiles_n = (p.N + bn_out - 1) / bn_out, tiles_m = (p.M + BM - 1) / BM;
-  const int total = tiles_m * tiles_n * p.splitk;
+  int total = tiles_m * tiles_n * p.splitk;
+  if constexpr (GRP) {
+    total = group_tiles(p.grp_start, p.grp_count, BM, tiles_n);
+    if (static_cast<int>(blockIdx.x) >= total) return;
+  }
 
   // The grid is at most one workgroup per CU and a workgroup walks the tiles blockIdx.x, blockIdx.x + gridDim.x,
   // ... (gridDim.x is a multiple of 8 or the whole tile count, so a workgroup stays on its XCD's range of
@@ -804,6 +809,9 @@ __global__ __launch_bounds__(512) void gemm256_kernel(GemmParams p) {
   struct Tile {
     int m0, n0, tn, ksplit, k_begin, nk;
     int voff_a[2], voff_w[2];      // per-lane source offsets of sub 0; sub 1 and the K-tile move the descriptor base
+    // grouped: the group's first row, its rows, its weights, and the offsets of A-sub1 (whose rows are gathered too)
+    int first, rows, voff_a1[2];
+    const bf16_t* w;
   };
   auto locate = [&](int t, Tile& c) {
     const int bid = xcd_remap(t, total);
@@ -812,7 +820,16 @@ __global__ __launch_bounds__(512) void gemm256_kernel(GemmParams p) {
     c.k_begin = c.ksplit * p.k_per_split;
     c.nk = min(p.k_per_split, p.K - c.k_begin) / BK;
     int tm, tnn;
-    tile_walk(tile, tiles_m, tiles_n, p.group_m, tm, tnn);
+    if constexpr (GRP) {
+      int within = bid;
+      const int e = max(group_of_tile(p.grp_start, p.grp_count, BM, tiles_n, within), 0);
+      c.first = p.grp_start[e];
+      c.rows = p.grp_start[e + 1] - c.first;
+      c.w = p.W + e * p.grp_wstride;
+      tile_walk(within, (c.rows + BM - 1) / BM, tiles_n, p.group_m, tm, tnn);
+    } else {
+      tile_walk(tile, tiles_m, tiles_n, p.group_m, tm, tnn);
+    }
     c.tn = tnn;
     c.m0 = tm * BM;
     c.n0 = c.tn * bn_out;
@@ -827,7 +844,14 @@ __global__ __launch_bounds__(512) void gemm256_kernel(GemmParams p) {
       } else {                 // image [BM / 2 rows][64 k]: rows = two runs of QR (wave rows 0 / 1)
         const int lr = (wid * LA + (i < LA ? i : 0)) * 8 + (lane >> 3);
         const int cc = (lane & 7) ^ ((lr >> 1) & 7);
-        c.voff_a[i] = ((c.m0 + (lr / QR) * (BM / 2) + (lr % QR)) * p.lda + cc * 8) * 2;
+        const int row = c.m0 + (lr / QR) * (BM / 2) + (lr % QR);
+        if constexpr (GRP) {         // (rows past the group are not stored)
+          const int r0 = c.first + min(row, c.rows - 1), r1 = c.first + min(row + QR, c.rows - 1);
+          c.voff_a[i] = ((p.grp_perm ? p.grp_perm[r0] / p.grp_top : r0) * p.lda + cc * 8) * 2;
+          c.voff_a1[i] = ((p.grp_perm ? p.grp_perm[r1] / p.grp_top : r1) * p.lda + cc * 8) * 2;
+        } else {
+          c.voff_a[i] = (row * p.lda + cc * 8) * 2;
+        }
       }
       if constexpr (BT) {      // columns = four runs of 32 (wave columns 0..3)
         const int lin = rg * 64 + lane;
@@ -847,18 +871,18 @@ __global__ __launch_bounds__(512) void gemm256_kernel(GemmParams p) {
     const int k0 = c.k_begin + kt * BK, h = which & 1;
     if (which < 2) {
       unsigned char* dst = smem + (kt & 1) * TILE + which * A_HALF + wid * (LA * 1024);
-      const long long adv = AT ? 2ll * k0 * p.lda + 2ll * h * 64 : 2ll * k0 + 2ll * h * QR * p.lda;
+      const long long adv = AT ? 2ll * k0 * p.lda + 2ll * h * 64 : 2ll * k0 + (GRP ? 0 : 2ll * h * QR * p.lda);
       const long long left = bytes_a - adv;
       const unsigned char* src = reinterpret_cast<const unsigned char*>(p.A) + adv;
       const int lim = static_cast<int>(left > 0 ? left : 0);
-      buffer_to_lds16(src, lim, dst, c.voff_a[0]);
-      if constexpr (LA == 2) buffer_to_lds16(src, lim, dst + 1024, c.voff_a[1]);
+      buffer_to_lds16(src, lim, dst, GRP && h ? c.voff_a1[0] : c.voff_a[0]);
+      if constexpr (LA == 2) buffer_to_lds16(src, lim, dst + 1024, GRP && h ? c.voff_a1[1] : c.voff_a[1]);
     } else {
       unsigned char* dst = smem + (kt & 1) * TILE + 2 * A_HALF + (which - 2) * W_HALF + wid * 2048;
       const long long adv = BT ? 2ll * k0 * p.ldw + 2ll * h * 32
                                : 2ll * k0 + 2ll * h * (p.glu_half ? p.glu_half : 32) * p.ldw;
       const long long left = bytes_w - adv;
-      const unsigned char* src = reinterpret_cast<const unsigned char*>(p.W) + adv;
+      const unsigned char* src = reinterpret_cast<const unsigned char*>(GRP ? c.w : p.W) + adv;
       const int lim = static_cast<int>(left > 0 ? left : 0);
       buffer_to_lds16(src, lim, dst, c.voff_w[0]);
       buffer_to_lds16(src, lim, dst + 1024, c.voff_w[1]);
@@ -987,6 +1011,11 @@ __global__ __launch_bounds__(512) void gemm256_kernel(GemmParams p) {
     if (wr == 0) fence();   // both wave rows are past their last LDS read
     wait_vm<0>();           // zero fills past K have landed: the LDS can be staged again (or handed on)
     const int m0 = cur.m0, n0 = cur.n0, tn = cur.tn, ksplit = cur.ksplit;
+    GemmParams out = p;
+    if constexpr (GRP) {
+      out.M = cur.rows;
+      out.C += static_cast<size_t>(cur.first) * p.ldc;
+    }
     t += gridDim.x;
     const bool more = t < total;
     if (more) {
@@ -995,8 +1024,8 @@ __global__ __launch_bounds__(512) void gemm256_kernel(GemmParams p) {
     }
     if constexpr (BMT == 256) {
       // plain bf16 output with whole 16-byte chunks per row: whole-line stores through LDS
-      if (p.rows_epilogue) gemm_epilogue_rows<TM, TN>(p, acc, m0, n0, wr, wc, lane, smem + TILE + wid * 2048);
-      else gemm_epilogue<TM, TN, BM / 2, 64, 4>(p, acc, m0, n0, wr, wc, tn, tiles_n, ksplit, lane);
+      if (p.rows_epilogue) gemm_epilogue_rows<TM, TN>(GRP ? out : p, acc, m0, n0, wr, wc, lane, smem + TILE + wid * 2048);
+      else gemm_epilogue<TM, TN, BM / 2, 64, 4>(GRP ? out : p, acc, m0, n0, wr, wc, tn, tiles_n, ksplit, lane);
     } else {
       gemm_epilogue<TM, TN, BM / 2, 64, 4>(p, acc, m0, n0, wr, wc, tn, tiles_n, ksplit, lane);
     }
@@ -1010,14 +1039,15 @@ static bool g_persist_256 = true;     // false: one workgroup per tile (A/B runs
 void gemm_persist_256(bool on) { g_persist_256 = on; }
 void gemm_group_m(int g) { g_group_m = g; }
 
-template <bool AT, bool BT, int BM = 256>
-static void launch_256(const GemmParams& p, hipStream_t st) {
+// grp_rows > 0: grouped, that many rows in all groups
+template <bool AT, bool BT, int BM = 256, bool GRP = false>
+static void launch_256(const GemmParams& p, hipStream_t st, int grp_rows = 0) {
   const int bn_out = p.glu_half ? 128 : 256;
-  const int tiles = ((p.M + BM - 1) / BM) * ((p.N + bn_out - 1) / bn_out) * p.splitk;
+  const int tiles = (GRP ? grp_rows / BM + p.grp_count : (p.M + BM - 1) / BM) * ((p.N + bn_out - 1) / bn_out) * p.splitk;
   constexpr int smem = 2 * (2 * BM * 64 + 2 * 16384);
   static bool attr_set = false;
   if (!attr_set) {
-    hipFuncSetAttribute(reinterpret_cast<const void*>(&gemm256_kernel<AT, BT, BM>),
+    hipFuncSetAttribute(reinterpret_cast<const void*>(&gemm256_kernel<AT, BT, BM, GRP>),
                         hipFuncAttributeMaxDynamicSharedMemorySize, smem);
     attr_set = true;
   }
@@ -1038,7 +1068,7 @@ static void launch_256(const GemmParams& p, hipStream_t st) {
                     !p.raw_partial && !p.rope_cos && p.N % 8 == 0 && p.ldc % 8 == 0 &&
                     (reinterpret_cast<uintptr_t>(p.C) & 15) == 0 &&
                     (!p.res || (reinterpret_cast<uintptr_t>(p.res) & 15) == 0);
-  hipLaunchKernelGGL((gemm256_kernel<AT, BT, BM>), dim3(grid), dim3(512), smem, st, q);
+  hipLaunchKernelGGL((gemm256_kernel<AT, BT, BM, GRP>), dim3(grid), dim3(512), smem, st, q);
 }
 
 // out = act(sum_s partial[s] + bias) + res, 4 columns per thread
@@ -1418,7 +1448,8 @@ void launch_gemm_grouped(const bf16_t* A, const bf16_t* W, bf16_t* C, const int*
   const int per = rows / E;             // rows of an average group
   if (per < 48) launch_grp<32, 128, 1, 4, 4>(p, rows, st);
   else if (per < 192) launch_grp<64, 128, 2, 2, 3>(p, rows, st);
-  else launch_grp<128, 128, 2, 2, 2>(p, rows, st);
+  else if (per < 768) launch_grp<128, 128, 2, 2, 2>(p, rows, st);
+  else launch_256<false, false, 256, true>(p, st, rows);
 }
 
 // H[M, I] = act(A · Wgate^T) * (A · Wup^T), act = silu or (glu_act) gelu, with W = [gate rows | up rows] ([2I, K]): the gate/up

@@ -115,40 +115,52 @@ __global__ __launch_bounds__((WIDE ? 256 : 64) * KW) void head_linear_kernel(Hea
   const int n0 = blockIdx.x * (16 * WN) + wn * 16;
   const T* wp = static_cast<const T*>(a.w) + (static_cast<long long>(h) * a.N + min(n0 + fr, a.N - 1)) * K + g * 8;
   if constexpr (MERGE) {
-    for (int r = wid; r < 16; r += NT / 64) {
+    // A wave takes a whole row (WIDE), or its share of the columns of every row with four groups of lanes on different
+    // splits.  Maxima and sums (a lane per split, at most 64) are on their way together with the first partial rows.
+    constexpr int LG = WIDE ? 1 : 4, CL = 64 / LG, U = WIDE ? 8 : 4, STEP = WIDE ? 512 : CL * 8 * KW;
+    const int sg = lane / CL, c_lane = ((WIDE ? 0 : wk * CL) + lane % CL) * 8;
+    for (int r = WIDE ? wid : 0; r < 16; r += WIDE ? NT / 64 : 1) {
       if (r >= nr) {
         const float z[8] = {0, 0, 0, 0, 0, 0, 0, 0};
-        for (int c = lane * 8; c < K; c += 512) store8(xs + r * ldx + c, z);
+        for (int c = c_lane; c < K; c += STEP)
+          if (sg == 0) store8(xs + r * ldx + c, z);
         continue;
       }
       const int row = r0 + r;
       const int len = latent_len(a.pos, row, a.cap), per = split_keys(len, a.nsplit), used = (len + per - 1) / per;
       const float* ml = a.part_ml + (static_cast<long long>(row) * a.H + h) * a.nsplit * 2;
       const float* po = a.part_o + (static_cast<long long>(row) * a.H + h) * a.nsplit * K;
-      float mx = -INFINITY;
-      for (int s = lane; s < used; s += 64) mx = fmaxf(mx, ml[2 * s]);
-      mx = wave_max(mx);
-      float l = 0.f;
-      for (int s = lane; s < used; s += 64) l += __builtin_amdgcn_exp2f(ml[2 * s] - mx) * ml[2 * s + 1];
-      const float inv = 1.f / wave_sum(l);
-      for (int c = lane * 8; c < K; c += 512) {
+      float m = ml[2 * min(lane, used - 1)], f = 0.f, inv = 0.f;
+      const float l = ml[2 * min(lane, used - 1) + 1];
+      for (int c0 = 0; c0 < K; c0 += STEP) {
+        const int c = min(c0 + c_lane, K - 8);
         float o[8] = {0, 0, 0, 0, 0, 0, 0, 0};
-        for (int s0 = 0; s0 < used; s0 += 8) {
-          float v[8][8], f[8];
+        for (int s0 = 0; s0 < used; s0 += LG * U) {
+          float v[U][8];
 #pragma unroll
-          for (int u = 0; u < 8; ++u) {
-            const int s = min(s0 + u, used - 1);
-            load8(po + static_cast<long long>(s) * K + c, v[u]);
-            f[u] = s0 + u < used ? __builtin_amdgcn_exp2f(ml[2 * s] - mx) : 0.f;
+          for (int u = 0; u < U; ++u) load8(po + static_cast<long long>(min(s0 + u * LG + sg, used - 1)) * K + c, v[u]);
+          if (c0 == 0 && s0 == 0) {
+            if (lane >= used) m = -INFINITY;
+            f = __builtin_amdgcn_exp2f(m - wave_max(m));   // 0 past the last split
+            inv = 1.f / wave_sum(lane < used ? f * l : 0.f);
           }
 #pragma unroll
-          for (int u = 0; u < 8; ++u)
+          for (int u = 0; u < U; ++u) {
+            const int s = s0 + u * LG + sg;
+            const float t = __shfl(f, s & 63, 64), fu = s < used ? t : 0.f;
 #pragma unroll
-            for (int i = 0; i < 8; ++i) o[i] += f[u] * v[u][i];
+            for (int i = 0; i < 8; ++i) o[i] += fu * v[u][i];
+          }
         }
 #pragma unroll
-        for (int i = 0; i < 8; ++i) o[i] *= inv;
-        store8(xs + r * ldx + c, o);
+        for (int i = 0; i < 8; ++i) {
+          if constexpr (LG == 4) {
+            o[i] += __shfl_xor(o[i], 16, 64);
+            o[i] += __shfl_xor(o[i], 32, 64);
+          }
+          o[i] *= inv;
+        }
+        if (sg == 0 && c0 + c_lane < K) store8(xs + r * ldx + c, o);
       }
     }
   } else {

@@ -796,7 +796,7 @@ Tensor latent_attend(const Tensor& q, const Tensor& cache, const OptTensor& row_
     return head_linear(o.view({M, H * R}), w_v, gate, gcol);
   }
   TORCH_CHECK(R == 64 || R % 128 == 0, "latent_attend: R 64 or a multiple of 128");
-  nsplit = std::min<int64_t>(std::max<int64_t>(nsplit, 1), 256);
+  nsplit = std::min<int64_t>(std::max<int64_t>(nsplit, 1), 64);
   Tensor po = at::empty({M, H, nsplit, R}, q.options().dtype(at::kFloat)), pm = at::empty({M, H, nsplit, 2}, q.options().dtype(at::kFloat));
   evgpt::launch_latent_attend(bptr(q), bptr(cache), po.data_ptr<float>(), pm.data_ptr<float>(), iptr(row_slot), pos.data_ptr<int>(), (int)M,
                               (int)H, (int)R, (int)cap, (int)nsplit, (float)scale, cur_stream());

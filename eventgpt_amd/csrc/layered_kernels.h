@@ -135,7 +135,7 @@ struct HeadLinearArgs {
 };
 void launch_head_linear(const HeadLinearArgs& a, bool f32, int rows, hipStream_t st);
 // partial attention of q [rows][H][R] over positions 0 .. pos[row] of the rows' caches: part_o [rows][H][nsplit][R],
-// part_ml [rows][H][nsplit][2] (maximum in log2 units, sum).  R: 64, 128, 256, 384 or 512
+// part_ml [rows][H][nsplit][2] (maximum in log2 units, sum).  R: 64, 128, 256, 384 or 512; at most 64 splits
 void launch_latent_attend(const bf16_t* q, const bf16_t* cache, float* part_o, float* part_ml, const int* row_slot,
                           const int* pos, int rows, int H, int R, int cap, int nsplit, float scale, hipStream_t st);
 

@@ -587,7 +587,7 @@ class MoE(Mixer):
             stream.leave(y)
             return
         xn = stream.normed(norm)
-        logits = raw.linear_slabs(xn, self.w_router) if rows.decode else raw.linear(xn, self.w_router, True)
+        logits = raw.linear_slabs(xn, self.w_router)
         idx, weights = raw.moe_route(logits, self.bias, top)
         perm, inv, start = raw.moe_group(idx, self.spec.experts)
         h = raw.moe_linear(xn, self.w_gate_up, start, perm, top, self.act)

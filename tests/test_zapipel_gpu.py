@@ -308,22 +308,26 @@ def test_sorting_by_expert(raw, dev, M, E, top):
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("counts", [[1], [3, 0, 7, 0, 1], [33, 64, 0, 65, 20], [100, 1, 130, 90], [300, 129, 0, 500, 128, 255]])
-def test_grouped_products(raw, dev, dtype, counts):
-    """Every tile size (by the average group), empty and uneven groups, gathered and consecutive rows, all activations."""
-    E, K, N, top = len(counts), 192, 320, 2
+@pytest.mark.parametrize("counts,K,N", [([1], 192, 320), ([3, 0, 7, 0, 1], 192, 320), ([33, 64, 0, 65, 20], 192, 320),
+                                        ([100, 1, 130, 90], 192, 320), ([300, 129, 0, 500, 128, 255], 192, 320),
+                                        ([1300, 257, 0, 1600], 192, 320), ([1800, 1500], 64, 4736)])
+def test_grouped_products(raw, dev, dtype, counts, K, N):
+    """Every tile size (by the average group), more tiles than workgroups, empty and uneven groups, gathered and consecutive
+    rows, all activations."""
+    E, top = len(counts), 2
     rows = sum(counts)
     M = -(-rows // top)
-    if M * top > rows:
-        counts = counts[:-1] + [counts[-1] + M * top - rows]
-        rows = M * top
+    counts = counts[:-1] + [counts[-1] + M * top - rows]
+    rows = M * top
     start = torch.tensor([0] + counts).cumsum(0)
-    who = torch.repeat_interleave(torch.arange(E), torch.tensor(counts))
     perm = torch.randperm(rows, generator=torch.Generator().manual_seed(rows))
     x, xr = typed(rnd(M, K), dtype, dev)
     w, wr = typed(rnd(E, N, K, seed=1, scale=K ** -0.5), dtype, dev)
     st, pm = start.to(dev, torch.int32), perm.to(dev, torch.int32)
-    y = (wr[who] @ xr[perm // top][..., None])[..., 0]
+
+    def grouped(a):
+        return torch.cat([a[start[e]:start[e + 1]] @ wr[e].T for e in range(E)])
+    y = grouped(xr[perm // top])
     tol = 2e-6 if dtype == F32 else 8e-3
     assert Z.rel_err(raw.moe_linear(x, w, st, pm, top, -1), y) < tol
     g, u = y.chunk(2, -1)
@@ -331,7 +335,7 @@ def test_grouped_products(raw, dev, dtype, counts):
     gelu = torch.nn.functional.gelu(g, approximate="tanh")
     assert Z.rel_err(raw.moe_linear(x, w, st, pm, top, GELU), gelu * u) < 2 * tol
     full, fr = typed(rnd(rows, K, seed=2), dtype, dev)
-    assert Z.rel_err(raw.moe_linear(full, w, st, None, 1, -1), (wr[who] @ fr[..., None])[..., 0]) < tol
+    assert Z.rel_err(raw.moe_linear(full, w, st, None, 1, -1), grouped(fr)) < tol
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
