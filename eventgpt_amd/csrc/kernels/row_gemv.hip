@@ -38,22 +38,23 @@ template <typename F> __device__ __forceinline__ void kept_chunks(int K, F f) {
   }
 }
 
-template <typename T>
+// ALL: either norm, the stream or columns of a projection; otherwise the RMS norm of the stream
+template <typename T, bool ALL>
 __device__ void prepare_norm(const GemvInput& in, int b, int K, T* xs, float* red, bool lead) {
   const float* x = static_cast<const float*>(in.x) + static_cast<long long>(b) * K;
-  const bool rows = in.kind == GV_ROWS;
+  const bool rows = ALL && in.kind == GV_ROWS;
   float keep[GV_KEEP][8], wk[GV_KEEP][8];
   auto value = [&](int c, float (&v)[8]) {
     if (!rows) load8(x + c, v);
     else section8(in.gate, b, in.gcol, in.n, c, v);
   };
   kept_chunks(K, [&](int k, int c) { value(c, keep[k]); load8(in.w + c, wk[k]); });
-  const RowStat st = row_stat<GV_KEEP>(keep, in.n, K, in.eps, in.layer != 0, red, value);
+  const RowStat st = row_stat<GV_KEEP>(keep, in.n, K, in.eps, ALL && in.layer != 0, red, value);
   auto put = [&](int c, const float (&v)[8], float (&w)[8]) {
 #pragma unroll
     for (int i = 0; i < 8; ++i) w[i] *= (v[i] - st.mean) * st.r;
     store8(xs + c, w);
-    if (lead && in.xn_out) store8(static_cast<T*>(in.xn_out) + static_cast<long long>(b) * K + c, w);
+    if (ALL && lead && in.xn_out) store8(static_cast<T*>(in.xn_out) + static_cast<long long>(b) * K + c, w);
   };
   kept_chunks(K, [&](int k, int c) { put(c, keep[k], wk[k]); });
   for (int c = (threadIdx.x + GV_KEEP * 256) * 8; c < K; c += 2048) {
@@ -205,16 +206,22 @@ __device__ void prepare_group(const GemvInput& in, int b, int K, T* xs, float* i
   }
 }
 
-// PLAIN: every problem reads its input rows from global memory; otherwise all are staged (PLAIN rows copied)
-template <typename T, int B, int EPI, bool PLAIN>
+// PREP_NONE: every problem reads its input rows from global memory; otherwise all are staged (PLAIN rows copied): PREP_RMS for
+// the RMS norm of the stream, branches and group norms, PREP_ALL for either norm of the stream, the norm after a
+// sublayer and columns of a projection, with the latent store and the finished rows.
+enum { PREP_NONE = 0, PREP_RMS = 1, PREP_ALL = 2 };
+template <typename T, int B, int EPI, int PREP>
 __global__ __launch_bounds__(256) void row_gemv_kernel(GemvCall call, int blocks0) {
   extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
   constexpr int CE = 16 / sizeof(T);                      // elements per 16-byte chunk
   __shared__ float part[2][4][GV_R * B];
   __shared__ float red[16];
-  if (call.latent.cache && blockIdx.x + 1 == gridDim.x) {
-    store_latents<T>(call.latent, B);
-    return;
+  constexpr bool PLAIN = PREP == PREP_NONE;
+  if constexpr (PREP == PREP_ALL) {
+    if (call.latent.cache && blockIdx.x + 1 == gridDim.x) {
+      store_latents<T>(call.latent, B);
+      return;
+    }
   }
   const bool second = call.count == 2 && static_cast<int>(blockIdx.x) >= blocks0;
   const GemvProblem& p = call.p[second ? 1 : 0];
@@ -243,8 +250,10 @@ __global__ __launch_bounds__(256) void row_gemv_kernel(GemvCall call, int blocks
   if constexpr (!PLAIN) {
     for (int b = 0; b < B; ++b) {
       T* xb = xs + static_cast<long long>(b) * K;
-      if (p.in.kind == GV_NORM || p.in.kind == GV_ROWS) prepare_norm(p.in, b, K, xb, red, blk == 0);
-      else if (p.in.kind == GV_POST) prepare_post(p.in, b, K, xb, red, blk == 0);
+      if constexpr (PREP == PREP_ALL) {
+        if (p.in.kind == GV_POST) prepare_post(p.in, b, K, xb, red, blk == 0);
+        else prepare_norm<T, true>(p.in, b, K, xb, red, blk == 0);
+      } else if (p.in.kind == GV_NORM) prepare_norm<T, false>(p.in, b, K, xb, red, blk == 0);
       else if (p.in.kind == GV_MERGE) prepare_merge(p.in, b, K, xb, red, blk == 0);
       else if (p.in.kind == GV_GROUP) prepare_group(p.in, b, K, xb, reinterpret_cast<float*>(smem + static_cast<long long>(B) * K * sizeof(T)));
       else
@@ -304,7 +313,7 @@ __global__ __launch_bounds__(256) void row_gemv_kernel(GemvCall call, int blocks
         const int r = tid / B, b = tid % B;
         float* y = p.y + static_cast<long long>(b) * p.ldy + u * GV_R + r;
         if constexpr (EPI == GV_ADD) *y += total(r * B + b);
-        else *y = call.finish ? soft_cap(total(r * B + b), call.scale, call.cap) : total(r * B + b);
+        else *y = PREP == PREP_ALL && call.finish ? soft_cap(total(r * B + b), call.scale, call.cap) : total(r * B + b);
       }
     }
     flip ^= 1;       // the next unit's partial sums go to the other buffer: one barrier per unit
@@ -338,11 +347,15 @@ static void launch_b(const GemvCall& c, size_t lds, hipStream_t st) {
   const int budget = g_blocks ? g_blocks : (B == 1 && c.count == 1 && (kind == GV_NORM || kind == GV_MERGE || kind == GV_POST) ? 512 : 768);
   const int b0 = blocks_of(c.p[0], c.count == 2 ? budget / 2 : budget), b1 = c.count == 2 ? blocks_of(c.p[1], budget / 2) : 0;
   const dim3 grid(b0 + b1 + (c.latent.cache ? 1 : 0)), block(256);
-  const bool plain = c.count == 1 && c.p[0].in.kind == GV_PLAIN;
-#define EVGPT_GEMV(E)                                                                              \
-  if (plain) hipLaunchKernelGGL((row_gemv_kernel<T, B, E, true>), grid, block, 0, st, c, b0);      \
-  else hipLaunchKernelGGL((row_gemv_kernel<T, B, E, false>), grid, block, lds, st, c, b0)
-  if (c.epilogue == GV_STORE) { EVGPT_GEMV(GV_STORE); }
+  const bool plain = c.count == 1 && kind == GV_PLAIN;
+  const bool all = c.count == 1 && (kind == GV_POST || kind == GV_ROWS || (kind == GV_NORM && (c.p[0].in.layer || c.p[0].in.xn_out || c.finish)));
+#define EVGPT_GEMV(E)                                                                                    \
+  if (plain) hipLaunchKernelGGL((row_gemv_kernel<T, B, E, PREP_NONE>), grid, block, 0, st, c, b0);       \
+  else hipLaunchKernelGGL((row_gemv_kernel<T, B, E, PREP_RMS>), grid, block, lds, st, c, b0)
+  // (nothing is added to the stream behind a PREP_ALL input)
+  if (all && c.epilogue == GV_GLU) hipLaunchKernelGGL((row_gemv_kernel<T, B, GV_GLU, PREP_ALL>), grid, block, lds, st, c, b0);
+  else if (all) hipLaunchKernelGGL((row_gemv_kernel<T, B, GV_STORE, PREP_ALL>), grid, block, lds, st, c, b0);
+  else if (c.epilogue == GV_STORE) { EVGPT_GEMV(GV_STORE); }
   else if (c.epilogue == GV_ADD) { EVGPT_GEMV(GV_ADD); }
   else { EVGPT_GEMV(GV_GLU); }
 #undef EVGPT_GEMV

@@ -568,7 +568,7 @@ Tensor gemv_norm(const Tensor& x, const Tensor& norm, int64_t n, double eps, con
     c.p[0].in.xn_out = xn_out->data_ptr();
   }
   if (scale.has_value()) {
-    TORCH_CHECK(act < 0 && cap >= 0, "gemv_norm: scaled rows");
+    TORCH_CHECK(act < 0 && cap >= 0 && c.p[0].in.kind != evgpt::GV_MERGE, "gemv_norm: scaled rows");
     c.finish = 1; c.scale = (float)*scale; c.cap = (float)cap;
   }
   const int64_t B = x.size(0), N = w.size(0);
